@@ -21,6 +21,8 @@ HEADERS = ["kh_common.h", "kh_gemv.h", "kh_attn.h", "kh_fused.h", "kh_q8ring.h",
            "kh_model_internal.h",
            "../../include/kuiper_hip.h"]
 ARCH = "gfx950"
+# no packed fp32 VALU forms (v_pk_{add,mul,fma}_f32): some have returned wrong results on this hardware pool
+DEVICE_FLAGS = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def _hipcc() -> str:
@@ -48,7 +50,7 @@ def build_lib(force: bool = False, verbose: bool = False) -> str:
     objs, procs = [], []
     for src in SOURCES:
         obj = os.path.join(LIB_DIR, os.path.splitext(src)[0] + ".o")
-        cmd = [_hipcc(), f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", "-Wall",
+        cmd = [_hipcc(), f"--offload-arch={ARCH}", *DEVICE_FLAGS, "-O3", "-std=c++17", "-fPIC", "-Wall",
                # no implicit FMA contraction: results must not depend on which kernel a stage is
                # inlined into (decode vs B-token prefill kernels are compared bit for bit) and the
                # CPU oracle is built the same way; explicit __builtin_fmaf calls stay FMAs
@@ -96,7 +98,7 @@ def build_variant(name: str, defines: list[str], commit: str | None = None) -> s
         if not os.path.exists(os.path.join(CSRC, src)):  # --variant-at an older commit: that source came later
             continue
         obj = os.path.join(od, os.path.splitext(src)[0] + ".o")
-        cmd = [_hipcc(), f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off", "-w"] + \
+        cmd = [_hipcc(), f"--offload-arch={ARCH}", *DEVICE_FLAGS, "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off", "-w"] + \
               [f"-D{d}" for d in defines] + ["-c", os.path.join(CSRC, src), "-o", obj]
         procs.append((cmd, subprocess.Popen(cmd)))
         objs.append(obj)

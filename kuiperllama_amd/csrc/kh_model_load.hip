@@ -323,13 +323,8 @@ static int kv_ensure_impl(kh_model* m, int row0, int rows, int layer);
 static void kv_release(kh_model* m);
 // Address ranges outlive the model that reserved them: kv_release hands a range (every chunk unmapped) to this
 // process-wide list and the next model whose caches reserve the same number of bytes takes it over; the list is never
-// emptied.  hipMemAddressFree is NOT called: on this runtime (ROCm 7.2) it dereferences a null pointer once in a few
-// thousand create / destroy cycles of a process that keeps mapping and unmapping chunks (tools/stress_destroy.py under
-// tools/dbg/segv_bt.c: the second of kv_release's two calls, inside libamdhip64; seen once in five runs of the GPU
-// suite, `profiles/r6_vmm_destroy_crash.txt`; the plain allocation survives 28 000 cycles).  A reservation is address
-// space only - no HBM, no page tables until a chunk is mapped - so the cost of keeping it is a few dozen distinct
-// sizes of a 47-bit space in the worst process this library has seen (its own test suite).
-// Hook KH_KV_VA_POOL=0: free the ranges as rounds 6's first version did (the stress tool uses it to show the crash).
+// emptied and hipMemAddressFree is never called: on ROCm 7.2 it can fail inside the runtime in a process that keeps
+// mapping and unmapping chunks.  A reservation is address space only - no HBM, no page tables until a chunk is mapped.
 struct VaPool {
   std::mutex mu;
   std::vector<std::pair<void*, size_t>> ranges;
@@ -358,10 +353,6 @@ static void* va_take(size_t bytes, size_t align) {
 }
 static void va_give(void* p, size_t bytes) {
   if (!p) return;
-  if (dbg_off("KH_KV_VA_POOL")) {
-    (void)hipMemAddressFree(p, bytes);
-    return;
-  }
   VaPool& vp = va_pool();
   std::lock_guard<std::mutex> g(vp.mu);
   vp.ranges.emplace_back(p, bytes);

@@ -6,7 +6,7 @@ cd "$(dirname "$0")/.."
 O=$PWD/gpurun_out; mkdir -p $O
 OUT=$O/r6_gemv_mfma_ab.txt
 B=$PWD/kuiperllama_amd/lib/mb_gemv_mfma
-[ -x $B ] || hipcc --offload-arch=gfx950 -O3 -std=c++17 -ffp-contract=off tools/mb_gemv_mfma.hip -o $B
+[ -x $B ] || hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -std=c++17 -ffp-contract=off tools/mb_gemv_mfma.hip -o $B
 : > $OUT
 for i in 1 2 3; do timeout 120 $B 16 20 2>&1 | grep -v amdgpu.ids | tee -a $OUT; done
 export TMPDIR=/tmp; cd /tmp

@@ -11,7 +11,7 @@
 //         B operand of the second product), O^T[d, head] += V^T[d, t] . P[t, head] as 16 more MFMAs (V rows as
 //         16-byte loads, the head dimension permuted d = 4 i + c so that a float4 feeds four d-tiles).
 // Both write the (M, L, o) partial of every (head, split); the host merges them and compares the two outputs.
-//   hipcc --offload-arch=gfx950 -O3 -std=c++17 -ffp-contract=off tools/mb_attn_mfma.hip -o kuiperllama_amd/lib/mb_attn_mfma
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -std=c++17 -ffp-contract=off tools/mb_attn_mfma.hip -o kuiperllama_amd/lib/mb_attn_mfma
 #include <hip/hip_runtime.h>
 #include <math.h>
 #include <stdio.h>

@@ -12,7 +12,7 @@
 // position: event-timed launch (hipGraph of the alternation, filler subtracted) and, from one traced launch per layer,
 // the critical path = per stamp the LATEST workgroup relative to the EARLIEST entry, and per-workgroup medians of the
 // phase lengths.
-//   hipcc --offload-arch=gfx950 -O3 -std=c++17 -ffp-contract=off -DKH_ATTN_TRACE tools/mb_attn_phases.hip -o kuiperllama_amd/lib/mb_attn_phases
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -std=c++17 -ffp-contract=off -DKH_ATTN_TRACE tools/mb_attn_phases.hip -o kuiperllama_amd/lib/mb_attn_phases
 #include <hip/hip_runtime.h>
 #include <math.h>
 #include <stdio.h>

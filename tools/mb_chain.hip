@@ -3,15 +3,14 @@
 //   Q2  slope / intercept of a hipGraph chain of dependent streaming kernels (what one hop costs)
 //   Q3  prefetching the wo slab on a parallel graph branch while a latency-bound "attention"
 //       kernel runs: does the consumer get faster?
-//   Q4  VALU issue rates that price the int8 dequant inner loop (v_fma_f32, v_pk_fma_f32,
+//   Q4  VALU issue rates that price the int8 dequant inner loop (v_fma_f32,
 //       v_cvt_f32_ubyteN, sdwa sign-extending convert)
-//   hipcc --offload-arch=gfx950 -O3 tools/mb_chain.hip -o kuiperllama_amd/lib/mb_chain
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 tools/mb_chain.hip -o kuiperllama_amd/lib/mb_chain
 #include <hip/hip_runtime.h>
 #include <cstdio>
 #include <cstdlib>
 #include <vector>
 typedef float f32x4 __attribute__((ext_vector_type(4)));
-typedef float f32x2 __attribute__((ext_vector_type(2)));
 #define CK(x) do { hipError_t e_ = (x); if (e_ != hipSuccess) { printf("HIP error %s at line %d\n", hipGetErrorString(e_), __LINE__); exit(1); } } while (0)
 
 // GEMV-shaped streaming read: one wave = one 2*U KiB tile (two "rows" of U KiB), tiles handed out
@@ -48,11 +47,9 @@ __global__ __launch_bounds__(512) void k_latency(const int* __restrict__ chase, 
   if (threadIdx.x == 0) out[blockIdx.x & 63] = (float)i;
 }
 
-template <int MODE>  // 0 v_fma_f32, 1 v_pk_fma_f32, 2 cvt_ubyte + fma, 3 sext byte cvt + fma
+template <int MODE>  // 0 v_fma_f32, 2 cvt_ubyte + fma, 3 sext byte cvt + fma
 __global__ __launch_bounds__(256) void k_alu(float* out, int iters, unsigned seed) {
   float a0 = threadIdx.x * 1e-3f, a1 = a0 + 1.f, a2 = a0 + 2.f, a3 = a0 + 3.f;
-  f32x2 p0 = {a0, a1}, p1 = {a2, a3}, p2 = {a1, a0}, p3 = {a3, a2};
-  const f32x2 m = {1.0001f, 0.9999f}, c = {1e-6f, -1e-6f};
   unsigned w = seed + threadIdx.x;
   for (int i = 0; i < iters; ++i) {
     if (MODE == 0) {
@@ -60,12 +57,6 @@ __global__ __launch_bounds__(256) void k_alu(float* out, int iters, unsigned see
       for (int k = 0; k < 16; ++k) {
         a0 = __builtin_fmaf(a0, 1.0001f, 1e-6f); a1 = __builtin_fmaf(a1, 0.9999f, 1e-6f);
         a2 = __builtin_fmaf(a2, 1.0001f, -1e-6f); a3 = __builtin_fmaf(a3, 0.9999f, -1e-6f);
-      }
-    } else if (MODE == 1) {
-#pragma unroll
-      for (int k = 0; k < 16; ++k) {
-        p0 = __builtin_elementwise_fma(p0, m, c); p1 = __builtin_elementwise_fma(p1, m, c);
-        p2 = __builtin_elementwise_fma(p2, m, c); p3 = __builtin_elementwise_fma(p3, m, c);
       }
     } else if (MODE == 2) {
 #pragma unroll
@@ -84,7 +75,7 @@ __global__ __launch_bounds__(256) void k_alu(float* out, int iters, unsigned see
       }
     }
   }
-  out[blockIdx.x * 256 + threadIdx.x] = a0 + a1 + a2 + a3 + p0.x + p0.y + p1.x + p1.y + p2.x + p2.y + p3.x + p3.y;
+  out[blockIdx.x * 256 + threadIdx.x] = a0 + a1 + a2 + a3;
 }
 
 static hipStream_t S, S2;
@@ -207,19 +198,18 @@ int main(int argc, char** argv) {
 
   // ---- Q4: VALU rates ------------------------------------------------------------------------------
   printf("## Q4 VALU: ns per 64 inner ops per wave-lane-set (grid 1024x256 = 16 waves/CU), lower = faster\n");
-  for (int mode = 0; mode < 4; ++mode) {
+  for (int mode : {0, 2, 3}) {
     const int iters = 4096;
     auto go = [&] {
       if (mode == 0) hipLaunchKernelGGL(k_alu<0>, dim3(1024), dim3(256), 0, S, out, iters, 7u);
-      else if (mode == 1) hipLaunchKernelGGL(k_alu<1>, dim3(1024), dim3(256), 0, S, out, iters, 7u);
       else if (mode == 2) hipLaunchKernelGGL(k_alu<2>, dim3(1024), dim3(256), 0, S, out, iters, 7u);
       else hipLaunchKernelGGL(k_alu<3>, dim3(1024), dim3(256), 0, S, out, iters, 7u);
     };
     float us = time_graph(go);
-    // per SIMD: 4 waves, each iters*64 "slots" (fma: 64 v_fma; pk: 64 v_pk_fma = 128 fma; cvt modes: 64 cvt+64 fma + lcg)
+    // per SIMD: 4 waves, each iters*64 "slots" (fma: 64 v_fma; cvt modes: 64 cvt+64 fma + lcg)
     const double slots = (double)iters * 64 * 4;  // wave-instruction slots per SIMD (nominal)
     printf("mode %d (%s): %.1f us -> %.2f cycles@2.4GHz per nominal slot per SIMD\n", mode,
-           mode == 0 ? "v_fma_f32" : mode == 1 ? "v_pk_fma_f32 (2 fma/slot)" : mode == 2 ? "cvt_ubyte+fma (2 ops/slot)" : "sext-byte cvt+fma",
+           mode == 0 ? "v_fma_f32" : mode == 2 ? "cvt_ubyte+fma (2 ops/slot)" : "sext-byte cvt+fma",
            us, us * 1e-6 * 2.4e9 / slots);
   }
   return 0;

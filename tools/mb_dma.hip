@@ -5,7 +5,7 @@
 //   V=2  as V=1 without nt
 //   V=3  plain global_load_dwordx4 into registers (16 per batch), no LDS (reference: the product's way)
 // DEPTH = batches of 16 pieces allowed in flight (vmcnt counts up to 63 only).
-//   hipcc --offload-arch=gfx950 -O3 tools/mb_dma.hip -o kuiperllama_amd/lib/mb_dma
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 tools/mb_dma.hip -o kuiperllama_amd/lib/mb_dma
 #include <hip/hip_runtime.h>
 #include <stdint.h>
 #include <stdio.h>

@@ -25,7 +25,7 @@
 // 64 only in this prototype; its summation order is its own (compared with tolerance, the GEMV stages
 // bit for bit).
 //
-//   hipcc --offload-arch=gfx950 -O3 -std=c++17 -ffp-contract=off tools/mb_engine.hip -o kuiperllama_amd/lib/mb_engine
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -std=c++17 -ffp-contract=off tools/mb_engine.hip -o kuiperllama_amd/lib/mb_engine
 //   mb_engine [1b|qwen|tiny] [pos] [reps]
 #include <hip/hip_runtime.h>
 #include <math.h>

@@ -2,7 +2,7 @@
 // (tools/f32ring.h) against the shipped register-tile kernels (kh_fused.h), same box, same slabs.
 // For every kernel: (1) outputs compared BITWISE with the shipped kernel's on the same inputs, (2) us per launch of a
 // hipGraph of NL launches over NL distinct weight slabs (nothing is served from a cache), best of 5.
-//   hipcc --offload-arch=gfx950 -O3 -ffp-contract=off -std=c++20 -w -I kuiperllama_amd/csrc -I tools tools/mb_f32ring.hip -o kuiperllama_amd/lib/mb_f32ring
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -ffp-contract=off -std=c++20 -w -I kuiperllama_amd/csrc -I tools tools/mb_f32ring.hip -o kuiperllama_amd/lib/mb_f32ring
 // argv[1]: 0 ffn13 only, 1 w2 only (default both); argv[2]: sweeps over the slabs per graph (default 2)
 #include <cstdio>
 #include <cstdlib>

@@ -11,7 +11,7 @@
 // Shapes: ffn13 (11008 (w1,w3) pairs x 4096, norm), qkv-like (6144 pairs x 4096, norm; the RoPE
 // epilogue is replaced by a plain store), wo (2048 pairs x 4096, SPLIT 2, no norm), w2 (2048 pairs
 // x 11008, SPLIT 4, 512 threads, no norm).  32 launches over distinct slabs per hipGraph, best of 5.
-//   hipcc --offload-arch=gfx950 -O3 -ffp-contract=off -I kuiperllama_amd/csrc tools/mb_gemv_ladder.hip -o kuiperllama_amd/lib/mb_gemv_ladder
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -ffp-contract=off -I kuiperllama_amd/csrc tools/mb_gemv_ladder.hip -o kuiperllama_amd/lib/mb_gemv_ladder
 #include <cstdio>
 #include <cstdlib>
 

@@ -19,7 +19,7 @@
 // in flight per wave (16 x dwordx4 per matrix pair tile), same launch geometry class (512 x 256 threads), the same
 // distinct weight slabs per launch of a captured graph (nothing is served from a cache).  Outputs are compared with
 // the VALU kernel's (summation order differs: tolerance, not bits).
-//   hipcc --offload-arch=gfx950 -O3 -std=c++17 -ffp-contract=off tools/mb_gemv_mfma.hip -o kuiperllama_amd/lib/mb_gemv_mfma
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -std=c++17 -ffp-contract=off tools/mb_gemv_mfma.hip -o kuiperllama_amd/lib/mb_gemv_mfma
 //   mb_gemv_mfma [slabs per graph = 16] [replays = 20] [only = 0 | 1 valu | 2 mfma16 | 3 mfma4]   (rocprofv3 passes)
 #include <hip/hip_runtime.h>
 #include <math.h>

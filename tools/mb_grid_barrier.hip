@@ -14,7 +14,7 @@
 //   E  nosync   : B without the barrier (wrong results; the pure streaming time of the phases)
 // The spin loops are bounded (an error flag is raised instead of hanging).  Results of A, B, C, D must be
 // identical (same arithmetic) — printed as a checksum.
-//   hipcc --offload-arch=gfx950 -O3 tools/mb_grid_barrier.hip -o kuiperllama_amd/lib/mb_grid_barrier
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 tools/mb_grid_barrier.hip -o kuiperllama_amd/lib/mb_grid_barrier
 #include <hip/hip_runtime.h>
 #include <cstdio>
 #include <cstdlib>

@@ -8,7 +8,7 @@
 //       re-reads its slice of the vector (sc1 loads) until every tag carries the current step.
 //       No counter, no fence, no barrier across workgroups.  Spins are bounded (error flag).
 // Same slabs, same tile shape (kh_gemv.h: a wave owns 2*U KiB), same vector length.
-//   hipcc --offload-arch=gfx950 -O3 tools/mb_handoff.hip -o kuiperllama_amd/lib/mb_handoff
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 tools/mb_handoff.hip -o kuiperllama_amd/lib/mb_handoff
 #include <hip/hip_runtime.h>
 #include <cstdint>
 #include <cstdio>

@@ -7,7 +7,7 @@
 // cannot be dropped).  32 launches over DISTINCT slabs in one hipGraph (weights never hit a cache),
 // timed with HIP events, best of 5; swept over grid sizes and U (16-byte loads per row in flight per
 // lane).  Output: us per launch and the fraction of 8 TB/s for the shape's algorithmic bytes.
-//   hipcc --offload-arch=gfx950 -O3 tools/mb_int8_floors.hip -o kuiperllama_amd/lib/mb_int8_floors
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 tools/mb_int8_floors.hip -o kuiperllama_amd/lib/mb_int8_floors
 #include <hip/hip_runtime.h>
 #include <cstdio>
 #include <cstdlib>

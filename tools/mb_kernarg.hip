@@ -9,7 +9,7 @@
 //     k_struct(Args a)                                    arguments through s_load
 //     k_scalar(const int* in, int* out, int a0 .. a5)     arguments preloaded (when the flag is given)
 //
-//   hipcc --offload-arch=gfx950 -O3 -std=c++17 -mllvm -amdgpu-kernarg-preload-count=16 tools/mb_kernarg.hip \
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -std=c++17 -mllvm -amdgpu-kernarg-preload-count=16 tools/mb_kernarg.hip \
 //         -o kuiperllama_amd/lib/mb_kernarg
 #include <hip/hip_runtime.h>
 #include <stdio.h>

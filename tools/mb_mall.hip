@@ -1,7 +1,7 @@
 // Microbenchmark: does the 256 MiB Infinity Cache (MALL) retain a weight slab between two
 // kernels, and do non-temporal loads hit in it?  Decides whether prefetching the next GEMV's
 // weights during the latency-bound attention kernel can pay.
-//   hipcc --offload-arch=gfx950 -O3 tools/mb_mall.hip -o kuiperllama_amd/lib/mb_mall
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 tools/mb_mall.hip -o kuiperllama_amd/lib/mb_mall
 #include <hip/hip_runtime.h>
 #include <cstdio>
 #include <vector>

@@ -2,7 +2,7 @@
 // 4.7-GB stream of non-temporal loads (the rest of a token's weights)?  If it did, a resident subset of the model
 // would be served from the memory-side cache in every token.  Per size S: A (S bytes) is read with plain loads, then
 // B (4.7 GB) with nt (or plain) loads, five rounds; the rate of A in rounds 2-5 against its cold rate.
-//   hipcc --offload-arch=gfx950 -O3 tools/mb_mall2.hip -o kuiperllama_amd/lib/mb_mall2
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 tools/mb_mall2.hip -o kuiperllama_amd/lib/mb_mall2
 #include <hip/hip_runtime.h>
 #include <cstdio>
 typedef float f32x4 __attribute__((ext_vector_type(4)));

@@ -23,7 +23,7 @@
 // recurrence stays bounded; the output of layer 15 feeds layer 0 of the next replay, so a stale read anywhere
 // changes the final bits: every variant must end with the SAME 2048 floats as the serial chain.
 //
-//   hipcc --offload-arch=gfx950 -O3 -std=c++17 -ffp-contract=off tools/mb_overlap.hip -o kuiperllama_amd/lib/mb_overlap
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -std=c++17 -ffp-contract=off tools/mb_overlap.hip -o kuiperllama_amd/lib/mb_overlap
 //   mb_overlap [reps]
 #include <hip/hip_runtime.h>
 #include <math.h>

@@ -2,7 +2,7 @@
 // LDS-DMA ring kernels (kh_fused_ring.h) on the Llama-2-7B int8 shapes (group 64), random weights.
 // For every kernel: (1) outputs compared BITWISE with the shipped kernel's on the same inputs, (2) us per launch of
 // a hipGraph of NL launches over NL distinct weight slabs (nothing is served from a cache), best of 5.
-//   hipcc --offload-arch=gfx950 -O3 -ffp-contract=off -std=c++20 -I kuiperllama_amd/csrc -I tools tools/mb_q8ring.hip -o kuiperllama_amd/lib/mb_q8ring
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -ffp-contract=off -std=c++20 -I kuiperllama_amd/csrc -I tools tools/mb_q8ring.hip -o kuiperllama_amd/lib/mb_q8ring
 #include <cstdio>
 #include <cstdlib>
 #include <cstring>

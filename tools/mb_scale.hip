@@ -5,7 +5,7 @@
 //   mode 1  + one dword scale load per dwordx4 (4 lanes share an address)      [shipped layout]
 //   mode 2  + ONE coalesced dword scale load per row per chunk (lane l <- scale[pi(l)])
 //   mode 3  + scale loads of mode 1 issued by one lane per quad only (exec-masked)
-//   hipcc --offload-arch=gfx950 -O3 tools/mb_scale.hip -o kuiperllama_amd/lib/mb_scale
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 tools/mb_scale.hip -o kuiperllama_amd/lib/mb_scale
 #include <hip/hip_runtime.h>
 #include <cstdio>
 #include <cstdlib>

@@ -3,7 +3,7 @@
 // distinct weight slabs as inside a decode step; the stamps of the last launch of the chain are read back: per wave
 // "last work item finished", per workgroup entry / end.  Reports percentiles of the wave finish times and the per-XCD
 // medians.  A wide spread at equal static work would mean a dynamic work distribution has something to win.
-//   hipcc --offload-arch=gfx950 -O3 -ffp-contract=off -std=c++20 -w -DKH_TRACE -I kuiperllama_amd/csrc -I tools tools/mb_skew.hip -o kuiperllama_amd/lib/mb_skew
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -ffp-contract=off -std=c++20 -w -DKH_TRACE -I kuiperllama_amd/csrc -I tools tools/mb_skew.hip -o kuiperllama_amd/lib/mb_skew
 #include <algorithm>
 #include <cstdio>
 #include <cstdlib>

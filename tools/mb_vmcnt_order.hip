@@ -5,7 +5,7 @@
 // older than the NDMA youngest operations has retired" if retirement is in order - and store the register.  A lane
 // that still holds the sentinel was read before its load landed.  Control: the same with NDMA further register loads
 // from the hot region instead of DMA (loads of one kind do retire in order).
-//   hipcc --offload-arch=gfx950 -O3 tools/mb_vmcnt_order.hip -o kuiperllama_amd/lib/mb_vmcnt_order
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 tools/mb_vmcnt_order.hip -o kuiperllama_amd/lib/mb_vmcnt_order
 #include <hip/hip_runtime.h>
 #include <stdint.h>
 #include <stdio.h>

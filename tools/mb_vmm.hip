@@ -6,7 +6,7 @@
 //           chunks and failed exactly there);
 //   part 2  mappings of ONE size (8 / 2 / 32 MiB) in random order over two interleaved 16-GiB reservations, unmapped and
 //           mapped again: never fails, 13-14 us per chunk - the form kv_ensure uses (and PyTorch's expandable segments).
-//   hipcc --offload-arch=gfx950 -O2 -std=c++17 -Wno-deprecated-declarations tools/mb_vmm.hip -o kuiperllama_amd/lib/mb_vmm
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O2 -std=c++17 -Wno-deprecated-declarations tools/mb_vmm.hip -o kuiperllama_amd/lib/mb_vmm
 #include <hip/hip_runtime.h>
 #include <stdio.h>
 #include <stdlib.h>

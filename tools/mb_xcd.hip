@@ -12,7 +12,7 @@
 // picks a same-XCD pair and a cross-XCD pair from what the launch reports.  Spins are bounded (a flavour that never
 // becomes visible reports "no progress").
 //
-//   hipcc --offload-arch=gfx950 -O3 -std=c++17 tools/mb_xcd.hip -o kuiperllama_amd/lib/mb_xcd
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -std=c++17 tools/mb_xcd.hip -o kuiperllama_amd/lib/mb_xcd
 #include <hip/hip_runtime.h>
 #include <stdio.h>
 #include <stdlib.h>
