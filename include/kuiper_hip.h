@@ -27,7 +27,7 @@
 extern "C" {
 #endif
 
-#define KH_VERSION 100 /* 0.1.0 */
+#define KH_VERSION 110 /* 0.1.1 */
 
 enum {
   KH_OK = 0,
@@ -47,7 +47,11 @@ int kh_version(void);
 int kh_device_count(void);
 
 enum { KH_ROPE_INTERLEAVED = 0, KH_ROPE_HALF = 1 };
-enum { KH_FAMILY_LLAMA = 0, KH_FAMILY_QWEN2 = 1 };
+/* KH_FAMILY_LAYERS: layer-list models - a checkpoint folder (config.json naming an architecture and its layers,
+ * model.safetensors).  The family and every constant come from config.json; opts->family, rope_* and rms_eps are ignored. */
+enum { KH_FAMILY_LLAMA = 0, KH_FAMILY_QWEN2 = 1, KH_FAMILY_LAYERS = 2 };
+/* storage type of weights, activations and cache; DEFAULT: fp32 for .bin images, bf16 for checkpoint folders */
+enum { KH_DTYPE_DEFAULT = 0, KH_DTYPE_BF16 = 1, KH_DTYPE_F32 = 2 };
 
 /* ============================ operator level ==========================================
  * One entry point per reference kernel typedef (kernels_interface.h). */
@@ -166,6 +170,8 @@ typedef struct kh_model_opts {
   int32_t max_seq_len; /* rows of KV cache + sin/cos to allocate; 0 = header seq_len */
   int32_t device;      /* HIP device ordinal (reference: cudaSetDevice(0)) */
   int32_t flags;       /* KH_FLAG_* bits, 0 = defaults */
+  int32_t dtype;       /* KH_DTYPE_* */
+  int32_t max_seqs;    /* sequences a layer-list model can hold at once (kh_seq_open); 0 = 1 */
 } kh_model_opts;
 /* decode attention at positions that need several time splits: merge the split partials inside the
  * attention launch (ticket + last arriver) instead of in the wo kernel that follows (the default) */
@@ -206,7 +212,8 @@ typedef struct kh_config {
   int32_t ring_selftest, attn_merge_selftest;
 } kh_config;
 
-/* Model::read_model_file + init (model.cpp:41-123, llama3.cpp:107-145) */
+/* Model::read_model_file + init (model.cpp:41-123, llama3.cpp:107-145).  A folder is taken as a checkpoint
+ * (config.json + model.safetensors), a file as a .bin image. */
 int kh_model_create_from_file(const char* path, const kh_model_opts* opts, kh_model** out);
 /* same, from the bytes of a .bin file already in host memory (header included) */
 int kh_model_create_from_host_image(const void* h_image, size_t nbytes,
@@ -217,6 +224,9 @@ int kh_model_create_from_host_image(const void* h_image, size_t nbytes,
 int kh_model_create_from_device_weights(const int32_t* h_header, const void* d_weight_data,
                                         size_t weight_nbytes, const kh_model_opts* opts,
                                         kh_model** out);
+/* a checkpoint already in host memory: the text of config.json and the bytes of model.safetensors */
+int kh_model_create_from_checkpoint(const char* h_config_json, size_t config_len, const void* h_safetensors,
+                                    size_t nbytes, const kh_model_opts* opts, kh_model** out);
 void kh_model_destroy(kh_model* m);
 int kh_model_get_config(const kh_model* m, kh_config* out);
 void* kh_model_stream(kh_model* m); /* the model's hipStream_t */
@@ -235,6 +245,34 @@ enum {
  * Synchronises the stream. exec: KH_EXEC_FUSED or KH_EXEC_UNFUSED. */
 int kh_model_predict(kh_model* m, int32_t token, int32_t pos, int32_t is_prompt, int32_t exec,
                      int32_t* h_next);
+/* Several sequences at once.  A sequence owns a slot: its cache rows and recurrent state.  kh_seq_open hands out a free
+ * slot at length 0 (KH_ERR_RANGE: all max_seqs slots are taken), kh_seq_close gives it back; what the slot held before
+ * never reaches the next sequence.  .bin models hold one sequence.  kh_model_generate* and kh_model_predict use slot 0
+ * and take it over from whoever opened it. */
+int kh_seq_open(kh_model* m, int32_t* seq);
+int kh_seq_close(kh_model* m, int32_t seq);
+int kh_seq_length(const kh_model* m, int32_t seq); /* tokens held; < 0: not open */
+/* One step of a batch: every entry appends n_tokens tokens to its sequence (different lengths in one batch; prompts,
+ * portions of prompts and single decoded tokens), each sequence at most once.  want = ascending places among an
+ * entry's tokens whose logits are copied to h_logits [sum of n_want][vocab], in the order of entries and want. */
+typedef struct kh_batch_entry {
+  int32_t seq, n_tokens;
+  const int32_t* tokens;
+  int32_t n_want;
+  const int32_t* want;
+} kh_batch_entry;
+int kh_model_forward(kh_model* m, const kh_batch_entry* entries, int32_t n_entries, float* h_logits);
+/* Greedy generation for several prompts as one batch (layer-list models): prompts run together, then every live
+ * sequence decodes one token per step; sequence i ends after max_new[i] tokens or at a token of h_stop.
+ * h_out [n_prompts][cap] receives the new tokens, h_n_out their numbers. */
+int kh_model_generate_batch(kh_model* m, int32_t n_prompts, const int32_t* const* h_prompts, const int32_t* n_prompt,
+                            const int32_t* max_new, const int32_t* h_stop, int32_t n_stop, int32_t* h_out, int32_t cap,
+                            int32_t* h_n_out);
+/* Residual stream after every layer run of the kh_model_forward calls that follow (tests, bring-up): run after run,
+ * [tokens of the call][dim], appended to h_buf (cap floats) until it is full; NULL ends it.  *n_written (may be NULL) =
+ * floats stored since the probe was set.  Layer-list models; a probed step runs on the pass kernels. */
+int kh_model_probe_residual(kh_model* m, float* h_buf, int64_t cap, int64_t* n_written);
+
 /* copy the last logits (kForwardOutput) to host */
 int kh_model_get_logits(kh_model* m, float* h_logits);
 /* device pointers of the KV cache [layer, cache_len, kv_dim] (tests) */

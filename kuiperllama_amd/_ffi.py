@@ -28,6 +28,8 @@ EXPORTS = [
     "kh_bpe_bos_id", "kh_bpe_eos_id", "kh_bpe_stop_id", "kh_bpe_encode", "kh_bpe_decode",
     "kh_model_generate", "kh_model_generate_until", "kh_model_first_sample", "kh_model_time_step", "kh_model_prefill", "kh_model_prefill_gemm", "kh_model_time_prefill", "kh_model_profile_kernel", "kh_model_profile_step", "kh_kclass_name",
     "kh_plan_decode_shapes", "kh_plan_decode_ring", "kh_plan_prefill_shape", "kh_plan_attention",
+    "kh_model_create_from_checkpoint", "kh_seq_open", "kh_seq_close", "kh_seq_length", "kh_model_forward",
+    "kh_model_generate_batch", "kh_model_probe_residual",
     "kh_debug_set", "kh_debug_get", "kh_debug_list",
 ]
 
@@ -38,6 +40,7 @@ KH_ERR_INTERNAL = -7
 KH_FLAG_ATTN_MERGE_IN_LAUNCH = 1
 KH_FLAG_ATTN_MERGE_FENCED = 2
 KH_FLAG_PREFILL_EXACT = 4
+KH_DTYPE_DEFAULT, KH_DTYPE_BF16, KH_DTYPE_F32 = 0, 1, 2
 
 
 class KhError(RuntimeError):
@@ -49,7 +52,12 @@ class KhError(RuntimeError):
 class ModelOpts(C.Structure):
     _fields_ = [("family", C.c_int32), ("is_quant", C.c_int32), ("rope_mode", C.c_int32),
                 ("rope_theta", C.c_float), ("rms_eps", C.c_float), ("max_seq_len", C.c_int32),
-                ("device", C.c_int32), ("flags", C.c_int32)]
+                ("device", C.c_int32), ("flags", C.c_int32), ("dtype", C.c_int32), ("max_seqs", C.c_int32)]
+
+
+class BatchEntry(C.Structure):
+    _fields_ = [("seq", C.c_int32), ("n_tokens", C.c_int32), ("tokens", C.POINTER(C.c_int32)), ("n_want", C.c_int32),
+                ("want", C.POINTER(C.c_int32))]
 
 
 class FirstSample(C.Structure):
@@ -114,6 +122,15 @@ def lib() -> C.CDLL:
                                                   C.POINTER(_vp)]
     L.kh_model_create_from_device_weights.argtypes = [C.POINTER(_i32), _vp, C.c_size_t,
                                                       C.POINTER(ModelOpts), C.POINTER(_vp)]
+    L.kh_model_create_from_checkpoint.argtypes = [C.c_char_p, C.c_size_t, _vp, C.c_size_t, C.POINTER(ModelOpts),
+                                                  C.POINTER(_vp)]
+    L.kh_seq_open.argtypes = [_vp, C.POINTER(_i32)]
+    L.kh_seq_close.argtypes = [_vp, _i32]
+    L.kh_seq_length.argtypes = [_vp, _i32]
+    L.kh_model_forward.argtypes = [_vp, C.POINTER(BatchEntry), _i32, _vp]
+    L.kh_model_generate_batch.argtypes = [_vp, _i32, C.POINTER(C.POINTER(_i32)), C.POINTER(_i32), C.POINTER(_i32),
+                                          C.POINTER(_i32), _i32, C.POINTER(_i32), _i32, C.POINTER(_i32)]
+    L.kh_model_probe_residual.argtypes = [_vp, _vp, _i64, C.POINTER(_i64)]
     L.kh_model_destroy.argtypes = [_vp]
     L.kh_model_destroy.restype = None
     L.kh_model_get_config.argtypes = [_vp, C.POINTER(Config)]

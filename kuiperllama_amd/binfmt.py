@@ -35,6 +35,7 @@ ROPE_INTERLEAVED = 0  # cpu/rope_kernel.cpp:98-121 (default build: llama2.c / Me
 ROPE_HALF = 1  # cpu/rope_kernel.cpp:18-42 / 58-82 (LLAMA3_SUPPORT / QWEN2_SUPPORT builds)
 FAMILY_LLAMA = 0
 FAMILY_QWEN2 = 1
+FAMILY_LAYERS = 2  # checkpoint folder: config.json + model.safetensors (kuiperllama_amd/checkpoint.py)
 
 HEADER_FP32_BYTES = 28  # 7 x int32 (model/config.h:5-13)
 HEADER_INT8_BYTES = 32  # + int32 group_size (model.cpp:64-70)

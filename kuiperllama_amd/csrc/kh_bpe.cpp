@@ -30,53 +30,12 @@
 #include <vector>
 
 #include "../../include/kuiper_hip.h"
+#include "kh_json.h"
 #include "kh_unicode_tables.h"
 
-namespace {
+using namespace khm;
 
-// ---- UTF-8 ---------------------------------------------------------------------------------------
-// decodes one code point at s[i]; malformed bytes come back as themselves (length 1), which keeps
-// the scanner total: such a byte is "other" for the pattern and goes through the byte-level BPE.
-inline uint32_t utf8_next(const std::string& s, size_t i, size_t* len) {
-  const unsigned char c = (unsigned char)s[i];
-  auto cont = [&](size_t k) { return i + k < s.size() && ((unsigned char)s[i + k] & 0xC0) == 0x80; };
-  if (c < 0x80) {
-    *len = 1;
-    return c;
-  }
-  if ((c & 0xE0) == 0xC0 && cont(1)) {
-    *len = 2;
-    return ((c & 0x1Fu) << 6) | ((unsigned char)s[i + 1] & 0x3Fu);
-  }
-  if ((c & 0xF0) == 0xE0 && cont(1) && cont(2)) {
-    *len = 3;
-    return ((c & 0x0Fu) << 12) | (((unsigned char)s[i + 1] & 0x3Fu) << 6) | ((unsigned char)s[i + 2] & 0x3Fu);
-  }
-  if ((c & 0xF8) == 0xF0 && cont(1) && cont(2) && cont(3)) {
-    *len = 4;
-    return ((c & 0x07u) << 18) | (((unsigned char)s[i + 1] & 0x3Fu) << 12) |
-           (((unsigned char)s[i + 2] & 0x3Fu) << 6) | ((unsigned char)s[i + 3] & 0x3Fu);
-  }
-  *len = 1;
-  return 0xFFFD0000u | c;  // not a code point: classified as "other"
-}
-inline void utf8_put(std::string& out, uint32_t cp) {
-  if (cp < 0x80) {
-    out += (char)cp;
-  } else if (cp < 0x800) {
-    out += (char)(0xC0 | (cp >> 6));
-    out += (char)(0x80 | (cp & 0x3F));
-  } else if (cp < 0x10000) {
-    out += (char)(0xE0 | (cp >> 12));
-    out += (char)(0x80 | ((cp >> 6) & 0x3F));
-    out += (char)(0x80 | (cp & 0x3F));
-  } else {
-    out += (char)(0xF0 | (cp >> 18));
-    out += (char)(0x80 | ((cp >> 12) & 0x3F));
-    out += (char)(0x80 | ((cp >> 6) & 0x3F));
-    out += (char)(0x80 | (cp & 0x3F));
-  }
-}
+namespace {
 
 template <size_t N>
 inline bool in_ranges(const KhCpRange (&t)[N], uint32_t cp) {
@@ -103,136 +62,6 @@ inline uint8_t classify(uint32_t cp) {
   if (in_ranges(kh_unicode_N, cp)) return C_N;
   return C_OTHER;
 }
-
-// ---- JSON (only what tokenizer.json needs) ------------------------------------------------------
-struct Json {
-  const char* p;
-  const char* end;
-  bool ok = true;
-  void ws() {
-    while (p < end && (*p == ' ' || *p == '\n' || *p == '\r' || *p == '\t')) ++p;
-  }
-  bool eat(char c) {
-    ws();
-    if (p < end && *p == c) {
-      ++p;
-      return true;
-    }
-    return false;
-  }
-  bool peek(char c) {
-    ws();
-    return p < end && *p == c;
-  }
-  static int hex4(const char* q) {
-    int v = 0;
-    for (int i = 0; i < 4; ++i) {
-      const char c = q[i];
-      v <<= 4;
-      if (c >= '0' && c <= '9') v |= c - '0';
-      else if (c >= 'a' && c <= 'f') v |= c - 'a' + 10;
-      else if (c >= 'A' && c <= 'F') v |= c - 'A' + 10;
-      else return -1;
-    }
-    return v;
-  }
-  bool str(std::string* out) {  // out may be null (skip)
-    ws();
-    if (p >= end || *p != '"') return ok = false;
-    ++p;
-    while (p < end && *p != '"') {
-      if (*p == '\\') {
-        if (p + 1 >= end) return ok = false;
-        const char e = p[1];
-        p += 2;
-        uint32_t cp;
-        switch (e) {
-          case 'n': cp = '\n'; break;
-          case 't': cp = '\t'; break;
-          case 'r': cp = '\r'; break;
-          case 'b': cp = '\b'; break;
-          case 'f': cp = '\f'; break;
-          case 'u': {
-            if (p + 4 > end) return ok = false;
-            int v = hex4(p);
-            if (v < 0) return ok = false;
-            p += 4;
-            cp = (uint32_t)v;
-            if (cp >= 0xD800 && cp < 0xDC00 && p + 6 <= end && p[0] == '\\' && p[1] == 'u') {
-              const int lo = hex4(p + 2);
-              if (lo >= 0xDC00 && lo < 0xE000) {
-                cp = 0x10000 + ((cp - 0xD800) << 10) + ((uint32_t)lo - 0xDC00);
-                p += 6;
-              }
-            }
-            break;
-          }
-          default: cp = (unsigned char)e; break;  // \" \\ \/
-        }
-        if (out) utf8_put(*out, cp);
-      } else {
-        if (out) *out += *p;
-        ++p;
-      }
-    }
-    if (p >= end) return ok = false;
-    ++p;
-    return true;
-  }
-  bool integer(long* v) {
-    // digits parsed by hand, bounded by `end`: the buffer (kh_bpe_create_from_memory's ptr/nbytes)
-    // is not NUL-terminated, so strtol could read past a file that is truncated inside a number
-    ws();
-    const char* q = p;
-    bool neg = false;
-    if (q < end && (*q == '-' || *q == '+')) neg = *q++ == '-';
-    if (q >= end || *q < '0' || *q > '9') return ok = false;
-    long x = 0;
-    while (q < end && *q >= '0' && *q <= '9') {
-      if (x > (0x7fffffffL - 9) / 10) return ok = false;  // ids are int32
-      x = x * 10 + (*q++ - '0');
-    }
-    // a fraction / exponent would not be an id
-    p = q;
-    if (v) *v = neg ? -x : x;
-    return true;
-  }
-  bool skip() {  // any value
-    ws();
-    if (p >= end) return ok = false;
-    if (*p == '"') return str(nullptr);
-    if (*p == '{') {
-      ++p;
-      if (eat('}')) return true;
-      do {
-        if (!str(nullptr) || !eat(':') || !skip()) return ok = false;
-      } while (eat(','));
-      return eat('}') ? true : (ok = false);
-    }
-    if (*p == '[') {
-      ++p;
-      if (eat(']')) return true;
-      do {
-        if (!skip()) return ok = false;
-      } while (eat(','));
-      return eat(']') ? true : (ok = false);
-    }
-    while (p < end && *p != ',' && *p != '}' && *p != ']' && *p != ' ' && *p != '\n' && *p != '\r' && *p != '\t') ++p;
-    return true;  // number / true / false / null
-  }
-  // iterate the members of an object: fn(key) must consume the value
-  template <class F>
-  bool object(F&& fn) {
-    if (!eat('{')) return ok = false;
-    if (eat('}')) return true;
-    do {
-      std::string key;
-      if (!str(&key) || !eat(':')) return ok = false;
-      if (!fn(key)) return ok = false;
-    } while (eat(','));
-    return eat('}') ? true : (ok = false);
-  }
-};
 
 }  // namespace
 

@@ -1,0 +1,331 @@
+// kh_latent.h — latent attention in its absorbed form.
+//
+// A cache row holds the normalised latent c (Rp elements, zero-padded) and the rotated key part shared by all heads
+// (drp elements): q_n . (W_uk c) = (W_uk^T q_n) . c, so a query row is [W_uk^T q_n | rotated q] and every head of a
+// token attends to the SAME rows; the values are the latents themselves, W_uv follows behind the softmax.  All
+// H x tokens query rows of a sequence therefore share each staged key tile - one read of the cache per 16 .. 64 rows.
+//
+// k_latent_attn: workgroup = 4 waves = WR row tiles of 16 query rows x CP column parts (WR CP = 4) of the latent.
+//   S^T = K Q^T: a lane ends with the scores of ONE query row (its column), so the running max / sum are lane scalars
+//   plus two cross-row swaps, and P^T is already the second operand of O^T = C^T P^T: no LDS round trip.  The key
+//   order inside a tile is permuted so that the four-score groups of the result layout are the contiguous fragment
+//   groups of the operand layout; the transposed tile is staged with the same permutation.
+// Softmax with a sink: m starts at sink_h and l at 1 in the first split (exp(sink - m), counted once, no value).
+// Scores, weights and sums are fp32; P is rounded to the storage type for its product with the values.
+#pragma once
+#include "kh_lops.h"
+
+namespace khm {
+
+// ---- per-token preparation: norms of the two latents, rotation of the shared key part, cache row -------------------
+template <class T>
+struct LatPrepArgs {
+  const float* raw;        // [T][ldr]: q latent (qr), kv latent (R), rotated part (dr)
+  const float *qn, *kvn;   // norm weights
+  const float2* rope;      // [positions][dims / 2] (cos, sin)
+  T* cq;                   // [T][ldq]
+  T* cache;                // + slot * slot_elems + pos * row
+  size_t slot_elems;
+  int ldr, ldq, qr, R, dr, Rp, row, dims;
+  float eps;
+  PassTabs p;
+};
+template <class T>
+__global__ __launch_bounds__(256) void k_latent_prep(const LatPrepArgs<T> a) {
+  __shared__ float red[KH_WAVES_MAX];
+  const int t = blockIdx.x;
+  const float* r = a.raw + (size_t)t * a.ldr;
+  const int pos = a.p.pos[t], slot = a.p.seg_slot[a.p.seg[t]];
+  float s = 0.f;
+  for (int i = threadIdx.x; i < a.qr; i += 256) s = __builtin_fmaf(r[i], r[i], s);
+  const float rq = 1.0f / sqrtf(block_sum(s, red) / (float)a.qr + a.eps);
+  for (int i = threadIdx.x; i < a.qr; i += 256) a.cq[(size_t)t * a.ldq + i] = (T)(r[i] * rq * a.qn[i]);
+  r += a.qr;
+  s = 0.f;
+  for (int i = threadIdx.x; i < a.R; i += 256) s = __builtin_fmaf(r[i], r[i], s);
+  const float rk = 1.0f / sqrtf(block_sum(s, red) / (float)a.R + a.eps);
+  T* row = a.cache + (size_t)slot * a.slot_elems + (size_t)pos * a.row;
+  for (int i = threadIdx.x; i < a.row; i += 256) {
+    float v = 0.f;
+    if (i < a.R) {
+      v = r[i] * rk * a.kvn[i];
+    } else if (i >= a.Rp && i - a.Rp < a.dr) {
+      const int j = i - a.Rp;
+      v = r[a.R + j];
+      if (j < a.dims) {
+        const float2 cs = a.rope[(size_t)pos * (a.dims >> 1) + (j >> 1)];
+        const float o = r[a.R + (j ^ 1)];
+        v = (j & 1) ? v * cs.x + o * cs.y : v * cs.x - o * cs.y;
+      }
+    }
+    row[i] = (T)v;
+  }
+}
+
+// rotated part of every head: q [T][H][dnp + drp] -> Q [T][H][Rp + drp] (pad columns zero).  grid T
+template <class T>
+struct RopeQArgs {
+  const T* q;
+  T* Q;
+  const float2* rope;
+  int H, dnp, dr, drp, Rp, dims;
+  PassTabs p;
+};
+template <class T>
+__global__ __launch_bounds__(256) void k_rope_q(const RopeQArgs<T> a) {
+  const int t = blockIdx.x, pos = a.p.pos[t];
+  for (int i = threadIdx.x; i < a.H * a.drp; i += 256) {
+    const int h = i / a.drp, j = i - h * a.drp;
+    const T* q = a.q + ((size_t)t * a.H + h) * (a.dnp + a.drp) + a.dnp;
+    float v = j < a.dr ? (float)q[j] : 0.f;
+    if (j < a.dims) {
+      const float2 cs = a.rope[(size_t)pos * (a.dims >> 1) + (j >> 1)];
+      const float o = (float)q[j ^ 1];
+      v = (j & 1) ? v * cs.x + o * cs.y : v * cs.x - o * cs.y;
+    }
+    a.Q[((size_t)t * a.H + h) * (a.Rp + a.drp) + a.Rp + j] = (T)v;
+  }
+}
+
+// ---- attention -------------------------------------------------------------------------------------------------
+struct LatTile {  // 16 WR query rows of one segment: flattened (token, head) rows r0 ..
+  int seg, r0;
+};
+struct LatArgs {
+  const void* Q;         // [T][H][row]
+  const void* cache;     // + slot * slot_elems + pos * row
+  size_t slot_elems;
+  const float* sink;     // [H]
+  void* out;             // T [T][H][Rp] (one split)
+  float* part;           // splits > 1: [T * H][splits][Rp + 2]: o (unnormalised), m, l
+  const LatTile* tiles;
+  int H, Rp, row, nsplit;
+  float scale2;          // scale * log2(e)
+  PassTabs p;
+};
+
+template <class T>
+struct LatCfg {
+  static constexpr int KT = 4 * Tile<T>::N;      // keys per tile: 32 bf16, 16 fp32 (a 64-byte row of the transposed tile)
+  static constexpr int MAXROT = 128;
+};
+template <class T>
+static inline size_t lat_lds(int row, int Rp) { return (size_t)LatCfg<T>::KT * row * sizeof(T) + (size_t)Rp * 64; }
+
+// position of key k of a tile in the permuted order (see above)
+template <class T>
+__device__ __forceinline__ int lat_perm(int k) {
+  return sizeof(T) == 2 ? ((k >> 2) & 3) * 8 + (k >> 4) * 4 + (k & 3) : k;
+}
+
+// RT: 16-column tiles of the latent this instantiation can hold (Rp <= 16 RT); CP: column parts
+template <class T, int RT, int CP>
+__global__ __launch_bounds__(256) void k_latent_attn(const LatArgs a) {
+  typedef Tile<T> TL;
+  typedef typename TL::frag frag;
+  constexpr int E = TL::N, KT = LatCfg<T>::KT;
+  constexpr int NQ = (RT * 16 + LatCfg<T>::MAXROT) / (4 * E);  // 64-byte k-blocks of a query row, at most
+  constexpr int NT = RT / CP;                                  // latent tiles per wave
+  constexpr int NS = KT / 16;                                  // score tiles
+  constexpr int NB = ((KT / E) * (RT * 16 + LatCfg<T>::MAXROT) / E + 255) / 256;  // E x E blocks per thread
+  extern __shared__ __attribute__((aligned(1024))) char smem_raw[];
+  char* const Kt = smem_raw;
+  char* const Vt = smem_raw + (size_t)KT * a.row * sizeof(T);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int fr = lane & 15, fh = lane >> 4;
+  const int wr = wave % (4 / CP), wc = wave / (4 / CP);
+  const LatTile tl = a.tiles[blockIdx.x];
+  const int n_rows = a.p.seg_n[tl.seg] * a.H, pos0 = a.p.seg_pos0[tl.seg], row0 = a.p.seg_row0[tl.seg];
+  const T* cache = (const T*)a.cache + (size_t)a.p.seg_slot[tl.seg] * a.slot_elems;
+  // this lane's query row
+  int r = tl.r0 + wr * 16 + fr;
+  const bool live = r < n_rows;
+  if (!live) r = n_rows - 1;
+  const int tok = r / a.H, head = r - tok * a.H;
+  const int my_pos = pos0 + tok;
+  // keys [k_lo, k_hi) of this split; k_hi = 1 + the last position any row of the workgroup sees
+  int rl = tl.r0 + 16 * (4 / CP) - 1;
+  if (rl >= n_rows) rl = n_rows - 1;
+  const int n_keys = pos0 + rl / a.H + 1;
+  int k_lo = 0, k_hi = n_keys;
+  if (a.nsplit > 1) {
+    const int per = ((n_keys + a.nsplit - 1) / a.nsplit + KT - 1) / KT * KT;
+    k_lo = (int)blockIdx.y * per;
+    k_hi = k_lo + per < n_keys ? k_lo + per : n_keys;
+  }
+  const int nqb = a.row / (4 * E);
+  const char* qrow = (const char*)((const T*)a.Q + ((size_t)(row0 + tok) * a.H + head) * a.row) + 16 * fh;
+  frag fq[NQ];
+#pragma unroll
+  for (int b = 0; b < NQ; ++b)
+    if (b < nqb) fq[b] = *(const frag*)(qrow + 64 * b);
+  const bool sinks = (a.nsplit == 1 || blockIdx.y == 0);
+  float m = sinks ? a.sink[head] * 1.44269504088896f : -INFINITY, l = sinks && fh == 0 ? 1.f : 0.f;
+  f32x4 o[NT];
+#pragma unroll
+  for (int n = 0; n < NT; ++n) o[n] = f32x4{0.f, 0.f, 0.f, 0.f};
+  // ---- staging: an E x E block (E keys x E columns) per thread and pass
+  const int cblk = a.row / E, nblk = (KT / E) * cblk;
+  frag pre[NB][E];
+  auto fetch = [&](int k0) __attribute__((always_inline)) {
+#pragma unroll
+    for (int q = 0; q < NB; ++q) {
+      const int b = q * 256 + (int)threadIdx.x;
+      const int kb = b / cblk, cb = b - kb * cblk;
+      if (b < nblk) {
+#pragma unroll
+        for (int e = 0; e < E; ++e) {
+          int k = k0 + kb * E + e;
+          k = k < n_keys ? k : n_keys - 1;
+          pre[q][e] = *(const frag*)(cache + (size_t)k * a.row + cb * E);
+        }
+      }
+    }
+  };
+  auto stash = [&]() __attribute__((always_inline)) {
+#pragma unroll
+    for (int q = 0; q < NB; ++q) {
+      const int b = q * 256 + (int)threadIdx.x;
+      const int kb = b / cblk, cb = b - kb * cblk;
+      if (b < nblk) {
+#pragma unroll
+        for (int e = 0; e < E; ++e) {
+          const int k = kb * E + e;
+          *(frag*)(Kt + ((size_t)k * cblk + (cb ^ (k & 7))) * 16) = pre[q][e];
+        }
+        if (cb * E < a.Rp) {
+          // transposed: column c gets its E keys.  The E keys of a block are two groups of four in the permuted order
+#pragma unroll
+          for (int c = 0; c < E; ++c) {
+            const int col = cb * E + c;
+            char* v = Vt + (size_t)col * 64;
+#pragma unroll
+            for (int g = 0; g < E / 4; ++g) {
+              typename TL::quad u;
+              u.x = pre[q][4 * g + 0][c];
+              u.y = pre[q][4 * g + 1][c];
+              u.z = pre[q][4 * g + 2][c];
+              u.w = pre[q][4 * g + 3][c];
+              const int kp = lat_perm<T>(kb * E + 4 * g);           // first key's place
+              const int chunk = (kp / E) ^ ((col >> 1) & 3);
+              *(typename TL::quad*)(v + chunk * 16 + (kp % E) * (int)sizeof(T)) = u;
+            }
+          }
+        }
+      }
+    }
+  };
+  if (k_lo < k_hi) fetch(k_lo);
+  for (int k0 = k_lo; k0 < k_hi; k0 += KT) {
+    __syncthreads();  // everyone is done with the previous tile
+    stash();
+    __syncthreads();
+    if (k0 + KT < k_hi) fetch(k0 + KT);
+    f32x4 s[NS];
+#pragma unroll
+    for (int n = 0; n < NS; ++n) s[n] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int b = 0; b < NQ; ++b) {
+      if (b < nqb) {
+#pragma unroll
+        for (int n = 0; n < NS; ++n) {
+          const int k = n * 16 + fr;
+          const frag fk = *(const frag*)(Kt + ((size_t)k * cblk + ((4 * b + fh) ^ (k & 7))) * 16);
+          s[n] = TL::mma(fk, fq[b], s[n]);
+        }
+      }
+    }
+    // lane: keys k0 + 16 n + 4 fh + i of row r
+    float mx = m;
+#pragma unroll
+    for (int n = 0; n < NS; ++n)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int k = k0 + 16 * n + 4 * fh + i;
+        s[n][i] = k <= my_pos && k < k_hi ? s[n][i] * a.scale2 : -INFINITY;
+        mx = fmaxf(mx, s[n][i]);
+      }
+    mx = xor16_max(mx);
+    mx = xor32_max(mx);
+    const float base = mx == -INFINITY ? 0.f : mx;  // nothing seen yet by this row
+    const float f = __builtin_amdgcn_exp2f(m - base);
+    m = mx;
+    l *= f;
+    frag p;
+#pragma unroll
+    for (int n = 0; n < NS; ++n)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float e = __builtin_amdgcn_exp2f(s[n][i] - base);
+        l += e;
+        p[4 * n + i] = (T)e;
+      }
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+      const int c0 = (wc * NT + n) * 16;
+      if (c0 < a.Rp) {
+        const int col = c0 + fr;
+        const frag fv = *(const frag*)(Vt + (size_t)col * 64 + ((fh ^ ((col >> 1) & 3)) << 4));
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[n][i] *= f;
+        o[n] = TL::mma(fv, p, o[n]);
+      }
+    }
+  }
+  l = xor16_sum(l);
+  l = xor32_sum(l);
+  if (!live) return;
+  const size_t orow = (size_t)(row0 + tok) * a.H + head;
+  if (a.nsplit == 1) {
+    const float inv = 1.0f / l;
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+      const int c0 = (wc * NT + n) * 16;
+      if (c0 < a.Rp) {
+        f32x4 v;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = o[n][i] * inv;
+        *(typename TL::quad*)((T*)a.out + orow * a.Rp + c0 + 4 * fh) = to_quad<T>(v);
+      }
+    }
+  } else {
+    float* p = a.part + (orow * a.nsplit + blockIdx.y) * (size_t)(a.Rp + 4);
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+      const int c0 = (wc * NT + n) * 16;
+      if (c0 < a.Rp) *(f32x4*)(p + c0 + 4 * fh) = o[n];
+    }
+    if (wc == 0 && fh == 0) {
+      p[a.Rp] = m;
+      p[a.Rp + 1] = l;
+    }
+  }
+}
+
+template <class T>
+int lat_attn_launch(hipStream_t s, const LatArgs& a, int ntiles, int cp) {
+  const size_t lds = lat_lds<T>(a.row, a.Rp);
+  auto go = [&](auto kern) -> int {
+    if (lds > 64 * 1024) {
+      const hipError_t e = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+      if (e != hipSuccess) return (int)e;
+    }
+    hipLaunchKernelGGL(kern, dim3(ntiles, a.nsplit), dim3(256), lds, s, a);
+    return KH_OK;
+  };
+  // column parts: 4 = 16-row tiles, 2 = 32-row tiles (latents of more than 256), 1 = 64-row tiles
+  if (cp == 4) {
+    if (a.Rp <= 64) return go(k_latent_attn<T, 4, 4>);
+    if (a.Rp <= 128) return go(k_latent_attn<T, 8, 4>);
+    if (a.Rp <= 256) return go(k_latent_attn<T, 16, 4>);
+    if (a.Rp <= 512) return go(k_latent_attn<T, 32, 4>);
+  } else if (cp == 2) {
+    if (a.Rp <= 512) return go(k_latent_attn<T, 32, 2>);
+  } else if (cp == 1) {
+    if (a.Rp <= 64) return go(k_latent_attn<T, 4, 1>);
+    if (a.Rp <= 128) return go(k_latent_attn<T, 8, 1>);
+    if (a.Rp <= 256) return go(k_latent_attn<T, 16, 1>);
+  }
+  return KH_ERR_UNSUPPORTED;
+}
+}  // namespace khm

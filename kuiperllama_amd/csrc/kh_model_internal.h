@@ -6,6 +6,7 @@
 //   kh_model_prefill.hip  B-token VALU prefill and the MFMA GEMM prefill (kh_prefill.h, kh_gemm.h,
 //                         kh_pattn.h kernels)
 //   kh_model_profile.hip  per-kernel / per-step timing entry points
+//   kh_hybrid_*.hip       the same roles for layer-list models (kh_hybrid.h)
 // gfx950 only.  No CPU fallback: every path launches HIP kernels.
 #pragma once
 #include <new>
@@ -44,11 +45,14 @@ struct LayerW {
   const float* ffn_norm;
 };
 
+struct Hybrid;  // kh_hybrid.h: a layer-list model
 }  // namespace khm
 using khm::LayerW;
 
 #define KH_STEP_VARIANTS 3  // kh_model_step.hip::step_variant
 struct kh_model {
+  khm::Hybrid* hy = nullptr;  // layer-list model (checkpoint folder); nullptr: a .bin image
+  std::vector<int> seq_len;   // .bin models: tokens of the one sequence kh_seq_open handed out
   kh_config cfg{};
   kh_model_opts opts{};
   hipStream_t stream = nullptr;
@@ -192,6 +196,11 @@ int step_graph_n(kh_model* m, int n_forced, int variant, int nsteps, hipGraphExe
 // (layer >= 0).  No-op for rows that are mapped already and for caches that are plainly allocated.  Newly mapped
 // memory is zeroed on the model's stream.
 int kv_ensure(kh_model* m, int rows, int layer = -1);
+// the parts of it that do not know a model's row geometry: reserve, and back a byte range of one cache
+int kv_allocate_bytes(kh_model* m, size_t total, int caches);
+int kv_map_range(kh_model* m, int which, size_t b0, size_t b1, int layer);
+// host memory -> device through pinned staging buffers
+hipError_t upload_chunked(char* d_dst, const char* h_src, size_t n, hipStream_t stream, float* ms_out);
 // ---- kh_model_selftest.hip ------------------------------------------------------------------
 // ring kernels vs register tiles, fence-free vs fenced split merge: once at the end of kh_model_create_*
 int run_selftests(kh_model* m);

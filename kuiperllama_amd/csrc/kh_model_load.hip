@@ -22,6 +22,7 @@
 #include <thread>
 #include <vector>
 
+#include "kh_hybrid.h"
 #include "kh_model_internal.h"
 
 using namespace khm;
@@ -69,6 +70,8 @@ int upload_threads() {
   n /= 2;
   return n < 1 ? 1 : (n > 8 ? 8 : (int)n);
 }
+}  // namespace
+namespace khm {
 hipError_t upload_chunked(char* d_dst, const char* h_src, size_t n, hipStream_t stream,
                           float* ms_out) {
   constexpr int NB = 4;
@@ -144,6 +147,8 @@ hipError_t upload_chunked(char* d_dst, const char* h_src, size_t n, hipStream_t 
     *ms_out = std::chrono::duration<float, std::milli>(std::chrono::steady_clock::now() - t0).count();
   return e;
 }
+}  // namespace khm
+namespace {
 
 // sin / cos table of the RoPE, rows [0, CL): computed on the host with libm exactly as the CPU backend does
 // (cpu/rope_kernel.cpp:4-16), so the fp32 table is bit-identical to the CPU reference's down to row 131071.  Every
@@ -284,6 +289,7 @@ int parse_header(const int32_t* h, const kh_model_opts* o, kh_config* c) {
   if (o->rope_mode != KH_ROPE_HALF && o->rope_mode != KH_ROPE_INTERLEAVED) return KH_ERR_INVALID_ARG;
   if (o->family != KH_FAMILY_LLAMA && o->family != KH_FAMILY_QWEN2) return KH_ERR_INVALID_ARG;
   if (!(o->rope_theta > 0.f) || !(o->rms_eps > 0.f)) return KH_ERR_INVALID_ARG;
+  if (o->dtype != KH_DTYPE_DEFAULT && o->dtype != KH_DTYPE_F32) return KH_ERR_UNSUPPORTED;  // .bin images run in fp32
   // vector-path preconditions of the fused kernels
   const int a = c->is_quant ? 16 : 4;
   if (c->dim % a || c->hidden_dim % a || c->head_size % 4 || (c->head_size & 1) ||
@@ -319,7 +325,6 @@ size_t expected_weight_bytes(const kh_config& c) {
 // model's stream).  Kernel addressing (model.cpp:226-243's slices) and captured graphs are unaffected: the base
 // pointers never change.  A 128-step run of Llama-3.2-1B commits 256 MiB of cache instead of 8.6 GB.
 // Hook KH_KV_VMM=0 (or a runtime without the virtual-memory API): one plain allocation, as before.
-static int kv_ensure_impl(kh_model* m, int row0, int rows, int layer);
 static void kv_release(kh_model* m);
 // Address ranges outlive the model that reserved them: kv_release hands a range (every chunk unmapped) to this
 // process-wide list and the next model whose caches reserve the same number of bytes takes it over; the list is never
@@ -357,10 +362,12 @@ static void va_give(void* p, size_t bytes) {
   std::lock_guard<std::mutex> g(vp.mu);
   vp.ranges.emplace_back(p, bytes);
 }
-static int kv_allocate(kh_model* m) {
-  const kh_config& c = m->cfg;
-  const size_t total = (size_t)c.layer_num * (size_t)c.cache_len * c.kv_dim * sizeof(float);
+}  // namespace
+namespace khm {
+// `caches` (1: m->kcache, 2: m->vcache as well) address ranges of `total` bytes each
+int kv_allocate_bytes(kh_model* m, size_t total, int caches) {
   kh_model::KvVmm& kv = m->kv;
+  float** const ptr[2] = {&m->kcache, &m->vcache};
   if (!dbg_off("KH_KV_VMM")) {
     hipMemAllocationProp prop = {};
     prop.type = hipMemAllocationTypePinned;
@@ -368,35 +375,41 @@ static int kv_allocate(kh_model* m) {
     prop.location.id = m->opts.device;
     size_t gran = 0;
     if (hipMemGetAllocationGranularity(&gran, &prop, hipMemAllocationGranularityRecommended) == hipSuccess && gran > 0) {
-      size_t chunk = (size_t)8 << 20;  // ONE size for every mapping of every model in the process (see kv_ensure)
+      size_t chunk = (size_t)8 << 20;  // ONE size for every mapping of every model in the process (see kv_map_range)
       chunk = (chunk + gran - 1) / gran * gran;
       const size_t reserved = (total + chunk - 1) / chunk * chunk;
-      void *pk = va_take(reserved, chunk), *pv = nullptr;
-      if (pk) {
-        if ((pv = va_take(reserved, chunk)) != nullptr) {
-          kv.on = true;
-          kv.chunk = chunk;
-          kv.reserved = reserved;
-          kv.have[0].assign(reserved / chunk, 0);
-          kv.have[1].assign(reserved / chunk, 0);
-          m->kcache = (float*)pk;
-          m->vcache = (float*)pv;
-          // trial: the first row of layer 0 (every sequence needs it).  A process in which this fails - e.g. one whose
-          // other users of the API mapped other sizes, see kv_ensure - takes the plain allocation below instead of
-          // failing at its first generate
-          if (kv_ensure_impl(m, 0, 1, 0) == KH_OK) return KH_OK;
-          kv_release(m);
-          kv = kh_model::KvVmm();
-        } else {
-          va_give(pk, reserved);
-        }
+      bool ok = true;
+      for (int w = 0; w < caches && ok; ++w) ok = (*ptr[w] = (float*)va_take(reserved, chunk)) != nullptr;
+      if (ok) {
+        kv.on = true;
+        kv.chunk = chunk;
+        kv.reserved = reserved;
+        for (int w = 0; w < caches; ++w) kv.have[w].assign(reserved / chunk, 0);
+        // trial: the first bytes (every sequence needs them).  A process in which this fails - e.g. one whose other
+        // users of the API map other sizes, see kv_map_range - takes the plain allocation below instead of failing at
+        // its first generate
+        for (int w = 0; w < caches && ok; ++w) ok = kv_map_range(m, w, 0, 1, 0) == KH_OK;
+        if (ok) return KH_OK;
+        kv_release(m);
+        kv = kh_model::KvVmm();
+      } else {
+        for (int w = 0; w < caches; ++w)
+          if (*ptr[w]) va_give(*ptr[w], reserved);
+        m->kcache = m->vcache = nullptr;
       }
     }
     (void)hipGetLastError();  // no virtual-memory API on this runtime / device: plain allocation
   }
   int rc;
-  if ((rc = dalloc(&m->kcache, total / sizeof(float))) != KH_OK) return rc;
-  return dalloc(&m->vcache, total / sizeof(float));
+  for (int w = 0; w < caches; ++w)
+    if ((rc = dalloc(ptr[w], total / sizeof(float) + 1)) != KH_OK) return rc;
+  return KH_OK;
+}
+}  // namespace khm
+namespace {
+static int kv_allocate(kh_model* m) {
+  const kh_config& c = m->cfg;
+  return kv_allocate_bytes(m, (size_t)c.layer_num * (size_t)c.cache_len * c.kv_dim * sizeof(float), 2);
 }
 static void kv_release(kh_model* m) {
   kh_model::KvVmm& kv = m->kv;
@@ -415,6 +428,68 @@ static void kv_release(kh_model* m) {
   }
   m->kcache = m->vcache = nullptr;
 }
+}  // namespace
+namespace khm {
+// bytes [b0, b1) of cache `which` backed by memory (no-op where they are, and for plain allocations); `layer` only
+// names the place in an error message
+int kv_map_range(kh_model* m, int which, size_t b0, size_t b1, int layer) {
+  kh_model::KvVmm& kv = m->kv;
+  if (!kv.on) return KH_OK;
+  hipMemAllocationProp prop = {};
+  prop.type = hipMemAllocationTypePinned;
+  prop.location.type = hipMemLocationTypeDevice;
+  prop.location.id = m->opts.device;
+  hipMemAccessDesc acc = {};
+  acc.location = prop.location;
+  acc.flags = hipMemAccessFlagsProtReadWrite;
+  char* base = (char*)(which ? m->vcache : m->kcache);
+  std::vector<uint8_t>& have = kv.have[which];
+  size_t ch = b0 / kv.chunk;
+  const size_t ch_end = (b1 + kv.chunk - 1) / kv.chunk;
+  while (ch < ch_end) {
+    if (have[ch]) {
+      ++ch;
+      continue;
+    }
+    size_t e = ch;
+    while (e < ch_end && !have[e]) ++e;  // a run of unmapped chunks: zeroed with one memset
+    // ONE handle per chunk, every handle the same size: on this runtime (ROCm 7.2) hipMemSetAccess returns
+    // "invalid argument" for a mapping that is smaller than one made earlier in the same process
+    // (tools/mb_vmm2.hip, profiles/r6_mb_vmm.txt); equal-sized mappings - what PyTorch's expandable segments
+    // use - are reliable, and a chunk costs 13 us to create + map + enable
+    for (size_t k = ch; k < e; ++k) {
+      kh_model::KvVmm::Run r;
+      r.va = base + k * kv.chunk;
+      r.len = kv.chunk;
+      const char* what = "hipMemCreate";
+      hipError_t err = hipMemCreate(&r.h, r.len, &prop, 0);
+      if (err == hipSuccess) {
+        what = "hipMemMap";
+        err = hipMemMap(r.va, r.len, 0, r.h, 0);
+        if (err == hipSuccess) {
+          what = "hipMemSetAccess";
+          err = hipMemSetAccess(r.va, r.len, &acc, 1);
+          if (err != hipSuccess) (void)hipMemUnmap(r.va, r.len);
+        }
+        if (err != hipSuccess) (void)hipMemRelease(r.h);
+      }
+      if (err != hipSuccess) {
+        fprintf(stderr, "[kh] KV cache: %s of %zu MiB at chunk %zu of the %s cache (layer %d) failed: %s\n", what,
+                r.len >> 20, k, which ? "V" : "K", layer, hipGetErrorString(err));
+        (void)hipGetLastError();
+        return (int)err;
+      }
+      kv.runs.push_back(r);
+      have[k] = 1;
+      kv.mapped += r.len;
+    }
+    KH_CHECK_HIP(hipMemsetAsync(base + ch * kv.chunk, 0, (e - ch) * kv.chunk, m->stream));
+    ch = e;
+  }
+  return KH_OK;
+}
+}  // namespace khm
+namespace {
 // rows [row0, rows) of one layer (layer >= 0) or of every layer
 static int kv_ensure_impl(kh_model* m, int row0, int rows, int layer) {
   kh_model::KvVmm& kv = m->kv;
@@ -423,65 +498,14 @@ static int kv_ensure_impl(kh_model* m, int row0, int rows, int layer) {
   if (rows > c.cache_len) rows = c.cache_len;
   if (rows <= kv.rows_all || row0 >= rows) return KH_OK;
   if (row0 < 0) row0 = 0;
-  hipMemAllocationProp prop = {};
-  prop.type = hipMemAllocationTypePinned;
-  prop.location.type = hipMemLocationTypeDevice;
-  prop.location.id = m->opts.device;
-  hipMemAccessDesc acc = {};
-  acc.location = prop.location;
-  acc.flags = hipMemAccessFlagsProtReadWrite;
   const size_t row_b = (size_t)c.kv_dim * sizeof(float), layer_b = (size_t)c.cache_len * row_b;
   const int l0 = layer >= 0 ? layer : 0, l1 = layer >= 0 ? layer + 1 : c.layer_num;
-  for (int which = 0; which < 2; ++which) {
-    char* base = (char*)(which ? m->vcache : m->kcache);
-    std::vector<uint8_t>& have = kv.have[which];
+  for (int which = 0; which < 2; ++which)
     for (int l = l0; l < l1; ++l) {
-      // bytes [b0, b1) of the reservation must be mapped
-      const size_t b0 = (size_t)l * layer_b + (size_t)row0 * row_b, b1 = (size_t)l * layer_b + (size_t)rows * row_b;
-      size_t ch = b0 / kv.chunk;
-      const size_t ch_end = (b1 + kv.chunk - 1) / kv.chunk;
-      while (ch < ch_end) {
-        if (have[ch]) {
-          ++ch;
-          continue;
-        }
-        size_t e = ch;
-        while (e < ch_end && !have[e]) ++e;  // a run of unmapped chunks: zeroed with one memset
-        // ONE handle per chunk, every handle the same size: on this runtime (ROCm 7.2) hipMemSetAccess returns
-        // "invalid argument" for a mapping that is smaller than one made earlier in the same process
-        // (tools/mb_vmm2.hip, profiles/r6_mb_vmm.txt); equal-sized mappings - what PyTorch's expandable segments
-        // use - are reliable, and a chunk costs 13 us to create + map + enable
-        for (size_t k = ch; k < e; ++k) {
-          kh_model::KvVmm::Run r;
-          r.va = base + k * kv.chunk;
-          r.len = kv.chunk;
-          const char* what = "hipMemCreate";
-          hipError_t err = hipMemCreate(&r.h, r.len, &prop, 0);
-          if (err == hipSuccess) {
-            what = "hipMemMap";
-            err = hipMemMap(r.va, r.len, 0, r.h, 0);
-            if (err == hipSuccess) {
-              what = "hipMemSetAccess";
-              err = hipMemSetAccess(r.va, r.len, &acc, 1);
-              if (err != hipSuccess) (void)hipMemUnmap(r.va, r.len);
-            }
-            if (err != hipSuccess) (void)hipMemRelease(r.h);
-          }
-          if (err != hipSuccess) {
-            fprintf(stderr, "[kh] KV cache: %s of %zu MiB at chunk %zu of the %s cache (layer %d) failed: %s\n", what,
-                    r.len >> 20, k, which ? "V" : "K", l, hipGetErrorString(err));
-            (void)hipGetLastError();
-            return (int)err;
-          }
-          kv.runs.push_back(r);
-          have[k] = 1;
-          kv.mapped += r.len;
-        }
-        KH_CHECK_HIP(hipMemsetAsync(base + ch * kv.chunk, 0, (e - ch) * kv.chunk, m->stream));
-        ch = e;
-      }
+      const int rc = kv_map_range(m, which, (size_t)l * layer_b + (size_t)row0 * row_b,
+                                  (size_t)l * layer_b + (size_t)rows * row_b, l);
+      if (rc != KH_OK) return rc;
     }
-  }
   if (layer < 0 && row0 == 0) kv.rows_all = rows;
   return KH_OK;
 }
@@ -624,7 +648,9 @@ int new_model(const int32_t* h_header, const kh_model_opts* opts, kh_model** out
 }  // namespace
 
 namespace khm {
-int kv_ensure(kh_model* m, int rows, int layer) { return kv_ensure_impl(m, 0, rows, layer); }
+int kv_ensure(kh_model* m, int rows, int layer) {
+  return m->hy ? hy_kv_ensure(m, 0, rows) : kv_ensure_impl(m, 0, rows, layer);
+}
 }  // namespace khm
 
 // =============================================================================================
@@ -651,6 +677,7 @@ extern "C" void kh_model_destroy(kh_model* m) {
   for (void* b : bufs)
     if (b) (void)hipFree(b);
   kv_release(m);
+  hy_destroy(m);
   if (m->owns_arena && m->arena) (void)hipFree(m->arena);
   if (m->stream) (void)hipStreamDestroy(m->stream);
   delete m;
@@ -772,6 +799,7 @@ extern "C" int kh_model_create_from_host_image(const void* h_image, size_t nbyte
 extern "C" int kh_model_create_from_file(const char* path, const kh_model_opts* opts,
                                          kh_model** out) {
   if (!path || !opts || !out) return KH_ERR_INVALID_ARG;
+  if (hy_is_folder(path)) return hy_create_from_folder(path, opts, out);  // config.json + model.safetensors
   // model.cpp:41-123: open + fstat + mmap(PROT_READ, MAP_PRIVATE)
   const int fd = open(path, O_RDONLY);
   if (fd == -1) return KH_ERR_IO;
@@ -819,7 +847,7 @@ extern "C" int kh_model_create_from_file(const char* path, const kh_model_opts* 
 extern "C" int kh_model_get_config(const kh_model* m, kh_config* out) {
   if (!m || !out) return KH_ERR_INVALID_ARG;
   *out = m->cfg;
-  out->launches_per_token = 5 * m->cfg.layer_num + 2;
+  out->launches_per_token = m->hy ? hy_launches(m) : 5 * m->cfg.layer_num + 2;
   return KH_OK;
 }
 extern "C" float kh_model_get_load_ms(const kh_model* m) { return m ? m->load_ms : -1.f; }
@@ -860,6 +888,7 @@ extern "C" int kh_model_first_sample(kh_model* m, kh_first_sample* out) {
 }
 extern "C" int kh_model_get_kv(kh_model* m, float** d_kcache, float** d_vcache) {
   if (!m || !d_kcache || !d_vcache) return KH_ERR_INVALID_ARG;
+  if (m->hy) return KH_ERR_UNSUPPORTED;  // latent rows and recurrent state, not a K / V pair
   // raw pointers leave the library: every row must be backed (a mapped-on-demand cache commits all of it here)
   KH_CHECK_HIP(hipSetDevice(m->opts.device));
   const int rc = kv_ensure(m, m->cfg.cache_len);
@@ -871,6 +900,11 @@ extern "C" int kh_model_get_kv(kh_model* m, float** d_kcache, float** d_vcache) 
 
 extern "C" int kh_model_kv_bytes(const kh_model* m, int64_t* reserved, int64_t* committed) {
   if (!m || !reserved || !committed) return KH_ERR_INVALID_ARG;
+  if (m->hy) {
+    *reserved = (int64_t)(m->hy->kv_slot * m->hy->slots * m->hy->elem());
+    *committed = m->kv.on ? (int64_t)m->kv.mapped : *reserved;
+    return KH_OK;
+  }
   const int64_t total = 2 * (int64_t)m->cfg.layer_num * m->cfg.cache_len * m->cfg.kv_dim * (int64_t)sizeof(float);
   *reserved = total;
   *committed = m->kv.on ? (int64_t)m->kv.mapped : total;
@@ -879,6 +913,7 @@ extern "C" int kh_model_kv_bytes(const kh_model* m, int64_t* reserved, int64_t* 
 
 extern "C" int kh_model_read_kv(kh_model* m, int32_t layer, int32_t row0, int32_t nrows,
                                 float* h_k, float* h_v) {
+  if (m && m->hy) return KH_ERR_UNSUPPORTED;
   if (!m || !h_k || !h_v || layer < 0 || layer >= m->cfg.layer_num || row0 < 0 || nrows <= 0 ||
       (int64_t)row0 + nrows > m->cfg.cache_len)
     return KH_ERR_INVALID_ARG;
@@ -897,6 +932,7 @@ extern "C" int kh_model_read_kv(kh_model* m, int32_t layer, int32_t row0, int32_
 
 extern "C" int kh_model_write_kv(kh_model* m, int32_t layer, int32_t row0, int32_t nrows,
                                  const float* h_k, const float* h_v) {
+  if (m && m->hy) return KH_ERR_UNSUPPORTED;
   if (!m || !h_k || !h_v || layer < 0 || layer >= m->cfg.layer_num || row0 < 0 || nrows <= 0 ||
       (int64_t)row0 + nrows > m->cfg.cache_len)
     return KH_ERR_INVALID_ARG;

@@ -9,6 +9,7 @@
 #include <vector>
 
 #include "kh_gemm.h"
+#include "kh_hybrid.h"
 #include "kh_model_internal.h"
 #include "kh_pattn.h"
 #include "kh_prefill.h"
@@ -20,6 +21,7 @@ namespace khm {
 // decode path uses at these sizes (in-register, at most 4 float4 per thread) and for the fast attention core.
 bool prefill_supported(const kh_model* m) {
   const kh_config& c = m->cfg;
+  if (m->hy) return false;
   if (c.head_size <= 32) return false;
   if (!kh_stage_fits4(c.dim, m->sh_qkv.wg) || !kh_stage_fits4(c.dim, m->sh_ffn.wg)) return false;
   if (m->sh_qkv.split > 2 || m->sh_ffn.split != 1) return false;
@@ -28,6 +30,7 @@ bool prefill_supported(const kh_model* m) {
   return true;
 }
 bool pg_supported(const kh_model* m) {
+  if (m->hy) return true;  // kh_hybrid_pass.hip
   const kh_config& c = m->cfg;
   if (c.head_size <= 32) return false;  // attention: the fast multi-token decode kernel
   const int kq = c.is_quant ? 64 : 16;  // K granule of one MFMA operand load
@@ -532,6 +535,10 @@ extern "C" int kh_model_prefill_gemm(kh_model* m, const int32_t* h_tokens, int32
   KH_CHECK_HIP(hipSetDevice(m->opts.device));
   int rc;
   if ((rc = kv_ensure(m, pos0 + n)) != KH_OK) return rc;
+  if (m->hy) {
+    const HyEntry e{0, n, pos0, h_tokens};
+    return kh_api_guard([&] { return hy_forward(m, &e, 1, nullptr, 0, nullptr); });
+  }
   if ((rc = ensure_pg_buffers(m)) != KH_OK) return rc;
   if ((rc = ensure_pg_ws(m)) != KH_OK) return rc;
   m->pg_launch_failed = false;
@@ -636,8 +643,10 @@ extern "C" int kh_model_time_prefill(kh_model* m, const int32_t* h_tokens, int32
     KH_CHECK_HIP(hipEventRecord(m->ev1, m->stream));
   } else if (mode == KH_PREFILL_GEMM) {
     if (!pg_supported(m)) return KH_ERR_UNSUPPORTED;
-    if ((rc = ensure_pg_buffers(m)) != KH_OK) return rc;
-    if ((rc = ensure_pg_ws(m)) != KH_OK) return rc;
+    if (!m->hy) {
+      if ((rc = ensure_pg_buffers(m)) != KH_OK) return rc;
+      if ((rc = ensure_pg_ws(m)) != KH_OK) return rc;
+    }
     KH_CHECK_HIP(hipEventRecord(m->ev0, m->stream));
     if ((rc = kh_model_prefill_gemm(m, h_tokens, n, pos0)) != KH_OK) return rc;
     KH_CHECK_HIP(hipEventRecord(m->ev1, m->stream));

@@ -10,6 +10,7 @@ extern "C" int kh_model_profile_kernel(kh_model* m, int32_t kclass, int32_t pos,
                                        float* h_avg_us) {
   if (!m || !h_avg_us || reps <= 0 || kclass < 0 || kclass >= KH_NUM_KCLASS)
     return KH_ERR_INVALID_ARG;
+  if (m->hy) return KH_ERR_UNSUPPORTED;  // the kernel classes are those of the .bin families' step
   const kh_config& c = m->cfg;
   if (pos < 0 || pos >= c.cache_len) return KH_ERR_RANGE;
   KH_CHECK_HIP(hipSetDevice(m->opts.device));
@@ -95,6 +96,7 @@ extern "C" const char* kh_kclass_name(int k) {
 extern "C" int kh_model_profile_step(kh_model* m, int32_t start_pos, int32_t n_steps,
                                      float* h_avg_us, int32_t* h_count) {
   if (!m || !h_avg_us || !h_count || n_steps <= 0 || start_pos < 0) return KH_ERR_INVALID_ARG;
+  if (m->hy) return KH_ERR_UNSUPPORTED;
   const kh_config& c = m->cfg;
   if (start_pos + n_steps > c.cache_len) return KH_ERR_RANGE;
   KH_CHECK_HIP(hipSetDevice(m->opts.device));

@@ -12,6 +12,7 @@
 
 #include "kh_fused.h"
 #include "kh_fused_ring.h"
+#include "kh_hybrid.h"
 #include "kh_model_internal.h"
 
 namespace khm {
@@ -398,6 +399,7 @@ void launch_sample(kh_model* m, int advance, int n_forced) {
 // OVERLAP) defer only up to 4 splits (profiles/r4_attn_defer_ab.txt: Llama-2-7B int8 loses from 8 on).
 int step_variant(const kh_model* m, int pos_lo, int pos_hi) {
   (void)pos_lo;
+  if (m->hy) return 0;
   if (pos_hi < KH_ATTN_MIN_TS) return 0;         // pos + 1 <= 256 everywhere: one split
   if (pos_hi + 1 >= m->attn_t_long) return 0;    // some step runs the group path
   if (m->attn_defer && attn_active_splits(pos_hi, m->attn_ns, m->attn_ts_shift) <= m->attn_defer_max) return 1;
@@ -409,6 +411,7 @@ int step_variant(const kh_model* m, int pos_lo, int pos_hi) {
 }
 // one fused decode step = 5L + 2 launches.  ev (optional) receives an event after each launch.
 void launch_step_fused(kh_model* m, int advance, int n_forced, hipEvent_t* ev, int variant) {
+  if (m->hy) return hy_launch_step(m, advance, n_forced);
   m->step_var = variant;
   int e = 0;
   auto mark = [&]() {
@@ -435,6 +438,10 @@ void launch_step_fused(kh_model* m, int advance, int n_forced, hipEvent_t* ev, i
 
 // the reference's own launch sequence, one C-ABI op per reference kernel (llama3.cpp:147-167)
 int launch_step_unfused(kh_model* m, int pos) {
+  if (m->hy) {
+    const int rc = hy_unfused_step(m);
+    return rc != KH_OK ? rc : kh_argmax_f32(m->logits, m->cfg.vocab_size, m->d_next, (void*)m->stream);
+  }
   const kh_config& c = m->cfg;
   void* s = (void*)m->stream;
   int rc;
@@ -478,7 +485,7 @@ int launch_step_unfused(kh_model* m, int pos) {
 
 void set_state(kh_model* m, int token, int pos) {
   hipLaunchKernelGGL(k_set_state, dim3(1), dim3(KH_WG), 0, m->stream, token, pos, m->d_token,
-                     m->d_pos, m->tok_emb, m->x, m->cfg.dim);
+                     m->d_pos, m->tok_emb, m->x, m->hy ? 0 : m->cfg.dim);  // layer lists gather it in their first kernel
 }
 
 int ensure_pinned_words(kh_model* m, int n) {

@@ -1,0 +1,133 @@
+// kh_moe.h — expert router and dispatch lists.
+// Scores s = softmax(z) over all router outputs (fp32); the `top` largest s + correction are chosen, ties to the lower
+// index; the weights are the chosen s.  Outputs from n_expert on are identity experts (no tensors).
+#pragma once
+#include "kh_lgemm.h"
+
+#define KH_MOE_MAX_OUT 1024  // router outputs (16 per lane)
+#define KH_MOE_MAX_TOP 32
+
+namespace khm {
+
+// The choice for one token by one wave; z in LDS or global [n_out].  Calls pick(k, id, weight) for k = 0 .. top - 1
+// on every lane, in order of decreasing choice score.
+template <class F>
+__device__ __forceinline__ void moe_route(const float* z, const float* corr, int n_out, int top, int lane, F&& pick) {
+  constexpr int PER = KH_MOE_MAX_OUT / 64;
+  float s[PER], key[PER];
+  float m = -INFINITY;
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int i = j * 64 + lane;
+    s[j] = i < n_out ? z[i] : -INFINITY;
+    m = fmaxf(m, s[j]);
+  }
+  m = wave_max(m);
+  float sum = 0.f;
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    s[j] = expf(s[j] - m);  // exp(-inf) = 0 beyond n_out
+    sum += s[j];
+  }
+  sum = wave_sum(sum);
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int i = j * 64 + lane;
+    s[j] /= sum;
+    key[j] = i < n_out ? s[j] + corr[i] : -INFINITY;
+  }
+  for (int k = 0; k < top; ++k) {
+    float v = -INFINITY, w = 0.f;
+    int id = 0x7fffffff;
+#pragma unroll
+    for (int j = 0; j < PER; ++j)
+      if (key[j] > v) {  // ascending j: the lowest index of a tie within the lane
+        v = key[j];
+        id = j * 64 + lane;
+        w = s[j];
+      }
+    wave_amax(v, id);
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const bool mine = j * 64 + lane == id;
+      if (mine) key[j] = -INFINITY;
+      if (mine) w = s[j];
+    }
+    w = __shfl(w, id & 63, 64);
+    pick(k, id, w);
+  }
+}
+
+struct RouteArgs {
+  const float* z;        // [T][ldz]: router outputs, then (shared expert) its gate logit
+  const float* corr;     // [n_out]
+  int32_t* id;           // [T][top]
+  float* w;              // [T][top]
+  float* id_w;           // [T] summed weight of the chosen identity experts
+  float* sh_g;           // [T] sigmoid of the shared expert's gate
+  int T, ldz, n_out, n_expert, top, shared;
+};
+static __global__ __launch_bounds__(256) void k_moe_route(const RouteArgs a) {
+  const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (t >= a.T) return;
+  const float* z = a.z + (size_t)t * a.ldz;
+  float idw = 0.f;
+  moe_route(z, a.corr, a.n_out, a.top, lane, [&](int k, int id, float w) __attribute__((always_inline)) {
+    if (id >= a.n_expert) idw += w;
+    if (lane == 0) {
+      a.id[(size_t)t * a.top + k] = id;
+      a.w[(size_t)t * a.top + k] = w;
+    }
+  });
+  if (lane == 0) {
+    a.id_w[t] = idw;
+    if (a.shared) a.sh_g[t] = sigmoid1(z[a.n_out]);
+  }
+}
+
+// Dispatch lists, one workgroup: rows grouped by expert (row -> token), slot of every (token, choice) in that order
+// (-1: identity expert), and the token tiles of the grouped GEMMs.
+struct ListArgs {
+  const int32_t* id;  // [T][top]
+  int32_t *rows, *slot;
+  LgTile* tiles;
+  int32_t* n_tiles;
+  int T, top, n_expert, bm;
+};
+static __global__ __launch_bounds__(1024) void k_moe_lists(const ListArgs a) {
+  __shared__ int32_t cnt[KH_MOE_MAX_OUT], off[KH_MOE_MAX_OUT], tile[KH_MOE_MAX_OUT];
+  for (int e = threadIdx.x; e < a.n_expert; e += 1024) cnt[e] = 0;
+  __syncthreads();
+  const int n = a.T * a.top;
+  for (int i = threadIdx.x; i < n; i += 1024) {
+    const int e = a.id[i];
+    if (e < a.n_expert) atomicAdd(&cnt[e], 1);
+  }
+  __syncthreads();
+  if (threadIdx.x == 0) {
+    int o = 0, q = 0;
+    for (int e = 0; e < a.n_expert; ++e) {
+      off[e] = o;
+      tile[e] = q;
+      o += cnt[e];
+      q += (cnt[e] + a.bm - 1) / a.bm;
+    }
+    *a.n_tiles = q;
+  }
+  __syncthreads();
+  for (int e = threadIdx.x; e < a.n_expert; e += 1024) {
+    const int c = cnt[e];
+    for (int r = 0, q = tile[e]; r < c; r += a.bm, ++q) a.tiles[q] = LgTile{e, off[e] + r, c - r < a.bm ? c - r : a.bm, 0};
+  }
+  __syncthreads();
+  for (int i = threadIdx.x; i < n; i += 1024) {
+    const int e = a.id[i];
+    int p = -1;
+    if (e < a.n_expert) {
+      p = atomicAdd(&off[e], 1);
+      a.rows[p] = i / a.top;
+    }
+    a.slot[i] = p;
+  }
+}
+}  // namespace khm

@@ -5,14 +5,16 @@
 from __future__ import annotations
 
 import ctypes as C
+import json
 from typing import List, Optional, Sequence, Tuple
 
 import numpy as np
 import torch
 
-from . import _ffi, binfmt
+from . import _ffi, binfmt, checkpoint
 from ._ffi import KH_EXEC_FUSED, KH_EXEC_GRAPH, KH_EXEC_UNFUSED  # noqa: F401
 
+DTYPES = {None: _ffi.KH_DTYPE_DEFAULT, "bfloat16": _ffi.KH_DTYPE_BF16, "float32": _ffi.KH_DTYPE_F32}
 EXEC = {"graph": KH_EXEC_GRAPH, "fused": KH_EXEC_FUSED, "unfused": KH_EXEC_UNFUSED}
 
 
@@ -25,7 +27,7 @@ def _opts(spec: binfmt.ModelSpec, max_seq_len: int, device: int, flags: int = 0)
 class KuiperModel:
     """Owns a kh_model handle.  Construct with one of the from_* classmethods."""
 
-    def __init__(self, handle: int, spec: binfmt.ModelSpec, keepalive=None):
+    def __init__(self, handle: int, spec: Optional[binfmt.ModelSpec], keepalive=None):
         self._h = C.c_void_p(handle)
         self.spec = spec
         self._keep = keepalive
@@ -86,6 +88,88 @@ class KuiperModel:
                                                                   C.byref(h)),
                    "kh_model_create_from_device_weights")
         return cls(h.value, spec, keepalive=keep)
+
+    # ---- checkpoint folders (layer-list models) -----------------------------------------
+    @staticmethod
+    def _layer_opts(max_seq_len: int, device: int, dtype: Optional[str], max_seqs: int) -> _ffi.ModelOpts:
+        return _ffi.ModelOpts(binfmt.FAMILY_LAYERS, 0, 0, 0.0, 0.0, max_seq_len, device, 0, DTYPES[dtype], max_seqs)
+
+    @classmethod
+    def from_checkpoint(cls, folder: str, max_seq_len: int = 0, device: int = 0, dtype: Optional[str] = None,
+                        max_seqs: int = 1) -> "KuiperModel":
+        """A folder with config.json and model.safetensors.  dtype: "bfloat16" (default) or "float32"; max_seqs:
+        sequences that can be live at once (open_seq / forward)."""
+        _ffi.sync_env()
+        h = C.c_void_p()
+        o = cls._layer_opts(max_seq_len, device, dtype, max_seqs)
+        _ffi.check(_ffi.lib().kh_model_create_from_file(folder.encode(), C.byref(o), C.byref(h)),
+                   "kh_model_create_from_file")
+        return cls(h.value, None)
+
+    @classmethod
+    def from_tensors(cls, config: dict, image: np.ndarray, max_seq_len: int = 0, device: int = 0,
+                     dtype: Optional[str] = None, max_seqs: int = 1) -> "KuiperModel":
+        """The same from memory: a configuration and the bytes of a safetensors file
+        (checkpoint.safetensors_image)."""
+        assert image.dtype == np.uint8 and image.flags["C_CONTIGUOUS"]
+        _ffi.sync_env()
+        h = C.c_void_p()
+        o = cls._layer_opts(max_seq_len, device, dtype, max_seqs)
+        text = json.dumps(config).encode()
+        _ffi.check(_ffi.lib().kh_model_create_from_checkpoint(text, len(text), image.ctypes.data, image.size,
+                                                              C.byref(o), C.byref(h)),
+                   "kh_model_create_from_checkpoint")
+        return cls(h.value, None)
+
+    # ---- sequences and batches ----------------------------------------------------------
+    def open_seq(self) -> int:
+        s = C.c_int32(-1)
+        _ffi.check(_ffi.lib().kh_seq_open(self._h, C.byref(s)), "kh_seq_open")
+        return int(s.value)
+
+    def close_seq(self, seq: int) -> None:
+        _ffi.check(_ffi.lib().kh_seq_close(self._h, seq), "kh_seq_close")
+
+    def seq_length(self, seq: int) -> int:
+        return int(_ffi.lib().kh_seq_length(self._h, seq))
+
+    def forward(self, entries: Sequence[Tuple[int, Sequence[int], Sequence[int]]]) -> np.ndarray:
+        """One step of a batch: entries = (sequence, its next tokens, places among them whose logits are wanted).
+        Returns the logits [wanted, vocab] in that order."""
+        arr = (_ffi.BatchEntry * len(entries))()
+        keep, n = [], 0
+        for a, (seq, toks, want) in zip(arr, entries):
+            t = (C.c_int32 * max(len(toks), 1))(*[int(x) for x in toks])
+            w = (C.c_int32 * max(len(want), 1))(*[int(x) for x in want])
+            keep += [t, w]
+            a.seq, a.n_tokens, a.tokens, a.n_want, a.want = seq, len(toks), t, len(want), w
+            n += len(want)
+        out = np.empty((n, self.cfg.vocab_size), np.float32)
+        _ffi.check(_ffi.lib().kh_model_forward(self._h, arr, len(entries), out.ctypes.data if n else None),
+                   "kh_model_forward")
+        return out
+
+    def generate_batch(self, prompts: Sequence[Sequence[int]], max_new: Sequence[int],
+                       stop: Optional[Sequence[int]] = None) -> List[List[int]]:
+        """Greedy continuation of several prompts decoded as one batch; the new tokens of each."""
+        n, cap = len(prompts), max(max_new)
+        bufs = [(C.c_int32 * len(p))(*[int(x) for x in p]) for p in prompts]
+        pp = (C.POINTER(C.c_int32) * n)(*[C.cast(b, C.POINTER(C.c_int32)) for b in bufs])
+        st = list(stop or [])
+        out, n_out = (C.c_int32 * (n * cap))(), (C.c_int32 * n)()
+        _ffi.check(_ffi.lib().kh_model_generate_batch(
+            self._h, n, pp, (C.c_int32 * n)(*[len(p) for p in prompts]), (C.c_int32 * n)(*max_new),
+            (C.c_int32 * max(len(st), 1))(*st), len(st), out, cap, n_out), "kh_model_generate_batch")
+        return [list(out[i * cap: i * cap + n_out[i]]) for i in range(n)]
+
+    def probe_residual(self, buf: Optional[np.ndarray]) -> int:
+        """Record the residual stream after every layer run of the following forward() calls into `buf` (float32);
+        None ends it.  Returns the floats written by the probe that ends."""
+        n = C.c_int64(0)
+        _ffi.check(_ffi.lib().kh_model_probe_residual(self._h, None if buf is None else buf.ctypes.data,
+                                                      0 if buf is None else buf.size, C.byref(n)),
+                   "kh_model_probe_residual")
+        return int(n.value)
 
     def close(self):
         if getattr(self, "_h", None) is not None and self._h.value:
