@@ -18,7 +18,7 @@
 #include "kh_scan.h"
 
 #define KH_HY_TMAX 2048       // tokens of one pass
-#define KH_HY_DECODE_B 8      // sequences of one fused decode step
+#define KH_HY_DECODE_B 4      // sequences of one fused decode step, at most
 
 namespace khm {
 
@@ -147,8 +147,17 @@ int hy_create_from_folder(const char* path, const kh_model_opts* o, kh_model** o
 int hy_forward(kh_model* m, const HyEntry* e, int n, const int32_t* want, int n_want, float* h_logits);
 // one token at (d_token, d_pos) of slot 0 on the pass kernels, logits to m->logits (the unfused step)
 int hy_unfused_step(kh_model* m);
+// query-row tile lists of latent attention: the kinds (heads, latents of more than 256) a model has, and the list for
+// segments of the given lengths
+typedef std::pair<int, int> LatKind;
+std::vector<LatKind> hy_lat_kinds(const Hybrid& hy);
+void hy_lat_tiles(const std::vector<int32_t>& seg_n, LatKind kind, int* cp, std::vector<int32_t>* tab);
+// argmax of m->logits as one sampler partial
+int kh_argmax_partial(kh_model* m);
 // ---- kh_hybrid_step.hip
 int hy_step_init(kh_model* m);
 void hy_launch_step(kh_model* m, int advance, int n_forced);
+int hy_decode_max(const kh_model* m);  // sequences the fused step can take at once
+int hy_decode(kh_model* m, const HyEntry* e, int n, float* h_logits);
 int hy_launches(const kh_model* m);  // kernel launches of one decode step
 }  // namespace khm

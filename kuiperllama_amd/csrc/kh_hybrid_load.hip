@@ -578,6 +578,11 @@ int finish(kh_model* m, Plan& pl) {
   KH_CHECK_HIP(hipEventCreate(&m->ev1));
   if ((rc = ensure_seq_cap(m, 256)) != KH_OK) return rc;
   if ((rc = hy_step_init(m)) != KH_OK) return rc;
+  // one eager step (token 0 at position 0 of slot 0, which every sequence starts by overwriting): kernel attributes and
+  // the one-token tables exist before a step is ever captured
+  if ((rc = hy_kv_ensure(m, 0, 1)) != KH_OK) return rc;
+  hy_launch_step(m, 0, 0);
+  if ((rc = kh_launch_status()) != KH_OK) return rc;
   KH_CHECK_HIP(hipStreamSynchronize(m->stream));
   return KH_OK;
 }

@@ -5,26 +5,431 @@
 
 #include "kh_fused.h"
 #include "kh_hybrid.h"
+#include "kh_ldecode.h"
 
 using namespace khm;
 
 namespace khm {
+// buffers and launch plan of the fused decode step for up to KH_HY_DECODE_B sequences
 struct Hybrid::Step {
-  int dummy = 0;
+  int bmax = 0;  // sequences one fused step can take (0: the geometry does not fit; everything runs as passes)
+  float *x[3] = {nullptr, nullptr, nullptr}, *xn2 = nullptr, *in = nullptr, *xc = nullptr, *mid = nullptr, *v = nullptr,
+        *he = nullptr, *hs = nullptr, *z = nullptr, *id_w = nullptr, *sh_g = nullptr, *part = nullptr, *logits = nullptr;
+  void* Q = nullptr;
+  int32_t *ids = nullptr, *tabs = nullptr, *tiles = nullptr;
+  int32_t* h_tabs = nullptr;
+  int nsplit = 1, head_wg = 1;
+  // per number of sequences B (1, 2, 4) and latent kind: tile list offset / count / column parts
+  struct Lat {
+    int B, H, big, cp, off, n;
+  };
+  std::vector<Lat> lat;
+  ~Step() {
+    for (void* p : {(void*)x[0], (void*)x[1], (void*)x[2], (void*)xn2, (void*)in, (void*)xc, (void*)mid, (void*)v, (void*)he,
+                    (void*)hs, (void*)z, (void*)id_w, (void*)sh_g, (void*)part, (void*)logits, Q, (void*)ids, (void*)tabs,
+                    (void*)tiles})
+      if (p) (void)hipFree(p);
+    if (h_tabs) (void)hipHostFree(h_tabs);
+  }
 };
 Hybrid::Hybrid() {}
 Hybrid::~Hybrid() {}
 
-int hy_step_init(kh_model* m) {
-  (void)m;
+namespace {
+constexpr int kMaxLds = 160 * 1024;
+// tabs: tok[B], pos[B], slot[B] (uploaded per batch) at 0, B, 2B of KH_HY_DECODE_B; ones and iota behind them
+enum { TB_TOK = 0, TB_POS = KH_HY_DECODE_B, TB_SLOT = 2 * KH_HY_DECODE_B, TB_ONE = 3 * KH_HY_DECODE_B,
+       TB_IOTA = 4 * KH_HY_DECODE_B, TB_ZERO = 5 * KH_HY_DECODE_B, TB_N = 6 * KH_HY_DECODE_B };
+
+template <class T>
+size_t vec_b(int n) { return Ld<T>::vec_bytes(n); }
+template <class T>
+size_t lds_out(const Hybrid& hy, const HyLayer& l, int B) {
+  const int nv = l.mixer == HY_MAMBA1 ? l.mb.innerp : l.la.H * l.la.dvp;
+  const int nbv = Ld<T>::blocks(nv);
+  const int nf = l.ff.on ? l.ff.top * Ld<T>::blocks(l.ff.ffp) + (l.ff.sffp ? Ld<T>::blocks(l.ff.sffp) : 0) : 0;
+  (void)hy;
+  return (size_t)(nbv + nf) * sizeof(LdBlk) + ((size_t)B * nbv + nf) * Ld<T>::BE * 4;
+}
+template <class T>
+bool fits(const Hybrid& hy, int B) {
+  const size_t room = kMaxLds - 2048;  // static shared memory of the kernels
+  if (B * vec_b<T>(hy.c.widthp) > room) return false;
+  for (auto& l : hy.layers) {
+    if (lds_out<T>(hy, l, B) > room) return false;
+    if (l.mixer == HY_MAMBA1 && B * vec_b<T>(l.mb.innerp) > room) return false;
+    if (l.mixer == HY_LATENT && (B * vec_b<T>(l.la.qrp) > room)) return false;
+  }
+  return true;
+}
+
+template <class K, class... A>
+int go(K kern, dim3 grid, size_t lds, hipStream_t s, A... args) {
+  if (lds > 64 * 1024) {
+    struct Done { int dev; const void* fn; size_t lds; };
+    static thread_local std::vector<Done> done;
+    int dev = 0;
+    (void)hipGetDevice(&dev);
+    bool hit = false;
+    for (const auto& d : done) hit = hit || (d.dev == dev && d.fn == (const void*)kern && d.lds >= lds);
+    if (!hit) {
+      const hipError_t e = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+      if (e != hipSuccess) return (int)e;
+      done.push_back({dev, (const void*)kern, lds});
+    }
+  }
+  hipLaunchKernelGGL(kern, grid, dim3(256), lds, s, args...);
   return KH_OK;
 }
-void hy_launch_step(kh_model* m, int advance, int n_forced) {
-  (void)hy_unfused_step(m);
-  (void)kh_argmax_f32(m->logits, m->cfg.vocab_size, m->d_next, (void*)m->stream);
-  (void)advance; (void)n_forced;
+#define TRY(e)                    \
+  do {                            \
+    const int _rc = (e);          \
+    if (_rc != KH_OK) return _rc; \
+  } while (0)
+
+int cdiv(int a, int b) { return (a + b - 1) / b; }
+
+template <class T, int B>
+int launch_scan(const LdScanArgs& a, hipStream_t s) {
+  int G = 1;
+  while (G * KH_SCAN_NS < a.N) G <<= 1;
+  const size_t lds = (size_t)(a.rankp + 2 * G * KH_SCAN_NS + 256 / G) * 4;
+  const dim3 grid(cdiv(a.C, 256 / G), B);
+  switch (G) {
+    case 1: return go(k_ld_scan<T, 1>, grid, lds, s, a);
+    case 2: return go(k_ld_scan<T, 2>, grid, lds, s, a);
+    case 4: return go(k_ld_scan<T, 4>, grid, lds, s, a);
+    case 8: return go(k_ld_scan<T, 8>, grid, lds, s, a);
+    case 16: return go(k_ld_scan<T, 16>, grid, lds, s, a);
+    default: return go(k_ld_scan<T, 32>, grid, lds, s, a);
+  }
 }
-int hy_launches(const kh_model* m) { return (int)m->hy->runs.size() * 15; }
+
+// One token of B sequences: tables at (tok, pos, slot); logits to `logits` [B][V]; argmax partials of sequence 0 to
+// the model's sampler buffers.
+template <class T, int B>
+int step(kh_model* m, const LdTabs tb, float* logits) {
+  Hybrid& hy = *m->hy;
+  Hybrid::Step& st = *hy.step_st;
+  hipStream_t s = m->stream;
+  const int W = hy.c.width, Wp = hy.c.widthp;
+  float* x_in = st.x[0];
+  for (size_t ri = 0; ri < hy.runs.size(); ++ri) {
+    const HyRun& r = hy.runs[ri];
+    const HyLayer& l = hy.layers[(size_t)r.layer];
+    const HyMoe& f = l.ff;
+    const bool mamba = l.mixer == HY_MAMBA1;
+    const bool changed = ri == 0 || r.pass >= 0;
+    float* x_cur = changed ? st.x[2] : x_in;
+    float* x_out = x_in == st.x[0] ? st.x[1] : st.x[0];
+    const int in_ld = mamba ? 2 * l.mb.inner : l.la.dqkv.N;
+    {
+      LdInArgs a{};
+      auto seg = [&](const HyMat& w, float* out, int rows, int ldo, int kind, int norm2) {
+        LdInSeg& g = a.seg[a.nseg++];
+        g.w = w.w;
+        g.out = out;
+        g.rows = rows;
+        g.ldo = ldo;
+        g.kind = kind;
+        g.norm2 = norm2;
+      };
+      seg(mamba ? l.mb.in : l.la.dqkv, st.in, in_ld, in_ld, mamba ? LDI_CONV : LDI_PLAIN, 0);
+      if (f.on) {
+        seg(f.zr, st.z, f.zr.N, f.zr.N, LDI_PLAIN, 1);
+        if (f.sff) seg(f.sgu, st.hs, f.sffp, f.sffp, LDI_SWIGLU, 1);
+      }
+      int total = 0, wg = 0;
+      auto items = [&](const LdInSeg& g) { return cdiv(g.rows, g.kind == LDI_SWIGLU ? 2 : 4); };
+      for (int i = 0; i < a.nseg; ++i) total += items(a.seg[i]);
+      const int ipw = cdiv(total, 2048);
+      for (int i = 0; i < a.nseg; ++i) {
+        a.seg[i].wg0 = wg;
+        a.seg[i].nwg = cdiv(items(a.seg[i]), 4 * ipw);
+        wg += a.seg[i].nwg;
+      }
+      a.x_in = x_in;
+      a.x_cur = changed ? x_cur : nullptr;
+      a.embed = hy.embed.w;
+      a.step = r.pass >= 0 ? hy.step.p + (size_t)r.pass * W : nullptr;
+      a.w1 = l.n1.p;
+      a.b1 = l.n1b.p;
+      a.w2 = f.on ? l.n2.p : nullptr;
+      a.b2 = f.on ? l.n2b.p : nullptr;
+      a.xn2 = f.on ? st.xn2 : nullptr;
+      a.W = W;
+      a.ld = Wp;
+      a.from_embed = ri == 0;
+      a.add_x0 = r.pass > 0;
+      a.eps = hy.c.eps;
+      a.t = tb;
+      if (mamba) {
+        a.conv_w = l.mb.conv.p;
+        a.conv_b = l.mb.conv_b.p;
+        a.conv_st = hy.state + r.conv_off;
+        a.slot_stride = hy.st_slot;
+        a.xc = st.xc;
+        a.inner = l.mb.inner;
+        a.taps = l.mb.taps;
+        a.xc_ld = l.mb.innerp;
+      }
+      TRY(go(k_ld_in<T, B>, dim3(wg), B * vec_b<T>(Wp), s, a));
+    }
+    {
+      LdMidArgs a{};
+      a.t = tb;
+      a.eps = hy.c.eps;
+      size_t lds = 0;
+      if (f.on) {
+        a.z = st.z;
+        a.corr = f.corr.p;
+        a.xn2 = st.xn2;
+        a.gu = f.gu.w;
+        a.he = st.he;
+        a.ids = st.ids;
+        a.id_w = st.id_w;
+        a.sh_g = st.sh_g;
+        a.top = f.top;
+        a.n_out = f.n_out();
+        a.n_expert = f.E;
+        a.shared = f.sff > 0;
+        a.ffp = f.ffp;
+        a.ldz = f.zr.N;
+        a.W = W;
+        a.ldw = f.gu.ld;
+        a.nwg_e = cdiv(f.ffp / 2, 4 * cdiv(B * f.top * f.ffp / 2, 3072));
+        lds = vec_b<T>(Wp);
+      }
+      const HyMat& wm = mamba ? l.mb.x : l.la.uq;
+      a.wm = wm.w;
+      a.rows = wm.N;
+      a.ldm = wm.ld;
+      a.n = mamba ? l.mb.inner : l.la.qr;
+      a.v = mamba ? st.xc : st.in;
+      a.ldv = mamba ? l.mb.innerp : in_ld;
+      a.vnorm = mamba ? nullptr : l.la.qn.p;
+      a.om = st.mid;
+      a.ldo = wm.N;
+      a.nwg_m = std::min(cdiv(cdiv(wm.N, 4), 4), 512);
+      lds = std::max(lds, B * vec_b<T>(wm.ld));
+      int extra = 0;
+      if (!mamba) {
+        const HyLatent& la = l.la;
+        extra = B;
+        a.latent = 1;
+        a.raw = st.in;
+        a.kvn = la.kvn.p;
+        a.rope = la.rope;
+        a.cache = (T*)m->kcache + r.kv_off;
+        a.slot_elems = hy.kv_slot;
+        a.qr = la.qr;
+        a.R = la.R;
+        a.dr = la.dr;
+        a.Rp = la.Rp;
+        a.row = la.row();
+        a.dims = la.dims;
+      }
+      TRY(go(k_ld_mid<T, B>, dim3(B * a.top * a.nwg_e + a.nwg_m + extra), lds, s, a));
+    }
+    if (mamba) {
+      const HyMamba& mb = l.mb;
+      LdScanArgs a{st.xc, st.in, st.mid, mb.dt.w, mb.dt_b.p, mb.A2.p, mb.D.p, hy.state + r.st_off, st.v, hy.st_slot,
+                   mb.inner, mb.state, mb.rankp, mb.innerp, mb.innerp, tb};
+      TRY((launch_scan<T, B>(a, s)));
+    } else {
+      const HyLatent& la = l.la;
+      LdAbsorbArgs ab{st.mid, la.ukT.w, la.rope, st.Q, la.H, std::max(1, std::min(cdiv(la.Rp, 32), cdiv(512, la.H * B))),
+                      la.dnp, la.dr, la.drp, la.Rp, la.row(), la.dims, tb};
+      TRY(go(k_ld_absorb<T>, dim3(la.H * ab.nwg, B), (size_t)la.dnp * 4, s, ab));
+      const Hybrid::Step::Lat* lt = nullptr;
+      for (auto& t : st.lat)
+        if (t.B == B && t.H == la.H && t.big == (la.Rp > 256)) lt = &t;
+      if (!lt) return KH_ERR_INTERNAL;
+      LatArgs at{};
+      at.Q = st.Q;
+      at.cache = (const T*)m->kcache + r.kv_off;
+      at.slot_elems = hy.kv_slot;
+      at.sink = la.sink.p;
+      at.part = st.part;
+      at.tiles = (const LatTile*)(st.tiles + lt->off);
+      at.H = la.H;
+      at.Rp = la.Rp;
+      at.row = la.row();
+      at.nsplit = st.nsplit;
+      at.scale2 = la.scale * 1.44269504088896f;
+      const int32_t* tabs = st.tabs;
+      at.p = PassTabs{tb.tok, tb.pos, tabs + TB_IOTA, tb.slot, tabs + TB_IOTA, tabs + TB_ONE, tb.pos};
+      TRY(lat_attn_launch<T>(s, at, lt->n, lt->cp));
+      LdValuesArgs va{st.part, la.uv.w, st.v, la.H, std::max(1, std::min(cdiv(la.dvp, 16), cdiv(512, la.H * B))), st.nsplit,
+                      la.Rp, la.dvp, tb.pos};
+      TRY(go(k_ld_values<T>, dim3(la.H * va.nwg, B), vec_b<T>(la.Rp), s, va));
+    }
+    {
+      const HyMat& wo = mamba ? l.mb.o : l.la.o;
+      LdOutArgs a{};
+      a.wo = wo.w;
+      a.v = st.v;
+      a.n_v = mamba ? l.mb.inner : l.la.H * l.la.dvp;
+      a.ld_v = mamba ? l.mb.innerp : l.la.H * l.la.dvp;
+      a.ldv = wo.ld;
+      a.x_cur = x_cur;
+      a.x_out = x_out;
+      a.W = W;
+      if (f.on) {
+        a.moe = 1;
+        a.down = f.down.w;
+        a.sdown = f.sdown.w;
+        a.he = st.he;
+        a.hs = st.hs;
+        a.ids = st.ids;
+        a.id_w = st.id_w;
+        a.sh_g = st.sh_g;
+        a.xn2 = st.xn2;
+        a.top = f.top;
+        a.ffp = f.ffp;
+        a.sffp = f.sffp;
+      }
+      a.nwg = std::min(cdiv(cdiv(W, 2), 4), 1024);
+      TRY(go(k_ld_out<T, B>, dim3(a.nwg), lds_out<T>(hy, l, B), s, a));
+    }
+    x_in = x_out;
+  }
+  LdHeadArgs h{x_in, hy.fnorm.p, hy.fnorm_b.p, hy.head.w, logits, m->part_val, m->part_idx, W, Wp, hy.c.vocab, hy.c.eps, hy.c.cap};
+  return go(k_ld_head<T, B>, dim3(st.head_wg), B * vec_b<T>(Wp), s, h);
+}
+template <class T>
+int step_b(kh_model* m, int B, const LdTabs& tb, float* logits) {
+  if (B == 1) return step<T, 1>(m, tb, logits);
+  if (B == 2) return step<T, 2>(m, tb, logits);
+  return step<T, 4>(m, tb, logits);
+}
+int step_any(kh_model* m, int B, const LdTabs& tb, float* logits) {
+  return m->hy->f32 ? step_b<float>(m, B, tb, logits) : step_b<bf16>(m, B, tb, logits);
+}
+}  // namespace
+
+int hy_step_init(kh_model* m) {
+  Hybrid& hy = *m->hy;
+  hy.step_st.reset(new Hybrid::Step());
+  Hybrid::Step& st = *hy.step_st;
+  for (int B : {1, 2, 4})
+    if (hy.f32 ? fits<float>(hy, B) : fits<bf16>(hy, B)) st.bmax = B;
+  const size_t B = KH_HY_DECODE_B, W = (size_t)hy.c.width;
+  size_t in = 1, xc = 1, mid = 1, v = 1, he = 1, hs = 1, z = 1, top = 1, Q = 1, part = 1;
+  auto up = [](size_t& a, size_t n) { a = a > n ? a : n; };
+  int hmin = 1 << 30;
+  for (auto& l : hy.layers) {
+    if (l.mixer == HY_MAMBA1) {
+      up(in, 2 * (size_t)l.mb.inner);
+      up(xc, (size_t)l.mb.innerp);
+      up(mid, (size_t)l.mb.x.N);
+      up(v, (size_t)l.mb.innerp);
+    } else {
+      up(in, (size_t)l.la.dqkv.N);
+      up(mid, (size_t)l.la.uq.N);
+      up(v, (size_t)l.la.H * l.la.dvp);
+      up(Q, (size_t)l.la.H * l.la.row());
+      up(part, (size_t)l.la.H * (l.la.Rp + 4));
+      hmin = std::min(hmin, l.la.H);
+    }
+    if (l.ff.on) {
+      up(he, (size_t)l.ff.top * l.ff.ffp);
+      up(hs, (size_t)l.ff.sffp);
+      up(z, (size_t)l.ff.zr.N);
+      up(top, (size_t)l.ff.top);
+    }
+  }
+  // time splits: about one workgroup per CU over the row tiles of one sequence
+  st.nsplit = 2;
+  while (st.nsplit < 64 && st.nsplit * KH_LAT_SPLIT_MIN < m->cfg.cache_len) st.nsplit *= 2;
+  auto f = [&](float** p, size_t n) -> int {
+    TRY(dalloc(p, n));
+    return (int)hipMemsetAsync(*p, 0, n * 4, m->stream);
+  };
+  for (float** p : {&st.x[0], &st.x[1], &st.x[2], &st.xn2}) TRY(f(p, B * W));
+  TRY(f(&st.in, B * in));
+  TRY(f(&st.xc, B * xc));
+  TRY(f(&st.mid, B * mid));
+  TRY(f(&st.v, B * v));
+  TRY(f(&st.he, B * he));
+  TRY(f(&st.hs, B * hs));
+  TRY(f(&st.z, B * z));
+  TRY(f(&st.id_w, B));
+  TRY(f(&st.sh_g, B));
+  TRY(f(&st.part, B * part * (size_t)st.nsplit));
+  TRY(f(&st.logits, B * (size_t)hy.c.vocab));
+  TRY(f((float**)&st.Q, B * Q));
+  TRY(dalloc(&st.ids, B * top));
+  TRY(dalloc(&st.tabs, TB_N));
+  KH_CHECK_HIP(hipHostMalloc((void**)&st.h_tabs, TB_N * 4, hipHostMallocDefault));
+  memset(st.h_tabs, 0, TB_N * 4);
+  for (int i = 0; i < KH_HY_DECODE_B; ++i) {
+    st.h_tabs[TB_ONE + i] = 1;
+    st.h_tabs[TB_IOTA + i] = i;
+  }
+  KH_CHECK_HIP(hipMemcpyAsync(st.tabs, st.h_tabs, TB_N * 4, hipMemcpyHostToDevice, m->stream));
+  std::vector<int32_t> all;
+  for (int b : {1, 2, 4})
+    for (const auto& k : hy_lat_kinds(hy)) {
+      Hybrid::Step::Lat t{b, k.first, k.second, 0, (int)all.size(), 0};
+      std::vector<int32_t> tab;
+      hy_lat_tiles(std::vector<int32_t>((size_t)b, 1), k, &t.cp, &tab);
+      t.n = (int)tab.size() / 2;
+      all.insert(all.end(), tab.begin(), tab.end());
+      st.lat.push_back(t);
+    }
+  TRY(dalloc(&st.tiles, all.size() + 1));
+  if (!all.empty()) KH_CHECK_HIP(hipMemcpy(st.tiles, all.data(), all.size() * 4, hipMemcpyHostToDevice));
+  st.head_wg = std::min(cdiv(cdiv(hy.c.vocab, 4), 4), 1024);
+  m->nparts = st.head_wg;
+  TRY(dalloc(&m->part_val, (size_t)m->nparts));
+  TRY(dalloc(&m->part_idx, (size_t)m->nparts));
+  return KH_OK;
+}
+
+// the generate loop's step: (d_token, d_pos) of slot 0, sampler behind it
+void hy_launch_step(kh_model* m, int advance, int n_forced) {
+  Hybrid& hy = *m->hy;
+  if (hy.step_st->bmax >= 1) {
+    const LdTabs tb{m->d_token, m->d_pos, hy.step_st->tabs + TB_ZERO};
+    (void)step_any(m, 1, tb, m->logits);
+  } else {  // the pass kernels leave logits; the sampler wants partials
+    (void)hy_unfused_step(m);
+    (void)kh_argmax_partial(m);
+  }
+  launch_sample(m, advance, n_forced);
+}
+int hy_launches(const kh_model* m) {
+  int n = 2;
+  for (const HyRun& r : m->hy->runs) n += m->hy->layers[(size_t)r.layer].mixer == HY_MAMBA1 ? 4 : 6;
+  return n;
+}
+int hy_decode_max(const kh_model* m) { return m->hy->step_st->bmax; }
+// one token of each of n sequences (n <= hy_decode_max), logits [n][vocab] to the host
+int hy_decode(kh_model* m, const HyEntry* e, int n, float* h_logits) {
+  Hybrid& hy = *m->hy;
+  Hybrid::Step& st = *hy.step_st;
+  KH_CHECK_HIP(hipSetDevice(m->opts.device));
+  KH_CHECK_HIP(hipStreamSynchronize(m->stream));  // the pinned table of the call before is free again
+  for (int i = 0; i < n; ++i) {
+    st.h_tabs[TB_TOK + i] = e[i].tok[0];
+    st.h_tabs[TB_POS + i] = e[i].pos0;
+    st.h_tabs[TB_SLOT + i] = e[i].slot;
+  }
+  KH_CHECK_HIP(hipMemcpyAsync(st.tabs, st.h_tabs, TB_ONE * 4, hipMemcpyHostToDevice, m->stream));
+  for (int i = 0; i < n;) {  // n = 3: 2 + 1
+    const int B = n - i >= 4 ? 4 : (n - i >= 2 ? 2 : 1);
+    const LdTabs tb{st.tabs + TB_TOK + i, st.tabs + TB_POS + i, st.tabs + TB_SLOT + i};
+    TRY(step_any(m, B, tb, st.logits));
+    if (h_logits)
+      KH_CHECK_HIP(hipMemcpyAsync(h_logits + (size_t)i * hy.c.vocab, st.logits, (size_t)B * hy.c.vocab * 4,
+                                  hipMemcpyDeviceToHost, m->stream));
+    i += B;
+  }
+  TRY(kh_launch_status());
+  if (h_logits) KH_CHECK_HIP(hipStreamSynchronize(m->stream));
+  return KH_OK;
+}
 }  // namespace khm
 
 // ---- sequences ---------------------------------------------------------------------------------------------------
@@ -82,7 +487,14 @@ int forward_layers(kh_model* m, const kh_batch_entry* e, int n, float* h_logits)
     base += e[i].n_tokens;
   }
   if (!want.empty() && !h_logits) return KH_ERR_INVALID_ARG;
-  if ((rc = hy_forward(m, es.data(), n, want.data(), (int)want.size(), want.empty() ? nullptr : h_logits)) != KH_OK) return rc;
+  bool single = n <= hy_decode_max(m) && !hy.probe && !dbg_off("KH_HY_DECODE");
+  for (const HyEntry& x : es) single = single && x.n == 1;
+  if (single) {  // the fused decode step computes every sequence's logits
+    std::vector<float> lg(want.empty() ? 0 : (size_t)n * hy.c.vocab);
+    if ((rc = hy_decode(m, es.data(), n, want.empty() ? nullptr : lg.data())) != KH_OK) return rc;
+    for (size_t k = 0; k < want.size(); ++k)
+      memcpy(h_logits + k * hy.c.vocab, lg.data() + (size_t)want[k] * hy.c.vocab, (size_t)hy.c.vocab * 4);
+  } else if ((rc = hy_forward(m, es.data(), n, want.data(), (int)want.size(), want.empty() ? nullptr : h_logits)) != KH_OK) return rc;
   for (int i = 0; i < n; ++i) hy.len[(size_t)e[i].seq] += e[i].n_tokens;
   return KH_OK;
 }

@@ -97,7 +97,8 @@ struct LatArgs {
   size_t slot_elems;
   const float* sink;     // [H]
   void* out;             // T [T][H][Rp] (one split)
-  float* part;           // splits > 1: [T * H][splits][Rp + 2]: o (unnormalised), m, l
+  float* part;           // splits > 1: [T * H][splits][Rp + 4]: o (unnormalised), m, l.  One token per segment then:
+                         // every row of a workgroup sees the same keys
   const LatTile* tiles;
   int H, Rp, row, nsplit;
   float scale2;          // scale * log2(e)
@@ -109,6 +110,16 @@ struct LatCfg {
   static constexpr int KT = 4 * Tile<T>::N;      // keys per tile: 32 bf16, 16 fp32 (a 64-byte row of the transposed tile)
   static constexpr int MAXROT = 128;
 };
+// keys per split and splits that have any: a split gets at least KH_LAT_SPLIT_MIN keys, whole tiles
+#define KH_LAT_SPLIT_MIN 64
+__host__ __device__ __forceinline__ int lat_split_len(int n_keys, int nsplit) {
+  const int per = (n_keys + nsplit - 1) / nsplit;
+  return (per + KH_LAT_SPLIT_MIN - 1) / KH_LAT_SPLIT_MIN * KH_LAT_SPLIT_MIN;
+}
+__host__ __device__ __forceinline__ int lat_active_splits(int n_keys, int nsplit) {
+  const int per = lat_split_len(n_keys, nsplit);
+  return (n_keys + per - 1) / per;
+}
 template <class T>
 static inline size_t lat_lds(int row, int Rp) { return (size_t)LatCfg<T>::KT * row * sizeof(T) + (size_t)Rp * 64; }
 
@@ -149,8 +160,9 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatArgs a) {
   const int n_keys = pos0 + rl / a.H + 1;
   int k_lo = 0, k_hi = n_keys;
   if (a.nsplit > 1) {
-    const int per = ((n_keys + a.nsplit - 1) / a.nsplit + KT - 1) / KT * KT;
+    const int per = lat_split_len(n_keys, a.nsplit);
     k_lo = (int)blockIdx.y * per;
+    if (k_lo >= n_keys) return;  // uniform; the merge does not read this split
     k_hi = k_lo + per < n_keys ? k_lo + per : n_keys;
   }
   const int nqb = a.row / (4 * E);

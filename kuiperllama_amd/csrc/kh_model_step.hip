@@ -384,7 +384,7 @@ void launch_sample(kh_model* m, int advance, int n_forced) {
   a.tok_emb = m->tok_emb;
   a.x = m->x;
   a.dim = c.dim;
-  a.vocab = c.vocab_size;
+  a.vocab = m->hy ? 0 : c.vocab_size;  // layer lists gather the embedding row in their first kernel
   a.advance = advance;
   hipLaunchKernelGGL(k_sample, dim3(1), dim3(KH_WG), 0, m->stream, a);
 }
