@@ -765,8 +765,102 @@ def assemble_line(spec, args, world, res, secondary, others, skipped, timing_bac
     return line
 
 
+# ---- layer-list models (--layers) ------------------------------------------------------------------------------------
+def layers_config(width: int, n_layers: int, vocab: int = 32000) -> dict:
+    """A Gufanex configuration with layers of a real model's proportions: mixers alternate, experts of half a width."""
+    ff, sff = width // 2, width
+    mlp = {"kind": "moe", "expert": {"ff": ff}, "shared": {"ff": sff},
+           "router": {"experts": 32, "identity": 4, "top": 6}}
+    mamba = {"type": "mamba1", "mlp": mlp,
+             "mixer": {"inner": 2 * width, "state": 16, "dt_rank": width // 16, "conv": 4}}
+    latent = {"type": "latent_attention", "mlp": mlp,
+              "mixer": {"heads": width // 128, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "q_rank": 1536,
+                        "scale": (128 + 64) ** -0.5, "rot": {"base": 10000.0, "dims": 64}}}
+    return {"architecture": "Gufanex", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "logit_softcap": 30.0,
+            "layers": [mamba if i % 2 == 0 else latent for i in range(n_layers)]}
+
+
+def layers_tensors(cfg: dict, seed: int = 0) -> dict:
+    """checkpoint.random_tensors with the large matrices drawn on the GPU (bf16 bits)."""
+    from kuiperllama_amd import checkpoint
+    small = {}
+    gen = torch.Generator(device="cuda")
+    gen.manual_seed(seed)
+    rng_cfg = checkpoint.tensor_shapes(cfg)
+    for k, sh in rng_cfg.items():
+        if len(sh) == 2 and sh[0] * sh[1] > 1 << 16 and not k.endswith("A_log"):
+            sc = 1.0 if k == "embed" else sh[1] ** -0.5
+            w = torch.randn(sh, device="cuda", generator=gen) * sc
+            small[k] = w.to(torch.bfloat16).view(torch.int16).cpu().numpy().view(np.uint16)
+        else:
+            small[k] = None
+    rest = checkpoint.random_tensors(cfg, seed, only=[k for k, v in small.items() if v is None])
+    return {k: (rest[k] if v is None else v) for k, v in small.items()}
+
+
+def layers_work(cfg: dict) -> tuple:
+    """(weight elements a decoded token reads, of which the head; linear MACs of a prompt token) - algorithmic."""
+    from kuiperllama_amd import checkpoint
+    active = 0
+    for k, sh in checkpoint.tensor_shapes(cfg).items():
+        if len(sh) != 2 or k in ("embed", "loop.step", "head") or k.endswith(("A_log", "conv")):
+            continue
+        n = sh[0] * sh[1]
+        if ".mlp.e" in k:
+            r = next(l for l in cfg["layers"])["mlp"]["router"]
+            n = n * r["top"] * (r["experts"] / (r["experts"] + r["identity"])) / r["experts"]
+        active += n
+    head = cfg["vocab"] * cfg["width"]
+    return active + head, head, active
+
+
+def layers_bench(args) -> None:
+    """Decode and prefill throughput of layer-list models beside the llama family at equal weights per token."""
+    from kuiperllama_amd import checkpoint
+    from kuiperllama_amd.model import KuiperModel
+    rows = []
+    rng = np.random.default_rng(1)
+    for width, n_layers in [(int(a), int(b)) for a, b in (x.split("x") for x in args.layers.split(","))]:
+        cfg = layers_config(width, n_layers)
+        elems, head, macs = layers_work(cfg)
+        t0 = time.time()
+        img = checkpoint.safetensors_image(layers_tensors(cfg))
+        m = KuiperModel.from_tensors(cfg, img, max_seq_len=4352)
+        del img
+        log(f"[bench] {width} x {n_layers}: built in {time.time() - t0:.1f} s, {m.cfg.weight_bytes / 1e9:.2f} GB")
+        hidden = int((macs / n_layers - 4 * width * width) / (3 * width)) // 64 * 64
+        sp = binfmt.ModelSpec(width, hidden, n_layers, width // 128, width // 128, cfg["vocab"], 4352, False,
+                              name=f"llama-{width}x{n_layers}")
+        for name, mk, wbytes, peak in (("gufanex", lambda: m, 2.0, 2.5e15),
+                                       ("llama", lambda: build_model(sp, 0)[0], 4.0, 157.3e12)):
+            mm = mk()
+            prompt = [int(t) for t in rng.integers(0, cfg["vocab"], 4096)]
+            mm.generate(prompt[:2], 32, exec="graph")
+            n = args.steps
+            best = min(mm.generate(prompt[:2], n, exec="graph")[1] for _ in range(3)) / n
+            nbytes = (elems if name == "gufanex" else sp.weight_elems()) * wbytes
+            row = {"model": name, "width": width, "layers": n_layers, "decode_us": round(best * 1e3, 1),
+                   "decode_tok_s": round(1e3 / best, 1), "weight_mb_per_token": round(nbytes / 1e6, 1),
+                   "decode_frac_of_8TBs": round(nbytes / (best * 1e-3) / 8e12, 3)}
+            row["decode_us_at_4095"] = round(float(np.median(mm.time_step(4095, 9))), 1)
+            for T in (512, 2048, 4096):
+                mm.time_prefill(prompt[:T], 0, mode="gemm")
+                ms = min(mm.time_prefill(prompt[:T], 0, mode="gemm") for _ in range(3))
+                fl = 2.0 * (macs if name == "gufanex" else sp.weight_elems() - cfg["vocab"] * width) * T
+                row[f"prefill{T}_tok_s"] = round(T / ms * 1e3)
+                row[f"prefill{T}_linear_frac_of_peak"] = round(fl / (ms * 1e-3) / peak, 3)
+            mm.close()
+            log("[bench] " + json.dumps(row))
+            rows.append(row)
+        torch.cuda.empty_cache()
+    print(json.dumps({"layers": rows}), flush=True)
+
+
 def main(argv=None):
     ap = argparse.ArgumentParser()
+    ap.add_argument("--layers", nargs="?", const="1024x8,2048x4,4096x2", default=None, metavar="WIDTHxLAYERS,...",
+                    help="measure layer-list models (Gufanex, bf16, random weights) of these sizes beside the llama "
+                         "family at equal weights per token instead of the default workload")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=128)  # generate(model, "a", 128), main.cpp:69
     ap.add_argument("--warmup", type=int, default=16)
@@ -801,6 +895,10 @@ def main(argv=None):
 
     if not torch.cuda.is_available():
         raise SystemExit("bench.py needs a GPU: the decode path has no CPU fallback")
+    if args.layers is not None:
+        torch.cuda.set_device(0)
+        layers_bench(args)
+        return
     from kuiperllama_amd import replicas
     local_rank = int(os.environ.get("LOCAL_RANK", "0"))
     torch.cuda.set_device(local_rank)

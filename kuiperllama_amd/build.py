@@ -19,7 +19,7 @@ SOURCES = ["kh_ops.hip", "kh_model_load.hip", "kh_model_step.hip", "kh_model_pre
            "kh_hybrid_load.hip", "kh_hybrid_pass.hip", "kh_hybrid_step.hip",
            "kh_tokenizer.cpp", "kh_bpe.cpp", "kh_debug.cpp"]
 HEADERS = ["kh_common.h", "kh_gemv.h", "kh_attn.h", "kh_fused.h", "kh_q8ring.h", "kh_fused_ring.h", "kh_prefill.h", "kh_gemm.h", "kh_pattn.h", "kh_unicode_tables.h", "kh_json.h",
-           "kh_tile.h", "kh_lgemm.h", "kh_lops.h", "kh_scan.h", "kh_moe.h", "kh_latent.h", "kh_hybrid.h", "kh_ldecode.h",
+           "kh_tile.h", "kh_lgemm.h", "kh_lops.h", "kh_scan.h", "kh_moe.h", "kh_latent.h", "kh_expanded.h", "kh_hybrid.h", "kh_ldecode.h",
            "kh_model_internal.h",
            "../../include/kuiper_hip.h"]
 ARCH = "gfx950"

@@ -7,7 +7,7 @@ from __future__ import annotations
 import json
 import os
 import struct
-from typing import Dict, Iterator, Tuple
+from typing import Dict, Iterator, Optional, Sequence, Tuple
 
 import numpy as np
 
@@ -110,12 +110,14 @@ def save(folder: str, cfg: dict, tensors: Dict[str, np.ndarray]) -> None:
     safetensors_image(tensors).tofile(os.path.join(folder, "model.safetensors"))
 
 
-def random_tensors(cfg: dict, seed: int = 0) -> Dict[str, np.ndarray]:
+def random_tensors(cfg: dict, seed: int = 0, only: Optional[Sequence[str]] = None) -> Dict[str, np.ndarray]:
     """Seeded random weights (bf16 bits) whose activations stay of order one: linear weights N(0, 1 / fan_in), norm
     weights around 1, A_log = log(1 .. state), dt biases that make softplus small."""
     rng = np.random.default_rng(seed)
     out: Dict[str, np.ndarray] = {}
     for k, s in tensor_shapes(cfg).items():
+        if only is not None and k not in only:
+            continue
         last = k.rsplit(".", 1)[-1]
         if k.endswith("norm") or last in ("norm1", "norm2", "D"):
             v = 1.0 + 0.1 * rng.standard_normal(s, np.float32)

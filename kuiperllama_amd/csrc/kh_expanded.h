@@ -1,0 +1,219 @@
+// kh_expanded.h — latent attention of long prompt segments in its expanded form.
+//
+// The absorbed form (kh_latent.h) contracts kv_rank + rot_dim per score; a prompt segment instead rebuilds its heads'
+// keys W_uk c and values W_uv c once per pass (two GEMMs over the cached latents) and contracts dim + rot_dim.  The
+// values are produced TRANSPOSED ([head value column][key]: the GEMM with its operands swapped), so every operand of
+// the attention kernel is a row of consecutive bytes and all staging is LDS-DMA.
+//
+// k_expanded_attn: workgroup = 4 waves x MR tiles of 16 tokens of ONE head; key tiles of KT (a 64-byte row of the
+// transposed values), double-buffered.  S^T = K Q^T and O^T = V^T P^T as in kh_latent.h; here the key order is
+// permuted where the K fragments are read (score tile n, row 4 h + i <- key 8 h + 4 n + i for bf16).
+#pragma once
+#include "kh_latent.h"
+#include "kh_lgemm.h"
+
+namespace khm {
+
+struct ExpArgs {
+  const void* Q;       // [T][H][dnp + drp], rotated
+  const void* Kx;      // [keys][H dnp]
+  const void* Vx;      // [H dvp][ldv]
+  const void* cache;   // rotated key parts: row k at + k * row (already offset to the part's first column)
+  const float* sink;
+  void* out;           // T [T][H dvp]
+  int H, dnp, drp, dvp, row, ldv;
+  int row0, n, pos0;   // the segment's rows in Q / out, their number, position of the first
+  float scale2;
+};
+
+// NQ: k-blocks (64 bytes) of a query row at most; NV: 16-column value tiles
+template <class T, int NQ, int NV, int MR>
+__global__ __launch_bounds__(256) void k_expanded_attn(const ExpArgs a) {
+  typedef Tile<T> TL;
+  typedef typename TL::frag frag;
+  constexpr int E = TL::N, KT = 4 * E, NS = KT / 16, ES = (int)sizeof(T);
+  extern __shared__ __attribute__((aligned(1024))) char smem_raw[];
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int fr = lane & 15, fh = lane >> 4;
+  const int head = blockIdx.x;
+  const int tile = (int)gridDim.y - 1 - (int)blockIdx.y;  // the longest key ranges first
+  const int q0 = tile * (64 * MR);
+  const int qc = a.dnp / E, rc = a.drp / E, vr = a.dvp;   // 16-byte chunks of the key parts, value rows
+  const int bytes_k = KT * a.dnp * ES, bytes_r = KT * a.drp * ES, stage = bytes_k + bytes_r + vr * 64;
+  int q_last = q0 + 64 * MR - 1;
+  q_last = q_last < a.n ? q_last : a.n - 1;
+  const int n_keys = a.pos0 + q_last + 1;
+  const int nb = (a.dnp + a.drp) / (4 * E);
+  const T* Q = (const T*)a.Q;
+  frag fq[MR][NQ];
+  int my_pos[MR];
+#pragma unroll
+  for (int m = 0; m < MR; ++m) {
+    int t = q0 + (wave * MR + m) * 16 + fr;
+    t = t < a.n ? t : a.n - 1;
+    my_pos[m] = a.pos0 + t;
+    const char* q = (const char*)(Q + ((size_t)(a.row0 + t) * a.H + head) * (a.dnp + a.drp)) + 16 * fh;
+#pragma unroll
+    for (int b = 0; b < NQ; ++b)
+      if (b < nb) fq[m][b] = *(const frag*)(q + 64 * b);
+  }
+  const unsigned lds0 = (unsigned)__builtin_amdgcn_readfirstlane((int)kh_lds_addr(smem_raw));
+  // slot s of a row of `c` chunks (c >= 8) holds chunk s ^ swz(row)
+  auto swz = [](int row) __attribute__((always_inline)) { return (row & 3) | ((row >> 1) & 4); };
+  const int nK = KT * qc / 64, nR = KT * rc / 64, nV = vr * 4 / 64;  // LDS-DMA requests of a stage (64 chunks each)
+  auto issue = [&](int slot, int k0) __attribute__((always_inline)) {
+    const unsigned d0 = lds0 + (unsigned)(slot * stage);
+    const char* kb = (const char*)a.Kx + ((size_t)k0 * a.H + head) * a.dnp * ES;
+    for (int j = wave; j < nK; j += 4) {
+      const int c = j * 64 + lane, r = c / qc, s = c - r * qc;
+      dma_x4_keep(kb, (unsigned)(r * a.H * a.dnp * ES + ((s ^ swz(r)) << 4)), d0 + 1024u * j);
+    }
+    for (int j = wave; j < nR; j += 4) {
+      const int c = j * 64 + lane, r = c / rc, s = c - r * rc;
+      const int k = k0 + r < n_keys ? k0 + r : n_keys - 1;  // rows behind the sequence's last are not backed
+      dma_x4_keep(a.cache, (unsigned)(k * a.row * ES + ((s ^ swz(r)) << 4)), d0 + bytes_k + 1024u * j);
+    }
+    const char* vb = (const char*)a.Vx + ((size_t)head * a.dvp * a.ldv + k0) * ES;
+    for (int j = wave; j < nV; j += 4) {
+      const int c = j * 64 + lane;
+      dma_x4_keep(vb, (unsigned)((c >> 2) * a.ldv * ES + ((c & 3) << 4)), d0 + bytes_k + bytes_r + 1024u * j);
+    }
+  };
+  float m[MR], l[MR];
+  f32x4 o[MR][NV];
+#pragma unroll
+  for (int q = 0; q < MR; ++q) {
+    m[q] = a.sink[head] * 1.44269504088896f;
+    l[q] = fh == 0 ? 1.f : 0.f;
+#pragma unroll
+    for (int n = 0; n < NV; ++n) o[q][n] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  const int wave_last = a.pos0 + q0 + (wave + 1) * MR * 16 - 1;  // last position any row of this wave sees
+  issue(0, 0);
+  int slot = 0;
+  for (int k0 = 0; k0 < n_keys; k0 += KT, slot ^= 1) {
+    wait_vm<0>();
+    __syncthreads();
+    if (k0 + KT < n_keys) issue(slot ^ 1, k0 + KT);
+    if (k0 > wave_last) continue;  // nothing in this tile for the wave (barriers stay uniform)
+    const char* Kt = smem_raw + slot * stage;
+    const char* Rt = Kt + bytes_k;
+    const char* Vt = Rt + bytes_r;
+    f32x4 s[MR][NS];
+#pragma unroll
+    for (int q = 0; q < MR; ++q)
+#pragma unroll
+      for (int n = 0; n < NS; ++n) s[q][n] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int b = 0; b < NQ; ++b) {
+      if (b < nb) {
+        const int c = 4 * b + fh;
+#pragma unroll
+        for (int n = 0; n < NS; ++n) {
+          const int k = NS == 2 ? 8 * (fr >> 2) + 4 * n + (fr & 3) : fr;
+          const char* src = 4 * b < qc ? Kt + ((size_t)k * qc + (c ^ swz(k))) * 16 : Rt + ((size_t)k * rc + ((c - qc) ^ swz(k))) * 16;
+          const frag fk = *(const frag*)src;
+#pragma unroll
+          for (int q = 0; q < MR; ++q) s[q][n] = TL::mma(fk, fq[q][b], s[q][n]);
+        }
+      }
+    }
+    frag p[MR];
+    float f[MR];
+    const bool edge = k0 + KT - 1 > a.pos0 + q0 + wave * MR * 16;  // the tile crosses the diagonal of some row
+#pragma unroll
+    for (int q = 0; q < MR; ++q) {
+      float mx = m[q];
+#pragma unroll
+      for (int n = 0; n < NS; ++n)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          float v = s[q][n][i] * a.scale2;
+          if (edge) {
+            const int k = k0 + (NS == 2 ? 8 * fh + 4 * n + i : 4 * fh + i);
+            v = k <= my_pos[q] ? v : -INFINITY;
+          }
+          s[q][n][i] = v;
+          mx = fmaxf(mx, v);
+        }
+      mx = xor16_max(mx);
+      mx = xor32_max(mx);  // finite: the sink
+      f[q] = __builtin_amdgcn_exp2f(m[q] - mx);
+      m[q] = mx;
+      float sum = 0.f;
+#pragma unroll
+      for (int n = 0; n < NS; ++n)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const float e = __builtin_amdgcn_exp2f(s[q][n][i] - mx);
+          sum += e;
+          p[q][4 * n + i] = (T)e;
+        }
+      l[q] = __builtin_fmaf(l[q], f[q], sum);
+    }
+#pragma unroll
+    for (int n = 0; n < NV; ++n) {
+      if (n * 16 < a.dvp) {
+        const frag fv = *(const frag*)(Vt + (size_t)(n * 16 + fr) * 64 + (fh << 4));
+#pragma unroll
+        for (int q = 0; q < MR; ++q) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) o[q][n][i] *= f[q];
+          o[q][n] = TL::mma(fv, p[q], o[q][n]);
+        }
+      }
+    }
+  }
+#pragma unroll
+  for (int q = 0; q < MR; ++q) {
+    float sum = xor16_sum(l[q]);
+    sum = xor32_sum(sum);
+    const float inv = 1.0f / sum;
+    const int t = q0 + (wave * MR + q) * 16 + fr;
+    if (t >= a.n) continue;
+    T* out = (T*)a.out + ((size_t)(a.row0 + t) * a.H + head) * a.dvp + 4 * fh;
+#pragma unroll
+    for (int n = 0; n < NV; ++n)
+      if (n * 16 < a.dvp) {
+        f32x4 v;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = o[q][n][i] * inv;
+        *(typename TL::quad*)(out + n * 16) = to_quad<T>(v);
+      }
+  }
+}
+
+// in-place rotation of the rotated part of every head of q [T][H][dnp + drp].  grid T
+template <class T>
+__global__ __launch_bounds__(256) void k_rope_inplace(T* q, const float2* rope, int H, int dnp, int drp, int dims, PassTabs p) {
+  const int t = blockIdx.x, half = dims >> 1;
+  const float2* rr = rope + (size_t)p.pos[t] * half;
+  for (int i = threadIdx.x; i < H * half; i += 256) {
+    const int h = i / half, j = i - h * half;
+    T* v = q + ((size_t)t * H + h) * (dnp + drp) + dnp + 2 * j;
+    const float2 cs = rr[j];
+    const float u = (float)v[0], w = (float)v[1];
+    v[0] = (T)(u * cs.x - w * cs.y);
+    v[1] = (T)(w * cs.x + u * cs.y);
+  }
+}
+
+static inline bool exp_supported(int dnp, int drp, int dvp) { return dnp + drp <= 256 && dvp <= 128 && drp > 0; }
+template <class T>
+int exp_attn_launch(hipStream_t s, const ExpArgs& a) {
+  constexpr int MR = sizeof(T) == 2 ? 2 : 1;
+  const size_t stage = (size_t)4 * Tile<T>::N * (a.dnp + a.drp) * sizeof(T) + (size_t)a.dvp * 64, lds = 2 * stage;
+  auto go = [&](auto kern) -> int {
+    if (lds > 64 * 1024) {
+      const hipError_t e = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+      if (e != hipSuccess) return (int)e;
+    }
+    hipLaunchKernelGGL(kern, dim3(a.H, (a.n + 64 * MR - 1) / (64 * MR)), dim3(256), lds, s, a);
+    return KH_OK;
+  };
+  constexpr int B = 4 * Tile<T>::N;  // elements of a k-block
+  if (a.dnp + a.drp <= 128 && a.dvp <= 64) return go(k_expanded_attn<T, 128 / B, 4, MR>);
+  if (a.dnp + a.drp <= 192) return go(k_expanded_attn<T, 192 / B, 8, MR>);
+  return go(k_expanded_attn<T, 256 / B, 8, MR>);
+}
+}  // namespace khm

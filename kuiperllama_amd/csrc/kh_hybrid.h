@@ -49,6 +49,7 @@ struct HyLatent {
   HyMat dqkv;  // [q latent | kv latent | rotated key part]
   HyMat uq;    // head by head [dnp | drp]
   HyMat ukT;   // head by head [Rp][dnp]: W_uk transposed
+  HyMat uk;    // head by head [dnp][Rp]
   HyMat uv;    // head by head [dvp][Rp]
   HyMat o;     // columns head by head, dvp each
   HyVec qn, kvn, sink;
@@ -111,6 +112,10 @@ struct Hybrid {
         *sh_g = nullptr, *part = nullptr, *wlogits = nullptr;
   void *xn1 = nullptr, *xn2 = nullptr, *a0 = nullptr, *a1 = nullptr, *a2 = nullptr, *h = nullptr, *hs = nullptr,
        *xw = nullptr;
+  // expanded latent attention: keys [exp_keys][H dnp] and transposed values [H dvp][exp_keys] of one segment
+  void *kx = nullptr, *vx = nullptr;
+  int exp_keys = 0;
+  bool any_latent = false;
   int32_t *moe_id = nullptr, *moe_rows = nullptr, *moe_slot = nullptr, *n_tiles = nullptr;
   LgTile* tiles = nullptr;
   int max_tiles = 0;
@@ -138,6 +143,7 @@ struct HyEntry {  // tokens of one sequence in a pass
 // ---- kh_hybrid_load.hip
 int hy_create(const char* config, size_t config_len, const void* tensors, size_t nbytes, const kh_model_opts* o, kh_model** out);
 void hy_destroy(kh_model* m);
+int hy_expand_buffers(kh_model* m, int keys);       // room for the expanded keys / values of that many tokens
 int hy_kv_ensure(kh_model* m, int slot, int rows);  // cache rows [0, rows) of a slot backed by memory
 bool hy_is_folder(const char* path);
 int hy_create_from_folder(const char* path, const kh_model_opts* o, kh_model** out);

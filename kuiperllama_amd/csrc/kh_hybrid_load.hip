@@ -12,6 +12,7 @@
 #include <sys/stat.h>
 #include <unistd.h>
 
+#include <algorithm>
 #include <atomic>
 #include <map>
 #include <thread>
@@ -266,6 +267,7 @@ int load_latent(Plan& pl, Tensors& ts, const std::string& p, const JsonValue& v,
   pl.put(la.dqkv, la.qr, ts.need(p + ".dkv", {la.R + la.dr, W}), 0, la.R + la.dr);
   la.uq = pl.mat(H * (la.dnp + la.drp), la.qr, la.qrp);
   la.ukT = pl.mat(H * la.Rp, la.dn, la.dnp);
+  la.uk = pl.mat(H * la.dnp, la.R, la.Rp);
   la.uv = pl.mat(H * la.dvp, la.R, la.Rp);
   la.o = pl.mat(W, H * la.dvp, H * la.dvp);
   const Tensor *uq = ts.need(p + ".uq", {(int64_t)H * (la.dn + la.dr), la.qr}), *uk = ts.need(p + ".uk", {(int64_t)H * la.dn, la.R}),
@@ -273,6 +275,7 @@ int load_latent(Plan& pl, Tensors& ts, const std::string& p, const JsonValue& v,
   for (int h = 0; h < H; ++h) {
     pl.put(la.uq, (int64_t)h * (la.dnp + la.drp), uq, (int64_t)h * (la.dn + la.dr), la.dn);
     pl.put(la.uq, (int64_t)h * (la.dnp + la.drp) + la.dnp, uq, (int64_t)h * (la.dn + la.dr) + la.dn, la.dr);
+    pl.put(la.uk, (int64_t)h * la.dnp, uk, (int64_t)h * la.dn, la.dn);
     pl.put_t(la.ukT, (int64_t)h * la.Rp, uk, (int64_t)h * la.dn, la.dn);
     pl.put(la.uv, (int64_t)h * la.dvp, uv, (int64_t)h * la.dv, la.dv);
     pl.put(la.o, 0, o, 0, W, (int64_t)h * la.dv, la.dv, (int64_t)h * la.dvp);
@@ -332,7 +335,7 @@ int load_gufanex(const JsonValue& cfg, Tensors& ts, Plan& pl, Hybrid& hy) {
   if (!(c.eps > 0)) return KH_ERR_FORMAT;
   const int W = c.width, L = (int)ls->arr.size();
   c.widthp = padk(W);
-  hy.embed = pl.mat(c.vocab, W, W);
+  hy.embed = pl.mat(c.vocab, W, c.widthp);
   pl.put(hy.embed, 0, ts.need("embed", {c.vocab, W}), 0, c.vocab);
   hy.head = pl.mat(c.vocab, W, c.widthp);
   pl.put(hy.head, 0, ts.need("head", {c.vocab, W}), 0, c.vocab);
@@ -344,7 +347,11 @@ int load_gufanex(const JsonValue& cfg, Tensors& ts, Plan& pl, Hybrid& hy) {
     c.loop_stop = lp->integer("stop", -1);
     c.loop_times = lp->integer("times", -1);
     if (c.loop_start < 0 || c.loop_stop <= c.loop_start || c.loop_stop > L || c.loop_times < 1) return KH_ERR_FORMAT;
-    hy.step = pl.vec(ts.need("loop.step", {c.loop_times, W}));
+    std::vector<float> step((size_t)c.loop_times * c.widthp, 0.f);
+    if (const Tensor* t = ts.need("loop.step", {c.loop_times, W}))
+      for (int p = 0; p < c.loop_times; ++p)
+        for (int i = 0; i < W; ++i) step[(size_t)p * c.widthp + i] = t->at((int64_t)p * W + i);
+    hy.step = pl.vec(std::move(step));
   }
   int rc;
   for (int i = 0; i < L; ++i) {
@@ -405,7 +412,7 @@ void each_mat(Hybrid& hy, F&& f) {
   f(hy.embed);
   f(hy.head);
   for (auto& l : hy.layers) {
-    for (HyMat* m : {&l.mb.in, &l.mb.x, &l.mb.dt, &l.mb.o, &l.la.dqkv, &l.la.uq, &l.la.ukT, &l.la.uv, &l.la.o, &l.ff.zr,
+    for (HyMat* m : {&l.mb.in, &l.mb.x, &l.mb.dt, &l.mb.o, &l.la.dqkv, &l.la.uq, &l.la.ukT, &l.la.uk, &l.la.uv, &l.la.o, &l.ff.zr,
                      &l.ff.gu, &l.ff.down, &l.ff.sgu, &l.ff.sdown})
       if (m->N) f(*m);
   }
@@ -421,7 +428,7 @@ void each_vec(Hybrid& hy, F&& f) {
 
 int alloc_workspace(kh_model* m) {
   Hybrid& hy = *m->hy;
-  const size_t T = KH_HY_TMAX, W = (size_t)hy.c.width, Wp = (size_t)hy.c.widthp, es = hy.elem();
+  const size_t T = KH_HY_TMAX, Wp = (size_t)hy.c.widthp, es = hy.elem();
   hy.tmax = KH_HY_TMAX;
   size_t f32a = 1, a0 = 1, a1 = 1, a2 = 1, dt = 1, bc = 1, z = 1, ends = 1, dtsum = 1, h = 1, hs = 1, y = 1, top = 1, tiles = 1;
   auto up = [](size_t& v, size_t n) { v = v > n ? v : n; };
@@ -443,6 +450,8 @@ int alloc_workspace(kh_model* m) {
       up(f32a, T * (size_t)(a.qr + a.R + a.dr));
       up(a0, T * (size_t)(a.qrp));
       up(a0, T * (size_t)(a.H * a.Rp));
+      up(a0, T * (size_t)(a.H * a.dvp));
+      hy.any_latent = true;
       up(a1, T * (size_t)(a.H * (a.dnp + a.drp)));
       up(a1, T * (size_t)(a.H * a.dvp));
       up(a2, T * (size_t)(a.H * a.row()));
@@ -451,7 +460,7 @@ int alloc_workspace(kh_model* m) {
       const HyMoe& f = l.ff;
       up(z, T * (size_t)f.zr.N);
       up(h, T * (size_t)f.top * (size_t)f.ffp);
-      up(y, T * (size_t)f.top * W);
+      up(y, T * (size_t)f.top * Wp);
       up(top, (size_t)f.top);
       up(hs, T * (size_t)f.sffp);
       up(tiles, T * (size_t)f.top / 32 + (size_t)f.E + 1);
@@ -473,17 +482,17 @@ int alloc_workspace(kh_model* m) {
   };
 #define TRY(e) \
   if ((rc = (e)) != KH_OK) return rc
-  TRY(zf(&hy.x, T * W));
-  TRY(zf(&hy.x0, T * W));
-  TRY(zf(&hy.mix, T * W));
-  TRY(zf(&hy.sh, T * W));
+  TRY(zf(&hy.x, T * Wp));
+  TRY(zf(&hy.x0, T * Wp));
+  TRY(zf(&hy.mix, T * Wp));
+  TRY(zt((void**)&hy.sh, T * Wp));
   TRY(zf(&hy.f32a, f32a));
   TRY(zf(&hy.dt, dt));
   TRY(zf(&hy.bc, bc));
   TRY(zf(&hy.z, z));
   TRY(zf(&hy.ends, ends));
   TRY(zf(&hy.dtsum, dtsum));
-  TRY(zf(&hy.y, y));
+  TRY(zt((void**)&hy.y, y));
   TRY(zf(&hy.moe_w, T * top));
   TRY(zf(&hy.id_w, T));
   TRY(zf(&hy.sh_g, T));
@@ -521,7 +530,7 @@ int finish(kh_model* m, Plan& pl) {
     KH_CHECK_HIP(upload_chunked(m->arena, img.data(), bytes, m->stream, &m->load_ms));
   }
   {
-    std::vector<float> f(pl.floats + 1, 0.f);
+    std::vector<float> f((pl.floats + 127) / 64 * 64, 0.f);  // vectors are read in whole padded rows
     for (auto& v : pl.vecs) memcpy(f.data() + v.first, v.second.data(), v.second.size() * 4);
     KH_CHECK_HIP(hipMalloc((void**)&hy.farena, f.size() * 4));
     KH_CHECK_HIP(hipMemcpy(hy.farena, f.data(), f.size() * 4, hipMemcpyHostToDevice));
@@ -668,7 +677,7 @@ void hy_destroy(kh_model* m) {
   if (!h) return;
   void* dev[] = {h->farena, h->state, h->x, h->x0, h->mix, h->f32a, h->y, h->sh, h->dt, h->bc, h->z, h->ends, h->dtsum,
                  h->moe_w, h->id_w, h->sh_g, h->part, h->wlogits, h->xn1, h->xn2, h->a0, h->a1, h->a2, h->h, h->hs, h->xw,
-                 h->moe_id, h->moe_rows, h->moe_slot, h->n_tiles, h->tiles, h->d_tab, h->d_one};
+                 h->moe_id, h->moe_rows, h->moe_slot, h->n_tiles, h->tiles, h->kx, h->vx, h->d_tab, h->d_one};
   for (void* p : dev)
     if (p) (void)hipFree(p);
   for (float2* t : h->rope_tabs) (void)hipFree(t);
@@ -689,6 +698,30 @@ int hy_kv_ensure(kh_model* m, int slot, int rows) {
     if (rc != KH_OK) return rc;
   }
   hy.rows_ok[(size_t)slot] = rows;
+  return KH_OK;
+}
+
+int hy_expand_buffers(kh_model* m, int keys) {
+  Hybrid& hy = *m->hy;
+  size_t k = 0, v = 0;
+  const size_t n = (size_t)pad_to(keys, 512);
+  for (auto& l : hy.layers)
+    if (l.mixer == HY_LATENT) {
+      k = std::max(k, n * l.la.H * l.la.dnp);
+      v = std::max(v, n * l.la.H * l.la.dvp);
+    }
+  for (void** p : {&hy.kx, &hy.vx}) {
+    if (*p) (void)hipFree(*p);
+    *p = nullptr;
+  }
+  hy.exp_keys = 0;
+  int rc;
+  if ((rc = dalloc((char**)&hy.kx, k * hy.elem())) != KH_OK) return rc;
+  if ((rc = dalloc((char**)&hy.vx, v * hy.elem())) != KH_OK) return rc;
+  // columns behind a sequence's last key are read as operands under zero weights: they must be finite
+  KH_CHECK_HIP(hipMemsetAsync(hy.kx, 0, k * hy.elem(), m->stream));
+  KH_CHECK_HIP(hipMemsetAsync(hy.vx, 0, v * hy.elem(), m->stream));
+  hy.exp_keys = (int)n;
   return KH_OK;
 }
 

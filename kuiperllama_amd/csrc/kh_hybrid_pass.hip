@@ -6,6 +6,7 @@
 
 #include <algorithm>
 
+#include "kh_expanded.h"
 #include "kh_hybrid.h"
 
 using namespace khm;
@@ -21,8 +22,13 @@ namespace {
 struct LatTiles {
   int H, big, cp, off, n;  // big: latents of more than 256; offset in ints from the table base
 };
+struct PassSeg {
+  int slot, row0, n, pos0;
+};
 // device view of one pass
 struct Pass {
+  std::vector<PassSeg> segs;
+  bool expand = false;  // few long segments: latent attention in its expanded form
   int T = 0, S = 0, n_chunks = 0, n_multi_segs = 0, n_multi_chunks = 0, n_want = 0;
   PassTabs p{};
   const ScanChunk* chunks = nullptr;
@@ -53,7 +59,7 @@ struct Runner {
   Hybrid& hy;
   const Pass& ps;
   hipStream_t s;
-  AddArgs pend{};
+  AddArgs<T> pend{};
   const T* pend_xn2 = nullptr;
 
   Runner(kh_model* mm, const Pass& p) : m(mm), hy(*mm->hy), ps(p), s(mm->stream) {}
@@ -83,7 +89,7 @@ struct Runner {
     a.ld = hy.c.widthp;
     a.from_embed = from_embed;
     a.add_x0 = pass_no > 0;
-    a.step = pass_no >= 0 ? hy.step.p + (size_t)pass_no * hy.c.width : nullptr;
+    a.step = pass_no >= 0 ? hy.step.p + (size_t)pass_no * hy.c.widthp : nullptr;
     a.eps = hy.c.eps;
     a.xn2_prev = (const T*)hy.xn2;
     a.xn1 = (T*)hy.xn1;
@@ -96,8 +102,8 @@ struct Runner {
         a.b2 = l->n2b.p;
       }
     }
-    pend = AddArgs{};
-    hipLaunchKernelGGL(k_combine<T>, dim3(ps.T), dim3(256), (size_t)hy.c.width * 4, s, a);
+    pend = AddArgs<T>{};
+    hipLaunchKernelGGL(k_combine<T>, dim3(ps.T), dim3(256), (size_t)hy.c.widthp * 4, s, a);
     return KH_OK;
   }
 
@@ -116,7 +122,8 @@ struct Runner {
     cv.ldo = mb.innerp;
     cv.taps = mb.taps;
     cv.p = ps.p;
-    hipLaunchKernelGGL(k_conv_silu<T>, dim3((I + 255) / 256, ps.T), dim3(256), 0, s, cv);
+    hipLaunchKernelGGL(k_conv_silu<T>, dim3((I + 256 * Tile<T>::N - 1) / (256 * Tile<T>::N), (ps.T + KH_CONV_TT - 1) / KH_CONV_TT),
+                       dim3(256), 0, s, cv, ps.T);
     hipLaunchKernelGGL(k_conv_state<T>, dim3((I + 255) / 256, ps.S), dim3(256), 0, s, cv);
     {
       LgArgs a = gemm(mb.x, hy.a1, mb.innerp, hy.a2, mb.rankp);
@@ -156,7 +163,30 @@ struct Runner {
     }
     TRY((scan_launch<T, true>(s, sc, ps.n_chunks)));
     if (state_only) return KH_OK;
-    return lg_launch<T, LG_F32>(s, gemm(mb.o, hy.a2, mb.innerp, hy.mix, hy.c.width));
+    return lg_launch<T, LG_F32>(s, gemm(mb.o, hy.a2, mb.innerp, hy.mix, hy.c.widthp));
+  }
+
+  // keys and values of every head of one segment, rebuilt from its cached latents, and its attention: q in a1 -> a0
+  int expanded(const HyRun& r, const HyLatent& la, const PassSeg& sg) {
+    const int H = la.H, keys = sg.pos0 + sg.n;
+    const T* cache = (const T*)m->kcache + (size_t)sg.slot * hy.kv_slot + r.kv_off;
+    LgArgs k = gemm(la.uk, cache, la.row(), hy.kx, H * la.dnp);
+    k.M = keys;
+    TRY((lg_launch<T, LG_T>(s, k)));
+    LgArgs v{};  // transposed: features are the keys
+    v.W = cache;
+    v.X = la.uv.w;
+    v.out = hy.vx;
+    v.M = H * la.dvp;
+    v.N = keys;
+    v.K = la.Rp;
+    v.ldw = la.row();
+    v.ldx = la.Rp;
+    v.ldo = hy.exp_keys;
+    TRY((lg_launch<T, LG_T>(s, v)));
+    ExpArgs a{hy.a1, hy.kx, hy.vx, cache + la.Rp, la.sink.p, hy.a0, H, la.dnp, la.drp, la.dvp, la.row(), hy.exp_keys,
+              sg.row0, sg.n, sg.pos0, la.scale * 1.44269504088896f};
+    return exp_attn_launch<T>(s, a);
   }
 
   int latent(const HyRun& r, const HyLatent& la, bool state_only) {
@@ -183,6 +213,12 @@ struct Runner {
     hipLaunchKernelGGL(k_latent_prep<T>, dim3(ps.T), dim3(256), 0, s, lp);
     if (state_only) return KH_OK;
     TRY((lg_launch<T, LG_T>(s, gemm(la.uq, hy.a0, la.qrp, hy.a1, H * qh))));
+    if (ps.expand && exp_supported(la.dnp, la.drp, la.dvp)) {
+      if (la.dims)
+        hipLaunchKernelGGL(k_rope_inplace<T>, dim3(ps.T), dim3(256), 0, s, (T*)hy.a1, la.rope, H, la.dnp, la.drp, la.dims, ps.p);
+      for (const PassSeg& sg : ps.segs) TRY(expanded(r, la, sg));
+      return lg_launch<T, LG_F32>(s, gemm(la.o, hy.a0, H * la.dvp, hy.mix, hy.c.widthp));
+    }
     {  // absorbed queries: per head, W_uk^T q_n
       LgArgs a = gemm(la.ukT, hy.a1, H * qh, hy.a2, H * row);
       a.N = la.Rp;
@@ -219,14 +255,14 @@ struct Runner {
       a.o_z = (size_t)la.dvp;
       TRY((lg_launch<T, LG_T>(s, a, H)));
     }
-    return lg_launch<T, LG_F32>(s, gemm(la.o, hy.a1, H * la.dvp, hy.mix, hy.c.width));
+    return lg_launch<T, LG_F32>(s, gemm(la.o, hy.a1, H * la.dvp, hy.mix, hy.c.widthp));
   }
 
   int moe(const HyMoe& f) {
     const int W = hy.c.width, Wp = hy.c.widthp;
     TRY((lg_launch<T, LG_F32>(s, gemm(f.zr, hy.xn2, Wp, hy.z, f.zr.N))));
     RouteArgs ra{hy.z, f.corr.p, hy.moe_id, hy.moe_w, hy.id_w, hy.sh_g, ps.T, f.zr.N, f.n_out(), f.E, f.top, f.sff > 0};
-    hipLaunchKernelGGL(k_moe_route, dim3((ps.T + 3) / 4), dim3(256), 0, s, ra);
+    moe_route_launch(s, ra);
     const int bm = lg_group_bm((long)ps.T * f.top, f.n_out());
     ListArgs li{hy.moe_id, hy.moe_rows, hy.moe_slot, hy.tiles, hy.n_tiles, ps.T, f.top, f.E, bm};
     hipLaunchKernelGGL(k_moe_lists, dim3(1), dim3(1024), 0, s, li);
@@ -242,22 +278,22 @@ struct Runner {
       TRY((lg_launch<T, LG_SWIGLU>(s, a, 1, bm, mt)));
     }
     {
-      LgArgs a = gemm(f.down, hy.h, f.ffp, hy.y, W);
+      LgArgs a = gemm(f.down, hy.h, f.ffp, hy.y, Wp);
       a.N = W;
       a.tiles = hy.tiles;
       a.n_tiles = hy.n_tiles;
       a.w_group = (size_t)W * f.down.ld;
-      TRY((lg_launch<T, LG_F32>(s, a, 1, bm, mt)));
+      TRY((lg_launch<T, LG_T>(s, a, 1, bm, mt)));
     }
-    pend.y = hy.y;
+    pend.y = (const T*)hy.y;
     pend.y_slot = hy.moe_slot;
     pend.y_w = hy.moe_w;
     pend.id_w = hy.id_w;
     pend.top = f.top;
     if (f.sff) {
       TRY((lg_launch<T, LG_SWIGLU>(s, gemm(f.sgu, hy.xn2, Wp, hy.hs, f.sffp))));
-      TRY((lg_launch<T, LG_F32>(s, gemm(f.sdown, hy.hs, f.sffp, hy.sh, W))));
-      pend.sh = hy.sh;
+      TRY((lg_launch<T, LG_T>(s, gemm(f.sdown, hy.hs, f.sffp, hy.sh, Wp))));
+      pend.sh = (const T*)hy.sh;
       pend.sh_g = hy.sh_g;
     }
     return KH_OK;
@@ -277,7 +313,8 @@ struct Runner {
         TRY(combine(nullptr, false, -1));
         const int64_t n = (int64_t)ps.T * hy.c.width;
         if (hy.probe_n + n <= hy.probe_cap) {
-          KH_CHECK_HIP(hipMemcpyAsync(hy.probe + hy.probe_n, hy.x, (size_t)n * 4, hipMemcpyDeviceToHost, s));
+          KH_CHECK_HIP(hipMemcpy2DAsync(hy.probe + hy.probe_n, (size_t)hy.c.width * 4, hy.x, (size_t)hy.c.widthp * 4,
+                                        (size_t)hy.c.width * 4, (size_t)ps.T, hipMemcpyDeviceToHost, s));
           KH_CHECK_HIP(hipStreamSynchronize(s));
           hy.probe_n += n;
         }
@@ -366,7 +403,7 @@ int hy_forward(kh_model* m, const HyEntry* e, int n, const int32_t* want, int n_
   };
   std::vector<Off> offs;
   std::vector<size_t> bases;
-  int ei = 0, eo = 0, row_base = 0, wi = 0;
+  int ei = 0, eo = 0, row_base = 0, wi = 0, exp_keys = 0;
   while (ei < n) {
     std::vector<int32_t> tok, pos, seg, slot, row0, sn, pos0, single, multi, m0, mn, wr, lt;
     while (ei < n && (int)tok.size() < hy.tmax) {
@@ -408,6 +445,13 @@ int hy_forward(kh_model* m, const HyEntry* e, int n, const int32_t* want, int n_
     while (wi < n_want && want[wi] < row_base + p.T) wr.push_back(want[wi++] - row_base);
     p.n_want = (int)wr.size();
     p.no_logits = wr.empty();
+    p.expand = hy.any_latent && p.S <= 8 && !dbg_off("KH_HY_EXPAND");
+    for (int i = 0; i < p.S; ++i) {
+      p.segs.push_back({slot[(size_t)i], row0[(size_t)i], sn[(size_t)i], pos0[(size_t)i]});
+      p.expand = p.expand && sn[(size_t)i] >= 32;
+    }
+    if (p.expand)
+      for (const PassSeg& sg : p.segs) exp_keys = std::max(exp_keys, sg.pos0 + sg.n);
     row_base += p.T;
     multi.insert(multi.end(), single.begin(), single.end());
     TabBuilder tb;
@@ -436,6 +480,7 @@ int hy_forward(kh_model* m, const HyEntry* e, int n, const int32_t* want, int n_
     offs.push_back(o);
     passes.push_back(std::move(p));
   }
+  if (exp_keys > hy.exp_keys) TRY(hy_expand_buffers(m, exp_keys));
   // ---- upload
   if (all.size() > hy.tab_cap) {
     if (hy.h_tab) (void)hipHostFree(hy.h_tab);

@@ -2,6 +2,7 @@
 #include <string.h>
 
 #include <algorithm>
+#include <type_traits>
 
 #include "kh_fused.h"
 #include "kh_hybrid.h"
@@ -49,12 +50,12 @@ size_t lds_out(const Hybrid& hy, const HyLayer& l, int B) {
   const int nbv = Ld<T>::blocks(nv);
   const int nf = l.ff.on ? l.ff.top * Ld<T>::blocks(l.ff.ffp) + (l.ff.sffp ? Ld<T>::blocks(l.ff.sffp) : 0) : 0;
   (void)hy;
-  return (size_t)(nbv + nf) * sizeof(LdBlk) + ((size_t)B * nbv + nf) * Ld<T>::BE * 4;
+  return (size_t)(nbv + nf) * sizeof(LdBlk) + ((size_t)B * nbv + nf) * Ld<T>::BE * 4;  // table, vectors
 }
 template <class T>
 bool fits(const Hybrid& hy, int B) {
   const size_t room = kMaxLds - 2048;  // static shared memory of the kernels
-  if (B * vec_b<T>(hy.c.widthp) > room) return false;
+  if (hy.c.widthp > 8192 || B * vec_b<T>(hy.c.widthp) > room) return false;
   for (auto& l : hy.layers) {
     if (lds_out<T>(hy, l, B) > room) return false;
     if (l.mixer == HY_MAMBA1 && B * vec_b<T>(l.mb.innerp) > room) return false;
@@ -64,7 +65,7 @@ bool fits(const Hybrid& hy, int B) {
 }
 
 template <class K, class... A>
-int go(K kern, dim3 grid, size_t lds, hipStream_t s, A... args) {
+int go(K kern, dim3 grid, int wg, size_t lds, hipStream_t s, A... args) {
   if (lds > 64 * 1024) {
     struct Done { int dev; const void* fn; size_t lds; };
     static thread_local std::vector<Done> done;
@@ -78,7 +79,7 @@ int go(K kern, dim3 grid, size_t lds, hipStream_t s, A... args) {
       done.push_back({dev, (const void*)kern, lds});
     }
   }
-  hipLaunchKernelGGL(kern, grid, dim3(256), lds, s, args...);
+  hipLaunchKernelGGL(kern, grid, dim3(wg), lds, s, args...);
   return KH_OK;
 }
 #define TRY(e)                    \
@@ -89,20 +90,29 @@ int go(K kern, dim3 grid, size_t lds, hipStream_t s, A... args) {
 
 int cdiv(int a, int b) { return (a + b - 1) / b; }
 
-template <class T, int B>
-int launch_scan(const LdScanArgs& a, hipStream_t s) {
-  int G = 1;
-  while (G * KH_SCAN_NS < a.N) G <<= 1;
-  const size_t lds = (size_t)(a.rankp + 2 * G * KH_SCAN_NS + 256 / G) * 4;
-  const dim3 grid(cdiv(a.C, 256 / G), B);
-  switch (G) {
-    case 1: return go(k_ld_scan<T, 1>, grid, lds, s, a);
-    case 2: return go(k_ld_scan<T, 2>, grid, lds, s, a);
-    case 4: return go(k_ld_scan<T, 4>, grid, lds, s, a);
-    case 8: return go(k_ld_scan<T, 8>, grid, lds, s, a);
-    case 16: return go(k_ld_scan<T, 16>, grid, lds, s, a);
-    default: return go(k_ld_scan<T, 32>, grid, lds, s, a);
-  }
+template <class T>
+int launch_scan(const LdScanArgs& a, int B, hipStream_t s) {
+  const dim3 grid(cdiv(a.C, 16), B);
+  if (a.N <= 16) return go(k_ld_scan<T, 1>, grid, 256, 0, s, a);
+  if (a.N <= 32) return go(k_ld_scan<T, 2>, grid, 256, 0, s, a);
+  if (a.N <= 64) return go(k_ld_scan<T, 4>, grid, 256, 0, s, a);
+  if (a.N <= 128) return go(k_ld_scan<T, 8>, grid, 256, 0, s, a);
+  return go(k_ld_scan<T, 16>, grid, 256, 0, s, a);
+}
+// staging depth (float4 per thread) that covers a padded row of the residual stream
+template <class T, class F>
+int with_nv(int ld, F&& f) {
+  const int n = cdiv(Ld<T>::blocks(ld) * Ld<T>::BE / 4, 256);
+  if (n <= 2) return f(std::integral_constant<int, 2>());
+  if (n <= 4) return f(std::integral_constant<int, 4>());
+  return f(std::integral_constant<int, 8>());
+}
+template <class F>
+int with_rp(int n_out, F&& f) {
+  const int per = moe_per(n_out);
+  if (per == 1) return f(std::integral_constant<int, 1>());
+  if (per == 4) return f(std::integral_constant<int, 4>());
+  return f(std::integral_constant<int, 16>());
 }
 
 // One token of B sequences: tables at (tok, pos, slot); logits to `logits` [B][V]; argmax partials of sequence 0 to
@@ -151,7 +161,7 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
       a.x_in = x_in;
       a.x_cur = changed ? x_cur : nullptr;
       a.embed = hy.embed.w;
-      a.step = r.pass >= 0 ? hy.step.p + (size_t)r.pass * W : nullptr;
+      a.step = r.pass >= 0 ? hy.step.p + (size_t)r.pass * Wp : nullptr;
       a.w1 = l.n1.p;
       a.b1 = l.n1b.p;
       a.w2 = f.on ? l.n2.p : nullptr;
@@ -173,7 +183,7 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
         a.taps = l.mb.taps;
         a.xc_ld = l.mb.innerp;
       }
-      TRY(go(k_ld_in<T, B>, dim3(wg), B * vec_b<T>(Wp), s, a));
+      TRY(with_nv<T>(Wp, [&](auto nv) { return go(k_ld_in<T, B, decltype(nv)::value>, dim3(wg), 256, B * vec_b<T>(Wp), s, a); }));
     }
     {
       LdMidArgs a{};
@@ -205,6 +215,7 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
       a.rows = wm.N;
       a.ldm = wm.ld;
       a.n = mamba ? l.mb.inner : l.la.qr;
+      a.n4 = l.mb.innerp / 4;  // convolved inputs are padded with zeros
       a.v = mamba ? st.xc : st.in;
       a.ldv = mamba ? l.mb.innerp : in_ld;
       a.vnorm = mamba ? nullptr : l.la.qn.p;
@@ -229,18 +240,23 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
         a.row = la.row();
         a.dims = la.dims;
       }
-      TRY(go(k_ld_mid<T, B>, dim3(B * a.top * a.nwg_e + a.nwg_m + extra), lds, s, a));
+      TRY(with_nv<T>(Wp, [&](auto nv) {
+        return with_rp(f.on ? f.n_out() : 1, [&](auto rp) {
+          return go(k_ld_mid<T, B, decltype(nv)::value, decltype(rp)::value>, dim3(B * a.top * a.nwg_e + a.nwg_m + extra), 256, lds,
+                    s, a);
+        });
+      }));
     }
     if (mamba) {
       const HyMamba& mb = l.mb;
       LdScanArgs a{st.xc, st.in, st.mid, mb.dt.w, mb.dt_b.p, mb.A2.p, mb.D.p, hy.state + r.st_off, st.v, hy.st_slot,
                    mb.inner, mb.state, mb.rankp, mb.innerp, mb.innerp, tb};
-      TRY((launch_scan<T, B>(a, s)));
+      TRY(launch_scan<T>(a, B, s));
     } else {
       const HyLatent& la = l.la;
       LdAbsorbArgs ab{st.mid, la.ukT.w, la.rope, st.Q, la.H, std::max(1, std::min(cdiv(la.Rp, 32), cdiv(512, la.H * B))),
                       la.dnp, la.dr, la.drp, la.Rp, la.row(), la.dims, tb};
-      TRY(go(k_ld_absorb<T>, dim3(la.H * ab.nwg, B), (size_t)la.dnp * 4, s, ab));
+      TRY(go(k_ld_absorb<T>, dim3(la.H * ab.nwg, B), 256, (size_t)la.dnp * 4, s, ab));
       const Hybrid::Step::Lat* lt = nullptr;
       for (auto& t : st.lat)
         if (t.B == B && t.H == la.H && t.big == (la.Rp > 256)) lt = &t;
@@ -262,14 +278,15 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
       TRY(lat_attn_launch<T>(s, at, lt->n, lt->cp));
       LdValuesArgs va{st.part, la.uv.w, st.v, la.H, std::max(1, std::min(cdiv(la.dvp, 16), cdiv(512, la.H * B))), st.nsplit,
                       la.Rp, la.dvp, tb.pos};
-      TRY(go(k_ld_values<T>, dim3(la.H * va.nwg, B), vec_b<T>(la.Rp), s, va));
+      TRY(go(k_ld_values<T>, dim3(la.H * va.nwg, B), 256, vec_b<T>(la.Rp), s, va));
     }
     {
       const HyMat& wo = mamba ? l.mb.o : l.la.o;
       LdOutArgs a{};
       a.wo = wo.w;
       a.v = st.v;
-      a.n_v = mamba ? l.mb.inner : l.la.H * l.la.dvp;
+      a.n4v = wo.ld / 4;
+      a.ld = Wp;
       a.ld_v = mamba ? l.mb.innerp : l.la.H * l.la.dvp;
       a.ldv = wo.ld;
       a.x_cur = x_cur;
@@ -289,13 +306,17 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
         a.ffp = f.ffp;
         a.sffp = f.sffp;
       }
-      a.nwg = std::min(cdiv(cdiv(W, 2), 4), 1024);
-      TRY(go(k_ld_out<T, B>, dim3(a.nwg), lds_out<T>(hy, l, B), s, a));
+      // waves of a row pair: as many as keep each wave's share within two tiles of the ring, while the launch has at
+      // most four workgroups per CU
+      const int nblk = Ld<T>::blocks(wo.ld) + (f.on ? f.top * Ld<T>::blocks(f.ffp) + (f.sff ? Ld<T>::blocks(f.sffp) : 0) : 0);
+      a.ks = 1;
+      while (a.ks < 8 && nblk / a.ks > 8 && cdiv(cdiv(W, 2) * a.ks * 2, 8) <= 1024) a.ks *= 2;
+      TRY(go(k_ld_out<T, B>, dim3(cdiv(cdiv(W, 2) * a.ks, 8)), 512, lds_out<T>(hy, l, B), s, a));
     }
     x_in = x_out;
   }
   LdHeadArgs h{x_in, hy.fnorm.p, hy.fnorm_b.p, hy.head.w, logits, m->part_val, m->part_idx, W, Wp, hy.c.vocab, hy.c.eps, hy.c.cap};
-  return go(k_ld_head<T, B>, dim3(st.head_wg), B * vec_b<T>(Wp), s, h);
+  return with_nv<T>(Wp, [&](auto nv) { return go(k_ld_head<T, B, decltype(nv)::value>, dim3(st.head_wg), 256, B * vec_b<T>(Wp), s, h); });
 }
 template <class T>
 int step_b(kh_model* m, int B, const LdTabs& tb, float* logits) {
@@ -314,7 +335,7 @@ int hy_step_init(kh_model* m) {
   Hybrid::Step& st = *hy.step_st;
   for (int B : {1, 2, 4})
     if (hy.f32 ? fits<float>(hy, B) : fits<bf16>(hy, B)) st.bmax = B;
-  const size_t B = KH_HY_DECODE_B, W = (size_t)hy.c.width;
+  const size_t B = KH_HY_DECODE_B, W = (size_t)hy.c.widthp;
   size_t in = 1, xc = 1, mid = 1, v = 1, he = 1, hs = 1, z = 1, top = 1, Q = 1, part = 1;
   auto up = [](size_t& a, size_t n) { a = a > n ? a : n; };
   int hmin = 1 << 30;

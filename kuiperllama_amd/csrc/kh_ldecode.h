@@ -33,6 +33,59 @@ struct Ld {
   }
 };
 
+// float4 group i (elements 4 i ..) of a staged vector: its 16-byte slot
+template <class T>
+__device__ __forceinline__ int ld_slot(int i) {
+  constexpr int B4 = Ld<T>::BE / 4, P = Ld<T>::P;
+  const int b = i / B4, r = i - b * B4;
+  return b * B4 + (r % P) * 64 + r / P;
+}
+__device__ __forceinline__ f32x4 f4_zero() { return f32x4{0.f, 0.f, 0.f, 0.f}; }
+// n4 valid float4 of src -> slots [0, total4), zeros behind them; times g
+template <class T, int NT>
+__device__ __forceinline__ void ld_stage(f32x4* xs, const float* src, int n4, int total4, float g, int tid) {
+  for (int i0 = tid; i0 < total4; i0 += 4 * NT) {
+    f32x4 v[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int i = i0 + j * NT;
+      v[j] = i < n4 ? ((const f32x4*)src)[i] : f4_zero();
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (i0 + j * NT < total4) xs[ld_slot<T>(i0 + j * NT)] = v[j] * g;
+  }
+}
+// Layer norm of one row (256 threads, NV float4 each, rows padded with zeros to ld) into LDS slots.  v: the row in
+// registers; returns the normalised values in v (also written to `out` when given).
+template <class T, int NV>
+__device__ __forceinline__ void ld_norm(f32x4 (&v)[NV], const f32x4 (&w)[NV], const f32x4 (&b)[NV], int W, int n4, int total4,
+                                        float eps, float* red, f32x4* xs, f32x4* out) {
+  float s = 0.f;
+#pragma unroll
+  for (int j = 0; j < NV; ++j) s += (v[j].x + v[j].y) + (v[j].z + v[j].w);
+  const float mean = block_sum(s, red) / (float)W;
+  float d2 = 0.f;
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int i = threadIdx.x + 256 * j;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const float d = 4 * i + k < W ? v[j][k] - mean : 0.f;
+      d2 = __builtin_fmaf(d, d, d2);
+    }
+  }
+  const float rstd = 1.0f / sqrtf(block_sum(d2, red) / (float)W + eps);
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int i = threadIdx.x + 256 * j;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) v[j][k] = (v[j][k] - mean) * rstd * w[j][k] + b[j][k];  // pads: zero weight and bias
+    if (i < total4) xs[ld_slot<T>(i)] = i < n4 ? v[j] : f4_zero();
+    if (out && i < n4) out[i] = v[j];
+  }
+}
+
 template <class T, int R, int U>
 struct LdTile {
   typename Tile<T>::frag v[R][U];
@@ -120,12 +173,12 @@ struct LdInSeg {
 struct LdInArgs {
   LdInSeg seg[3];
   int nseg;
-  const float* x_in;   // [B][W]
+  const float* x_in;   // [B][ld]
   float* x_cur;        // written by workgroup 0 when the input is modified
   const void* embed;
   const float* step;
   const float *w1, *b1, *w2, *b2;
-  float* xn2;          // [B][W], written by workgroup 0 (nullptr: no feed-forward)
+  float* xn2;          // [B][ld], written by the router's first workgroup (nullptr: no feed-forward)
   int W, ld, from_embed, add_x0;
   float eps;
   LdTabs t;
@@ -136,7 +189,7 @@ struct LdInArgs {
   int inner, taps, xc_ld;
 };
 
-template <class T, int B>
+template <class T, int B, int NV>
 __global__ __launch_bounds__(256) void k_ld_in(const LdInArgs a) {
   constexpr int R = 4, U = 4;
   extern __shared__ __attribute__((aligned(16))) char smem_raw[];
@@ -181,37 +234,40 @@ __global__ __launch_bounds__(256) void k_ld_in(const LdInArgs a) {
     ld_load<T, R, U>(t, row, 0, nblk, nch, lane);
   }
   // ---- layer norm of B rows
-  const int xstride = nblk * Ld<T>::BE;
-  for (int q = 0; q < B; ++q) {
-    const int tok = a.t.tok[q];
-    const T* e = (const T*)a.embed + (size_t)tok * a.W;
-    float* x = xs + (size_t)q * xstride;
-    float s = 0.f;
-    for (int i = threadIdx.x; i < xstride; i += 256) {
-      float v = 0.f;
-      if (i < a.W) {
-        v = a.from_embed ? (float)e[i] : a.x_in[(size_t)q * a.W + i];
-        if (a.add_x0) v += (float)e[i];
-        if (a.step) v += a.step[i];
-        if (a.x_cur && wg == 0) a.x_cur[(size_t)q * a.W + i] = v;
+  const int xstride = nblk * Ld<T>::BE, n4 = a.ld >> 2, total4 = xstride >> 2;
+  {
+    f32x4 nw[NV], nb[NV], v[NV];
+    const f32x4 *wp = (const f32x4*)(norm2 ? a.w2 : a.w1), *bp = (const f32x4*)(norm2 ? a.b2 : a.b1);
+    auto get = [&](int q) __attribute__((always_inline)) {
+      const T* e = (const T*)a.embed + (size_t)a.t.tok[q] * a.ld;
+#pragma unroll
+      for (int j = 0; j < NV; ++j) {
+        const int i = threadIdx.x + 256 * j;
+        v[j] = f4_zero();
+        if (i < n4) {
+          v[j] = a.from_embed ? quad_f(e + 4 * i) : ((const f32x4*)(a.x_in + (size_t)q * a.ld))[i];
+          if (a.add_x0) v[j] += quad_f(e + 4 * i);
+          if (a.step) v[j] += ((const f32x4*)a.step)[i];
+        }
       }
-      x[Ld<T>::place(i)] = v;
-      s += v;
+    };
+    get(0);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int i = threadIdx.x + 256 * j;
+      nw[j] = i < n4 ? wp[i] : f4_zero();
+      nb[j] = i < n4 ? bp[i] : f4_zero();
     }
-    const float mean = block_sum(s, red) / (float)a.W;
-    float d2 = 0.f;
-    for (int i = threadIdx.x; i < a.W; i += 256) {
-      const float d = x[Ld<T>::place(i)] - mean;
-      d2 = __builtin_fmaf(d, d, d2);
-    }
-    const float rstd = 1.0f / sqrtf(block_sum(d2, red) / (float)a.W + a.eps);
-    for (int i = threadIdx.x; i < a.W; i += 256) {
-      const float n = (x[Ld<T>::place(i)] - mean) * rstd;
-      float y1 = 0.f;
-      if (norm2) y1 = n * a.w2[i] + a.b2[i];
-      else y1 = n * a.w1[i] + a.b1[i];
-      x[Ld<T>::place(i)] = y1;
-      if (a.xn2 && wg == 0) a.xn2[(size_t)q * a.W + i] = n * a.w2[i] + a.b2[i];
+    for (int q = 0; q < B; ++q) {
+      if (q) get(q);
+      if (a.x_cur && wg == 0) {
+#pragma unroll
+        for (int j = 0; j < NV; ++j)
+          if ((int)threadIdx.x + 256 * j < n4) ((f32x4*)(a.x_cur + (size_t)q * a.ld))[threadIdx.x + 256 * j] = v[j];
+      }
+      // the router's first workgroup leaves the second norm for the launches that follow
+      f32x4* keep = a.xn2 && wg == a.seg[1].wg0 ? (f32x4*)(a.xn2 + (size_t)q * a.ld) : nullptr;
+      ld_norm<T, NV>(v, nw, nb, a.W, n4, total4, a.eps, red, (f32x4*)(xs + (size_t)q * xstride), keep);
     }
   }
   __syncthreads();
@@ -274,7 +330,7 @@ struct LdMidArgs {
   const float* v;        // [B][ldv] input vectors (n valid entries)
   const float* vnorm;    // RMS norm weight (nullptr: none)
   float* om;             // [B][ldo]
-  int nwg_m, rows, ldm, n, ldv, ldo;
+  int nwg_m, rows, ldm, n, n4, ldv, ldo;  // n4: float4 of a row that may be read (no norm)
   // cache rows of latent attention: the last B workgroups
   int latent;
   const float* raw;      // [B][ldv]: q latent, kv latent, rotated part
@@ -286,14 +342,12 @@ struct LdMidArgs {
   float eps;
   LdTabs t;
 };
-template <class T, int B>
+template <class T, int B, int NV, int RP>
 __global__ __launch_bounds__(256) void k_ld_mid(const LdMidArgs a) {
   constexpr int R = 4, U = 4;
   extern __shared__ __attribute__((aligned(16))) char smem_raw[];
   float* xs = (float*)smem_raw;
   __shared__ float red[KH_WAVES_MAX];
-  __shared__ int s_id;
-  __shared__ float s_w;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   int wg = blockIdx.x;
   LdTile<T, R, U> t;
@@ -301,44 +355,64 @@ __global__ __launch_bounds__(256) void k_ld_mid(const LdMidArgs a) {
   const int ne = B * a.top * a.nwg_e;
   if (wg < ne) {  // ---- one chosen expert of one sequence
     const int pair = wg / a.nwg_e, part = wg - pair * a.nwg_e, q = pair / a.top, k = pair - q * a.top;
-    if (wave == 0) {
-      float idw = 0.f;
-      moe_route(a.z + (size_t)q * a.ldz, a.corr, a.n_out, a.top, lane, [&](int kk, int id, float w) __attribute__((always_inline)) {
-        const bool ident = id >= a.n_expert;
-        if (ident) idw += w;
-        if (kk == k && lane == 0) {
-          s_id = ident ? -1 : id;
-          s_w = w;
-          if (part == 0) a.ids[q * a.top + k] = ident ? -1 : id;
-        }
-      });
-      if (k == 0 && part == 0 && lane == 0) {
+    const int nblk = Ld<T>::blocks(a.ldw), nch = a.ldw / Ld<T>::E;
+    const int n4 = a.ldw >> 2, total4 = nblk * Ld<T>::BE / 4;
+    f32x4 x[NV];  // requested first: in flight while the choice is made
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int i = threadIdx.x + 256 * j;
+      x[j] = i < n4 ? ((const f32x4*)(a.xn2 + (size_t)q * a.ldw))[i] : f4_zero();
+    }
+    // every wave makes the choice for itself: its weight loads leave without a barrier
+    float idw = 0.f, w = 0.f;
+    int id = -1;
+    moe_route<RP>(a.z + (size_t)q * a.ldz, a.corr, a.n_out, a.top, lane, [&](int kk, int i, float wt) __attribute__((always_inline)) {
+      const bool ident = i >= a.n_expert;
+      if (ident) idw += wt;
+      if (kk == k) {
+        id = ident ? -1 : i;
+        w = wt;
+      }
+    });
+    if (part == 0 && threadIdx.x == 0) {
+      a.ids[q * a.top + k] = id;
+      if (k == 0) {
         a.id_w[q] = idw;
         if (a.shared) a.sh_g[q] = sigmoid1(a.z[(size_t)q * a.ldz + a.n_out]);
       }
     }
-    const int nblk = Ld<T>::blocks(a.ldw), nch = a.ldw / Ld<T>::E;
-    for (int i = threadIdx.x; i < nblk * Ld<T>::BE; i += 256)
-      xs[Ld<T>::place(i)] = i < a.W ? a.xn2[(size_t)q * a.W + i] : 0.f;
-    __syncthreads();
-    const int id = s_id;
-    if (id < 0) return;  // identity expert: no tensors
-    const float w = s_w;
+    if (id < 0) return;  // identity expert: no tensors (the whole workgroup agrees)
     const T* base = (const T*)a.gu + (size_t)id * 2 * a.ffp * a.ldw;
     const int items = a.ffp / 2;
-    for (int it = part * 4 + wave; it < items; it += a.nwg_e * 4) {
+    int it = part * 4 + wave;
+    auto set_rows = [&](int i) __attribute__((always_inline)) {
 #pragma unroll
       for (int r = 0; r < R; ++r) {
-        const int j = it * 2 + (r & 1);
+        const int j = i * 2 + (r & 1);
         row[r] = base + (size_t)((j >> 4) * 32 + (j & 15) + (r >> 1) * 16) * a.ldw;
       }
-      float acc[R][1] = {};
+    };
+    if (it < items) {
+      set_rows(it);
       ld_load<T, R, U>(t, row, 0, nblk, nch, lane);
+    }
+#pragma unroll
+    for (int j = 0; j < NV; ++j)
+      if ((int)threadIdx.x + 256 * j < total4) ((f32x4*)xs)[ld_slot<T>(threadIdx.x + 256 * j)] = x[j];
+    __syncthreads();
+    while (it < items) {
+      float acc[R][1] = {};
       ld_rows<T, R, U, 1>(t, row, nblk, nch, xs, 0, lane, acc);
+      const int cur = it;
+      it += a.nwg_e * 4;
+      if (it < items) {
+        set_rows(it);
+        ld_load<T, R, U>(t, row, 0, nblk, nch, lane);
+      }
       ld_reduce<R, 1>(acc);
       if (lane < 2) {
         const float g = ld_pick<R, 1>(acc, lane, 0), u = ld_pick<R, 1>(acc, lane + 2, 0);
-        a.he[(size_t)pair * a.ffp + it * 2 + lane] = w * (silu1(g) * u);
+        a.he[(size_t)pair * a.ffp + cur * 2 + lane] = w * (silu1(g) * u);
       }
     }
     return;
@@ -361,15 +435,16 @@ __global__ __launch_bounds__(256) void k_ld_mid(const LdMidArgs a) {
       ld_load<T, R, U>(t, row, 0, nblk, nch, lane);
     }
     for (int q = 0; q < B; ++q) {
-      float s = 0.f;
-      for (int i = threadIdx.x; i < xstride; i += 256) {
-        const float v = i < a.n ? a.v[(size_t)q * a.ldv + i] : 0.f;
-        xs[(size_t)q * xstride + Ld<T>::place(i)] = v;
-        s = __builtin_fmaf(v, v, s);
-      }
-      if (a.vnorm) {
+      const float* v = a.v + (size_t)q * a.ldv;
+      f32x4* x4 = (f32x4*)(xs + (size_t)q * xstride);
+      if (!a.vnorm) {
+        ld_stage<T, 256>(x4, v, a.n4, xstride >> 2, 1.f, threadIdx.x);
+      } else {
+        float s = 0.f;
+        for (int i = threadIdx.x; i < a.n; i += 256) s = __builtin_fmaf(v[i], v[i], s);
         const float rs = 1.0f / sqrtf(block_sum(s, red) / (float)a.n + a.eps);
-        for (int i = threadIdx.x; i < a.n; i += 256) xs[(size_t)q * xstride + Ld<T>::place(i)] *= rs * a.vnorm[i];
+        for (int i = threadIdx.x; i < xstride; i += 256)
+          xs[(size_t)q * xstride + Ld<T>::place(i)] = i < a.n ? v[i] * rs * a.vnorm[i] : 0.f;
       }
     }
     __syncthreads();
@@ -416,7 +491,7 @@ __global__ __launch_bounds__(256) void k_ld_mid(const LdMidArgs a) {
   }
 }
 
-// ---- k_ld_scan: grid (channels / (256 / G), B) --------------------------------------------------------------------
+// ---- k_ld_scan: 16 lanes per channel, 16 channels per workgroup.  grid (channels / 16, B) ----------------------------
 struct LdScanArgs {
   const float *xc, *xz, *dbc;  // [B][xc_ld], [B][2 C] (z half), [B][rankp + 2 N]
   const void* wdt;             // [C][rankp]
@@ -427,63 +502,44 @@ struct LdScanArgs {
   int C, N, rankp, xc_ld, y_ld;
   LdTabs t;
 };
-template <class T, int G>
+template <class T, int NSL /* states per lane */>
 __global__ __launch_bounds__(256) void k_ld_scan(const LdScanArgs a) {
-  extern __shared__ __attribute__((aligned(16))) char smem_raw[];
-  constexpr int CW = 256 / G;           // channels of a workgroup
   constexpr int E = Tile<T>::N;
-  float* v = (float*)smem_raw;          // dt inputs [rankp], B [G 8], C [G 8]
-  const int NP = G * KH_SCAN_NS;
-  float* bc = v + a.rankp;
-  float* dts = bc + 2 * NP;             // [CW]
-  const int q = blockIdx.y, c0 = blockIdx.x * CW;
-  const float* dbc = a.dbc + (size_t)q * (a.rankp + 2 * a.N);
-  const int g = threadIdx.x & (G - 1), cl = (int)threadIdx.x / G;
-  const int c = c0 + cl;
+  const int q = blockIdx.y, g = threadIdx.x & 15;
+  const int c = blockIdx.x * 16 + ((int)threadIdx.x >> 4);
   const bool live = c < a.C;
   const int cc = live ? c : a.C - 1;
+  const float* dbc = a.dbc + (size_t)q * (a.rankp + 2 * a.N);
   float* st = a.state + (size_t)a.t.slot[q] * a.slot_stride + (size_t)cc * a.N;
   const bool fresh = a.t.pos[q] == 0;
-  float A2[KH_SCAN_NS], S[KH_SCAN_NS];
+  float A2[NSL], S[NSL], Bn[NSL], Cn[NSL];
 #pragma unroll
-  for (int j = 0; j < KH_SCAN_NS; ++j) {
-    const int n = g * KH_SCAN_NS + j;
-    A2[j] = n < a.N ? a.A2[(size_t)cc * a.N + n] : 0.f;
-    S[j] = n < a.N && !fresh ? st[n] : 0.f;
+  for (int j = 0; j < NSL; ++j) {  // neighbouring lanes own neighbouring states
+    const int n = j * 16 + g;
+    const bool in = n < a.N;
+    A2[j] = in ? a.A2[(size_t)cc * a.N + n] : 0.f;
+    S[j] = in && !fresh ? st[n] : 0.f;
+    Bn[j] = in ? dbc[a.rankp + n] : 0.f;
+    Cn[j] = in ? dbc[a.rankp + a.N + n] : 0.f;
   }
-  for (int i = threadIdx.x; i < a.rankp; i += 256) v[i] = dbc[i];
-  for (int i = threadIdx.x; i < 2 * NP; i += 256) {
-    const int which = i >= NP, n = i - which * NP;
-    bc[i] = n < a.N ? dbc[a.rankp + which * a.N + n] : 0.f;
-  }
-  __syncthreads();
-  // dt: eight lanes per channel
-  for (int i = (int)threadIdx.x >> 3; i < CW; i += 32) {
-    const int ch = c0 + i < a.C ? c0 + i : a.C - 1;
-    float s = 0.f;
-    for (int k = (threadIdx.x & 7) * E; k < a.rankp; k += 8 * E) {
-      const typename Tile<T>::frag w = *(const typename Tile<T>::frag*)((const T*)a.wdt + (size_t)ch * a.rankp + k);
+  const float x = a.xc[(size_t)q * a.xc_ld + cc], z = a.xz[(size_t)q * 2 * a.C + a.C + cc];
+  float s = 0.f;
+  for (int k = g * E; k < a.rankp; k += 16 * E) {
+    const typename Tile<T>::frag w = *(const typename Tile<T>::frag*)((const T*)a.wdt + (size_t)cc * a.rankp + k);
 #pragma unroll
-      for (int e = 0; e < E; ++e) s = __builtin_fmaf((float)w[e], v[k + e], s);
-    }
-    s = group_sum<8>(s);
-    if ((threadIdx.x & 7) == 0) dts[i] = softplus1(s + a.dt_b[ch]);
+    for (int e = 0; e < E; ++e) s = __builtin_fmaf((float)w[e], dbc[k + e], s);
   }
-  __syncthreads();
-  const float dt = dts[cl], x = a.xc[(size_t)q * a.xc_ld + cc], dx = dt * x;
+  const float dt = softplus1(group_sum<16>(s) + a.dt_b[cc]), dx = dt * x;
   float y = 0.f;
 #pragma unroll
-  for (int j = 0; j < KH_SCAN_NS; ++j) {
-    const int n = g * KH_SCAN_NS + j;
-    S[j] = __builtin_fmaf(__builtin_amdgcn_exp2f(dt * A2[j]), S[j], dx * bc[n]);
-    y = __builtin_fmaf(S[j], bc[NP + n], y);
+  for (int j = 0; j < NSL; ++j) {
+    const int n = j * 16 + g;
+    S[j] = __builtin_fmaf(__builtin_amdgcn_exp2f(dt * A2[j]), S[j], dx * Bn[j]);
+    y = __builtin_fmaf(S[j], Cn[j], y);
     if (live && n < a.N) st[n] = S[j];
   }
-  y = group_sum<G>(y);
-  if (g == 0 && live) {
-    y = __builtin_fmaf(a.D[c], x, y);
-    a.y[(size_t)q * a.y_ld + c] = y * silu1(a.xz[(size_t)q * 2 * a.C + a.C + c]);
-  }
+  y = group_sum<16>(y);
+  if (g == 0 && live) a.y[(size_t)q * a.y_ld + c] = __builtin_fmaf(a.D[c], x, y) * silu1(z);
 }
 
 // ---- k_ld_absorb: Q row of every head: W_uk^T q_n and the rotated part.  grid (H nwg, B) ------------------------------
@@ -599,132 +655,130 @@ __global__ __launch_bounds__(256) void k_ld_values(const LdValuesArgs a) {
 // ---- k_ld_out ----------------------------------------------------------------------------------------------------
 struct LdOutArgs {
   const void* wo;         // [W][ldv]
-  const float* v;         // [B][ld_v] mixer vector (n_v valid)
+  const float* v;         // [B][ld_v] mixer vector (4 n4v readable)
   const void *down, *sdown;  // experts [W][ffp] each; shared [W][sffp]
   const float *he, *hs;   // [B][top][ffp] (weighted), [B][sffp]
   const int32_t* ids;     // [B][top]
   const float *id_w, *sh_g, *xn2, *x_cur;
-  float* x_out;           // [B][W]
-  int W, n_v, ld_v, ldv, top, ffp, sffp, moe, nwg;
+  float* x_out;           // [B][ld]
+  int W, ld, n4v, ld_v, ldv, top, ffp, sffp, moe, ks;
 };
-// A row of the concatenation is a list of blocks: table entry = weight pointer of row 0 at the block, row stride and
-// valid chunks.  Vector parts lie block by block in the same order.
+// Workgroup = 8 waves = 8 / ks groups of ks waves; a group owns R rows, its waves share the blocks of the concatenation
+// [mixer | shared | expert 0 | expert 1 ...] (identity experts: blocks with no chunks, skipped).  Experts differ between
+// sequences, so for B > 1 the feed-forward part runs once per sequence.
 struct LdBlk {
-  const void* p;
-  int stride, nch;  // elements between rows; 16-byte chunks valid in this block
+  const void* p;    // row 0 at this block
+  int stride, nch;  // elements between rows; 16-byte chunks of a row in this block (0: skip)
 };
 template <class T, int B>
-__global__ __launch_bounds__(256) void k_ld_out(const LdOutArgs a) {
-  constexpr int R = 2, U = 8;
+__global__ __launch_bounds__(512) void k_ld_out(const LdOutArgs a) {
+  constexpr int R = 2, U = 4;
   extern __shared__ __attribute__((aligned(16))) char smem_raw[];
   typedef typename Tile<T>::frag frag;
   constexpr int BE = Ld<T>::BE, E = Ld<T>::E;
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  __shared__ float comb[8][R * B];
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int nbv = Ld<T>::blocks(a.ldv);
   const int nbe = a.moe ? Ld<T>::blocks(a.ffp) : 0, nbs = a.moe && a.sffp ? Ld<T>::blocks(a.sffp) : 0;
-  const int nb_ff = a.top * nbe + nbs;  // blocks of one sequence's feed-forward part (identity experts: skipped)
-  // LDS: block table [nbv + nb_ff], vectors: v [B][nbv], feed-forward [nb_ff] of one sequence at a time
+  const int nb = nbv + nbs + a.top * nbe;
   LdBlk* tab = (LdBlk*)smem_raw;
-  float* xv = (float*)(smem_raw + (size_t)(nbv + nb_ff) * sizeof(LdBlk));
+  float* xv = (float*)(smem_raw + (size_t)nb * sizeof(LdBlk));
   float* xf = xv + (size_t)B * nbv * BE;
-  const int items = (a.W + R - 1) / R;
-  for (int b = threadIdx.x; b < nbv; b += 256) {
-    const int left = a.ldv / E - b * 64;
-    tab[b] = LdBlk{(const T*)a.wo + (size_t)b * BE, a.ldv, left < 64 ? left : 64};
-  }
-  auto tile_of = [&](frag (&w)[R][U], int b0, int b1, const int (&ri)[R]) __attribute__((always_inline)) {
+  const int kp = wave % a.ks, grp = (int)blockIdx.x * (8 / a.ks) + wave / a.ks;
+  const int item = grp * R;
+  int ri[R];
 #pragma unroll
-    for (int u = 0; u < U; ++u) {
-      if (b0 + u < b1) {
-        const LdBlk k = tab[b0 + u];
-        const int c = lane < k.nch ? lane : k.nch - 1;
-#pragma unroll
-        for (int r = 0; r < R; ++r)
-          w[r][u] = ld_nt((const frag*)((const T*)k.p + (size_t)ri[r] * k.stride) + c);
-      }
+  for (int r = 0; r < R; ++r) ri[r] = item + r < a.W ? item + r : a.W - 1;
+  auto part = [&](int n, const T* base, int stride, int len, LdBlk* out, int tid0) __attribute__((always_inline)) {
+    for (int b = (int)threadIdx.x - tid0; b >= 0 && b < n; b += 512) {
+      const int left = len / E - b * 64;
+      out[b] = LdBlk{base + (size_t)b * BE, stride, left < 64 ? left : 64};
     }
   };
-  // first item of this wave; later items reload everything
+  part(nbv, (const T*)a.wo, a.ldv, a.ldv, tab, 0);
+  if (nbs) part(nbs, (const T*)a.sdown, a.sffp, a.sffp, tab + nbv, 64);
   for (int q = 0; q < B; ++q)
-    for (int i = threadIdx.x; i < nbv * BE; i += 256)
-      xv[(size_t)q * nbv * BE + Ld<T>::place(i)] = i < a.n_v ? a.v[(size_t)q * a.ld_v + i] : 0.f;
-  for (int it0 = blockIdx.x * 4; it0 < items; it0 += a.nwg * 4) {  // uniform per workgroup: barriers inside
-    const int item = it0 + wave;
-    int ri[R];
+    ld_stage<T, 512>((f32x4*)(xv + (size_t)q * nbv * BE), a.v + (size_t)q * a.ld_v, a.n4v, nbv * BE / 4, 1.f, threadIdx.x);
+  float acc[R][B] = {};
 #pragma unroll
-    for (int r = 0; r < R; ++r) ri[r] = item * R + r < a.W ? item * R + r : a.W - 1;
-    float acc[R][B] = {};
-#pragma unroll
-    for (int q = 0; q < (B > 1 ? B : 1); ++q) {
-      int nb = 0;  // feed-forward blocks of sequence q in the table
-      if (a.moe) {
-        __syncthreads();  // the part of the sequence before has been consumed
-        int slot = 0;
-        for (int k = 0; k < a.top; ++k) {
-          const int id = a.ids[q * a.top + k];
-          if (id < 0) continue;
-          const float* he = a.he + (size_t)(q * a.top + k) * a.ffp;
-          for (int i = threadIdx.x; i < nbe * BE; i += 256)
-            xf[(size_t)slot * BE + Ld<T>::place(i)] = i < a.ffp ? he[i] : 0.f;
-          for (int b = threadIdx.x; b < nbe; b += 256) {
-            const int left = a.ffp / E - b * 64;
-            tab[nbv + slot + b] = LdBlk{(const T*)a.down + (size_t)id * a.W * a.ffp + (size_t)b * BE, a.ffp, left < 64 ? left : 64};
-          }
-          slot += nbe;
-        }
-        if (nbs) {
-          const float g = a.sh_g[q];
-          for (int i = threadIdx.x; i < nbs * BE; i += 256)
-            xf[(size_t)slot * BE + Ld<T>::place(i)] = i < a.sffp ? g * a.hs[(size_t)q * a.sffp + i] : 0.f;
-          for (int b = threadIdx.x; b < nbs; b += 256) {
-            const int left = a.sffp / E - b * 64;
-            tab[nbv + slot + b] = LdBlk{(const T*)a.sdown + (size_t)b * BE, a.sffp, left < 64 ? left : 64};
-          }
-          slot += nbs;
-        }
-        nb = slot;
+  for (int q = 0; q < B; ++q) {
+    if (a.moe) {
+      if (q) __syncthreads();  // the part of the sequence before has been consumed
+      for (int b = (int)threadIdx.x - 128; b >= 0 && b < a.top * nbe; b += 384) {
+        const int k = b / nbe, bb = b - k * nbe, id = a.ids[q * a.top + k];
+        const int left = a.ffp / E - bb * 64;
+        tab[nbv + nbs + b] = LdBlk{(const T*)a.down + ((size_t)(id < 0 ? 0 : id) * a.W) * a.ffp + (size_t)bb * BE, a.ffp,
+                                   id < 0 ? 0 : (left < 64 ? left : 64)};
       }
-      __syncthreads();
-      const int b_lo = q == 0 ? 0 : nbv, b_hi = nbv + nb;  // the mixer part runs once, for all sequences
-      frag w[R][U];
-      for (int b0 = b_lo; b0 < b_hi; b0 += U) {
-        tile_of(w, b0, b_hi, ri);
-#pragma unroll
-        for (int u = 0; u < U; ++u) {
-          const int b = b0 + u;
-          if (b >= b_hi) continue;
-          if (b < nbv) {
-#pragma unroll
-            for (int j = 0; j < B; ++j) {
-              const f32x4* x = (const f32x4*)(xv + ((size_t)j * nbv + b) * BE) + lane;
-#pragma unroll
-              for (int r = 0; r < R; ++r) acc[r][j] = ld_dot<T>(w[r][u], x, acc[r][j]);
-            }
-          } else {
-            const f32x4* x = (const f32x4*)(xf + (size_t)(b - nbv) * BE) + lane;
-#pragma unroll
-            for (int r = 0; r < R; ++r) acc[r][q] = ld_dot<T>(w[r][u], x, acc[r][q]);
-          }
-        }
-      }
+      if (nbs) ld_stage<T, 512>((f32x4*)xf, a.hs + (size_t)q * a.sffp, a.sffp >> 2, nbs * BE / 4, a.sh_g[q], threadIdx.x);
+      for (int k = 0; k < a.top; ++k)
+        ld_stage<T, 512>((f32x4*)(xf + (size_t)(nbs + k * nbe) * BE), a.he + (size_t)(q * a.top + k) * a.ffp, a.ffp >> 2,
+                         nbe * BE / 4, 1.f, threadIdx.x);
     }
-    ld_reduce<R, B>(acc);
-    if (lane < R * B && item < items) {
-      const int r = lane & (R - 1), q = lane / R, i = item * R + r;
-      const float v = ld_pick<R, B>(acc, r, q);
-      if (i < a.W) {
-        const size_t o = (size_t)q * a.W + i;
-        float y = v;
-        if (a.moe) y = __builtin_fmaf(a.id_w[q], a.xn2[o], y);
-        a.x_out[o] = a.x_cur[o] + y;
+    __syncthreads();
+    const int b_lo = q == 0 ? 0 : nbv, n = nb - b_lo, per = (n + a.ks - 1) / a.ks;
+    const int b0 = b_lo + kp * per, b1 = b0 + per < nb ? b0 + per : nb;
+    frag w[2][R][U];
+    int nc[2][U];
+    auto fetch = [&](int set, int b) __attribute__((always_inline)) {
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        nc[set][u] = 0;
+        if (b + u < b1) {
+          const LdBlk k = tab[b + u];
+          nc[set][u] = __builtin_amdgcn_readfirstlane(k.nch);
+          if (nc[set][u]) {
+            const int c = lane < k.nch ? lane : k.nch - 1;
+#pragma unroll
+            for (int r = 0; r < R; ++r) w[set][r][u] = ld_nt((const frag*)((const T*)k.p + (size_t)ri[r] * k.stride) + c);
+          }
+        }
       }
+    };
+    auto use = [&](int set, int b) __attribute__((always_inline)) {
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        if (!nc[set][u]) continue;
+        if (b + u < nbv) {
+#pragma unroll
+          for (int j = 0; j < B; ++j) {
+            const f32x4* x = (const f32x4*)(xv + ((size_t)j * nbv + b + u) * BE) + lane;
+#pragma unroll
+            for (int r = 0; r < R; ++r) acc[r][j] = ld_dot<T>(w[set][r][u], x, acc[r][j]);
+          }
+        } else {
+          const f32x4* x = (const f32x4*)(xf + (size_t)(b + u - nbv) * BE) + lane;
+#pragma unroll
+          for (int r = 0; r < R; ++r) acc[r][q] = ld_dot<T>(w[set][r][u], x, acc[r][q]);
+        }
+      }
+    };
+    fetch(0, b0);
+    for (int b = b0; b < b1; b += 2 * U) {
+      fetch(1, b + U);
+      use(0, b);
+      fetch(0, b + 2 * U);
+      use(1, b + U);
+    }
+  }
+  ld_reduce<R, B>(acc);
+  if (lane < R * B) comb[wave][lane] = ld_pick<R, B>(acc, lane & (R - 1), lane / R);
+  __syncthreads();
+  if (kp == 0 && lane < R * B) {
+    float v = 0.f;
+    for (int k = 0; k < a.ks; ++k) v += comb[wave + k][lane];
+    const int q = lane / R, i = item + (lane & (R - 1));
+    if (i < a.W) {
+      const size_t o = (size_t)q * a.ld + i;
+      if (a.moe) v = __builtin_fmaf(a.id_w[q], a.xn2[o], v);
+      a.x_out[o] = a.x_cur[o] + v;
     }
   }
 }
 
 // ---- k_ld_head ---------------------------------------------------------------------------------------------------
 struct LdHeadArgs {
-  const float* x;        // [B][W]
+  const float* x;        // [B][ld]
   const float *w, *b;    // final norm
   const void* head;      // [V][ld]
   float* logits;         // [B][V]
@@ -733,7 +787,7 @@ struct LdHeadArgs {
   int W, ld, V;
   float eps, cap;
 };
-template <class T, int B>
+template <class T, int B, int NV>
 __global__ __launch_bounds__(256) void k_ld_head(const LdHeadArgs a) {
   constexpr int R = 4, U = 4;
   extern __shared__ __attribute__((aligned(16))) char smem_raw[];
@@ -759,23 +813,23 @@ __global__ __launch_bounds__(256) void k_ld_head(const LdHeadArgs a) {
     set_rows(item);
     ld_load<T, R, U>(t, row, 0, nblk, nch, lane);
   }
-  for (int q = 0; q < B; ++q) {
-    float* x = xs + (size_t)q * xstride;
-    float s = 0.f;
-    for (int i = threadIdx.x; i < xstride; i += 256) {
-      const float v = i < a.W ? a.x[(size_t)q * a.W + i] : 0.f;
-      x[Ld<T>::place(i)] = v;
-      s += v;
+  {
+    const int n4 = a.ld >> 2;
+    f32x4 nw[NV], nb[NV], v[NV];
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int i = threadIdx.x + 256 * j;
+      nw[j] = i < n4 ? ((const f32x4*)a.w)[i] : f4_zero();
+      nb[j] = i < n4 ? ((const f32x4*)a.b)[i] : f4_zero();
     }
-    const float mean = block_sum(s, red) / (float)a.W;
-    float d2 = 0.f;
-    for (int i = threadIdx.x; i < a.W; i += 256) {
-      const float d = x[Ld<T>::place(i)] - mean;
-      d2 = __builtin_fmaf(d, d, d2);
+    for (int q = 0; q < B; ++q) {
+#pragma unroll
+      for (int j = 0; j < NV; ++j) {
+        const int i = threadIdx.x + 256 * j;
+        v[j] = i < n4 ? ((const f32x4*)(a.x + (size_t)q * a.ld))[i] : f4_zero();
+      }
+      ld_norm<T, NV>(v, nw, nb, a.W, n4, xstride >> 2, a.eps, red, (f32x4*)(xs + (size_t)q * xstride), nullptr);
     }
-    const float rstd = 1.0f / sqrtf(block_sum(d2, red) / (float)a.W + a.eps);
-    for (int i = threadIdx.x; i < a.W; i += 256)
-      x[Ld<T>::place(i)] = (x[Ld<T>::place(i)] - mean) * rstd * a.w[i] + a.b[i];
   }
   __syncthreads();
   float bv = -INFINITY;

@@ -12,98 +12,124 @@ struct PassTabs {
 };
 
 // what one layer leaves to be added to the residual stream
+template <class T>
 struct AddArgs {
-  const float* mix;       // [T][W] mixer output (nullptr: nothing pending)
+  const float* mix;       // [T][ld] mixer output (nullptr: nothing pending)
   // experts: sum_k w[t][k] y[slot[t][k]] (slot < 0: not a stored row), identity weight, gated shared expert
-  const float* y;         // expert output rows [rows][W]
+  const T* y;             // expert output rows [rows][ld]
   const int32_t* y_slot;  // [T][top]
   const float* y_w;       // [T][top]
   const float* id_w;      // [T]
-  const float* sh;        // [T][W] shared expert's output
+  const T* sh;            // [T][ld] shared expert's output
   const float* sh_g;      // [T] its gate
   int top;
 };
 
 // One workgroup per token.  x += pending; (loop entry) x += x0, x += step; then xn1 / xn2 = layer norms of x.
-// x_src: 0 = x itself, 1 = the embedding row (first layer; also fills x0).
+// Rows of every array are ld (a multiple of KH_LPAD) elements with zeros behind the W valid ones.
 template <class T>
 struct CombineArgs {
   float *x, *x0;
-  AddArgs add;
+  AddArgs<T> add;
   const T* embed;
   const int32_t* tok;
-  const float* step;                       // [W] or nullptr
+  const float* step;                       // one row or nullptr
   const float *w1, *b1, *w2, *b2;          // norm parameters (w1 nullptr: no norm output)
-  T *xn1, *xn2;                            // [T][ld]
+  T *xn1, *xn2;
   const T* xn2_prev;                       // identity experts' input: the xn2 the pending layer read
   int W, ld, from_embed, add_x0;
   float eps;
 };
 template <class T>
+__device__ __forceinline__ f32x4 quad_f(const T* p) {
+  const typename Tile<T>::quad q = *(const typename Tile<T>::quad*)p;
+  return f32x4{(float)q.x, (float)q.y, (float)q.z, (float)q.w};
+}
+__device__ __forceinline__ f32x4 fma_s(float s, f32x4 a, f32x4 b) {
+  f32x4 r;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) r[i] = __builtin_fmaf(s, a[i], b[i]);
+  return r;
+}
+template <class T>
 __global__ __launch_bounds__(256) void k_combine(const CombineArgs<T> a) {
   extern __shared__ __attribute__((aligned(16))) char smem_raw[];
-  float* row = (float*)smem_raw;
+  f32x4* row = (f32x4*)smem_raw;  // [ld / 4]
   __shared__ float red[KH_WAVES_MAX];
-  const int t = blockIdx.x;
-  const size_t o = (size_t)t * a.W;
-  float* x = a.x + o;
+  const int t = blockIdx.x, n4 = a.ld >> 2;
+  const size_t o = (size_t)t * a.ld;
   float s = 0.f;
-  const T* e = a.from_embed ? a.embed + (size_t)a.tok[t] * a.W : nullptr;
+  const T* e = a.from_embed ? a.embed + (size_t)a.tok[t] * a.ld : nullptr;
   float idw = 0.f, shg = 0.f;
   const int top = a.add.y ? a.add.top : 0;
   if (a.add.y) {
     idw = a.add.id_w[t];
     shg = a.add.sh ? a.add.sh_g[t] : 0.f;
   }
-  for (int i = threadIdx.x; i < a.W; i += 256) {
-    float v;
+  for (int i = threadIdx.x; i < n4; i += 256) {
+    const int c = 4 * i;
+    f32x4 v;
     if (a.from_embed) {
-      v = (float)e[i];
-      a.x0[o + i] = v;
+      v = quad_f(e + c);
+      *(f32x4*)(a.x0 + o + c) = v;
     } else {
-      v = x[i];
+      v = *(const f32x4*)(a.x + o + c);
     }
     if (a.add.mix) {
-      float d = a.add.mix[o + i];
+      f32x4 d = *(const f32x4*)(a.add.mix + o + c);
       if (a.add.y) {
-        float f = 0.f;
+        f32x4 f = {0.f, 0.f, 0.f, 0.f};
         for (int k = 0; k < top; ++k) {
           const int sl = a.add.y_slot[(size_t)t * top + k];
-          if (sl >= 0) f = __builtin_fmaf(a.add.y_w[(size_t)t * top + k], a.add.y[(size_t)sl * a.W + i], f);
+          if (sl >= 0) f = fma_s(a.add.y_w[(size_t)t * top + k], quad_f(a.add.y + (size_t)sl * a.ld + c), f);
         }
-        if (idw != 0.f) f = __builtin_fmaf(idw, (float)a.xn2_prev[(size_t)t * a.ld + i], f);
-        if (a.add.sh) f = __builtin_fmaf(shg, a.add.sh[o + i], f);
+        if (idw != 0.f) f = fma_s(idw, quad_f(a.xn2_prev + o + c), f);
+        if (a.add.sh) f = fma_s(shg, quad_f(a.add.sh + o + c), f);
         d += f;
       }
       v += d;
     }
-    if (a.add_x0) v += a.x0[o + i];
-    if (a.step) v += a.step[i];
-    x[i] = v;
+    if (a.add_x0) v += *(const f32x4*)(a.x0 + o + c);
+    if (a.step) v += *(const f32x4*)(a.step + c);
+    *(f32x4*)(a.x + o + c) = v;
     row[i] = v;
-    s += v;
+    s += (v.x + v.y) + (v.z + v.w);
   }
   if (!a.w1) return;
   const float mean = block_sum(s, red) / (float)a.W;
   float q = 0.f;
-  for (int i = threadIdx.x; i < a.W; i += 256) {
-    const float d = row[i] - mean;
-    q = __builtin_fmaf(d, d, q);
+  for (int i = threadIdx.x; i < n4; i += 256) {
+    const f32x4 v = row[i];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const float d = 4 * i + k < a.W ? v[k] - mean : 0.f;
+      q = __builtin_fmaf(d, d, q);
+    }
   }
   const float rstd = 1.0f / sqrtf(block_sum(q, red) / (float)a.W + a.eps);
-  for (int i = threadIdx.x; i < a.W; i += 256) {
-    const float n = (row[i] - mean) * rstd;
-    a.xn1[(size_t)t * a.ld + i] = (T)(n * a.w1[i] + a.b1[i]);
-    if (a.w2) a.xn2[(size_t)t * a.ld + i] = (T)(n * a.w2[i] + a.b2[i]);
+  for (int i = threadIdx.x; i < n4; i += 256) {
+    const int c = 4 * i;
+    const f32x4 v = row[i];
+    f32x4 y;
+    const f32x4 w1 = *(const f32x4*)(a.w1 + c), b1 = *(const f32x4*)(a.b1 + c);
+#pragma unroll
+    for (int k = 0; k < 4; ++k) y[k] = (v[k] - mean) * rstd * w1[k] + b1[k];  // pads: weights and biases are zero
+    *(typename Tile<T>::quad*)(a.xn1 + o + c) = to_quad<T>(y);
+    if (a.w2) {
+      const f32x4 w2 = *(const f32x4*)(a.w2 + c), b2 = *(const f32x4*)(a.b2 + c);
+#pragma unroll
+      for (int k = 0; k < 4; ++k) y[k] = (v[k] - mean) * rstd * w2[k] + b2[k];
+      *(typename Tile<T>::quad*)(a.xn2 + o + c) = to_quad<T>(y);
+    }
   }
 }
 
-// layer norm of gathered rows: out[r] = norm(x[rows[r]])
+// layer norm of gathered rows: out[r] = norm(x[rows[r]]); rows of ld elements on both sides
 template <class T>
 __global__ __launch_bounds__(256) void k_gather_norm(const float* x, const int32_t* rows, const float* w, const float* b,
                                                      T* out, int W, int ld, float eps) {
   __shared__ float red[KH_WAVES_MAX];
-  const float* r = x + (size_t)rows[blockIdx.x] * W;
+  const float* r = x + (size_t)rows[blockIdx.x] * ld;
   float s = 0.f;
   for (int i = threadIdx.x; i < W; i += 256) s += r[i];
   const float mean = block_sum(s, red) / (float)W;
@@ -130,22 +156,54 @@ struct ConvArgs {
   int C, ldx, ldo, taps;
   PassTabs p;
 };
+// E channels (16 bytes) of KH_CONV_TT consecutive tokens per thread.  grid (C / (256 E), T / KH_CONV_TT)
+#define KH_CONV_TT 4
 template <class T>
-__global__ __launch_bounds__(256) void k_conv_silu(const ConvArgs<T> a) {
-  const int c = blockIdx.x * 256 + threadIdx.x, t = blockIdx.y;
+__global__ __launch_bounds__(256) void k_conv_silu(const ConvArgs<T> a, int T_all) {
+  constexpr int E = Tile<T>::N;
+  const int c = (blockIdx.x * 256 + threadIdx.x) * E;
   if (c >= a.C) return;
-  const int sg = a.p.seg[t], i = t - a.p.seg_row0[sg];
-  const bool fresh = a.p.seg_pos0[sg] == 0;
-  const float* st = a.state + (size_t)a.p.seg_slot[sg] * a.slot_stride;
-  float v = a.b[c];
-  for (int k = 0; k < a.taps; ++k) {
-    const int j = i - (a.taps - 1) + k;  // row of the segment
-    float in = 0.f;
-    if (j >= 0) in = (float)a.xz[(size_t)(t - i + j) * a.ldx + c];
-    else if (!fresh) in = st[(size_t)(a.taps - 1 + j) * a.C + c];
-    v = __builtin_fmaf(a.w[(size_t)c * a.taps + k], in, v);
+  const bool vec = c + E <= a.C && (a.ldx & (E - 1)) == 0;
+  for (int u = 0; u < KH_CONV_TT; ++u) {
+    const int t = blockIdx.y * KH_CONV_TT + u;
+    if (t >= T_all) return;
+    const int sg = a.p.seg[t], i = t - a.p.seg_row0[sg];
+    const bool fresh = a.p.seg_pos0[sg] == 0;
+    const float* st = a.state + (size_t)a.p.seg_slot[sg] * a.slot_stride;
+    float v[E];
+#pragma unroll
+    for (int e = 0; e < E; ++e) v[e] = c + e < a.C ? a.b[c + e] : 0.f;
+    for (int k = 0; k < a.taps; ++k) {
+      const int j = i - (a.taps - 1) + k;  // row of the segment
+      float in[E];
+#pragma unroll
+      for (int e = 0; e < E; ++e) in[e] = 0.f;
+      if (j >= 0) {
+        const T* x = a.xz + (size_t)(t - i + j) * a.ldx + c;
+        if (vec) {
+          const typename Tile<T>::frag f = *(const typename Tile<T>::frag*)x;
+#pragma unroll
+          for (int e = 0; e < E; ++e) in[e] = (float)f[e];
+        } else {
+#pragma unroll
+          for (int e = 0; e < E; ++e)
+            if (c + e < a.C) in[e] = (float)x[e];
+        }
+      } else if (!fresh) {
+#pragma unroll
+        for (int e = 0; e < E; ++e)
+          if (c + e < a.C) in[e] = st[(size_t)(a.taps - 1 + j) * a.C + c + e];
+      }
+#pragma unroll
+      for (int e = 0; e < E; ++e)
+        if (c + e < a.C) v[e] = __builtin_fmaf(a.w[(size_t)(c + e) * a.taps + k], in[e], v[e]);
+    }
+    T* o = a.out + (size_t)t * a.ldo + c;  // rows are padded to whole fragments
+    typename Tile<T>::frag f;
+#pragma unroll
+    for (int e = 0; e < E; ++e) f[e] = (T)(c + e < a.C ? silu1(v[e]) : 0.f);
+    *(typename Tile<T>::frag*)o = f;
   }
-  a.out[(size_t)t * a.ldo + c] = (T)silu1(v);
 }
 // the last taps - 1 inputs of every segment become its sequence's state.  grid (C / 256, S)
 template <class T>

@@ -9,17 +9,17 @@
 
 namespace khm {
 
-// The choice for one token by one wave; z in LDS or global [n_out].  Calls pick(k, id, weight) for k = 0 .. top - 1
-// on every lane, in order of decreasing choice score.
-template <class F>
+// The choice for one token by one wave; z in LDS or global [n_out], n_out <= 64 PER.  Calls pick(k, id, weight) for
+// k = 0 .. top - 1 on every lane with wave-uniform values, in order of decreasing choice score.
+template <int PER, class F>
 __device__ __forceinline__ void moe_route(const float* z, const float* corr, int n_out, int top, int lane, F&& pick) {
-  constexpr int PER = KH_MOE_MAX_OUT / 64;
   float s[PER], key[PER];
   float m = -INFINITY;
 #pragma unroll
   for (int j = 0; j < PER; ++j) {
     const int i = j * 64 + lane;
     s[j] = i < n_out ? z[i] : -INFINITY;
+    key[j] = i < n_out ? corr[i] : 0.f;
     m = fmaxf(m, s[j]);
   }
   m = wave_max(m);
@@ -32,29 +32,28 @@ __device__ __forceinline__ void moe_route(const float* z, const float* corr, int
   sum = wave_sum(sum);
 #pragma unroll
   for (int j = 0; j < PER; ++j) {
-    const int i = j * 64 + lane;
     s[j] /= sum;
-    key[j] = i < n_out ? s[j] + corr[i] : -INFINITY;
+    key[j] = j * 64 + lane < n_out ? s[j] + key[j] : -INFINITY;
   }
   for (int k = 0; k < top; ++k) {
-    float v = -INFINITY, w = 0.f;
-    int id = 0x7fffffff;
+    float v = key[0];
 #pragma unroll
-    for (int j = 0; j < PER; ++j)
-      if (key[j] > v) {  // ascending j: the lowest index of a tie within the lane
-        v = key[j];
-        id = j * 64 + lane;
-        w = s[j];
-      }
-    wave_amax(v, id);
+    for (int j = 1; j < PER; ++j) v = fmaxf(v, key[j]);
+    v = wave_max(v);
+    // lowest index that holds the maximum (indices are exact in fp32)
+    float first = 1e9f;
+#pragma unroll
+    for (int j = PER - 1; j >= 0; --j) first = key[j] == v ? (float)(j * 64 + lane) : first;
+    const int id = (int)(-wave_max(-first));
+    float w = 0.f;
 #pragma unroll
     for (int j = 0; j < PER; ++j) {
       const bool mine = j * 64 + lane == id;
-      if (mine) key[j] = -INFINITY;
-      if (mine) w = s[j];
+      w = mine ? s[j] : w;
+      key[j] = mine ? -INFINITY : key[j];
     }
-    w = __shfl(w, id & 63, 64);
-    pick(k, id, w);
+    w = wave_sum(w);  // one lane holds it, the others zero
+    pick(k, __builtin_amdgcn_readfirstlane(id), w);
   }
 }
 
@@ -67,12 +66,13 @@ struct RouteArgs {
   float* sh_g;           // [T] sigmoid of the shared expert's gate
   int T, ldz, n_out, n_expert, top, shared;
 };
-static __global__ __launch_bounds__(256) void k_moe_route(const RouteArgs a) {
+template <int PER>
+__global__ __launch_bounds__(256) void k_moe_route(const RouteArgs a) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= a.T) return;
   const float* z = a.z + (size_t)t * a.ldz;
   float idw = 0.f;
-  moe_route(z, a.corr, a.n_out, a.top, lane, [&](int k, int id, float w) __attribute__((always_inline)) {
+  moe_route<PER>(z, a.corr, a.n_out, a.top, lane, [&](int k, int id, float w) __attribute__((always_inline)) {
     if (id >= a.n_expert) idw += w;
     if (lane == 0) {
       a.id[(size_t)t * a.top + k] = id;
@@ -83,6 +83,15 @@ static __global__ __launch_bounds__(256) void k_moe_route(const RouteArgs a) {
     a.id_w[t] = idw;
     if (a.shared) a.sh_g[t] = sigmoid1(z[a.n_out]);
   }
+}
+
+static inline int moe_per(int n_out) { return n_out <= 64 ? 1 : (n_out <= 256 ? 4 : 16); }
+static inline void moe_route_launch(hipStream_t s, const RouteArgs& a) {
+  const dim3 g((a.T + 3) / 4), b(256);
+  const int per = moe_per(a.n_out);
+  if (per == 1) hipLaunchKernelGGL(k_moe_route<1>, g, b, 0, s, a);
+  else if (per == 4) hipLaunchKernelGGL(k_moe_route<4>, g, b, 0, s, a);
+  else hipLaunchKernelGGL(k_moe_route<16>, g, b, 0, s, a);
 }
 
 // Dispatch lists, one workgroup: rows grouped by expert (row -> token), slot of every (token, choice) in that order
