@@ -6,11 +6,15 @@
 // the attention kernel is a row of consecutive bytes and all staging is LDS-DMA.
 //
 // k_expanded_attn: workgroup = 4 waves x MR tiles of 16 tokens of ONE head; key tiles of KT (a 64-byte row of the
-// transposed values), double-buffered.  S^T = K Q^T and O^T = V^T P^T as in kh_latent.h; here the key order is
+// transposed values) through a ring of KH_EXP_STAGES LDS stages.  S^T = K Q^T and O^T = V^T P^T as in kh_latent.h; here the key order is
 // permuted where the K fragments are read (score tile n, row 4 h + i <- key 8 h + 4 n + i for bf16).
 #pragma once
 #include "kh_latent.h"
 #include "kh_lgemm.h"
+
+#ifndef KH_EXP_STAGES
+#define KH_EXP_STAGES 3
+#endif
 
 namespace khm {
 
@@ -26,24 +30,24 @@ struct ExpArgs {
   float scale2;
 };
 
-// NQ: k-blocks (64 bytes) of a query row at most; NV: 16-column value tiles
-template <class T, int NQ, int NV, int MR>
+// KN, KR, KV: unrotated key part, rotated part and value size in units of 64 (compile-time: see kh_latent.h)
+template <class T, int KN, int KR, int KV, int MR>
 __global__ __launch_bounds__(256) void k_expanded_attn(const ExpArgs a) {
   typedef Tile<T> TL;
   typedef typename TL::frag frag;
   constexpr int E = TL::N, KT = 4 * E, NS = KT / 16, ES = (int)sizeof(T);
+  constexpr int DN = 64 * KN, DRP = 64 * KR, DV = 64 * KV, NQ = (DN + DRP) / (4 * E), NV = DV / 16;
   extern __shared__ __attribute__((aligned(1024))) char smem_raw[];
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int fr = lane & 15, fh = lane >> 4;
   const int head = blockIdx.x;
   const int tile = (int)gridDim.y - 1 - (int)blockIdx.y;  // the longest key ranges first
   const int q0 = tile * (64 * MR);
-  const int qc = a.dnp / E, rc = a.drp / E, vr = a.dvp;   // 16-byte chunks of the key parts, value rows
-  const int bytes_k = KT * a.dnp * ES, bytes_r = KT * a.drp * ES, stage = bytes_k + bytes_r + vr * 64;
+  constexpr int qc = DN / E, rc = DRP / E;  // 16-byte chunks of the key parts
+  constexpr int bytes_k = KT * DN * ES, bytes_r = KT * DRP * ES, stage = bytes_k + bytes_r + DV * 64;
   int q_last = q0 + 64 * MR - 1;
   q_last = q_last < a.n ? q_last : a.n - 1;
   const int n_keys = a.pos0 + q_last + 1;
-  const int nb = (a.dnp + a.drp) / (4 * E);
   const T* Q = (const T*)a.Q;
   frag fq[MR][NQ];
   int my_pos[MR];
@@ -52,32 +56,46 @@ __global__ __launch_bounds__(256) void k_expanded_attn(const ExpArgs a) {
     int t = q0 + (wave * MR + m) * 16 + fr;
     t = t < a.n ? t : a.n - 1;
     my_pos[m] = a.pos0 + t;
-    const char* q = (const char*)(Q + ((size_t)(a.row0 + t) * a.H + head) * (a.dnp + a.drp)) + 16 * fh;
+    const char* q = (const char*)(Q + ((size_t)(a.row0 + t) * a.H + head) * (DN + DRP)) + 16 * fh;
 #pragma unroll
-    for (int b = 0; b < NQ; ++b)
-      if (b < nb) fq[m][b] = *(const frag*)(q + 64 * b);
+    for (int b = 0; b < NQ; ++b) fq[m][b] = *(const frag*)(q + 64 * b);
   }
   const unsigned lds0 = (unsigned)__builtin_amdgcn_readfirstlane((int)kh_lds_addr(smem_raw));
   // slot s of a row of `c` chunks (c >= 8) holds chunk s ^ swz(row)
   auto swz = [](int row) __attribute__((always_inline)) { return (row & 3) | ((row >> 1) & 4); };
-  const int nK = KT * qc / 64, nR = KT * rc / 64, nV = vr * 4 / 64;  // LDS-DMA requests of a stage (64 chunks each)
+  // LDS-DMA requests of a wave and stage (64 chunks each): request j covers chunks (4 j + wave) 64 ..
+  constexpr int nK = KT * qc / 256, nR = KT * rc / 256, nV = DV * 4 / 256, NL = nK + nR + nV;
+  unsigned vk[nK], vr[nR], vv[nV];
+  int rr[nR];
+#pragma unroll
+  for (int j = 0; j < nK; ++j) {
+    const int c = (4 * j + wave) * 64 + lane, r = c / qc, s = c - r * qc;
+    vk[j] = (unsigned)(r * a.H * DN * ES + ((s ^ swz(r)) << 4));
+  }
+#pragma unroll
+  for (int j = 0; j < nR; ++j) {
+    const int c = (4 * j + wave) * 64 + lane, r = c / rc, s = c - r * rc;
+    rr[j] = r;
+    vr[j] = (unsigned)((s ^ swz(r)) << 4);
+  }
+#pragma unroll
+  for (int j = 0; j < nV; ++j) {
+    const int c = (4 * j + wave) * 64 + lane;
+    vv[j] = (unsigned)((c >> 2) * a.ldv * ES + ((c & 3) << 4));
+  }
   auto issue = [&](int slot, int k0) __attribute__((always_inline)) {
-    const unsigned d0 = lds0 + (unsigned)(slot * stage);
-    const char* kb = (const char*)a.Kx + ((size_t)k0 * a.H + head) * a.dnp * ES;
-    for (int j = wave; j < nK; j += 4) {
-      const int c = j * 64 + lane, r = c / qc, s = c - r * qc;
-      dma_x4_keep(kb, (unsigned)(r * a.H * a.dnp * ES + ((s ^ swz(r)) << 4)), d0 + 1024u * j);
+    const unsigned d0 = lds0 + (unsigned)(slot * stage) + 1024u * wave;
+    const char* kb = (const char*)a.Kx + ((size_t)k0 * a.H + head) * DN * ES;
+#pragma unroll
+    for (int j = 0; j < nK; ++j) dma_x4_keep(kb, vk[j], d0 + 4096u * j);
+#pragma unroll
+    for (int j = 0; j < nR; ++j) {
+      const int k = k0 + rr[j] < n_keys ? k0 + rr[j] : n_keys - 1;  // rows behind the sequence's last are not backed
+      dma_x4_keep(a.cache, (unsigned)(k * a.row * ES) + vr[j], d0 + bytes_k + 4096u * j);
     }
-    for (int j = wave; j < nR; j += 4) {
-      const int c = j * 64 + lane, r = c / rc, s = c - r * rc;
-      const int k = k0 + r < n_keys ? k0 + r : n_keys - 1;  // rows behind the sequence's last are not backed
-      dma_x4_keep(a.cache, (unsigned)(k * a.row * ES + ((s ^ swz(r)) << 4)), d0 + bytes_k + 1024u * j);
-    }
-    const char* vb = (const char*)a.Vx + ((size_t)head * a.dvp * a.ldv + k0) * ES;
-    for (int j = wave; j < nV; j += 4) {
-      const int c = j * 64 + lane;
-      dma_x4_keep(vb, (unsigned)((c >> 2) * a.ldv * ES + ((c & 3) << 4)), d0 + bytes_k + bytes_r + 1024u * j);
-    }
+    const char* vb = (const char*)a.Vx + ((size_t)head * DV * a.ldv + k0) * ES;
+#pragma unroll
+    for (int j = 0; j < nV; ++j) dma_x4_keep(vb, vv[j], d0 + bytes_k + bytes_r + 4096u * j);
   };
   float m[MR], l[MR];
   f32x4 o[MR][NV];
@@ -89,12 +107,19 @@ __global__ __launch_bounds__(256) void k_expanded_attn(const ExpArgs a) {
     for (int n = 0; n < NV; ++n) o[q][n] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
   const int wave_last = a.pos0 + q0 + (wave + 1) * MR * 16 - 1;  // last position any row of this wave sees
-  issue(0, 0);
-  int slot = 0;
-  for (int k0 = 0; k0 < n_keys; k0 += KT, slot ^= 1) {
-    wait_vm<0>();
+  constexpr int NST = KH_EXP_STAGES;
+#pragma unroll
+  for (int i = 0; i < NST - 1; ++i)
+    if (i * KT < n_keys) issue(i, i * KT);
+  int slot = -1, fill = NST - 2;
+  for (int k0 = 0; k0 < n_keys; k0 += KT) {
+    slot = slot + 1 == NST ? 0 : slot + 1;
+    fill = fill + 1 == NST ? 0 : fill + 1;
+    // this stage has landed when only the younger NST - 2 stages are outstanding
+    if (k0 + (NST - 2) * KT < n_keys) wait_vm<(NST - 2) * NL>();
+    else wait_vm<0>();
     __syncthreads();
-    if (k0 + KT < n_keys) issue(slot ^ 1, k0 + KT);
+    if (k0 + (NST - 1) * KT < n_keys) issue(fill, k0 + (NST - 1) * KT);
     if (k0 > wave_last) continue;  // nothing in this tile for the wave (barriers stay uniform)
     const char* Kt = smem_raw + slot * stage;
     const char* Rt = Kt + bytes_k;
@@ -106,16 +131,14 @@ __global__ __launch_bounds__(256) void k_expanded_attn(const ExpArgs a) {
       for (int n = 0; n < NS; ++n) s[q][n] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int b = 0; b < NQ; ++b) {
-      if (b < nb) {
-        const int c = 4 * b + fh;
+      const int c = 4 * b + fh;
 #pragma unroll
-        for (int n = 0; n < NS; ++n) {
-          const int k = NS == 2 ? 8 * (fr >> 2) + 4 * n + (fr & 3) : fr;
-          const char* src = 4 * b < qc ? Kt + ((size_t)k * qc + (c ^ swz(k))) * 16 : Rt + ((size_t)k * rc + ((c - qc) ^ swz(k))) * 16;
-          const frag fk = *(const frag*)src;
+      for (int n = 0; n < NS; ++n) {
+        const int k = NS == 2 ? 8 * (fr >> 2) + 4 * n + (fr & 3) : fr;
+        const char* src = 4 * b < qc ? Kt + ((size_t)k * qc + (c ^ swz(k))) * 16 : Rt + ((size_t)k * rc + ((c - qc) ^ swz(k))) * 16;
+        const frag fk = *(const frag*)src;
 #pragma unroll
-          for (int q = 0; q < MR; ++q) s[q][n] = TL::mma(fk, fq[q][b], s[q][n]);
-        }
+        for (int q = 0; q < MR; ++q) s[q][n] = TL::mma(fk, fq[q][b], s[q][n]);
       }
     }
     frag p[MR];
@@ -153,14 +176,12 @@ __global__ __launch_bounds__(256) void k_expanded_attn(const ExpArgs a) {
     }
 #pragma unroll
     for (int n = 0; n < NV; ++n) {
-      if (n * 16 < a.dvp) {
-        const frag fv = *(const frag*)(Vt + (size_t)(n * 16 + fr) * 64 + (fh << 4));
+      const frag fv = *(const frag*)(Vt + (size_t)(n * 16 + fr) * 64 + (fh << 4));
 #pragma unroll
-        for (int q = 0; q < MR; ++q) {
+      for (int q = 0; q < MR; ++q) {
 #pragma unroll
-          for (int i = 0; i < 4; ++i) o[q][n][i] *= f[q];
-          o[q][n] = TL::mma(fv, p[q], o[q][n]);
-        }
+        for (int i = 0; i < 4; ++i) o[q][n][i] *= f[q];
+        o[q][n] = TL::mma(fv, p[q], o[q][n]);
       }
     }
   }
@@ -171,15 +192,14 @@ __global__ __launch_bounds__(256) void k_expanded_attn(const ExpArgs a) {
     const float inv = 1.0f / sum;
     const int t = q0 + (wave * MR + q) * 16 + fr;
     if (t >= a.n) continue;
-    T* out = (T*)a.out + ((size_t)(a.row0 + t) * a.H + head) * a.dvp + 4 * fh;
+    T* out = (T*)a.out + ((size_t)(a.row0 + t) * a.H + head) * DV + 4 * fh;
 #pragma unroll
-    for (int n = 0; n < NV; ++n)
-      if (n * 16 < a.dvp) {
+    for (int n = 0; n < NV; ++n) {
         f32x4 v;
 #pragma unroll
         for (int i = 0; i < 4; ++i) v[i] = o[q][n][i] * inv;
         *(typename TL::quad*)(out + n * 16) = to_quad<T>(v);
-      }
+    }
   }
 }
 
@@ -198,11 +218,16 @@ __global__ __launch_bounds__(256) void k_rope_inplace(T* q, const float2* rope, 
   }
 }
 
-static inline bool exp_supported(int dnp, int drp, int dvp) { return dnp + drp <= 256 && dvp <= 128 && drp > 0; }
+static inline bool exp_supported(int dnp, int drp, int dvp) {
+  return dnp + drp <= 256 && dnp >= 64 && dnp <= 192 && (drp == 64 || drp == 128) && (dvp == 64 || dvp == 128);
+}
 template <class T>
 int exp_attn_launch(hipStream_t s, const ExpArgs& a) {
-  constexpr int MR = sizeof(T) == 2 ? 2 : 1;
-  const size_t stage = (size_t)4 * Tile<T>::N * (a.dnp + a.drp) * sizeof(T) + (size_t)a.dvp * 64, lds = 2 * stage;
+#ifndef KH_EXP_MR
+#define KH_EXP_MR 1
+#endif
+  constexpr int MR = sizeof(T) == 2 ? KH_EXP_MR : 1;
+  const size_t stage = (size_t)4 * Tile<T>::N * (a.dnp + a.drp) * sizeof(T) + (size_t)a.dvp * 64, lds = KH_EXP_STAGES * stage;
   auto go = [&](auto kern) -> int {
     if (lds > 64 * 1024) {
       const hipError_t e = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
@@ -211,9 +236,21 @@ int exp_attn_launch(hipStream_t s, const ExpArgs& a) {
     hipLaunchKernelGGL(kern, dim3(a.H, (a.n + 64 * MR - 1) / (64 * MR)), dim3(256), lds, s, a);
     return KH_OK;
   };
-  constexpr int B = 4 * Tile<T>::N;  // elements of a k-block
-  if (a.dnp + a.drp <= 128 && a.dvp <= 64) return go(k_expanded_attn<T, 128 / B, 4, MR>);
-  if (a.dnp + a.drp <= 192) return go(k_expanded_attn<T, 192 / B, 8, MR>);
-  return go(k_expanded_attn<T, 256 / B, 8, MR>);
+  auto val = [&](auto kv) -> int {
+    constexpr int KV = decltype(kv)::value;
+    const int kn = a.dnp / 64, kr = a.drp / 64;
+    if (kr == 1) {
+      if (kn == 1) return go(k_expanded_attn<T, 1, 1, KV, MR>);
+      if (kn == 2) return go(k_expanded_attn<T, 2, 1, KV, MR>);
+      if (kn == 3) return go(k_expanded_attn<T, 3, 1, KV, MR>);
+    } else if (kr == 2) {
+      if (kn == 1) return go(k_expanded_attn<T, 1, 2, KV, MR>);
+      if (kn == 2) return go(k_expanded_attn<T, 2, 2, KV, MR>);
+    }
+    return KH_ERR_UNSUPPORTED;
+  };
+  if (a.dvp == 64) return val(std::integral_constant<int, 1>());
+  if (a.dvp == 128) return val(std::integral_constant<int, 2>());
+  return KH_ERR_UNSUPPORTED;
 }
 }  // namespace khm

@@ -215,6 +215,7 @@ int load_mamba(Plan& pl, Tensors& ts, const std::string& p, const JsonValue& v, 
   mb.rank = size_of(v, "dt_rank", ts.dim(p + ".dt", 1));
   mb.taps = size_of(v, "conv", ts.dim(p + ".conv", 1));
   if (mb.inner <= 0 || mb.state <= 0 || mb.rank <= 0 || mb.taps <= 0) return KH_ERR_FORMAT;
+  if (mb.taps > 64) return KH_ERR_UNSUPPORTED;
   if (mb.state > KH_SCAN_MAX_STATE) return KH_ERR_UNSUPPORTED;
   const int I = mb.inner, N = mb.state, r = mb.rank;
   mb.innerp = padk(I);
@@ -256,11 +257,11 @@ int load_latent(Plan& pl, Tensors& ts, const std::string& p, const JsonValue& v,
   }
   if (la.dims < 0 || la.dims > la.dr || la.dims % 2 || !(la.base > 0)) return KH_ERR_FORMAT;
   la.dnp = padk(la.dn);
-  la.drp = padk(la.dr);
+  la.drp = lat_pad_rot(la.dr);
   la.dvp = padk(la.dv);
-  la.Rp = padk(la.R);
+  la.Rp = lat_pad_latent(la.R);
   la.qrp = padk(la.qr);
-  if (la.Rp > 512 || la.drp > LatCfg<bf16>::MAXROT) return KH_ERR_UNSUPPORTED;
+  if (!la.Rp || !la.drp) return KH_ERR_UNSUPPORTED;
   const int H = la.H;
   la.dqkv = pl.mat(la.qr + la.R + la.dr, W, padk(W));
   pl.put(la.dqkv, 0, ts.need(p + ".dq", {la.qr, W}), 0, la.qr);

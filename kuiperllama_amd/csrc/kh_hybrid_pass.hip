@@ -122,8 +122,7 @@ struct Runner {
     cv.ldo = mb.innerp;
     cv.taps = mb.taps;
     cv.p = ps.p;
-    hipLaunchKernelGGL(k_conv_silu<T>, dim3((I + 256 * Tile<T>::N - 1) / (256 * Tile<T>::N), (ps.T + KH_CONV_TT - 1) / KH_CONV_TT),
-                       dim3(256), 0, s, cv, ps.T);
+    conv_launch<T>(s, cv, ps.T);
     hipLaunchKernelGGL(k_conv_state<T>, dim3((I + 255) / 256, ps.S), dim3(256), 0, s, cv);
     {
       LgArgs a = gemm(mb.x, hy.a1, mb.innerp, hy.a2, mb.rankp);

@@ -17,18 +17,12 @@ struct Hybrid::Step {
   float *x[3] = {nullptr, nullptr, nullptr}, *xn2 = nullptr, *in = nullptr, *xc = nullptr, *mid = nullptr, *v = nullptr,
         *he = nullptr, *hs = nullptr, *z = nullptr, *id_w = nullptr, *sh_g = nullptr, *part = nullptr, *logits = nullptr;
   void* Q = nullptr;
-  int32_t *ids = nullptr, *tabs = nullptr, *tiles = nullptr;
+  int32_t *ids = nullptr, *tabs = nullptr;
   int32_t* h_tabs = nullptr;
   int nsplit = 1, head_wg = 1;
-  // per number of sequences B (1, 2, 4) and latent kind: tile list offset / count / column parts
-  struct Lat {
-    int B, H, big, cp, off, n;
-  };
-  std::vector<Lat> lat;
   ~Step() {
     for (void* p : {(void*)x[0], (void*)x[1], (void*)x[2], (void*)xn2, (void*)in, (void*)xc, (void*)mid, (void*)v, (void*)he,
-                    (void*)hs, (void*)z, (void*)id_w, (void*)sh_g, (void*)part, (void*)logits, Q, (void*)ids, (void*)tabs,
-                    (void*)tiles})
+                    (void*)hs, (void*)z, (void*)id_w, (void*)sh_g, (void*)part, (void*)logits, Q, (void*)ids, (void*)tabs})
       if (p) (void)hipFree(p);
     if (h_tabs) (void)hipHostFree(h_tabs);
   }
@@ -38,9 +32,9 @@ Hybrid::~Hybrid() {}
 
 namespace {
 constexpr int kMaxLds = 160 * 1024;
-// tabs: tok[B], pos[B], slot[B] (uploaded per batch) at 0, B, 2B of KH_HY_DECODE_B; ones and iota behind them
-enum { TB_TOK = 0, TB_POS = KH_HY_DECODE_B, TB_SLOT = 2 * KH_HY_DECODE_B, TB_ONE = 3 * KH_HY_DECODE_B,
-       TB_IOTA = 4 * KH_HY_DECODE_B, TB_ZERO = 5 * KH_HY_DECODE_B, TB_N = 6 * KH_HY_DECODE_B };
+// tabs: tok[B], pos[B], slot[B] (uploaded per batch) at 0, B, 2B of KH_HY_DECODE_B; zeros behind them
+enum { TB_TOK = 0, TB_POS = KH_HY_DECODE_B, TB_SLOT = 2 * KH_HY_DECODE_B, TB_ZERO = 3 * KH_HY_DECODE_B,
+       TB_N = 4 * KH_HY_DECODE_B };
 
 template <class T>
 size_t vec_b(int n) { return Ld<T>::vec_bytes(n); }
@@ -257,28 +251,24 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
       LdAbsorbArgs ab{st.mid, la.ukT.w, la.rope, st.Q, la.H, std::max(1, std::min(cdiv(la.Rp, 32), cdiv(512, la.H * B))),
                       la.dnp, la.dr, la.drp, la.Rp, la.row(), la.dims, tb};
       TRY(go(k_ld_absorb<T>, dim3(la.H * ab.nwg, B), 256, (size_t)la.dnp * 4, s, ab));
-      const Hybrid::Step::Lat* lt = nullptr;
-      for (auto& t : st.lat)
-        if (t.B == B && t.H == la.H && t.big == (la.Rp > 256)) lt = &t;
-      if (!lt) return KH_ERR_INTERNAL;
+      const int cp = la.H <= 32 ? 4 : (la.Rp > 256 ? 2 : 1), tiles = B * cdiv(la.H, 64 / cp);
       LatArgs at{};
       at.Q = st.Q;
       at.cache = (const T*)m->kcache + r.kv_off;
       at.slot_elems = hy.kv_slot;
       at.sink = la.sink.p;
       at.part = st.part;
-      at.tiles = (const LatTile*)(st.tiles + lt->off);
       at.H = la.H;
       at.Rp = la.Rp;
       at.row = la.row();
       at.nsplit = st.nsplit;
       at.scale2 = la.scale * 1.44269504088896f;
-      const int32_t* tabs = st.tabs;
-      at.p = PassTabs{tb.tok, tb.pos, tabs + TB_IOTA, tb.slot, tabs + TB_IOTA, tabs + TB_ONE, tb.pos};
-      TRY(lat_attn_launch<T>(s, at, lt->n, lt->cp));
-      LdValuesArgs va{st.part, la.uv.w, st.v, la.H, std::max(1, std::min(cdiv(la.dvp, 16), cdiv(512, la.H * B))), st.nsplit,
+      at.p.seg_slot = tb.slot;
+      at.p.seg_pos0 = tb.pos;
+      TRY(lat_attn_launch<T>(s, at, tiles, cp));
+      LdValuesArgs va{st.part, la.uv.w, st.v, la.H, std::max(1, std::min(cdiv(la.dvp, 16), cdiv(128, la.H * B))), st.nsplit,
                       la.Rp, la.dvp, tb.pos};
-      TRY(go(k_ld_values<T>, dim3(la.H * va.nwg, B), 256, vec_b<T>(la.Rp), s, va));
+      TRY(go(k_ld_values<T>, dim3(la.H * va.nwg, B), 256, vec_b<T>(la.Rp) + 256 * 16 + (size_t)la.Rp * 4, s, va));
     }
     {
       const HyMat& wo = mamba ? l.mb.o : l.la.o;
@@ -362,7 +352,7 @@ int hy_step_init(kh_model* m) {
   }
   // time splits: about one workgroup per CU over the row tiles of one sequence
   st.nsplit = 2;
-  while (st.nsplit < 64 && st.nsplit * KH_LAT_SPLIT_MIN < m->cfg.cache_len) st.nsplit *= 2;
+  while (st.nsplit < 128 && st.nsplit * KH_LAT_SPLIT_MIN < m->cfg.cache_len) st.nsplit *= 2;
   auto f = [&](float** p, size_t n) -> int {
     TRY(dalloc(p, n));
     return (int)hipMemsetAsync(*p, 0, n * 4, m->stream);
@@ -384,23 +374,7 @@ int hy_step_init(kh_model* m) {
   TRY(dalloc(&st.tabs, TB_N));
   KH_CHECK_HIP(hipHostMalloc((void**)&st.h_tabs, TB_N * 4, hipHostMallocDefault));
   memset(st.h_tabs, 0, TB_N * 4);
-  for (int i = 0; i < KH_HY_DECODE_B; ++i) {
-    st.h_tabs[TB_ONE + i] = 1;
-    st.h_tabs[TB_IOTA + i] = i;
-  }
   KH_CHECK_HIP(hipMemcpyAsync(st.tabs, st.h_tabs, TB_N * 4, hipMemcpyHostToDevice, m->stream));
-  std::vector<int32_t> all;
-  for (int b : {1, 2, 4})
-    for (const auto& k : hy_lat_kinds(hy)) {
-      Hybrid::Step::Lat t{b, k.first, k.second, 0, (int)all.size(), 0};
-      std::vector<int32_t> tab;
-      hy_lat_tiles(std::vector<int32_t>((size_t)b, 1), k, &t.cp, &tab);
-      t.n = (int)tab.size() / 2;
-      all.insert(all.end(), tab.begin(), tab.end());
-      st.lat.push_back(t);
-    }
-  TRY(dalloc(&st.tiles, all.size() + 1));
-  if (!all.empty()) KH_CHECK_HIP(hipMemcpy(st.tiles, all.data(), all.size() * 4, hipMemcpyHostToDevice));
   st.head_wg = std::min(cdiv(cdiv(hy.c.vocab, 4), 4), 1024);
   m->nparts = st.head_wg;
   TRY(dalloc(&m->part_val, (size_t)m->nparts));
@@ -437,7 +411,7 @@ int hy_decode(kh_model* m, const HyEntry* e, int n, float* h_logits) {
     st.h_tabs[TB_POS + i] = e[i].pos0;
     st.h_tabs[TB_SLOT + i] = e[i].slot;
   }
-  KH_CHECK_HIP(hipMemcpyAsync(st.tabs, st.h_tabs, TB_ONE * 4, hipMemcpyHostToDevice, m->stream));
+  KH_CHECK_HIP(hipMemcpyAsync(st.tabs, st.h_tabs, TB_ZERO * 4, hipMemcpyHostToDevice, m->stream));
   for (int i = 0; i < n;) {  // n = 3: 2 + 1
     const int B = n - i >= 4 ? 4 : (n - i >= 2 ? 2 : 1);
     const LdTabs tb{st.tabs + TB_TOK + i, st.tabs + TB_POS + i, st.tabs + TB_SLOT + i};

@@ -13,6 +13,8 @@
 // Softmax with a sink: m starts at sink_h and l at 1 in the first split (exp(sink - m), counted once, no value).
 // Scores, weights and sums are fp32; P is rounded to the storage type for its product with the values.
 #pragma once
+#include <type_traits>
+
 #include "kh_lops.h"
 
 namespace khm {
@@ -99,7 +101,7 @@ struct LatArgs {
   void* out;             // T [T][H][Rp] (one split)
   float* part;           // splits > 1: [T * H][splits][Rp + 4]: o (unnormalised), m, l.  One token per segment then:
                          // every row of a workgroup sees the same keys
-  const LatTile* tiles;
+  const LatTile* tiles;  // nullptr: one token per segment, ceil(H / rows of a tile) workgroups each
   int H, Rp, row, nsplit;
   float scale2;          // scale * log2(e)
   PassTabs p;
@@ -108,10 +110,11 @@ struct LatArgs {
 template <class T>
 struct LatCfg {
   static constexpr int KT = 4 * Tile<T>::N;      // keys per tile: 32 bf16, 16 fp32 (a 64-byte row of the transposed tile)
-  static constexpr int MAXROT = 128;
 };
 // keys per split and splits that have any: a split gets at least KH_LAT_SPLIT_MIN keys, whole tiles
-#define KH_LAT_SPLIT_MIN 64
+#ifndef KH_LAT_SPLIT_MIN
+#define KH_LAT_SPLIT_MIN 32
+#endif
 __host__ __device__ __forceinline__ int lat_split_len(int n_keys, int nsplit) {
   const int per = (n_keys + nsplit - 1) / nsplit;
   return (per + KH_LAT_SPLIT_MIN - 1) / KH_LAT_SPLIT_MIN * KH_LAT_SPLIT_MIN;
@@ -129,24 +132,39 @@ __device__ __forceinline__ int lat_perm(int k) {
   return sizeof(T) == 2 ? ((k >> 2) & 3) * 8 + (k >> 4) * 4 + (k & 3) : k;
 }
 
-// RT: 16-column tiles of the latent this instantiation can hold (Rp <= 16 RT); CP: column parts
-template <class T, int RT, int CP>
+// RT: 16-column tiles of the latent (Rp = 16 RT); DR: rotated part / 64; CP: column parts.  The row geometry is a
+// compile-time constant: a size guard around each fragment would end a scheduling block after every LDS read.
+template <class T, int RT, int DR, int CP>
 __global__ __launch_bounds__(256) void k_latent_attn(const LatArgs a) {
   typedef Tile<T> TL;
   typedef typename TL::frag frag;
   constexpr int E = TL::N, KT = LatCfg<T>::KT;
-  constexpr int NQ = (RT * 16 + LatCfg<T>::MAXROT) / (4 * E);  // 64-byte k-blocks of a query row, at most
+  constexpr int Rp = RT * 16, ROW = Rp + 64 * DR;
+  constexpr int NQ = ROW / (4 * E);                            // 64-byte k-blocks of a query row
   constexpr int NT = RT / CP;                                  // latent tiles per wave
   constexpr int NS = KT / 16;                                  // score tiles
-  constexpr int NB = ((KT / E) * (RT * 16 + LatCfg<T>::MAXROT) / E + 255) / 256;  // E x E blocks per thread
+  constexpr int cblk = ROW / E, nblk = (KT / E) * cblk;
+  constexpr int NB = (nblk + 255) / 256;                       // E x E blocks per thread
   extern __shared__ __attribute__((aligned(1024))) char smem_raw[];
   char* const Kt = smem_raw;
-  char* const Vt = smem_raw + (size_t)KT * a.row * sizeof(T);
+  char* const Vt = smem_raw + (size_t)KT * ROW * sizeof(T);
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int fr = lane & 15, fh = lane >> 4;
   const int wr = wave % (4 / CP), wc = wave / (4 / CP);
-  const LatTile tl = a.tiles[blockIdx.x];
-  const int n_rows = a.p.seg_n[tl.seg] * a.H, pos0 = a.p.seg_pos0[tl.seg], row0 = a.p.seg_row0[tl.seg];
+  LatTile tl;
+  int n_rows, pos0, row0;
+  if (a.tiles) {
+    tl = a.tiles[blockIdx.x];
+    n_rows = a.p.seg_n[tl.seg] * a.H;
+    row0 = a.p.seg_row0[tl.seg];
+  } else {  // one token per segment: no tables to wait for
+    const int per = (a.H + 64 / CP - 1) / (64 / CP);
+    tl.seg = (int)blockIdx.x / per;
+    tl.r0 = ((int)blockIdx.x - tl.seg * per) * (64 / CP);
+    n_rows = a.H;
+    row0 = tl.seg;
+  }
+  pos0 = a.p.seg_pos0[tl.seg];
   const T* cache = (const T*)a.cache + (size_t)a.p.seg_slot[tl.seg] * a.slot_elems;
   // this lane's query row
   int r = tl.r0 + wr * 16 + fr;
@@ -165,19 +183,10 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatArgs a) {
     if (k_lo >= n_keys) return;  // uniform; the merge does not read this split
     k_hi = k_lo + per < n_keys ? k_lo + per : n_keys;
   }
-  const int nqb = a.row / (4 * E);
-  const char* qrow = (const char*)((const T*)a.Q + ((size_t)(row0 + tok) * a.H + head) * a.row) + 16 * fh;
-  frag fq[NQ];
-#pragma unroll
-  for (int b = 0; b < NQ; ++b)
-    if (b < nqb) fq[b] = *(const frag*)(qrow + 64 * b);
-  const bool sinks = (a.nsplit == 1 || blockIdx.y == 0);
-  float m = sinks ? a.sink[head] * 1.44269504088896f : -INFINITY, l = sinks && fh == 0 ? 1.f : 0.f;
   f32x4 o[NT];
 #pragma unroll
   for (int n = 0; n < NT; ++n) o[n] = f32x4{0.f, 0.f, 0.f, 0.f};
   // ---- staging: an E x E block (E keys x E columns) per thread and pass
-  const int cblk = a.row / E, nblk = (KT / E) * cblk;
   frag pre[NB][E];
   auto fetch = [&](int k0) __attribute__((always_inline)) {
 #pragma unroll
@@ -189,7 +198,7 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatArgs a) {
         for (int e = 0; e < E; ++e) {
           int k = k0 + kb * E + e;
           k = k < n_keys ? k : n_keys - 1;
-          pre[q][e] = *(const frag*)(cache + (size_t)k * a.row + cb * E);
+          pre[q][e] = *(const frag*)(cache + (size_t)k * ROW + cb * E);
         }
       }
     }
@@ -205,7 +214,7 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatArgs a) {
           const int k = kb * E + e;
           *(frag*)(Kt + ((size_t)k * cblk + (cb ^ (k & 7))) * 16) = pre[q][e];
         }
-        if (cb * E < a.Rp) {
+        if (cb * E < Rp) {
           // transposed: column c gets its E keys.  The E keys of a block are two groups of four in the permuted order
 #pragma unroll
           for (int c = 0; c < E; ++c) {
@@ -228,6 +237,12 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatArgs a) {
     }
   };
   if (k_lo < k_hi) fetch(k_lo);
+  const char* qrow = (const char*)((const T*)a.Q + ((size_t)(row0 + tok) * a.H + head) * ROW) + 16 * fh;
+  frag fq[NQ];
+#pragma unroll
+  for (int b = 0; b < NQ; ++b) fq[b] = *(const frag*)(qrow + 64 * b);
+  const bool sinks = (a.nsplit == 1 || blockIdx.y == 0);
+  float m = sinks ? a.sink[head] * 1.44269504088896f : -INFINITY, l = sinks && fh == 0 ? 1.f : 0.f;
   for (int k0 = k_lo; k0 < k_hi; k0 += KT) {
     __syncthreads();  // everyone is done with the previous tile
     stash();
@@ -237,16 +252,13 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatArgs a) {
 #pragma unroll
     for (int n = 0; n < NS; ++n) s[n] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int b = 0; b < NQ; ++b) {
-      if (b < nqb) {
+    for (int b = 0; b < NQ; ++b)
 #pragma unroll
-        for (int n = 0; n < NS; ++n) {
-          const int k = n * 16 + fr;
-          const frag fk = *(const frag*)(Kt + ((size_t)k * cblk + ((4 * b + fh) ^ (k & 7))) * 16);
-          s[n] = TL::mma(fk, fq[b], s[n]);
-        }
+      for (int n = 0; n < NS; ++n) {
+        const int k = n * 16 + fr;
+        const frag fk = *(const frag*)(Kt + ((size_t)k * cblk + ((4 * b + fh) ^ (k & 7))) * 16);
+        s[n] = TL::mma(fk, fq[b], s[n]);
       }
-    }
     // lane: keys k0 + 16 n + 4 fh + i of row r
     float mx = m;
 #pragma unroll
@@ -274,14 +286,11 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatArgs a) {
       }
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
-      const int c0 = (wc * NT + n) * 16;
-      if (c0 < a.Rp) {
-        const int col = c0 + fr;
-        const frag fv = *(const frag*)(Vt + (size_t)col * 64 + ((fh ^ ((col >> 1) & 3)) << 4));
+      const int col = (wc * NT + n) * 16 + fr;
+      const frag fv = *(const frag*)(Vt + (size_t)col * 64 + ((fh ^ ((col >> 1) & 3)) << 4));
 #pragma unroll
-        for (int i = 0; i < 4; ++i) o[n][i] *= f;
-        o[n] = TL::mma(fv, p, o[n]);
-      }
+      for (int i = 0; i < 4; ++i) o[n][i] *= f;
+      o[n] = TL::mma(fv, p, o[n]);
     }
   }
   l = xor16_sum(l);
@@ -293,23 +302,21 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatArgs a) {
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
       const int c0 = (wc * NT + n) * 16;
-      if (c0 < a.Rp) {
-        f32x4 v;
+      f32x4 v;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = o[n][i] * inv;
-        *(typename TL::quad*)((T*)a.out + orow * a.Rp + c0 + 4 * fh) = to_quad<T>(v);
-      }
+      for (int i = 0; i < 4; ++i) v[i] = o[n][i] * inv;
+      *(typename TL::quad*)((T*)a.out + orow * Rp + c0 + 4 * fh) = to_quad<T>(v);
     }
   } else {
-    float* p = a.part + (orow * a.nsplit + blockIdx.y) * (size_t)(a.Rp + 4);
+    float* p = a.part + (orow * a.nsplit + blockIdx.y) * (size_t)(Rp + 4);
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
       const int c0 = (wc * NT + n) * 16;
-      if (c0 < a.Rp) *(f32x4*)(p + c0 + 4 * fh) = o[n];
+      *(f32x4*)(p + c0 + 4 * fh) = o[n];
     }
     if (wc == 0 && fh == 0) {
-      p[a.Rp] = m;
-      p[a.Rp + 1] = l;
+      p[Rp] = m;
+      p[Rp + 1] = l;
     }
   }
 }
@@ -326,18 +333,27 @@ int lat_attn_launch(hipStream_t s, const LatArgs& a, int ntiles, int cp) {
     return KH_OK;
   };
   // column parts: 4 = 16-row tiles, 2 = 32-row tiles (latents of more than 256), 1 = 64-row tiles
-  if (cp == 4) {
-    if (a.Rp <= 64) return go(k_latent_attn<T, 4, 4>);
-    if (a.Rp <= 128) return go(k_latent_attn<T, 8, 4>);
-    if (a.Rp <= 256) return go(k_latent_attn<T, 16, 4>);
-    if (a.Rp <= 512) return go(k_latent_attn<T, 32, 4>);
-  } else if (cp == 2) {
-    if (a.Rp <= 512) return go(k_latent_attn<T, 32, 2>);
-  } else if (cp == 1) {
-    if (a.Rp <= 64) return go(k_latent_attn<T, 4, 1>);
-    if (a.Rp <= 128) return go(k_latent_attn<T, 8, 1>);
-    if (a.Rp <= 256) return go(k_latent_attn<T, 16, 1>);
-  }
+  auto pick = [&](auto dr) -> int {
+    constexpr int DR = decltype(dr)::value;
+    if (cp == 4) {
+      if (a.Rp == 64) return go(k_latent_attn<T, 4, DR, 4>);
+      if (a.Rp == 128) return go(k_latent_attn<T, 8, DR, 4>);
+      if (a.Rp == 256) return go(k_latent_attn<T, 16, DR, 4>);
+      if (a.Rp == 512) return go(k_latent_attn<T, 32, DR, 4>);
+    } else if (cp == 2) {
+      if (a.Rp == 512) return go(k_latent_attn<T, 32, DR, 2>);
+    } else if (cp == 1) {
+      if (a.Rp == 64) return go(k_latent_attn<T, 4, DR, 1>);
+      if (a.Rp == 128) return go(k_latent_attn<T, 8, DR, 1>);
+      if (a.Rp == 256) return go(k_latent_attn<T, 16, DR, 1>);
+    }
+    return KH_ERR_UNSUPPORTED;
+  };
+  if (a.row - a.Rp == 64) return pick(std::integral_constant<int, 1>());
+  if (a.row - a.Rp == 128) return pick(std::integral_constant<int, 2>());
   return KH_ERR_UNSUPPORTED;
 }
+// padded sizes of a cache row the kernel is instantiated for: latent and rotated part (0: none)
+static inline int lat_pad_latent(int R) { return R <= 64 ? 64 : (R <= 128 ? 128 : (R <= 256 ? 256 : (R <= 512 ? 512 : 0))); }
+static inline int lat_pad_rot(int dr) { return dr <= 64 ? 64 : (dr <= 128 ? 128 : 0); }
 }  // namespace khm

@@ -631,11 +631,30 @@ __global__ __launch_bounds__(256) void k_ld_values(const LdValuesArgs a) {
   }
   l = block_sum(l, red);
   const float inv = 1.0f / l;
-  for (int i = threadIdx.x; i < nblk * Ld<T>::BE; i += 256) {
-    float v = 0.f;
-    if (i < a.Rp)
-      for (int s = 0; s < ns; ++s) v = __builtin_fmaf(fac[s], p[(size_t)s * (a.Rp + 4) + i], v);
-    xs[Ld<T>::place(i)] = v * inv;
+  // column groups of four; 256 / (Rp / 4) thread groups share the splits and meet in LDS
+  const int c4 = a.Rp >> 2, grp = c4 < 256 ? 256 / c4 : 1, g = (int)threadIdx.x / c4;
+  f32x4* sum = (f32x4*)(xs + (size_t)nblk * Ld<T>::BE);  // [grp][c4]
+  if (g < grp) {
+    for (int i = (int)threadIdx.x - g * c4; i < c4; i += 256) {
+      f32x4 v = f4_zero();
+      int s = g;
+      for (; s + 7 * grp < ns; s += 8 * grp) {
+        f32x4 x[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] = *(const f32x4*)(p + (size_t)(s + j * grp) * (a.Rp + 4) + 4 * i);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v = fma_s(fac[s + j * grp], x[j], v);
+      }
+      for (; s < ns; s += grp) v = fma_s(fac[s], *(const f32x4*)(p + (size_t)s * (a.Rp + 4) + 4 * i), v);
+      sum[g * c4 + i] = v;
+    }
+  }
+  __syncthreads();
+  for (int i = threadIdx.x; i < nblk * Ld<T>::BE / 4; i += 256) {
+    f32x4 v = f4_zero();
+    if (i < c4)
+      for (int k = 0; k < grp; ++k) v += sum[k * c4 + i];
+    ((f32x4*)xs)[ld_slot<T>(i)] = v * inv;
   }
   __syncthreads();
   while (item < items) {

@@ -156,54 +156,94 @@ struct ConvArgs {
   int C, ldx, ldo, taps;
   PassTabs p;
 };
-// E channels (16 bytes) of KH_CONV_TT consecutive tokens per thread.  grid (C / (256 E), T / KH_CONV_TT)
-#define KH_CONV_TT 4
-template <class T>
+// E channels (16 bytes) of KH_CONV_TT consecutive tokens per thread; the taps of the channels stay in registers.
+// TAPS: number of taps, 0 = any (weights re-read per token).  grid (C / (256 E), T / KH_CONV_TT)
+#define KH_CONV_TT 8
+template <class T, int TAPS>
 __global__ __launch_bounds__(256) void k_conv_silu(const ConvArgs<T> a, int T_all) {
   constexpr int E = Tile<T>::N;
+  typedef typename Tile<T>::frag frag;
   const int c = (blockIdx.x * 256 + threadIdx.x) * E;
   if (c >= a.C) return;
   const bool vec = c + E <= a.C && (a.ldx & (E - 1)) == 0;
+  const int taps = TAPS ? TAPS : a.taps;
+  float w[E][TAPS ? TAPS : 1], bias[E];
+#pragma unroll
+  for (int e = 0; e < E; ++e) {
+    bias[e] = c + e < a.C ? a.b[c + e] : 0.f;
+    if (TAPS)
+#pragma unroll
+      for (int k = 0; k < TAPS; ++k) w[e][k] = c + e < a.C ? a.w[(size_t)(c + e) * TAPS + k] : 0.f;
+  }
   for (int u = 0; u < KH_CONV_TT; ++u) {
     const int t = blockIdx.y * KH_CONV_TT + u;
     if (t >= T_all) return;
     const int sg = a.p.seg[t], i = t - a.p.seg_row0[sg];
-    const bool fresh = a.p.seg_pos0[sg] == 0;
-    const float* st = a.state + (size_t)a.p.seg_slot[sg] * a.slot_stride;
     float v[E];
 #pragma unroll
-    for (int e = 0; e < E; ++e) v[e] = c + e < a.C ? a.b[c + e] : 0.f;
-    for (int k = 0; k < a.taps; ++k) {
-      const int j = i - (a.taps - 1) + k;  // row of the segment
-      float in[E];
-#pragma unroll
-      for (int e = 0; e < E; ++e) in[e] = 0.f;
-      if (j >= 0) {
-        const T* x = a.xz + (size_t)(t - i + j) * a.ldx + c;
-        if (vec) {
-          const typename Tile<T>::frag f = *(const typename Tile<T>::frag*)x;
-#pragma unroll
-          for (int e = 0; e < E; ++e) in[e] = (float)f[e];
-        } else {
-#pragma unroll
-          for (int e = 0; e < E; ++e)
-            if (c + e < a.C) in[e] = (float)x[e];
-        }
-      } else if (!fresh) {
-#pragma unroll
-        for (int e = 0; e < E; ++e)
-          if (c + e < a.C) in[e] = st[(size_t)(a.taps - 1 + j) * a.C + c + e];
-      }
+    for (int e = 0; e < E; ++e) v[e] = bias[e];
+    auto tap = [&](int k, const float (&in)[E]) __attribute__((always_inline)) {
 #pragma unroll
       for (int e = 0; e < E; ++e)
-        if (c + e < a.C) v[e] = __builtin_fmaf(a.w[(size_t)(c + e) * a.taps + k], in[e], v[e]);
+        v[e] = __builtin_fmaf(TAPS ? w[e][TAPS ? k : 0] : (c + e < a.C ? a.w[(size_t)(c + e) * taps + k] : 0.f), in[e], v[e]);
+    };
+    auto from_row = [&](int j, float (&in)[E]) __attribute__((always_inline)) {
+      const T* x = a.xz + (size_t)(t - i + j) * a.ldx + c;
+      if (vec) {
+        const frag f = *(const frag*)x;
+#pragma unroll
+        for (int e = 0; e < E; ++e) in[e] = (float)f[e];
+      } else {
+#pragma unroll
+        for (int e = 0; e < E; ++e) in[e] = c + e < a.C ? (float)x[e] : 0.f;
+      }
+    };
+    float in[E];
+    if (i >= taps - 1) {  // every input is a row of the segment
+      if (TAPS) {
+#pragma unroll
+        for (int k = 0; k < TAPS; ++k) {
+          from_row(i - (TAPS - 1) + k, in);
+          tap(k, in);
+        }
+      } else {
+        for (int k = 0; k < taps; ++k) {
+          from_row(i - (taps - 1) + k, in);
+          tap(k, in);
+        }
+      }
+    } else {
+      const bool fresh = a.p.seg_pos0[sg] == 0;
+      const float* st = a.state + (size_t)a.p.seg_slot[sg] * a.slot_stride;
+      auto edge = [&](int k) __attribute__((always_inline)) {
+        const int j = i - (taps - 1) + k;
+        if (j >= 0) {
+          from_row(j, in);
+        } else {
+#pragma unroll
+          for (int e = 0; e < E; ++e) in[e] = !fresh && c + e < a.C ? st[(size_t)(taps - 1 + j) * a.C + c + e] : 0.f;
+        }
+        tap(k, in);
+      };
+      if constexpr (TAPS != 0) {
+#pragma unroll
+        for (int k = 0; k < TAPS; ++k) edge(k);
+      } else {
+        for (int k = 0; k < taps; ++k) edge(k);
+      }
     }
-    T* o = a.out + (size_t)t * a.ldo + c;  // rows are padded to whole fragments
-    typename Tile<T>::frag f;
+    frag f;  // output rows are padded to whole fragments
 #pragma unroll
     for (int e = 0; e < E; ++e) f[e] = (T)(c + e < a.C ? silu1(v[e]) : 0.f);
-    *(typename Tile<T>::frag*)o = f;
+    *(frag*)(a.out + (size_t)t * a.ldo + c) = f;
   }
+}
+template <class T>
+void conv_launch(hipStream_t s, const ConvArgs<T>& a, int T_all) {
+  constexpr int CW = 256 * Tile<T>::N;
+  const dim3 g((a.C + CW - 1) / CW, (T_all + KH_CONV_TT - 1) / KH_CONV_TT);
+  if (a.taps == 4) hipLaunchKernelGGL((k_conv_silu<T, 4>), g, dim3(256), 0, s, a, T_all);
+  else hipLaunchKernelGGL((k_conv_silu<T, 0>), g, dim3(256), 0, s, a, T_all);
 }
 // the last taps - 1 inputs of every segment become its sequence's state.  grid (C / 256, S)
 template <class T>
