@@ -8,7 +8,7 @@
 // the reference's space -> "Ġ" replacement unless --hf-spaces, two stop ids); the decoded text is
 // printed like main.cpp:43-45.
 //
-//   kuiper_demo model.bin [--family llama|qwen2] [--quant] [--rope interleaved|half]
+//   kuiper_demo model.bin | checkpoint-folder [--dtype bfloat16|float32] [--family llama|qwen2] [--quant] [--rope interleaved|half]
 //               [--theta 10000] [--eps 1e-5] [--steps 128] [--prompt 1,263] [--stop 2]
 //               [--exec graph|fused|unfused] [--max-seq-len N] [--device 0]
 //               [--tokenizer tokenizer.model | --tokenizer-json tokenizer.json [--hf-spaces]] [--text "a"]
@@ -17,6 +17,8 @@
 // --exact-prefill = KH_FLAG_PREFILL_EXACT: the prompt phase bit for bit the reference's one-token-per-pass prompt
 // phase (demo/main.cpp:20-22); without it prompts of 17+ tokens run as fp32-MFMA GEMMs (tolerance parity, 8-10 x the
 // prompt tokens/s).  --fenced-merge = KH_FLAG_ATTN_MERGE_FENCED.  The self-checks of kh_model_create_* are printed.
+// A folder (config.json + model.safetensors) is a layer-list model: family, rotation and epsilon come from its
+// configuration, --dtype picks the storage type.
 // Prints the generated ids and "steps/s" like demo/main.cpp:70-72.
 #include <chrono>
 #include <cstdio>
@@ -29,7 +31,7 @@
 
 static void usage() {
   std::fprintf(stderr,
-               "usage: kuiper_demo model.bin [--family llama|qwen2] [--quant] [--rope interleaved|half]\n"
+               "usage: kuiper_demo model.bin|folder [--dtype bfloat16|float32] [--family llama|qwen2] [--quant] [--rope interleaved|half]\n"
                "       [--theta F] [--eps F] [--steps N] [--prompt id,id,...] [--stop id,id] [--exec graph|fused|unfused]\n"
                "       [--max-seq-len N] [--device D] [--tokenizer tokenizer.model | --tokenizer-json tokenizer.json\n"
                "       [--hf-spaces]] [--text \"...\"] [--exact-prefill] [--fenced-merge]\n");
@@ -41,7 +43,7 @@ int main(int argc, char** argv) {
     return 2;
   }
   const char* path = argv[1];
-  kh_model_opts o{KH_FAMILY_LLAMA, 0, KH_ROPE_INTERLEAVED, 10000.f, 1e-5f, 0, 0, 0};
+  kh_model_opts o{KH_FAMILY_LLAMA, 0, KH_ROPE_INTERLEAVED, 10000.f, 1e-5f, 0, 0, 0, KH_DTYPE_DEFAULT, 1};
   int steps = 128, exec = KH_EXEC_GRAPH;
   std::vector<int32_t> stop;  // is_sentence_ending ids (main.cpp:30): eos / <|eot_id|> / ...
   std::vector<int32_t> prompt{1, 263};  // BOS + "a": the reference demo's prompt (main.cpp:64)
@@ -62,6 +64,7 @@ int main(int argc, char** argv) {
     if (a == "--family") o.family = std::string(next()) == "qwen2" ? KH_FAMILY_QWEN2 : KH_FAMILY_LLAMA;
     else if (a == "--quant") o.is_quant = 1;
     else if (a == "--rope") o.rope_mode = std::string(next()) == "half" ? KH_ROPE_HALF : KH_ROPE_INTERLEAVED;
+    else if (a == "--dtype") o.dtype = std::string(next()) == "float32" ? KH_DTYPE_F32 : KH_DTYPE_BF16;
     else if (a == "--theta") o.rope_theta = (float)std::atof(next());
     else if (a == "--eps") o.rms_eps = (float)std::atof(next());
     else if (a == "--steps") steps = std::atoi(next());
