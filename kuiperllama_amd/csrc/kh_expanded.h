@@ -41,7 +41,9 @@ __global__ __launch_bounds__(256) void k_expanded_attn(const ExpArgs a) {
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int fr = lane & 15, fh = lane >> 4;
   const int head = blockIdx.x;
-  const int tile = (int)gridDim.y - 1 - (int)blockIdx.y;  // the longest key ranges first
+  // longest key ranges first; a launch of at most two workgroups per CU pairs the longest with the shortest instead
+  const int nt = (int)gridDim.y, half = (nt + 1) >> 1, by = (int)blockIdx.y;
+  const int tile = nt * (int)gridDim.x <= 512 && by >= half ? by - half : nt - 1 - by;
   const int q0 = tile * (64 * MR);
   constexpr int qc = DN / E, rc = DRP / E;  // 16-byte chunks of the key parts
   constexpr int bytes_k = KT * DN * ES, bytes_r = KT * DRP * ES, stage = bytes_k + bytes_r + DV * 64;

@@ -6,15 +6,17 @@
 // H x tokens query rows of a sequence therefore share each staged key tile - one read of the cache per 16 .. 64 rows.
 //
 // k_latent_attn: workgroup = 4 waves = WR row tiles of 16 query rows x CP column parts (WR CP = 4) of the latent.
-//   S^T = K Q^T: a lane ends with the scores of ONE query row (its column), so the running max / sum are lane scalars
-//   plus two cross-row swaps, and P^T is already the second operand of O^T = C^T P^T: no LDS round trip.  The key
-//   order inside a tile is permuted so that the four-score groups of the result layout are the contiguous fragment
-//   groups of the operand layout; the transposed tile is staged with the same permutation.
+//   Key tiles of KT rows go straight from the cache to LDS (LDS-DMA, a ring of two).  S^T = K Q^T: a lane ends with the
+//   scores of ONE query row (its column), so the running max / sum are lane scalars plus two cross-row swaps, and P^T
+//   is already the second operand of O^T = C^T P^T.  The first operand, columns of the tile, comes from the same LDS
+//   rows: bf16 through the transposing read (ds_read_b64_tr_b16: lane i of 16 receives element i of four rows), fp32
+//   one element at a time.
 // Softmax with a sink: m starts at sink_h and l at 1 in the first split (exp(sink - m), counted once, no value).
 // Scores, weights and sums are fp32; P is rounded to the storage type for its product with the values.
 #pragma once
 #include <type_traits>
 
+#include "kh_lgemm.h"
 #include "kh_lops.h"
 
 namespace khm {
@@ -109,7 +111,7 @@ struct LatArgs {
 
 template <class T>
 struct LatCfg {
-  static constexpr int KT = 4 * Tile<T>::N;      // keys per tile: 32 bf16, 16 fp32 (a 64-byte row of the transposed tile)
+  static constexpr int KT = 4 * Tile<T>::N;  // keys per tile: 32 bf16, 16 fp32 (one k-block of the second product)
 };
 // keys per split and splits that have any: a split gets at least KH_LAT_SPLIT_MIN keys, whole tiles
 #ifndef KH_LAT_SPLIT_MIN
@@ -124,12 +126,36 @@ __host__ __device__ __forceinline__ int lat_active_splits(int n_keys, int nsplit
   return (n_keys + per - 1) / per;
 }
 template <class T>
-static inline size_t lat_lds(int row, int Rp) { return (size_t)LatCfg<T>::KT * row * sizeof(T) + (size_t)Rp * 64; }
+static inline size_t lat_lds(int row) { return (size_t)2 * LatCfg<T>::KT * row * sizeof(T); }
 
-// position of key k of a tile in the permuted order (see above)
-template <class T>
-__device__ __forceinline__ int lat_perm(int k) {
-  return sizeof(T) == 2 ? ((k >> 2) & 3) * 8 + (k >> 4) * 4 + (k & 3) : k;
+// First operand of the second product: the lane's column `col`, keys 4 fh .. + 3 (and + 16 for bf16) of a tile whose
+// 16-byte chunk c of row k lies in slot c ^ (k & 7)
+template <int CB /* chunks per row */>
+__device__ __forceinline__ bf16x8 lat_col(const char* tile, int c0, int lane, bf16) {
+  typedef short s16x4 __attribute__((ext_vector_type(4)));
+  const int fh = lane >> 4, k = 4 * fh + ((lane >> 2) & 3), c = (c0 >> 3) + ((lane & 3) >> 1);
+  bf16x8 r;
+#pragma unroll
+  for (int n = 0; n < 2; ++n) {
+    const int kk = k + 16 * n;
+    const char* p = tile + ((size_t)kk * CB + (c ^ (kk & 7))) * 16 + (lane & 1) * 8;
+    const s16x4 v = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)p);
+    const bf16x4 q = __builtin_bit_cast(bf16x4, v);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) r[4 * n + i] = q[i];
+  }
+  return r;
+}
+template <int CB>
+__device__ __forceinline__ f32x4 lat_col(const char* tile, int c0, int lane, float) {
+  const int fh = lane >> 4, col = c0 + (lane & 15), c = col >> 2;
+  f32x4 r;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int k = 4 * fh + i;
+    r[i] = *(const float*)(tile + ((size_t)k * CB + (c ^ (k & 7))) * 16 + (col & 3) * 4);
+  }
+  return r;
 }
 
 // RT: 16-column tiles of the latent (Rp = 16 RT); DR: rotated part / 64; CP: column parts.  The row geometry is a
@@ -143,12 +169,10 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatArgs a) {
   constexpr int NQ = ROW / (4 * E);                            // 64-byte k-blocks of a query row
   constexpr int NT = RT / CP;                                  // latent tiles per wave
   constexpr int NS = KT / 16;                                  // score tiles
-  constexpr int cblk = ROW / E, nblk = (KT / E) * cblk;
-  constexpr int NB = (nblk + 255) / 256;                       // E x E blocks per thread
+  constexpr int cblk = ROW / E, NL = KT * cblk / 256;          // chunks of a row; LDS-DMA requests per wave and tile
+  constexpr int TB = KT * ROW * (int)sizeof(T);                // bytes of a tile
   extern __shared__ __attribute__((aligned(1024))) char smem_raw[];
-  char* const Kt = smem_raw;
-  char* const Vt = smem_raw + (size_t)KT * ROW * sizeof(T);
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int fr = lane & 15, fh = lane >> 4;
   const int wr = wave % (4 / CP), wc = wave / (4 / CP);
   LatTile tl;
@@ -186,68 +210,37 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatArgs a) {
   f32x4 o[NT];
 #pragma unroll
   for (int n = 0; n < NT; ++n) o[n] = f32x4{0.f, 0.f, 0.f, 0.f};
-  // ---- staging: an E x E block (E keys x E columns) per thread and pass
-  frag pre[NB][E];
-  auto fetch = [&](int k0) __attribute__((always_inline)) {
+  // ---- staging: request j of a wave covers chunks (4 j + wave) 64 .. of the tile
+  int kr[NL];
+  unsigned kc[NL];
 #pragma unroll
-    for (int q = 0; q < NB; ++q) {
-      const int b = q * 256 + (int)threadIdx.x;
-      const int kb = b / cblk, cb = b - kb * cblk;
-      if (b < nblk) {
+  for (int j = 0; j < NL; ++j) {
+    const int c = (4 * j + wave) * 64 + lane;
+    kr[j] = c / cblk;
+    kc[j] = (unsigned)(((c - kr[j] * cblk) ^ (kr[j] & 7)) << 4);
+  }
+  const unsigned lds0 = (unsigned)__builtin_amdgcn_readfirstlane((int)kh_lds_addr(smem_raw)) + 1024u * wave;
+  auto issue = [&](int slot, int k0) __attribute__((always_inline)) {
+    const char* base = (const char*)(cache + (size_t)k0 * ROW);
 #pragma unroll
-        for (int e = 0; e < E; ++e) {
-          int k = k0 + kb * E + e;
-          k = k < n_keys ? k : n_keys - 1;
-          pre[q][e] = *(const frag*)(cache + (size_t)k * ROW + cb * E);
-        }
-      }
+    for (int j = 0; j < NL; ++j) {
+      const int k = k0 + kr[j] < n_keys ? kr[j] : n_keys - 1 - k0;  // rows behind the sequence's last may not be backed
+      dma_x4_keep(base, (unsigned)(k * (ROW * (int)sizeof(T))) + kc[j], lds0 + (unsigned)(slot * TB + 4096 * j));
     }
   };
-  auto stash = [&]() __attribute__((always_inline)) {
-#pragma unroll
-    for (int q = 0; q < NB; ++q) {
-      const int b = q * 256 + (int)threadIdx.x;
-      const int kb = b / cblk, cb = b - kb * cblk;
-      if (b < nblk) {
-#pragma unroll
-        for (int e = 0; e < E; ++e) {
-          const int k = kb * E + e;
-          *(frag*)(Kt + ((size_t)k * cblk + (cb ^ (k & 7))) * 16) = pre[q][e];
-        }
-        if (cb * E < Rp) {
-          // transposed: column c gets its E keys.  The E keys of a block are two groups of four in the permuted order
-#pragma unroll
-          for (int c = 0; c < E; ++c) {
-            const int col = cb * E + c;
-            char* v = Vt + (size_t)col * 64;
-#pragma unroll
-            for (int g = 0; g < E / 4; ++g) {
-              typename TL::quad u;
-              u.x = pre[q][4 * g + 0][c];
-              u.y = pre[q][4 * g + 1][c];
-              u.z = pre[q][4 * g + 2][c];
-              u.w = pre[q][4 * g + 3][c];
-              const int kp = lat_perm<T>(kb * E + 4 * g);           // first key's place
-              const int chunk = (kp / E) ^ ((col >> 1) & 3);
-              *(typename TL::quad*)(v + chunk * 16 + (kp % E) * (int)sizeof(T)) = u;
-            }
-          }
-        }
-      }
-    }
-  };
-  if (k_lo < k_hi) fetch(k_lo);
+  if (k_lo < k_hi) issue(0, k_lo);
   const char* qrow = (const char*)((const T*)a.Q + ((size_t)(row0 + tok) * a.H + head) * ROW) + 16 * fh;
   frag fq[NQ];
 #pragma unroll
   for (int b = 0; b < NQ; ++b) fq[b] = *(const frag*)(qrow + 64 * b);
   const bool sinks = (a.nsplit == 1 || blockIdx.y == 0);
   float m = sinks ? a.sink[head] * 1.44269504088896f : -INFINITY, l = sinks && fh == 0 ? 1.f : 0.f;
-  for (int k0 = k_lo; k0 < k_hi; k0 += KT) {
-    __syncthreads();  // everyone is done with the previous tile
-    stash();
-    __syncthreads();
-    if (k0 + KT < k_hi) fetch(k0 + KT);
+  int slot = 0;
+  for (int k0 = k_lo; k0 < k_hi; k0 += KT, slot ^= 1) {
+    wait_vm<0>();     // this tile has landed (the next one is requested behind the barrier)
+    __syncthreads();  // ... for every wave, and everyone is done with the tile before
+    if (k0 + KT < k_hi) issue(slot ^ 1, k0 + KT);
+    const char* Kt = smem_raw + slot * TB;
     f32x4 s[NS];
 #pragma unroll
     for (int n = 0; n < NS; ++n) s[n] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -286,8 +279,7 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatArgs a) {
       }
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
-      const int col = (wc * NT + n) * 16 + fr;
-      const frag fv = *(const frag*)(Vt + (size_t)col * 64 + ((fh ^ ((col >> 1) & 3)) << 4));
+      const frag fv = lat_col<cblk>(Kt, (wc * NT + n) * 16, lane, T());
 #pragma unroll
       for (int i = 0; i < 4; ++i) o[n][i] *= f;
       o[n] = TL::mma(fv, p, o[n]);
@@ -323,7 +315,7 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatArgs a) {
 
 template <class T>
 int lat_attn_launch(hipStream_t s, const LatArgs& a, int ntiles, int cp) {
-  const size_t lds = lat_lds<T>(a.row, a.Rp);
+  const size_t lds = lat_lds<T>(a.row);
   auto go = [&](auto kern) -> int {
     if (lds > 64 * 1024) {
       const hipError_t e = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
