@@ -44,7 +44,7 @@ size_t lds_out(const Hybrid& hy, const HyLayer& l, int B) {
   const int nbv = Ld<T>::blocks(nv);
   const int nf = l.ff.on ? l.ff.top * Ld<T>::blocks(l.ff.ffp) + (l.ff.sffp ? Ld<T>::blocks(l.ff.sffp) : 0) : 0;
   (void)hy;
-  return (size_t)(nbv + nf) * sizeof(LdBlk) + ((size_t)B * nbv + nf) * Ld<T>::BE * 4;  // table, vectors
+  return ((size_t)B * nbv + nf) * Ld<T>::BE * 4;
 }
 template <class T>
 bool fits(const Hybrid& hy, int B) {
@@ -296,11 +296,13 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
         a.ffp = f.ffp;
         a.sffp = f.sffp;
       }
-      // waves of a row pair: as many as keep each wave's share within two tiles of the ring, while the launch has at
-      // most four workgroups per CU
+      // waves of a row pair: as many as keep each wave's share within its two tiles and give every CU a workgroup, while
+      // the launch has at most four per CU
       const int nblk = Ld<T>::blocks(wo.ld) + (f.on ? f.top * Ld<T>::blocks(f.ffp) + (f.sff ? Ld<T>::blocks(f.sffp) : 0) : 0);
       a.ks = 1;
-      while (a.ks < 8 && nblk / a.ks > 8 && cdiv(cdiv(W, 2) * a.ks * 2, 8) <= 1024) a.ks *= 2;
+      while (a.ks < 8 && nblk >= 2 * a.ks && (nblk / a.ks > 8 || cdiv(cdiv(W, 2) * a.ks, 8) < 256) &&
+             cdiv(cdiv(W, 2) * a.ks * 2, 8) <= 1024)
+        a.ks *= 2;
       TRY(go(k_ld_out<T, B>, dim3(cdiv(cdiv(W, 2) * a.ks, 8)), 512, lds_out<T>(hy, l, B), s, a));
     }
     x_in = x_out;

@@ -57,25 +57,36 @@ __device__ __forceinline__ void ld_stage(f32x4* xs, const float* src, int n4, in
   }
 }
 // Layer norm of one row (256 threads, NV float4 each, rows padded with zeros to ld) into LDS slots.  v: the row in
-// registers; returns the normalised values in v (also written to `out` when given).
+// registers; returns the normalised values in v (also written to `out` when given).  Mean and variance come from ONE
+// workgroup reduction of (x - shift) and (x - shift)^2, shift = an element of the row: no cancellation beyond the
+// distance of that element from the mean.  red: 2 KH_WAVES_MAX floats.
 template <class T, int NV>
-__device__ __forceinline__ void ld_norm(f32x4 (&v)[NV], const f32x4 (&w)[NV], const f32x4 (&b)[NV], int W, int n4, int total4,
-                                        float eps, float* red, f32x4* xs, f32x4* out) {
-  float s = 0.f;
-#pragma unroll
-  for (int j = 0; j < NV; ++j) s += (v[j].x + v[j].y) + (v[j].z + v[j].w);
-  const float mean = block_sum(s, red) / (float)W;
-  float d2 = 0.f;
+__device__ __forceinline__ void ld_norm(f32x4 (&v)[NV], const f32x4 (&w)[NV], const f32x4 (&b)[NV], float shift, int W, int n4,
+                                        int total4, float eps, float* red, f32x4* xs, f32x4* out) {
+  float s1 = 0.f, s2 = 0.f;
 #pragma unroll
   for (int j = 0; j < NV; ++j) {
     const int i = threadIdx.x + 256 * j;
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
-      const float d = 4 * i + k < W ? v[j][k] - mean : 0.f;
-      d2 = __builtin_fmaf(d, d, d2);
+      const float d = 4 * i + k < W ? v[j][k] - shift : 0.f;
+      s1 += d;
+      s2 = __builtin_fmaf(d, d, s2);
     }
   }
-  const float rstd = 1.0f / sqrtf(block_sum(d2, red) / (float)W + eps);
+  s1 = wave_sum(s1);
+  s2 = wave_sum(s2);
+  const int wave = threadIdx.x >> 6;
+  if ((threadIdx.x & 63) == 0) {
+    red[wave] = s1;
+    red[KH_WAVES_MAX + wave] = s2;
+  }
+  __syncthreads();
+  s1 = (red[0] + red[1]) + (red[2] + red[3]);
+  s2 = (red[KH_WAVES_MAX] + red[KH_WAVES_MAX + 1]) + (red[KH_WAVES_MAX + 2] + red[KH_WAVES_MAX + 3]);
+  const float m = s1 / (float)W, mean = shift + m;
+  const float var = fmaxf(s2 / (float)W - m * m, 0.f);
+  const float rstd = 1.0f / sqrtf(var + eps);
 #pragma unroll
   for (int j = 0; j < NV; ++j) {
     const int i = threadIdx.x + 256 * j;
@@ -194,7 +205,7 @@ __global__ __launch_bounds__(256) void k_ld_in(const LdInArgs a) {
   constexpr int R = 4, U = 4;
   extern __shared__ __attribute__((aligned(16))) char smem_raw[];
   float* xs = (float*)smem_raw;
-  __shared__ float red[KH_WAVES_MAX];
+  __shared__ float red[2 * KH_WAVES_MAX];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, wg = blockIdx.x;
   int si = 0;
   if (a.nseg > 1 && wg >= a.seg[1].wg0) si = 1;
@@ -233,6 +244,25 @@ __global__ __launch_bounds__(256) void k_ld_in(const LdInArgs a) {
     set_rows(item);
     ld_load<T, R, U>(t, row, 0, nblk, nch, lane);
   }
+  // convolution operands of the wave's first item: requested with its weights (up to four taps)
+  constexpr int CT = 4;
+  float cw[CT], cs[CT];
+  float cb = 0.f;
+  const bool conv_pre = kind == LDI_CONV && a.taps <= CT;
+  if (conv_pre && item < items && lane < R * B) {
+    const int c = item * R + (lane & (R - 1)), q = lane / R;
+    if (c < a.inner) {
+      const float* st = a.conv_st + (size_t)a.t.slot[q] * a.slot_stride + c;
+      const bool fresh = a.t.pos[q] == 0;
+      cb = a.conv_b[c];
+#pragma unroll
+      for (int k = 0; k < CT; ++k) {
+        cw[k] = k < a.taps ? a.conv_w[(size_t)c * a.taps + k] : 0.f;
+        cs[k] = k + 1 < a.taps && !fresh ? st[(size_t)k * a.inner] : 0.f;
+      }
+    }
+  }
+  const int first_item = item;
   // ---- layer norm of B rows
   const int xstride = nblk * Ld<T>::BE, n4 = a.ld >> 2, total4 = xstride >> 2;
   {
@@ -267,7 +297,9 @@ __global__ __launch_bounds__(256) void k_ld_in(const LdInArgs a) {
       }
       // the router's first workgroup leaves the second norm for the launches that follow
       f32x4* keep = a.xn2 && wg == a.seg[1].wg0 ? (f32x4*)(a.xn2 + (size_t)q * a.ld) : nullptr;
-      ld_norm<T, NV>(v, nw, nb, a.W, n4, total4, a.eps, red, (f32x4*)(xs + (size_t)q * xstride), keep);
+      float shift = a.from_embed ? (float)((const T*)a.embed)[(size_t)a.t.tok[q] * a.ld] : a.x_in[(size_t)q * a.ld];
+      if (q) __syncthreads();  // red is free again
+      ld_norm<T, NV>(v, nw, nb, shift, a.W, n4, total4, a.eps, red, (f32x4*)(xs + (size_t)q * xstride), keep);
     }
   }
   __syncthreads();
@@ -295,15 +327,29 @@ __global__ __launch_bounds__(256) void k_ld_in(const LdInArgs a) {
         if (i < rows) {
           if (kind == LDI_CONV && i < a.inner) {
             float* st = a.conv_st + (size_t)a.t.slot[q] * a.slot_stride + i;
-            const bool fresh = a.t.pos[q] == 0;
-            const float* cw = a.conv_w + (size_t)i * a.taps;
-            float c = a.conv_b[i];
-            for (int k = 0; k + 1 < a.taps; ++k) {
-              const float in = fresh ? 0.f : st[(size_t)k * a.inner];
-              c = __builtin_fmaf(cw[k], in, c);
-              if (k) st[(size_t)(k - 1) * a.inner] = in;
+            float c;
+            if (conv_pre && cur == first_item) {
+              c = cb;
+#pragma unroll
+              for (int k = 0; k < CT; ++k) {
+                if (k + 1 < a.taps) {
+                  c = __builtin_fmaf(cw[k], cs[k], c);
+                  if (k) st[(size_t)(k - 1) * a.inner] = cs[k];
+                } else if (k + 1 == a.taps) {
+                  c = __builtin_fmaf(cw[k], v, c);
+                }
+              }
+            } else {
+              const bool fresh = a.t.pos[q] == 0;
+              const float* w1 = a.conv_w + (size_t)i * a.taps;
+              c = a.conv_b[i];
+              for (int k = 0; k + 1 < a.taps; ++k) {
+                const float in = fresh ? 0.f : st[(size_t)k * a.inner];
+                c = __builtin_fmaf(w1[k], in, c);
+                if (k) st[(size_t)(k - 1) * a.inner] = in;
+              }
+              c = __builtin_fmaf(w1[a.taps - 1], v, c);
             }
-            c = __builtin_fmaf(cw[a.taps - 1], v, c);
             if (a.taps > 1) st[(size_t)(a.taps - 2) * a.inner] = v;
             a.xc[(size_t)q * a.xc_ld + i] = silu1(c);
           } else {
@@ -683,12 +729,9 @@ struct LdOutArgs {
   int W, ld, n4v, ld_v, ldv, top, ffp, sffp, moe, ks;
 };
 // Workgroup = 8 waves = 8 / ks groups of ks waves; a group owns R rows, its waves share the blocks of the concatenation
-// [mixer | shared | expert 0 | expert 1 ...] (identity experts: blocks with no chunks, skipped).  Experts differ between
-// sequences, so for B > 1 the feed-forward part runs once per sequence.
-struct LdBlk {
-  const void* p;    // row 0 at this block
-  int stride, nch;  // elements between rows; 16-byte chunks of a row in this block (0: skip)
-};
+// [mixer | shared | expert 0 | expert 1 ...] (blocks of identity experts are skipped).  Experts differ between
+// sequences, so for B > 1 the feed-forward part runs once per sequence.  A block's place follows from its number, so
+// the first two tiles of a wave are requested before the vectors are staged.
 template <class T, int B>
 __global__ __launch_bounds__(512) void k_ld_out(const LdOutArgs a) {
   constexpr int R = 2, U = 4;
@@ -698,62 +741,79 @@ __global__ __launch_bounds__(512) void k_ld_out(const LdOutArgs a) {
   __shared__ float comb[8][R * B];
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int nbv = Ld<T>::blocks(a.ldv);
-  const int nbe = a.moe ? Ld<T>::blocks(a.ffp) : 0, nbs = a.moe && a.sffp ? Ld<T>::blocks(a.sffp) : 0;
-  const int nb = nbv + nbs + a.top * nbe;
-  LdBlk* tab = (LdBlk*)smem_raw;
-  float* xv = (float*)(smem_raw + (size_t)nb * sizeof(LdBlk));
+  const int nbe = a.moe ? Ld<T>::blocks(a.ffp) : 1, nbs = a.moe && a.sffp ? Ld<T>::blocks(a.sffp) : 0;
+  const int nb = nbv + nbs + (a.moe ? a.top * nbe : 0);
+  float* xv = (float*)smem_raw;
   float* xf = xv + (size_t)B * nbv * BE;
   const int kp = wave % a.ks, grp = (int)blockIdx.x * (8 / a.ks) + wave / a.ks;
   const int item = grp * R;
   int ri[R];
 #pragma unroll
   for (int r = 0; r < R; ++r) ri[r] = item + r < a.W ? item + r : a.W - 1;
-  auto part = [&](int n, const T* base, int stride, int len, LdBlk* out, int tid0) __attribute__((always_inline)) {
-    for (int b = (int)threadIdx.x - tid0; b >= 0 && b < n; b += 512) {
-      const int left = len / E - b * 64;
-      out[b] = LdBlk{base + (size_t)b * BE, stride, left < 64 ? left : 64};
+  // residual operands of the rows this wave will finish
+  float rx = 0.f, rn = 0.f, rw = 0.f;
+  if (kp == 0 && lane < R * B) {
+    const int q = lane / R, i = item + (lane & (R - 1));
+    if (i < a.W) {
+      rx = a.x_cur[(size_t)q * a.ld + i];
+      if (a.moe) {
+        rn = a.xn2[(size_t)q * a.ld + i];
+        rw = a.id_w[q];
+      }
+    }
+  }
+  frag w[2][R][U];
+  int nc[2][U];
+  auto fetch = [&](int set, int b0, int b1, int q) __attribute__((always_inline)) {
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int b = b0 + u;  // wave-uniform
+      nc[set][u] = 0;
+      if (b < b1) {
+        const T* p = (const T*)a.wo;
+        int stride = a.ldv, bb = b;
+        bool have = true;
+        if (b >= nbv + nbs) {
+          const int e = b - nbv - nbs, k = e / nbe, id = a.ids[q * a.top + k];
+          bb = e - k * nbe;
+          stride = a.ffp;
+          have = id >= 0;
+          p = (const T*)a.down + (size_t)(have ? id : 0) * a.W * a.ffp;
+        } else if (b >= nbv) {
+          bb = b - nbv;
+          stride = a.sffp;
+          p = (const T*)a.sdown;
+        }
+        const int left = stride / E - bb * 64, n = left < 64 ? left : 64;
+        nc[set][u] = have ? n : 0;
+        if (have) {
+          const int c = lane < n ? lane : n - 1;
+#pragma unroll
+          for (int r = 0; r < R; ++r) w[set][r][u] = ld_nt((const frag*)(p + (size_t)ri[r] * stride + (size_t)bb * BE) + c);
+        }
+      }
     }
   };
-  part(nbv, (const T*)a.wo, a.ldv, a.ldv, tab, 0);
-  if (nbs) part(nbs, (const T*)a.sdown, a.sffp, a.sffp, tab + nbv, 64);
-  for (int q = 0; q < B; ++q)
-    ld_stage<T, 512>((f32x4*)(xv + (size_t)q * nbv * BE), a.v + (size_t)q * a.ld_v, a.n4v, nbv * BE / 4, 1.f, threadIdx.x);
   float acc[R][B] = {};
 #pragma unroll
   for (int q = 0; q < B; ++q) {
+    const int b_lo = q == 0 ? 0 : nbv, per = (nb - b_lo + a.ks - 1) / a.ks;
+    const int b0 = b_lo + kp * per, b1 = b0 + per < nb ? b0 + per : nb;
+    fetch(0, b0, b1, q);
+    fetch(1, b0 + U, b1, q);
+    if (q == 0) {
+      for (int j = 0; j < B; ++j)
+        ld_stage<T, 512>((f32x4*)(xv + (size_t)j * nbv * BE), a.v + (size_t)j * a.ld_v, a.n4v, nbv * BE / 4, 1.f, threadIdx.x);
+    } else {
+      __syncthreads();  // the feed-forward vectors of the sequence before have been consumed
+    }
     if (a.moe) {
-      if (q) __syncthreads();  // the part of the sequence before has been consumed
-      for (int b = (int)threadIdx.x - 128; b >= 0 && b < a.top * nbe; b += 384) {
-        const int k = b / nbe, bb = b - k * nbe, id = a.ids[q * a.top + k];
-        const int left = a.ffp / E - bb * 64;
-        tab[nbv + nbs + b] = LdBlk{(const T*)a.down + ((size_t)(id < 0 ? 0 : id) * a.W) * a.ffp + (size_t)bb * BE, a.ffp,
-                                   id < 0 ? 0 : (left < 64 ? left : 64)};
-      }
       if (nbs) ld_stage<T, 512>((f32x4*)xf, a.hs + (size_t)q * a.sffp, a.sffp >> 2, nbs * BE / 4, a.sh_g[q], threadIdx.x);
       for (int k = 0; k < a.top; ++k)
         ld_stage<T, 512>((f32x4*)(xf + (size_t)(nbs + k * nbe) * BE), a.he + (size_t)(q * a.top + k) * a.ffp, a.ffp >> 2,
                          nbe * BE / 4, 1.f, threadIdx.x);
     }
     __syncthreads();
-    const int b_lo = q == 0 ? 0 : nbv, n = nb - b_lo, per = (n + a.ks - 1) / a.ks;
-    const int b0 = b_lo + kp * per, b1 = b0 + per < nb ? b0 + per : nb;
-    frag w[2][R][U];
-    int nc[2][U];
-    auto fetch = [&](int set, int b) __attribute__((always_inline)) {
-#pragma unroll
-      for (int u = 0; u < U; ++u) {
-        nc[set][u] = 0;
-        if (b + u < b1) {
-          const LdBlk k = tab[b + u];
-          nc[set][u] = __builtin_amdgcn_readfirstlane(k.nch);
-          if (nc[set][u]) {
-            const int c = lane < k.nch ? lane : k.nch - 1;
-#pragma unroll
-            for (int r = 0; r < R; ++r) w[set][r][u] = ld_nt((const frag*)((const T*)k.p + (size_t)ri[r] * k.stride) + c);
-          }
-        }
-      }
-    };
     auto use = [&](int set, int b) __attribute__((always_inline)) {
 #pragma unroll
       for (int u = 0; u < U; ++u) {
@@ -772,12 +832,11 @@ __global__ __launch_bounds__(512) void k_ld_out(const LdOutArgs a) {
         }
       }
     };
-    fetch(0, b0);
     for (int b = b0; b < b1; b += 2 * U) {
-      fetch(1, b + U);
       use(0, b);
-      fetch(0, b + 2 * U);
+      fetch(0, b + 2 * U, b1, q);
       use(1, b + U);
+      fetch(1, b + 3 * U, b1, q);
     }
   }
   ld_reduce<R, B>(acc);
@@ -787,11 +846,7 @@ __global__ __launch_bounds__(512) void k_ld_out(const LdOutArgs a) {
     float v = 0.f;
     for (int k = 0; k < a.ks; ++k) v += comb[wave + k][lane];
     const int q = lane / R, i = item + (lane & (R - 1));
-    if (i < a.W) {
-      const size_t o = (size_t)q * a.ld + i;
-      if (a.moe) v = __builtin_fmaf(a.id_w[q], a.xn2[o], v);
-      a.x_out[o] = a.x_cur[o] + v;
-    }
+    if (i < a.W) a.x_out[(size_t)q * a.ld + i] = rx + __builtin_fmaf(rw, rn, v);
   }
 }
 
@@ -811,7 +866,7 @@ __global__ __launch_bounds__(256) void k_ld_head(const LdHeadArgs a) {
   constexpr int R = 4, U = 4;
   extern __shared__ __attribute__((aligned(16))) char smem_raw[];
   float* xs = (float*)smem_raw;
-  __shared__ float red[KH_WAVES_MAX];
+  __shared__ float red[2 * KH_WAVES_MAX];
   __shared__ float sv[4];
   __shared__ int si[4];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -847,7 +902,8 @@ __global__ __launch_bounds__(256) void k_ld_head(const LdHeadArgs a) {
         const int i = threadIdx.x + 256 * j;
         v[j] = i < n4 ? ((const f32x4*)(a.x + (size_t)q * a.ld))[i] : f4_zero();
       }
-      ld_norm<T, NV>(v, nw, nb, a.W, n4, xstride >> 2, a.eps, red, (f32x4*)(xs + (size_t)q * xstride), nullptr);
+      if (q) __syncthreads();
+      ld_norm<T, NV>(v, nw, nb, a.x[(size_t)q * a.ld], a.W, n4, xstride >> 2, a.eps, red, (f32x4*)(xs + (size_t)q * xstride), nullptr);
     }
   }
   __syncthreads();

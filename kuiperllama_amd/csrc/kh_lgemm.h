@@ -229,7 +229,7 @@ f32x4 y = v;
 // launches: BM = the row granule the tile list was built with (lg_group_bm).
 static inline int lg_group_bm(long rows, int groups) {
   const long per = rows / (groups > 0 ? groups : 1);
-  return per >= 96 ? 128 : (per > 24 ? 64 : 32);
+  return per > 64 ? 128 : (per > 24 ? 64 : 32);
 }
 template <class T, int EPI>
 int lg_launch(hipStream_t s, const LgArgs& a, int zdim = 1, int group_bm = 0, int max_tiles = 0) {
