@@ -799,19 +799,23 @@ def layers_tensors(cfg: dict, seed: int = 0) -> dict:
 
 
 def layers_work(cfg: dict) -> tuple:
-    """(weight elements a decoded token reads, of which the head; linear MACs of a prompt token) - algorithmic."""
+    """(weight elements a decoded token reads, of which the head; linear multiply-adds of a prompt token whose logits
+    nobody asks for: the last layer only leaves its state or cache rows) - algorithmic."""
     from kuiperllama_amd import checkpoint
-    active = 0
+    active, prompt, last = 0.0, 0.0, len(cfg["layers"]) - 1
     for k, sh in checkpoint.tensor_shapes(cfg).items():
-        if len(sh) != 2 or k in ("embed", "loop.step", "head") or k.endswith(("A_log", "conv")):
+        if len(sh) != 2 or not k.startswith("l") or k == "loop.step" or k.endswith(("A_log", "conv")):
             continue
-        n = sh[0] * sh[1]
+        layer = int(k[1:k.index(".")])
+        n = float(sh[0] * sh[1])
         if ".mlp.e" in k:
-            r = next(l for l in cfg["layers"])["mlp"]["router"]
-            n = n * r["top"] * (r["experts"] / (r["experts"] + r["identity"])) / r["experts"]
+            r = cfg["layers"][layer]["mlp"]["router"]
+            n *= r["top"] / (r["experts"] + r["identity"])
         active += n
+        if layer < last or k.endswith((".mix.in", ".mix.x", ".mix.dt", ".mix.dq", ".mix.dkv")):
+            prompt += n
     head = cfg["vocab"] * cfg["width"]
-    return active + head, head, active
+    return active + head, head, prompt
 
 
 def layers_bench(args) -> None:
@@ -822,13 +826,13 @@ def layers_bench(args) -> None:
     rng = np.random.default_rng(1)
     for width, n_layers in [(int(a), int(b)) for a, b in (x.split("x") for x in args.layers.split(","))]:
         cfg = layers_config(width, n_layers)
-        elems, head, macs = layers_work(cfg)
+        elems, head, prompt_macs = layers_work(cfg)
         t0 = time.time()
         img = checkpoint.safetensors_image(layers_tensors(cfg))
         m = KuiperModel.from_tensors(cfg, img, max_seq_len=4352)
         del img
         log(f"[bench] {width} x {n_layers}: built in {time.time() - t0:.1f} s, {m.cfg.weight_bytes / 1e9:.2f} GB")
-        hidden = int((macs / n_layers - 4 * width * width) / (3 * width)) // 64 * 64
+        hidden = int(((elems - head) / n_layers - 4 * width * width) / (3 * width)) // 64 * 64
         sp = binfmt.ModelSpec(width, hidden, n_layers, width // 128, width // 128, cfg["vocab"], 4352, False,
                               name=f"llama-{width}x{n_layers}")
         for name, mk, wbytes, peak in (("gufanex", lambda: m, 2.0, 2.5e15),
@@ -846,7 +850,9 @@ def layers_bench(args) -> None:
             for T in (512, 2048, 4096):
                 mm.time_prefill(prompt[:T], 0, mode="gemm")
                 ms = min(mm.time_prefill(prompt[:T], 0, mode="gemm") for _ in range(3))
-                fl = 2.0 * (macs if name == "gufanex" else sp.weight_elems() - cfg["vocab"] * width) * T
+                # both families leave the last layer's output projections and feed-forward out of a prompt pass
+                fl = 2.0 * T * (prompt_macs if name == "gufanex" else
+                                (n_layers - 1) * (4 * width * width + 3 * width * hidden) + 3 * width * width)
                 row[f"prefill{T}_tok_s"] = round(T / ms * 1e3)
                 row[f"prefill{T}_linear_frac_of_peak"] = round(fl / (ms * 1e-3) / peak, 3)
             mm.close()

@@ -95,11 +95,11 @@ def test_trace_runner_asks_for_its_arguments(capsys):
 def test_layers_bench_configuration_counts_its_weights():
     import bench
     cfg = bench.layers_config(512, 2)
-    elems, head, linear = bench.layers_work(cfg)
-    assert elems == linear + head and head == 512 * cfg["vocab"]
+    elems, head, prompt = bench.layers_work(cfg)
+    assert head == 512 * cfg["vocab"]
     m, a = cfg["layers"][0]["mixer"], cfg["layers"][1]["mixer"]
     mam = 512 * 2 * m["inner"] + (m["dt_rank"] + 32) * m["inner"] + m["inner"] * m["dt_rank"] + 512 * m["inner"]
-    H = a["heads"]
-    lat = 512 * (1536 + 512 + 64) + 1536 * H * 192 + 512 * H * 256 + 512 * H * 128
+    H, down = a["heads"], 512 * (1536 + 512 + 64)
+    lat = down + 1536 * H * 192 + 512 * H * 256 + 512 * H * 128
     ff = 36 * 512 + 512 + 3 * 512 * 512 + 6 * (32 / 36) * 3 * 512 * 256
-    assert abs(linear - (mam + lat + 2 * ff)) < 1
+    assert abs(elems - head - (mam + lat + 2 * ff)) < 1 and abs(prompt - (mam + ff + down)) < 1
