@@ -237,15 +237,17 @@ def ref_cpu_flavor(spec) -> str | None:
 
 
 def kernel_sources_sha1() -> str:
-    """sha1 over the device-code headers of the decode / prefill kernels (csrc/kh_*.h except the host-only
-    kh_model_internal.h), in name order.  profiles/pmc_traffic.json is stamped with it when the PMC passes are
+    """sha1 over the device-code headers of the .bin families' decode / prefill kernels (csrc/kh_*.h except the
+    host-only ones and the layer-list models' own), in name order.  profiles/pmc_traffic.json is stamped with it when the PMC passes are
     collected; bench.py recomputes it, so a kernel change after the collection shows in the record
     (roofline.traffic_source.kernel_sources_unchanged) instead of silently keeping a stale traffic ratio."""
     import hashlib
+    other = ("kh_model_internal.h", "kh_json.h", "kh_hybrid.h", "kh_tile.h", "kh_lgemm.h", "kh_lops.h", "kh_scan.h",
+             "kh_moe.h", "kh_latent.h", "kh_expanded.h", "kh_ldecode.h")
     h = hashlib.sha1()
     d = os.path.join(os.path.dirname(os.path.abspath(__file__)), "csrc")
     for f in sorted(os.listdir(d)):
-        if f.startswith("kh_") and f.endswith(".h") and f != "kh_model_internal.h":
+        if f.startswith("kh_") and f.endswith(".h") and f not in other:
             h.update(f.encode())
             h.update(open(os.path.join(d, f), "rb").read())
     return h.hexdigest()

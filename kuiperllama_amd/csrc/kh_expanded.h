@@ -126,23 +126,31 @@ __global__ __launch_bounds__(256) void k_expanded_attn(const ExpArgs a) {
     const char* Kt = smem_raw + slot * stage;
     const char* Rt = Kt + bytes_k;
     const char* Vt = Rt + bytes_r;
-    f32x4 s[MR][NS];
-#pragma unroll
-    for (int q = 0; q < MR; ++q)
-#pragma unroll
-      for (int n = 0; n < NS; ++n) s[q][n] = f32x4{0.f, 0.f, 0.f, 0.f};
+    // keys, then values, are requested from LDS together: the values arrive under the scores and the softmax
+    frag fk[NQ][NS], fv[NV];
 #pragma unroll
     for (int b = 0; b < NQ; ++b) {
       const int c = 4 * b + fh;
 #pragma unroll
       for (int n = 0; n < NS; ++n) {
         const int k = NS == 2 ? 8 * (fr >> 2) + 4 * n + (fr & 3) : fr;
-        const char* src = 4 * b < qc ? Kt + ((size_t)k * qc + (c ^ swz(k))) * 16 : Rt + ((size_t)k * rc + ((c - qc) ^ swz(k))) * 16;
-        const frag fk = *(const frag*)src;
-#pragma unroll
-        for (int q = 0; q < MR; ++q) s[q][n] = TL::mma(fk, fq[q][b], s[q][n]);
+        fk[b][n] = *(const frag*)(4 * b < qc ? Kt + ((size_t)k * qc + (c ^ swz(k))) * 16 : Rt + ((size_t)k * rc + ((c - qc) ^ swz(k))) * 16);
       }
     }
+#pragma unroll
+    for (int n = 0; n < NV; ++n) fv[n] = *(const frag*)(Vt + (size_t)(n * 16 + fr) * 64 + (fh << 4));
+    __builtin_amdgcn_sched_barrier(0);
+    f32x4 s[MR][NS];
+#pragma unroll
+    for (int q = 0; q < MR; ++q)
+#pragma unroll
+      for (int n = 0; n < NS; ++n) s[q][n] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int b = 0; b < NQ; ++b)
+#pragma unroll
+      for (int n = 0; n < NS; ++n)
+#pragma unroll
+        for (int q = 0; q < MR; ++q) s[q][n] = TL::mma(fk[b][n], fq[q][b], s[q][n]);
     frag p[MR];
     float f[MR];
     const bool edge = k0 + KT - 1 > a.pos0 + q0 + wave * MR * 16;  // the tile crosses the diagonal of some row
@@ -178,12 +186,11 @@ __global__ __launch_bounds__(256) void k_expanded_attn(const ExpArgs a) {
     }
 #pragma unroll
     for (int n = 0; n < NV; ++n) {
-      const frag fv = *(const frag*)(Vt + (size_t)(n * 16 + fr) * 64 + (fh << 4));
 #pragma unroll
       for (int q = 0; q < MR; ++q) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) o[q][n][i] *= f[q];
-        o[q][n] = TL::mma(fv, p[q], o[q][n]);
+        o[q][n] = TL::mma(fv[n], p[q], o[q][n]);
       }
     }
   }

@@ -4,7 +4,7 @@
 //   * One workgroup = 4 waves (2 x 2) = a BM-token x BN-feature tile; K advances 128 bytes per stage through a ring
 //     of NSTAGE LDS stages filled by the LDS-DMA path (global_load_lds_dwordx4): no staging registers, and
 //     NSTAGE - 1 stages are in flight while one is multiplied.  The big tiles use two stages, which leaves room for
-//     two workgroups per CU: one multiplies while the other waits (128 x 128: 0.40 - 0.46 of the bf16 peak, against
+//     two workgroups per CU: one multiplies while the other waits (128 x 128: 0.43 - 0.50 of the bf16 peak, against
 //     0.28 - 0.33 with three stages and one workgroup).
 //   * LDS rows are 128 bytes.  Chunk c (16 bytes) of row r sits in slot c ^ (r & 7): the lanes of a fragment read
 //     (16 rows, same chunk) touch all 64 banks.  The DMA writes slots in lane order, so the permutation is applied
@@ -142,24 +142,29 @@ __global__ __launch_bounds__(256) void k_lgemm(const LgArgs a) {
     __syncthreads();
     if (k + NST - 1 < nk) issue(fill);
     const char* st = smem_raw + slot * STAGE;
+    // both halves of the stage are requested from LDS before the first product: the second half arrives under the
+    // products of the first (left to itself the compiler reads one half at a time; 0.40 -> 0.43 ... 0.50 of the peak)
+    frag fx[2][TM], fw[2][TN];
 #pragma unroll
     for (int b = 0; b < 2; ++b) {
-      frag fx[TM], fw[TN];
 #pragma unroll
       for (int m = 0; m < TM; ++m) {
         const int r = wm * (BM / 2) + m * 16 + fr;
-        fx[m] = *(const frag*)(st + r * 128 + (((4 * b + fh) ^ (r & 7)) << 4));
+        fx[b][m] = *(const frag*)(st + r * 128 + (((4 * b + fh) ^ (r & 7)) << 4));
       }
 #pragma unroll
       for (int n = 0; n < TN; ++n) {
         const int r = BM + wn * (BN / 2) + n * 16 + fr;
-        fw[n] = *(const frag*)(st + r * 128 + (((4 * b + fh) ^ (r & 7)) << 4));
+        fw[b][n] = *(const frag*)(st + r * 128 + (((4 * b + fh) ^ (r & 7)) << 4));
       }
+    }
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
 #pragma unroll
       for (int n = 0; n < TN; ++n)
 #pragma unroll
-        for (int m = 0; m < TM; ++m) acc[n][m] = TL::mma(fw[n], fx[m], acc[n][m]);
-    }
+        for (int m = 0; m < TM; ++m) acc[n][m] = TL::mma(fw[b][n], fx[b][m], acc[n][m]);
     slot = slot + 1 == NST ? 0 : slot + 1;
     fill = fill + 1 == NST ? 0 : fill + 1;
   }
