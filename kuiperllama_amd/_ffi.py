@@ -206,7 +206,7 @@ def debug_get(key: str) -> Optional[str]:
     return None if v is None else v.decode()
 
 
-_HOOK_PREFIXES = ("KH_SHAPE_", "KH_ATTN_", "KH_PG_", "KH_PREFILL", "KH_RING", "KH_SELFTEST", "KH_KV_")
+_HOOK_PREFIXES = ("KH_SHAPE_", "KH_ATTN_", "KH_PG_", "KH_PREFILL", "KH_RING", "KH_SELFTEST", "KH_KV_", "KH_HY_")
 _ENV_MIRRORED = {}  # hook -> value, as last written into the table FROM os.environ by sync_env()
 _ENV_SEEDED = False
 

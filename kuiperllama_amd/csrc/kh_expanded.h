@@ -27,7 +27,7 @@ struct ExpArgs {
   void* out;           // T [T][H dvp]
   int H, dnp, drp, dvp, row, ldv;
   int row0, n, pos0;   // the segment's rows in Q / out, their number, position of the first
-  float scale2;
+  float scale2;        // > 0
 };
 
 // KN, KR, KV: unrotated key part, rotated part and value size in units of 64 (compile-time: see kh_latent.h)
@@ -152,47 +152,52 @@ __global__ __launch_bounds__(256) void k_expanded_attn(const ExpArgs a) {
 #pragma unroll
         for (int q = 0; q < MR; ++q) s[q][n] = TL::mma(fk[b][n], fq[q][b], s[q][n]);
     frag p[MR];
-    float f[MR];
     const bool edge = k0 + KT - 1 > a.pos0 + q0 + wave * MR * 16;  // the tile crosses the diagonal of some row
 #pragma unroll
     for (int q = 0; q < MR; ++q) {
-      float mx = m[q];
+      if (edge) {
+#pragma unroll
+        for (int n = 0; n < NS; ++n)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int k = k0 + (NS == 2 ? 8 * fh + 4 * n + i : 4 * fh + i);
+            s[q][n][i] = k <= my_pos[q] ? s[q][n][i] : -INFINITY;
+          }
+      }
+      float mx = s[q][0][0];
 #pragma unroll
       for (int n = 0; n < NS; ++n)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          float v = s[q][n][i] * a.scale2;
-          if (edge) {
-            const int k = k0 + (NS == 2 ? 8 * fh + 4 * n + i : 4 * fh + i);
-            v = k <= my_pos[q] ? v : -INFINITY;
-          }
-          s[q][n][i] = v;
-          mx = fmaxf(mx, v);
-        }
-      mx = xor16_max(mx);
-      mx = xor32_max(mx);  // finite: the sink
-      f[q] = __builtin_amdgcn_exp2f(m[q] - mx);
-      m[q] = mx;
+        for (int i = 0; i < 4; ++i) mx = fmaxf(mx, s[q][n][i]);
+      mx *= a.scale2;
+      // the running maximum (at least the sink) rarely moves after the first tiles: rescale only when some row's does
+      if (__any(mx > m[q])) {
+        mx = fmaxf(mx, m[q]);
+        mx = xor16_max(mx);
+        mx = xor32_max(mx);
+        const float f = __builtin_amdgcn_exp2f(m[q] - mx);
+        m[q] = mx;
+        l[q] *= f;
+#pragma unroll
+        for (int n = 0; n < NV; ++n)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) o[q][n][i] *= f;
+      }
       float sum = 0.f;
 #pragma unroll
       for (int n = 0; n < NS; ++n)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const float e = __builtin_amdgcn_exp2f(s[q][n][i] - mx);
+          const float e = __builtin_amdgcn_exp2f(__builtin_fmaf(s[q][n][i], a.scale2, -m[q]));
           sum += e;
           p[q][4 * n + i] = (T)e;
         }
-      l[q] = __builtin_fmaf(l[q], f[q], sum);
+      l[q] += sum;
     }
 #pragma unroll
-    for (int n = 0; n < NV; ++n) {
+    for (int n = 0; n < NV; ++n)
 #pragma unroll
-      for (int q = 0; q < MR; ++q) {
-#pragma unroll
-        for (int i = 0; i < 4; ++i) o[q][n][i] *= f[q];
-        o[q][n] = TL::mma(fv[n], p[q], o[q][n]);
-      }
-    }
+      for (int q = 0; q < MR; ++q) o[q][n] = TL::mma(fv[n], p[q], o[q][n]);
   }
 #pragma unroll
   for (int q = 0; q < MR; ++q) {

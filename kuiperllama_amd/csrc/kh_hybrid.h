@@ -109,7 +109,7 @@ struct Hybrid {
   int tmax = 0;
   float *x = nullptr, *x0 = nullptr, *mix = nullptr, *f32a = nullptr, *y = nullptr, *sh = nullptr, *dt = nullptr,
         *bc = nullptr, *z = nullptr, *ends = nullptr, *dtsum = nullptr, *moe_w = nullptr, *id_w = nullptr,
-        *sh_g = nullptr, *part = nullptr, *wlogits = nullptr;
+        *sh_g = nullptr, *wlogits = nullptr;
   void *xn1 = nullptr, *xn2 = nullptr, *a0 = nullptr, *a1 = nullptr, *a2 = nullptr, *h = nullptr, *hs = nullptr,
        *xw = nullptr;
   // expanded latent attention: keys [exp_keys][H dnp] and transposed values [H dvp][exp_keys] of one segment
@@ -153,13 +153,8 @@ int hy_create_from_folder(const char* path, const kh_model_opts* o, kh_model** o
 int hy_forward(kh_model* m, const HyEntry* e, int n, const int32_t* want, int n_want, float* h_logits);
 // one token at (d_token, d_pos) of slot 0 on the pass kernels, logits to m->logits (the unfused step)
 int hy_unfused_step(kh_model* m);
-// query-row tile lists of latent attention: the kinds (heads, latents of more than 256) a model has, and the list for
-// segments of the given lengths
-typedef std::pair<int, int> LatKind;
-std::vector<LatKind> hy_lat_kinds(const Hybrid& hy);
-void hy_lat_tiles(const std::vector<int32_t>& seg_n, LatKind kind, int* cp, std::vector<int32_t>* tab);
 // argmax of m->logits as one sampler partial
-int kh_argmax_partial(kh_model* m);
+int hy_argmax_partial(kh_model* m);
 // ---- kh_hybrid_step.hip
 int hy_step_init(kh_model* m);
 void hy_launch_step(kh_model* m, int advance, int n_forced);

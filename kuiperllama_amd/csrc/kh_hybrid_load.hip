@@ -433,7 +433,6 @@ int alloc_workspace(kh_model* m) {
   hy.tmax = KH_HY_TMAX;
   size_t f32a = 1, a0 = 1, a1 = 1, a2 = 1, dt = 1, bc = 1, z = 1, ends = 1, dtsum = 1, h = 1, hs = 1, y = 1, top = 1, tiles = 1;
   auto up = [](size_t& v, size_t n) { v = v > n ? v : n; };
-  const size_t chunks = T / KH_SCAN_CH + T;  // every segment of a pass can end in a partial chunk
   const size_t multi = T / KH_SCAN_CH * 2 + 2;  // chunks of segments that have more than one
   for (auto& l : hy.layers) {
     if (l.mixer == HY_MAMBA1) {
@@ -467,7 +466,6 @@ int alloc_workspace(kh_model* m) {
       up(tiles, T * (size_t)f.top / 32 + (size_t)f.E + 1);
     }
   }
-  (void)chunks;
   int rc;
   auto zf = [&](float** p, size_t n) -> int {
     if ((rc = dalloc(p, n)) != KH_OK) return rc;
@@ -677,7 +675,7 @@ void hy_destroy(kh_model* m) {
   Hybrid* h = m->hy;
   if (!h) return;
   void* dev[] = {h->farena, h->state, h->x, h->x0, h->mix, h->f32a, h->y, h->sh, h->dt, h->bc, h->z, h->ends, h->dtsum,
-                 h->moe_w, h->id_w, h->sh_g, h->part, h->wlogits, h->xn1, h->xn2, h->a0, h->a1, h->a2, h->h, h->hs, h->xw,
+                 h->moe_w, h->id_w, h->sh_g, h->wlogits, h->xn1, h->xn2, h->a0, h->a1, h->a2, h->h, h->hs, h->xw,
                  h->moe_id, h->moe_rows, h->moe_slot, h->n_tiles, h->tiles, h->kx, h->vx, h->d_tab, h->d_one};
   for (void* p : dev)
     if (p) (void)hipFree(p);

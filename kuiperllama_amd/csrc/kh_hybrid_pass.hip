@@ -50,7 +50,33 @@ struct TabBuilder {
   int put(const std::vector<int32_t>& x) { return put(x.data(), x.size()); }
 };
 
+// query-row tile lists of latent attention a pass needs: one per (heads, latent of more than 256)
+typedef std::pair<int, int> LatKind;
 LatKind lat_kind(const HyLatent& la) { return {la.H, la.Rp > 256}; }
+std::vector<LatKind> lat_kinds(const Hybrid& hy) {
+  std::vector<LatKind> r;
+  for (auto& l : hy.layers)
+    if (l.mixer == HY_LATENT && std::find(r.begin(), r.end(), lat_kind(l.la)) == r.end()) r.push_back(lat_kind(l.la));
+  return r;
+}
+// 64 rows per tile (32 for big latents, whose accumulators would not fit), or 16 where the rows of the segments would
+// leave most of those empty
+void lat_tiles(const std::vector<int32_t>& seg_n, LatKind kind, int* cp, std::vector<int32_t>* tab) {
+  const int H = kind.first;
+  long rows = 0, t64 = 0;
+  for (int n : seg_n) {
+    rows += (long)n * H;
+    t64 += ((long)n * H + 63) / 64;
+  }
+  *cp = t64 * 64 > 2 * rows ? 4 : (kind.second ? 2 : 1);
+  const int step = 64 / *cp;
+  tab->clear();
+  for (size_t s = 0; s < seg_n.size(); ++s)
+    for (int r = (seg_n[s] * H - 1) / step * step; r >= 0; r -= step) {  // the longest key ranges first
+      tab->push_back((int)s);
+      tab->push_back(r);
+    }
+}
 
 // ---- the pass ----------------------------------------------------------------------------------------------------
 template <class T>
@@ -212,7 +238,7 @@ struct Runner {
     hipLaunchKernelGGL(k_latent_prep<T>, dim3(ps.T), dim3(256), 0, s, lp);
     if (state_only) return KH_OK;
     TRY((lg_launch<T, LG_T>(s, gemm(la.uq, hy.a0, la.qrp, hy.a1, H * qh))));
-    if (ps.expand && exp_supported(la.dnp, la.drp, la.dvp)) {
+    if (ps.expand && la.scale > 0.f && exp_supported(la.dnp, la.drp, la.dvp)) {
       if (la.dims)
         hipLaunchKernelGGL(k_rope_inplace<T>, dim3(ps.T), dim3(256), 0, s, (T*)hy.a1, la.rope, H, la.dnp, la.drp, la.dims, ps.p);
       for (const PassSeg& sg : ps.segs) TRY(expanded(r, la, sg));
@@ -353,37 +379,13 @@ int run_pass(kh_model* m, const Pass& ps, float* h_logits) {
 
 namespace khm {
 
-std::vector<LatKind> hy_lat_kinds(const Hybrid& hy) {
-  std::vector<LatKind> r;
-  for (auto& l : hy.layers)
-    if (l.mixer == HY_LATENT && std::find(r.begin(), r.end(), lat_kind(l.la)) == r.end()) r.push_back(lat_kind(l.la));
-  return r;
-}
-// 64 rows per tile (32 for big latents, whose accumulators would not fit), or 16 where the rows of the segments would
-// leave most of those empty
-void hy_lat_tiles(const std::vector<int32_t>& seg_n, LatKind kind, int* cp, std::vector<int32_t>* tab) {
-  const int H = kind.first;
-  long rows = 0, t64 = 0;
-  for (int n : seg_n) {
-    rows += (long)n * H;
-    t64 += ((long)n * H + 63) / 64;
-  }
-  *cp = t64 * 64 > 2 * rows ? 4 : (kind.second ? 2 : 1);
-  const int step = 64 / *cp;
-  tab->clear();
-  for (size_t s = 0; s < seg_n.size(); ++s)
-    for (int r = (seg_n[s] * H - 1) / step * step; r >= 0; r -= step) {  // the longest key ranges first
-      tab->push_back((int)s);
-      tab->push_back(r);
-    }
-}
 static __global__ void k_one_partial(const int32_t* idx, float* val, int32_t* out, int n) {
   for (int i = threadIdx.x; i < n; i += 64) {
     val[i] = i ? -INFINITY : 0.f;
     out[i] = *idx;
   }
 }
-int kh_argmax_partial(kh_model* m) {
+int hy_argmax_partial(kh_model* m) {
   TRY(kh_argmax_f32(m->logits, m->cfg.vocab_size, m->d_next, (void*)m->stream));
   hipLaunchKernelGGL(k_one_partial, dim3(1), dim3(64), 0, m->stream, (const int32_t*)m->d_next, m->part_val, m->part_idx, m->nparts);
   return kh_launch_status();
@@ -393,7 +395,7 @@ int hy_forward(kh_model* m, const HyEntry* e, int n, const int32_t* want, int n_
   Hybrid& hy = *m->hy;
   KH_CHECK_HIP(hipSetDevice(m->opts.device));
   KH_CHECK_HIP(hipStreamSynchronize(m->stream));  // the pinned tables of the call before are free again
-  const std::vector<LatKind> kinds = hy_lat_kinds(hy);
+  const std::vector<LatKind> kinds = lat_kinds(hy);
   // ---- cut the concatenated tokens into passes and build every pass's tables
   std::vector<Pass> passes;
   std::vector<int32_t> all;
@@ -468,7 +470,7 @@ int hy_forward(kh_model* m, const HyEntry* e, int n, const int32_t* want, int n_
     o.want = tb.put(wr);
     for (const LatKind& kd : kinds) {
       LatTiles t{kd.first, kd.second, 0, 0, 0};
-      hy_lat_tiles(sn, kd, &t.cp, &lt);
+      lat_tiles(sn, kd, &t.cp, &lt);
       t.n = (int)lt.size() / 2;
       t.off = tb.put(lt);
       p.lat.push_back(t);
@@ -523,9 +525,9 @@ int hy_unfused_step(kh_model* m) {
   Hybrid& hy = *m->hy;
   Pass p;
   std::vector<int32_t> tab{0, 0, 0, 0, 0, 1, 0, 0, 0, 0, 1, 3, 0, 0, 0, 0}, lt;
-  for (const LatKind& kd : hy_lat_kinds(hy)) {
+  for (const LatKind& kd : lat_kinds(hy)) {
     LatTiles t{kd.first, kd.second, 0, 0, 0};
-    hy_lat_tiles({1}, kd, &t.cp, &lt);
+    lat_tiles({1}, kd, &t.cp, &lt);
     t.n = (int)lt.size() / 2;
     t.off = (int)tab.size();
     tab.insert(tab.end(), lt.begin(), lt.end());

@@ -392,7 +392,7 @@ void hy_launch_step(kh_model* m, int advance, int n_forced) {
     (void)step_any(m, 1, tb, m->logits);
   } else {  // the pass kernels leave logits; the sampler wants partials
     (void)hy_unfused_step(m);
-    (void)kh_argmax_partial(m);
+    (void)hy_argmax_partial(m);
   }
   launch_sample(m, advance, n_forced);
 }

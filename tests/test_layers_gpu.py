@@ -335,6 +335,18 @@ def test_greedy_generation(gpu, mixed, n_prompt):
     m.close()
 
 
+def test_geometry_beyond_the_fused_step(gpu):
+    """A mixer vector that does not fit LDS: decoding and generation run on the pass kernels."""
+    mod = U.Model(U.config([U.mamba(40000, 2, 2, 4), U.with_ff(U.latent())], width=16, vocab=30))
+    toks = mod.tokens(9)
+    m = mod.load()
+    U.check(U.run_alone(m, toks, (4, 5, 6, 7, 8)), mod.logits(toks), "float32")
+    want = toks[1:3] + mod.greedy(toks[:3], 6)
+    for ex in ("graph", "fused", "unfused", "graph"):
+        assert m.generate(toks[:3], 8, exec=ex)[0] == want, ex
+    m.close()
+
+
 def test_greedy_batch(gpu, mixed):
     ps = [mixed.tokens(n, seed=30 + n) for n in (3, 17, 1, 8, 33)]
     want = [mixed.greedy(p, 9 + i) for i, p in enumerate(ps)]
