@@ -16,10 +16,10 @@ CSRC = os.path.join(_PKG, "csrc")
 LIB_DIR = os.path.join(_PKG, "lib")
 LIB_PATH = os.path.join(LIB_DIR, "libkuiper_hip.so")
 SOURCES = ["kh_ops.hip", "kh_model_load.hip", "kh_model_step.hip", "kh_model_prefill.hip", "kh_model_profile.hip", "kh_model_selftest.hip",
-           "kh_hybrid_load.hip", "kh_hybrid_pass.hip", "kh_hybrid_step.hip",
+           "kh_hybrid_load.hip", "kh_hybrid_pass.hip", "kh_hybrid_step.hip", "kh_heads.hip",
            "kh_tokenizer.cpp", "kh_bpe.cpp", "kh_debug.cpp"]
 HEADERS = ["kh_common.h", "kh_gemv.h", "kh_attn.h", "kh_fused.h", "kh_q8ring.h", "kh_fused_ring.h", "kh_prefill.h", "kh_gemm.h", "kh_pattn.h", "kh_unicode_tables.h", "kh_json.h",
-           "kh_tile.h", "kh_lgemm.h", "kh_lops.h", "kh_scan.h", "kh_moe.h", "kh_latent.h", "kh_expanded.h", "kh_hybrid.h", "kh_ldecode.h",
+           "kh_tile.h", "kh_lgemm.h", "kh_lops.h", "kh_scan.h", "kh_moe.h", "kh_latent.h", "kh_expanded.h", "kh_heads.h", "kh_hybrid.h", "kh_ldecode.h",
            "kh_model_internal.h",
            "../../include/kuiper_hip.h"]
 ARCH = "gfx950"
@@ -243,7 +243,7 @@ def kernel_sources_sha1() -> str:
     (roofline.traffic_source.kernel_sources_unchanged) instead of silently keeping a stale traffic ratio."""
     import hashlib
     other = ("kh_model_internal.h", "kh_json.h", "kh_hybrid.h", "kh_tile.h", "kh_lgemm.h", "kh_lops.h", "kh_scan.h",
-             "kh_moe.h", "kh_latent.h", "kh_expanded.h", "kh_ldecode.h")
+             "kh_moe.h", "kh_latent.h", "kh_expanded.h", "kh_heads.h", "kh_ldecode.h")
     h = hashlib.sha1()
     d = os.path.join(os.path.dirname(os.path.abspath(__file__)), "csrc")
     for f in sorted(os.listdir(d)):

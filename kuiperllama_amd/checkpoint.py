@@ -11,7 +11,10 @@ from typing import Dict, Iterator, Optional, Sequence, Tuple
 
 import numpy as np
 
-ARCHITECTURES = ("Gufanex",)
+ARCHITECTURES = ("Gufanex", "Gusorax")
+
+
+DISTANCE_ROWS = 32  # rows of a distance table that a configuration does not size (the loader reads them off the tensor)
 
 
 def load_config(folder: str) -> dict:
@@ -34,6 +37,18 @@ def _mixer_tensors(p: str, kind: str, m: dict, W: int) -> Iterator[Tuple[str, tu
         yield from ((p + ".dq", (q, W)), (p + ".dq.norm", (q,)), (p + ".uq", (H * (dn + dr), q)),
                     (p + ".dkv", (R + dr, W)), (p + ".dkv.norm", (R,)), (p + ".uk", (H * dn, R)),
                     (p + ".uv", (H * dv, R)), (p + ".sink", (H,)), (p + ".o", (W, H * dv)))
+    elif kind in ("attention", "attention_2"):
+        H, G, dk, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        biased = kind == "attention_2"
+        for n, rows in (("q", H * dk), ("k", G * dk), ("v", G * dv)):
+            yield f"{p}.{n}", (rows, W)
+            if biased:
+                yield f"{p}.{n}.b", (rows,)
+        yield from ((p + ".q.norm", (dk,)), (p + ".k.norm", (dk,)))
+        yield (p + ".g", (H * dv, W)) if biased else (p + ".rel", (m.get("rel_rows", DISTANCE_ROWS), H))
+        yield p + ".o", (W, H * dv)
+        if biased:
+            yield p + ".o.b", (W,)
     else:
         raise ValueError(f"unknown mixer {kind!r}")
 
@@ -42,12 +57,17 @@ def _gated(p: str, ff: int, W: int) -> Iterator[Tuple[str, tuple]]:
     yield from ((p + ".gate", (ff, W)), (p + ".up", (ff, W)), (p + ".down", (W, ff)))
 
 
-def _moe_tensors(p: str, m: dict, W: int) -> Iterator[Tuple[str, tuple]]:
+def _moe_tensors(p: str, m: dict, W: int, correction: bool = True) -> Iterator[Tuple[str, tuple]]:
+    if m["kind"] == "dense":
+        yield from _gated(p, m["ff"], W)
+        return
     r = m["router"]
     n_out = r["experts"] + r.get("identity", 0)
     for e in range(r["experts"]):
         yield from _gated(f"{p}.e{e}", m["expert"]["ff"], W)
-    yield from ((p + ".router", (n_out, W)), (p + ".correction", (n_out,)))
+    yield p + ".router", (n_out, W)
+    if correction:
+        yield p + ".correction", (n_out,)
     if m.get("shared"):
         yield from _gated(p + ".shared", m["shared"]["ff"], W)
         yield p + ".shared.sg", (1, W)
@@ -58,17 +78,27 @@ def tensor_shapes(cfg: dict) -> Dict[str, tuple]:
     if cfg.get("architecture") not in ARCHITECTURES:
         raise ValueError(f"unknown architecture {cfg.get('architecture')!r}")
     W, V = cfg["width"], cfg["vocab"]
+    gufanex = cfg["architecture"] == "Gufanex"  # else: one RMS norm per layer, positions, a matrix into the loop
     out: Dict[str, tuple] = {"embed": (V, W)}
+    if not gufanex:
+        out["pos"] = (cfg["max_positions"], W)
     if cfg.get("loop"):
-        out["loop.step"] = (cfg["loop"]["times"], W)
+        out.update({"loop.step": (cfg["loop"]["times"], W)} if gufanex else {"loop.in": (W, 2 * W)})
+
+    def norm(name):
+        out[name] = (W,)
+        if gufanex:
+            out[name + ".b"] = (W,)
+
     for i, l in enumerate(cfg["layers"]):
         p = f"l{i}"
-        for n in (".norm1", ".norm2") if l.get("mlp") else (".norm1",):
-            out[p + n] = out[p + n + ".b"] = (W,)
+        norm(p + ".norm1")
+        if l.get("mlp") and gufanex:
+            norm(p + ".norm2")
         out.update(_mixer_tensors(p + ".mix", l["type"], l["mixer"], W))
         if l.get("mlp"):
-            out.update(_moe_tensors(p + ".mlp", l["mlp"], W))
-    out["final.norm"] = out["final.norm.b"] = (W,)
+            out.update(_moe_tensors(p + ".mlp", l["mlp"], W, gufanex))
+    norm("final.norm")
     out["head"] = (V, W)
     return out
 
@@ -112,14 +142,22 @@ def save(folder: str, cfg: dict, tensors: Dict[str, np.ndarray]) -> None:
 
 def random_tensors(cfg: dict, seed: int = 0, only: Optional[Sequence[str]] = None) -> Dict[str, np.ndarray]:
     """Seeded random weights (bf16 bits) whose activations stay of order one: linear weights N(0, 1 / fan_in), norm
-    weights around 1, A_log = log(1 .. state), dt biases that make softplus small."""
+    weights around 1 (around 0 where the norm adds one), A_log = log(1 .. state), dt biases that make softplus small,
+    embeddings that the configuration's scale brings to order one."""
+    one_plus = cfg["architecture"] != "Gufanex"
     rng = np.random.default_rng(seed)
     out: Dict[str, np.ndarray] = {}
     for k, s in tensor_shapes(cfg).items():
         if only is not None and k not in only:
             continue
         last = k.rsplit(".", 1)[-1]
-        if k.endswith("norm") or last in ("norm1", "norm2", "D"):
+        if one_plus and (last == "norm1" or k == "final.norm"):
+            v = 0.1 * rng.standard_normal(s, np.float32)
+        elif k == "pos":
+            v = 0.3 * rng.standard_normal(s, np.float32)
+        elif k.endswith(".rel"):
+            v = rng.standard_normal(s, np.float32)
+        elif k.endswith("norm") or last in ("norm1", "norm2", "D"):
             v = 1.0 + 0.1 * rng.standard_normal(s, np.float32)
         elif k.endswith("A_log"):
             v = np.log(np.arange(1, s[1] + 1, dtype=np.float32))[None, :] + 0.1 * rng.standard_normal(s, np.float32)
@@ -132,7 +170,7 @@ def random_tensors(cfg: dict, seed: int = 0, only: Optional[Sequence[str]] = Non
         elif len(s) == 1 or k == "loop.step":
             v = 0.1 * rng.standard_normal(s, np.float32)
         elif k == "embed":
-            v = rng.standard_normal(s, np.float32)
+            v = rng.standard_normal(s, np.float32) / float(cfg.get("embedding", {}).get("scale", 1.0))
         else:
             v = rng.standard_normal(s, np.float32) * (1.0 / np.sqrt(s[-1]))
         out[k] = to_bf16(v)

@@ -10,6 +10,7 @@
 #include <string>
 #include <vector>
 
+#include "kh_heads.h"
 #include "kh_json.h"
 #include "kh_latent.h"
 #include "kh_lgemm.h"
@@ -30,10 +31,11 @@ struct HyMat {
 };
 struct HyVec {  // fp32 parameters
   size_t off = 0;
-  const float* p = nullptr;
+  const float* p = nullptr;  // nullptr: the model has none
+  bool on = false;
 };
 
-enum HyMixer { HY_MAMBA1 = 0, HY_LATENT = 1 };
+enum HyMixer { HY_MAMBA1 = 0, HY_LATENT = 1, HY_HEADS = 2 };
 
 struct HyMamba {
   int inner = 0, state = 0, rank = 0, taps = 0;
@@ -56,9 +58,29 @@ struct HyLatent {
   const float2* rope = nullptr;
   int row() const { return Rp + drp; }
 };
+struct HyHeads {  // attention over cached keys and values, grouped heads
+  int H = 0, G = 0, dk = 0, dv = 0;
+  int dkr = 0, dvr = 0;  // rows of a projected head (multiples of 16)
+  int dkp = 0, dvp = 0;  // elements of a cached head (multiples of 64)
+  float scale = 1.f;
+  KeySpan span{0, 0};
+  int nbias = 0, ring = 0, nsplit = 1;
+  bool gate = false, sink = false;
+  HyMat qkvg;  // query heads, key heads, value heads, gate rows
+  HyMat o;     // columns head by head, dvr each
+  HyVec qkvg_b, o_b, qn, kn, bias;
+  int row() const { return G * (dkp + dvp); }
+  int k_off() const { return H * dkr; }
+  int v_off() const { return k_off() + G * dkr; }
+  int g_off() const { return v_off() + G * dvr; }
+  HeadRow head_row(float eps) const { return {kn.p, G, dk, dv, dkr, dvr, dkp, dvp, k_off(), v_off(), ring, eps}; }
+};
+// Feed-forward: routed experts and / or one every token takes (a dense feed-forward is the latter alone)
 struct HyMoe {
-  bool on = false;
-  int E = 0, ident = 0, top = 0, ff = 0, ffp = 0, sff = 0, sffp = 0;  // sff 0: no shared expert
+  bool on = false, over_chosen = false;
+  int E = 0, ident = 0, top = 0, ff = 0, ffp = 0, sff = 0, sffp = 0;  // top 0: no router; sff 0: no shared expert
+  bool sgate = false;  // the shared expert has a gate row
+  GateAct act{INFINITY, 1.f, 0.f}, sact{INFINITY, 1.f, 0.f};
   HyMat zr;    // router rows, then the shared expert's gate row
   HyMat gu;    // experts, each [2 ffp]: 16 gate rows, 16 up rows, ...
   HyMat down;  // experts, each [W][ffp]
@@ -70,8 +92,13 @@ struct HyLayer {
   int mixer = HY_MAMBA1;
   HyMamba mb;
   HyLatent la;
+  HyHeads ha;
   HyMoe ff;
-  HyVec n1, n1b, n2, n2b;
+  HyVec n1, n1b, n2, n2b;  // n2 off: the feed-forward reads the first norm
+  const HyMat& out_mat() const { return mixer == HY_MAMBA1 ? mb.o : (mixer == HY_LATENT ? la.o : ha.o); }
+  const HyVec& norm2() const { return n2.on ? n2 : n1; }
+  const HyVec& norm2_b() const { return n2.on ? n2b : n1b; }
+  int cache_row() const { return mixer == HY_LATENT ? la.row() : (mixer == HY_HEADS ? ha.row() : 0); }  // elements
 };
 // one run of a layer: a looped layer has one per pass, each with its own cache or state
 struct HyRun {
@@ -83,7 +110,9 @@ struct HyRun {
 struct HyConfig {
   std::string arch;
   int width = 0, vocab = 0, widthp = 0;
-  float eps = 1e-5f, cap = 0.f;
+  float eps = 1e-5f, cap = 0.f, mult = 1.f, emb_scale = 1.f;
+  bool rms = false;    // RMS norms without biases (else layer norms)
+  int max_pos = 0;     // positions the model has (0: any)
   int loop_start = 0, loop_stop = 0, loop_times = 1;
   bool loop = false;
 };
@@ -93,7 +122,8 @@ struct Hybrid {
   bool f32 = false;  // storage type: fp32 instead of bf16
   std::vector<HyLayer> layers;
   std::vector<HyRun> runs;
-  HyMat embed, head;
+  HyMat embed, head, pos_emb;
+  HyMat enter;  // a pass of the loop starts with x <- enter [x ; embedding output]
   HyVec fnorm, fnorm_b, step;
   char* farena = nullptr;  // fp32 parameters
   std::vector<float2*> rope_tabs;
@@ -139,6 +169,31 @@ struct HyEntry {  // tokens of one sequence in a pass
   int slot, n, pos0;
   const int32_t* tok;
 };
+
+// the attention arguments that follow from the model; the caller adds rows, output and splits
+inline HeadsArgs heads_args(const Hybrid& hy, const HyHeads& a, const void* cache) {
+  HeadsArgs h{};
+  h.g_off = a.gate ? a.g_off() : -1;
+  h.qn = a.qn.p;
+  h.cache = cache;
+  h.slot_elems = hy.kv_slot;
+  h.bias = a.bias.p;
+  h.H = a.H;
+  h.G = a.G;
+  h.dk = a.dk;
+  h.dkr = a.dkr;
+  h.dkp = a.dkp;
+  h.dvr = a.dvr;
+  h.dvp = a.dvp;
+  h.ring = a.ring;
+  h.nsplit = 1;
+  h.nbias = a.nbias;
+  h.sink = a.sink;
+  h.span = a.span;
+  h.eps = hy.c.eps;
+  h.scale2 = a.scale * 1.44269504088896f;
+  return h;
+}
 
 // ---- kh_hybrid_load.hip
 int hy_create(const char* config, size_t config_len, const void* tensors, size_t nbytes, const kh_model_opts* o, kh_model** out);

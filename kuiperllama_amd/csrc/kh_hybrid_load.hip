@@ -152,6 +152,7 @@ struct Plan {
     HyVec r;
     floats = align(floats, 64);
     r.off = floats;
+    r.on = true;
     floats += v.size();
     vecs.emplace_back(r.off, std::move(v));
     return r;
@@ -192,6 +193,15 @@ struct Plan {
     for (auto& t : team) t.join();
   }
 };
+
+// a vector of `heads` pieces of n elements, each padded with zeros to np
+std::vector<float> head_vec(const Tensor* t, int heads, int n, int np) {
+  std::vector<float> v((size_t)heads * np, 0.f);
+  if (t)
+    for (int h = 0; h < heads; ++h)
+      for (int i = 0; i < n; ++i) v[(size_t)h * np + i] = t->at((int64_t)h * n + i);
+  return v;
+}
 
 // gate and up rows interleaved in groups of 16: destination rows base + 32 (r / 16) + r % 16 (+ 16 for up)
 void put_gate_up(Plan& pl, const HyMat& m, int64_t base, const Tensor* gate, const Tensor* up, int ff) {
@@ -287,7 +297,101 @@ int load_latent(Plan& pl, Tensors& ts, const std::string& p, const JsonValue& v,
   return KH_OK;
 }
 
-int load_moe(Plan& pl, Tensors& ts, const std::string& p, const JsonValue& v, int W, HyMoe& ff) {
+// Entry of a distance table of `rows` entries that holds for distance n: one entry per distance below half of them, then
+// entries of equal width in log distance up to `far`, the last one for everything beyond.
+int distance_entry(int n, int rows, double far) {
+  const int half = rows / 2;
+  if (n < half || rows <= 1) return std::min(n, rows - 1);
+  double x = log((double)n / half) / log(far / half) * (rows - half);
+  if (!(x < rows)) return rows - 1;  // beyond `far`, or a degenerate far
+  const double r = nearbyint(x);
+  if (fabs(x - r) < 1e-9) x = r;  // a border up to rounding of the logarithms
+  return std::max(0, std::min(rows - 1, half + (int)floor(x)));
+}
+
+enum HeadsFlags { HEADS_BIASES = 1, HEADS_REL = 2, HEADS_WINDOW = 4, HEADS_CHUNK = 8, HEADS_SINK = 16, HEADS_GATE = 32 };
+// Attention over grouped heads with query / key norms; flags: projection biases, a learned distance bias, what mask.size
+// means, a sink, an output gate.
+int load_heads(Plan& pl, Tensors& ts, const std::string& p, const JsonValue& v, int W, int flags, HyHeads& a) {
+  a.H = v.integer("heads", -1);
+  a.G = v.integer("kv_heads", a.H);
+  a.dk = size_of(v, "dim", ts.dim(p + ".q.norm", 0));
+  if (a.H <= 0 || a.G <= 0 || a.H % a.G || a.dk <= 0) return KH_ERR_FORMAT;
+  a.dv = size_of(v, "vdim", ts.dim(p + ".v", 0) / a.G);
+  if (a.dv <= 0) return KH_ERR_FORMAT;
+  if (a.dk > KH_HEADS_MAX_DIM || a.dv > KH_HEADS_MAX_DIM) return KH_ERR_UNSUPPORTED;
+  a.scale = (float)v.number("scale", 1.0 / sqrt((double)a.dk));
+  const JsonValue* mask = v.get("mask");
+  const int size = mask ? mask->integer("size", 0) : 0;
+  if (flags & (HEADS_WINDOW | HEADS_CHUNK)) {
+    if (size <= 0) return KH_ERR_FORMAT;
+    ((flags & HEADS_WINDOW) ? a.span.window : a.span.chunk) = size;
+  }
+  a.sink = (flags & HEADS_SINK) != 0;
+  a.gate = (flags & HEADS_GATE) != 0;
+  a.dkr = pad_to(a.dk, 16);
+  a.dvr = pad_to(a.dv, 16);
+  a.dkp = padk(a.dk);
+  a.dvp = padk(a.dv);
+  const int H = a.H, G = a.G, N = a.g_off() + (a.gate ? H * a.dvr : 0);
+  a.qkvg = pl.mat(N, W, padk(W));
+  std::vector<float> b;
+  auto part = [&](const char* name, int at, int heads, int d, int dr, bool bias) {
+    const Tensor* t = ts.need(p + name, {(int64_t)heads * d, W});
+    for (int h = 0; h < heads; ++h) pl.put(a.qkvg, at + (int64_t)h * dr, t, (int64_t)h * d, d);
+    std::vector<float> x((size_t)heads * dr, 0.f);
+    if (bias) x = head_vec(ts.need(p + name + ".b", {(int64_t)heads * d}), heads, d, dr);
+    b.insert(b.end(), x.begin(), x.end());
+  };
+  const bool biases = (flags & HEADS_BIASES) != 0;
+  part(".q", 0, H, a.dk, a.dkr, biases);
+  part(".k", a.k_off(), G, a.dk, a.dkr, biases);
+  part(".v", a.v_off(), G, a.dv, a.dvr, biases);
+  if (a.gate) part(".g", a.g_off(), H, a.dv, a.dvr, false);
+  const int hv = H * a.dvr;
+  a.o = pl.mat(W, hv, padk(hv));
+  const Tensor* o = ts.need(p + ".o", {W, (int64_t)H * a.dv});
+  for (int h = 0; h < H; ++h) pl.put(a.o, 0, o, 0, W, (int64_t)h * a.dv, a.dv, (int64_t)h * a.dvr);
+  if (biases) {
+    a.qkvg_b = pl.vec(std::move(b));
+    a.o_b = pl.vec(ts.need(p + ".o.b", {W}));
+  }
+  a.qn = pl.vec(head_vec(ts.need(p + ".q.norm", {a.dk}), 1, a.dk, a.dkp));
+  a.kn = pl.vec(head_vec(ts.need(p + ".k.norm", {a.dk}), 1, a.dk, a.dkp));
+  if (flags & HEADS_REL) {
+    const int rows = (int)ts.dim(p + ".rel", 0);
+    const double far = v.number("bias_max", -1.0);
+    if (rows <= 0 || !(far > 0)) return KH_ERR_FORMAT;
+    const Tensor* rel = ts.need(p + ".rel", {rows, H});
+    // by distance, up to the last entry's first distance or the farthest visible one
+    std::vector<int> entry{distance_entry(0, rows, far)};
+    const int most = a.span.window > 0 ? a.span.window : 1 << 20;
+    while ((int)entry.size() < most && entry.back() < rows - 1) entry.push_back(distance_entry((int)entry.size(), rows, far));
+    a.nbias = (int)entry.size();
+    std::vector<float> t((size_t)H * a.nbias, 0.f);
+    if (rel)
+      for (int h = 0; h < H; ++h)
+        for (int n = 0; n < a.nbias; ++n) t[(size_t)h * a.nbias + n] = rel->at((int64_t)entry[(size_t)n] * H + h) * 1.4426950408889634f;
+    a.bias = pl.vec(std::move(t));
+  }
+  return KH_OK;
+}
+
+// dense feed-forward, SwiGLU: an expert every token takes
+int load_dense(Plan& pl, Tensors& ts, const std::string& p, const JsonValue& v, int W, HyMoe& ff) {
+  ff.on = true;
+  ff.sff = size_of(v, "ff", ts.dim(p + ".gate", 0));
+  if (ff.sff <= 0) return KH_ERR_FORMAT;
+  ff.sffp = padk(ff.sff);
+  ff.sgu = pl.mat(2 * ff.sffp, W, padk(W));
+  put_gate_up(pl, ff.sgu, 0, ts.need(p + ".gate", {ff.sff, W}), ts.need(p + ".up", {ff.sff, W}), ff.sff);
+  ff.sdown = pl.mat(W, ff.sff, ff.sffp);
+  pl.put(ff.sdown, 0, ts.need(p + ".down", {W, ff.sff}), 0, W);
+  return KH_OK;
+}
+
+// correction: the choice is by softmax over all outputs plus a correction; else weights are the softmax over the chosen
+int load_moe(Plan& pl, Tensors& ts, const std::string& p, const JsonValue& v, int W, bool correction, HyMoe& ff) {
   if (v.text("kind") != "moe") return KH_ERR_UNSUPPORTED;
   const JsonValue *r = v.get("router"), *ex = v.get("expert"), *sh = v.get("shared");
   if (!r) return KH_ERR_FORMAT;
@@ -306,7 +410,8 @@ int load_moe(Plan& pl, Tensors& ts, const std::string& p, const JsonValue& v, in
   }
   ff.zr = pl.mat(ff.n_out() + (sh ? 1 : 0), W, padk(W));
   pl.put(ff.zr, 0, ts.need(p + ".router", {ff.n_out(), W}), 0, ff.n_out());
-  ff.corr = pl.vec(ts.need(p + ".correction", {ff.n_out()}));
+  ff.over_chosen = !correction;
+  if (correction) ff.corr = pl.vec(ts.need(p + ".correction", {ff.n_out()}));
   ff.gu = pl.mat(ff.E * 2 * ff.ffp, W, padk(W));
   ff.down = pl.mat(ff.E * W, ff.ff, ff.ffp);
   for (int e = 0; e < ff.E; ++e) {
@@ -315,6 +420,7 @@ int load_moe(Plan& pl, Tensors& ts, const std::string& p, const JsonValue& v, in
     pl.put(ff.down, (int64_t)e * W, ts.need(q + ".down", {W, ff.ff}), 0, W);
   }
   if (sh) {
+    ff.sgate = true;
     pl.put(ff.zr, ff.n_out(), ts.need(p + ".shared.sg", {1, W}), 0, 1);
     ff.sgu = pl.mat(2 * ff.sffp, W, padk(W));
     put_gate_up(pl, ff.sgu, 0, ts.need(p + ".shared.gate", {ff.sff, W}), ts.need(p + ".shared.up", {ff.sff, W}), ff.sff);
@@ -324,39 +430,54 @@ int load_moe(Plan& pl, Tensors& ts, const std::string& p, const JsonValue& v, in
   return KH_OK;
 }
 
-// Gufanex: parallel blocks with two layer norms, mixers mamba1 / latent_attention, mixture of experts, one looped range
-int load_gufanex(const JsonValue& cfg, Tensors& ts, Plan& pl, Hybrid& hy) {
+// What every architecture has: sizes, norm constant, embedding, head, the looped range
+int load_common(const JsonValue& cfg, Tensors& ts, Plan& pl, Hybrid& hy) {
   HyConfig& c = hy.c;
   c.width = size_of(cfg, "width", ts.dim("embed", 1));
   c.vocab = size_of(cfg, "vocab", ts.dim("embed", 0));
   const JsonValue *ls = cfg.get("layers"), *nm = cfg.get("norm"), *lp = cfg.get("loop");
   if (c.width <= 0 || c.vocab <= 0 || !ls || ls->kind != JsonValue::ARR || ls->arr.empty() || !nm) return KH_ERR_FORMAT;
   c.eps = (float)nm->number("eps", -1.0);
-  c.cap = (float)cfg.number("logit_softcap", 0.0);
   if (!(c.eps > 0)) return KH_ERR_FORMAT;
-  const int W = c.width, L = (int)ls->arr.size();
+  const int W = c.width;
   c.widthp = padk(W);
   hy.embed = pl.mat(c.vocab, W, c.widthp);
   pl.put(hy.embed, 0, ts.need("embed", {c.vocab, W}), 0, c.vocab);
   hy.head = pl.mat(c.vocab, W, c.widthp);
   pl.put(hy.head, 0, ts.need("head", {c.vocab, W}), 0, c.vocab);
-  hy.fnorm = pl.vec(ts.need("final.norm", {W}));
-  hy.fnorm_b = pl.vec(ts.need("final.norm.b", {W}));
   if (lp) {
     c.loop = true;
     c.loop_start = lp->integer("start", -1);
     c.loop_stop = lp->integer("stop", -1);
     c.loop_times = lp->integer("times", -1);
-    if (c.loop_start < 0 || c.loop_stop <= c.loop_start || c.loop_stop > L || c.loop_times < 1) return KH_ERR_FORMAT;
+    if (c.loop_start < 0 || c.loop_stop <= c.loop_start || c.loop_stop > (int)ls->arr.size() || c.loop_times < 1) return KH_ERR_FORMAT;
+  }
+  return KH_OK;
+}
+int unknown_mixer(int layer, const std::string& type) {
+  fprintf(stderr, "[kh] layer %d: unknown mixer '%s'\n", layer, type.c_str());
+  return KH_ERR_UNSUPPORTED;
+}
+
+// Gufanex: parallel blocks with two layer norms, mixers mamba1 / latent_attention, mixture of experts, one looped range
+// whose passes add the embedding output and a step vector
+int load_gufanex(const JsonValue& cfg, Tensors& ts, Plan& pl, Hybrid& hy) {
+  HyConfig& c = hy.c;
+  int rc = load_common(cfg, ts, pl, hy);
+  if (rc != KH_OK) return rc;
+  const int W = c.width, L = (int)cfg.get("layers")->arr.size();
+  c.cap = (float)cfg.number("logit_softcap", 0.0);
+  hy.fnorm = pl.vec(ts.need("final.norm", {W}));
+  hy.fnorm_b = pl.vec(ts.need("final.norm.b", {W}));
+  if (c.loop) {
     std::vector<float> step((size_t)c.loop_times * c.widthp, 0.f);
     if (const Tensor* t = ts.need("loop.step", {c.loop_times, W}))
       for (int p = 0; p < c.loop_times; ++p)
         for (int i = 0; i < W; ++i) step[(size_t)p * c.widthp + i] = t->at((int64_t)p * W + i);
     hy.step = pl.vec(std::move(step));
   }
-  int rc;
   for (int i = 0; i < L; ++i) {
-    const JsonValue& v = ls->arr[(size_t)i];
+    const JsonValue& v = cfg.get("layers")->arr[(size_t)i];
     const std::string p = "l" + std::to_string(i), type = v.text("type");
     const JsonValue *mx = v.get("mixer"), *ml = v.get("mlp");
     HyLayer ly;
@@ -370,14 +491,65 @@ int load_gufanex(const JsonValue& cfg, Tensors& ts, Plan& pl, Hybrid& hy) {
       ly.mixer = HY_LATENT;
       rc = load_latent(pl, ts, p + ".mix", mx ? *mx : none, W, ly.la);
     } else {
-      fprintf(stderr, "[kh] layer %d: unknown mixer '%s'\n", i, type.c_str());
-      return KH_ERR_UNSUPPORTED;
+      return unknown_mixer(i, type);
     }
     if (rc != KH_OK) return rc;
     if (ml) {
       ly.n2 = pl.vec(ts.need(p + ".norm2", {W}));
       ly.n2b = pl.vec(ts.need(p + ".norm2.b", {W}));
-      if ((rc = load_moe(pl, ts, p + ".mlp", *ml, W, ly.ff)) != KH_OK) return rc;
+      if ((rc = load_moe(pl, ts, p + ".mlp", *ml, W, true, ly.ff)) != KH_OK) return rc;
+    }
+    hy.layers.push_back(ly);
+  }
+  return KH_OK;
+}
+
+// Gusorax: parallel blocks behind one RMS norm (weights around zero) with a residual multiplier, mixers attention
+// (sliding window, distance bias) / attention_2 (chunks, sink, gate, biases), dense feed-forwards or clamped experts,
+// scaled embeddings with learned positions, one looped range whose passes enter through a matrix
+int load_gusorax(const JsonValue& cfg, Tensors& ts, Plan& pl, Hybrid& hy) {
+  HyConfig& c = hy.c;
+  int rc = load_common(cfg, ts, pl, hy);
+  if (rc != KH_OK) return rc;
+  const int W = c.width, L = (int)cfg.get("layers")->arr.size();
+  c.rms = true;
+  c.mult = (float)cfg.number("residual_mult", 1.0);
+  if (const JsonValue* e = cfg.get("embedding")) c.emb_scale = (float)e->number("scale", 1.0);
+  c.max_pos = size_of(cfg, "max_positions", ts.dim("pos", 0));
+  if (c.max_pos <= 0) return KH_ERR_FORMAT;
+  hy.pos_emb = pl.mat(c.max_pos, W, c.widthp);
+  pl.put(hy.pos_emb, 0, ts.need("pos", {c.max_pos, W}), 0, c.max_pos);
+  auto norm = [&](const std::string& name) {
+    std::vector<float> v = head_vec(ts.need(name, {W}), 1, W, W);
+    for (float& x : v) x += 1.f;
+    return pl.vec(std::move(v));
+  };
+  hy.fnorm = norm("final.norm");
+  if (c.loop) {
+    const Tensor* t = ts.need("loop.in", {W, 2 * W});
+    hy.enter = pl.mat(W, 2 * c.widthp, 2 * c.widthp);
+    pl.put(hy.enter, 0, t, 0, W, 0, W, 0);
+    pl.put(hy.enter, 0, t, 0, W, W, W, c.widthp);
+  }
+  for (int i = 0; i < L; ++i) {
+    const JsonValue& v = cfg.get("layers")->arr[(size_t)i];
+    const std::string p = "l" + std::to_string(i), type = v.text("type");
+    const JsonValue *mx = v.get("mixer"), *ml = v.get("mlp");
+    HyLayer ly;
+    ly.n1 = norm(p + ".norm1");
+    int flags;
+    if (type == "attention") flags = HEADS_REL | HEADS_WINDOW;
+    else if (type == "attention_2") flags = HEADS_BIASES | HEADS_CHUNK | HEADS_SINK | HEADS_GATE;
+    else return unknown_mixer(i, type);
+    if (!mx) return KH_ERR_FORMAT;
+    ly.mixer = HY_HEADS;
+    if ((rc = load_heads(pl, ts, p + ".mix", *mx, W, flags, ly.ha)) != KH_OK) return rc;
+    if (ml && ml->text("kind") == "dense") {
+      if ((rc = load_dense(pl, ts, p + ".mlp", *ml, W, ly.ff)) != KH_OK) return rc;
+    } else if (ml) {
+      if ((rc = load_moe(pl, ts, p + ".mlp", *ml, W, false, ly.ff)) != KH_OK) return rc;
+      const JsonValue* ex = ml->get("expert");
+      ly.ff.act = GateAct{(float)(ex ? ex->number("limit", INFINITY) : INFINITY), 1.702f, 1.f};
     }
     hy.layers.push_back(ly);
   }
@@ -388,7 +560,7 @@ struct Arch {
   const char* name;
   int (*load)(const JsonValue&, Tensors&, Plan&, Hybrid&);
 };
-const Arch kArchs[] = {{"Gufanex", load_gufanex}};
+const Arch kArchs[] = {{"Gufanex", load_gufanex}, {"Gusorax", load_gusorax}};
 
 // runs in execution order, and where each finds its part of a slot's state
 void build_runs(Hybrid& hy) {
@@ -410,30 +582,34 @@ void build_runs(Hybrid& hy) {
 
 template <class F>
 void each_mat(Hybrid& hy, F&& f) {
-  f(hy.embed);
-  f(hy.head);
+  for (HyMat* m : {&hy.embed, &hy.head, &hy.pos_emb, &hy.enter})
+    if (m->N) f(*m);
   for (auto& l : hy.layers) {
-    for (HyMat* m : {&l.mb.in, &l.mb.x, &l.mb.dt, &l.mb.o, &l.la.dqkv, &l.la.uq, &l.la.ukT, &l.la.uk, &l.la.uv, &l.la.o, &l.ff.zr,
-                     &l.ff.gu, &l.ff.down, &l.ff.sgu, &l.ff.sdown})
+    for (HyMat* m : {&l.mb.in, &l.mb.x, &l.mb.dt, &l.mb.o, &l.la.dqkv, &l.la.uq, &l.la.ukT, &l.la.uk, &l.la.uv, &l.la.o, &l.ha.qkvg,
+                     &l.ha.o, &l.ff.zr, &l.ff.gu, &l.ff.down, &l.ff.sgu, &l.ff.sdown})
       if (m->N) f(*m);
   }
 }
 template <class F>
 void each_vec(Hybrid& hy, F&& f) {
-  for (HyVec* v : {&hy.fnorm, &hy.fnorm_b, &hy.step}) f(*v);
+  for (HyVec* v : {&hy.fnorm, &hy.fnorm_b, &hy.step})
+    if (v->on) f(*v);
   for (auto& l : hy.layers)
     for (HyVec* v : {&l.n1, &l.n1b, &l.n2, &l.n2b, &l.mb.conv, &l.mb.conv_b, &l.mb.dt_b, &l.mb.A2, &l.mb.D, &l.la.qn,
-                     &l.la.kvn, &l.la.sink, &l.ff.corr})
-      f(*v);
+                     &l.la.kvn, &l.la.sink, &l.ha.qkvg_b, &l.ha.o_b, &l.ha.qn, &l.ha.kn, &l.ha.bias, &l.ff.corr})
+      if (v->on) f(*v);
 }
+
+// cache rows a run of the layer keeps per sequence
+int cache_rows(const HyLayer& l, int cache_len) { return l.mixer == HY_HEADS ? l.ha.ring : cache_len; }
 
 int alloc_workspace(kh_model* m) {
   Hybrid& hy = *m->hy;
-  const size_t T = KH_HY_TMAX, Wp = (size_t)hy.c.widthp, es = hy.elem();
-  hy.tmax = KH_HY_TMAX;
+  const size_t T = (size_t)hy.tmax, Wp = (size_t)hy.c.widthp, es = hy.elem();
   size_t f32a = 1, a0 = 1, a1 = 1, a2 = 1, dt = 1, bc = 1, z = 1, ends = 1, dtsum = 1, h = 1, hs = 1, y = 1, top = 1, tiles = 1;
   auto up = [](size_t& v, size_t n) { v = v > n ? v : n; };
   const size_t multi = T / KH_SCAN_CH * 2 + 2;  // chunks of segments that have more than one
+  if (hy.enter.N) up(a2, T * 2 * Wp);
   for (auto& l : hy.layers) {
     if (l.mixer == HY_MAMBA1) {
       const size_t I = (size_t)l.mb.inner, Ip = (size_t)l.mb.innerp;
@@ -445,6 +621,9 @@ int alloc_workspace(kh_model* m) {
       up(bc, T * 2 * (size_t)l.mb.state);
       up(ends, multi * I * (size_t)l.mb.state);
       up(dtsum, multi * I);
+    } else if (l.mixer == HY_HEADS) {
+      up(a1, T * (size_t)l.ha.qkvg.N);
+      up(a0, T * (size_t)l.ha.o.ld);
     } else {
       const HyLatent& a = l.la;
       up(f32a, T * (size_t)(a.qr + a.R + a.dr));
@@ -556,6 +735,20 @@ int finish(kh_model* m, Plan& pl) {
     l.la.rope = d;
   }
   // ---- state manager
+  const char* tm = dbg("KH_HY_TMAX");
+  hy.tmax = tm ? std::max(32, std::min(atoi(tm), KH_HY_TMAX)) : KH_HY_TMAX;
+  for (auto& l : hy.layers) {
+    if (l.mixer != HY_HEADS) continue;
+    HyHeads& a = l.ha;
+    // a query's span and the tokens of one pass, which are all written before the first of them attends
+    const int span = a.span.window > 0 ? a.span.window : a.span.chunk;
+    a.ring = span > 0 && span < CL - hy.tmax ? std::min(CL, pad_to(span + hy.tmax, 64)) : CL;
+    // time splits of a decoded token: tiles of the visible keys over about two workgroups per CU
+    const int keys = span > 0 ? std::min(span, CL) : CL;
+    a.nsplit = 2;
+    while (a.nsplit < 128 && a.nsplit * KH_LAT_SPLIT_MIN < keys && a.nsplit * a.G < 512) a.nsplit *= 2;
+    if ((double)a.ring * a.row() * hy.elem() >= 4294967296.0) return KH_ERR_UNSUPPORTED;  // 32-bit offsets within a run
+  }
   build_runs(hy);
   for (auto& r : hy.runs) {
     const HyLayer& l = hy.layers[(size_t)r.layer];
@@ -566,7 +759,7 @@ int finish(kh_model* m, Plan& pl) {
       hy.st_slot += ((size_t)l.mb.inner * (l.mb.taps - 1) + 63) / 64 * 64;
     } else {
       r.kv_off = hy.kv_slot;
-      hy.kv_slot += (size_t)CL * l.la.row();
+      hy.kv_slot += (size_t)cache_rows(l, CL) * l.cache_row();
     }
   }
   hy.len.assign((size_t)hy.slots, -1);
@@ -644,16 +837,23 @@ int create_impl(const char* config, size_t config_len, const void* tensors, size
   c.family = KH_FAMILY_LAYERS;
   c.rms_eps = h.c.eps;
   c.cache_len = c.seq_len = o->max_seq_len > 0 ? o->max_seq_len : 8192;
+  if (h.c.max_pos > 0 && c.cache_len > h.c.max_pos) c.cache_len = c.seq_len = h.c.max_pos;
+  c.kv_mul = 1;
   for (auto& l : h.layers) {
     if (l.mixer == HY_LATENT) {
       c.head_num = c.kv_head_num = l.la.H;
       c.kv_dim = l.la.R + l.la.dr;
       c.head_size = l.la.dn + l.la.dr;
       c.rope_theta = (float)l.la.base;
+    } else if (l.mixer == HY_HEADS) {
+      c.head_num = l.ha.H;
+      c.kv_head_num = l.ha.G;
+      c.kv_dim = l.ha.G * l.ha.dk;
+      c.kv_mul = l.ha.H / l.ha.G;
+      c.head_size = l.ha.dk;
     }
-    if (l.ff.on) c.hidden_dim = l.ff.ff;
+    if (l.ff.on) c.hidden_dim = l.ff.top ? l.ff.ff : l.ff.sff;
   }
-  c.kv_mul = 1;
   return finish(m, pl);
 }
 
@@ -690,10 +890,10 @@ int hy_kv_ensure(kh_model* m, int slot, int rows) {
   if (rows <= hy.rows_ok[(size_t)slot] || !hy.kv_slot) return KH_OK;
   for (const HyRun& r : hy.runs) {
     const HyLayer& l = hy.layers[(size_t)r.layer];
-    if (l.mixer != HY_LATENT) continue;
-    const size_t row_b = (size_t)l.la.row() * hy.elem();
+    if (!l.cache_row()) continue;
+    const size_t row_b = (size_t)l.cache_row() * hy.elem();
     const size_t b0 = ((size_t)slot * hy.kv_slot + r.kv_off) * hy.elem();
-    const int rc = kv_map_range(m, 0, b0, b0 + (size_t)rows * row_b, r.layer);
+    const int rc = kv_map_range(m, 0, b0, b0 + (size_t)std::min(rows, cache_rows(l, m->cfg.cache_len)) * row_b, r.layer);
     if (rc != KH_OK) return rc;
   }
   hy.rows_ok[(size_t)slot] = rows;

@@ -19,8 +19,15 @@ namespace {
     if (_rc != KH_OK) return _rc;    \
   } while (0)
 
-struct LatTiles {
-  int H, big, cp, off, n;  // big: latents of more than 256; offset in ints from the table base
+// Query-row tiles of an attention kernel: `per` rows a token, `lanes` workgroups per tile (key / value heads), big tiles of
+// `big` rows.  Layers of one kind share a tile list.
+struct RowKind {
+  int per, lanes, big;
+  bool operator==(const RowKind& o) const { return per == o.per && lanes == o.lanes && big == o.big; }
+};
+struct RowTiles {
+  RowKind kind;
+  int rows, off, n;  // rows of a tile; offset in ints from the table base; tiles
 };
 struct PassSeg {
   int slot, row0, n, pos0;
@@ -34,7 +41,7 @@ struct Pass {
   const ScanChunk* chunks = nullptr;
   const int32_t *multi0 = nullptr, *multin = nullptr, *want = nullptr;
   const int32_t* base = nullptr;
-  std::vector<LatTiles> lat;
+  std::vector<RowTiles> tiles;
   bool no_logits = false;  // nothing of the last layer's output is wanted: only its cache rows / state
 };
 
@@ -50,32 +57,35 @@ struct TabBuilder {
   int put(const std::vector<int32_t>& x) { return put(x.data(), x.size()); }
 };
 
-// query-row tile lists of latent attention a pass needs: one per (heads, latent of more than 256)
-typedef std::pair<int, int> LatKind;
-LatKind lat_kind(const HyLatent& la) { return {la.H, la.Rp > 256}; }
-std::vector<LatKind> lat_kinds(const Hybrid& hy) {
-  std::vector<LatKind> r;
-  for (auto& l : hy.layers)
-    if (l.mixer == HY_LATENT && std::find(r.begin(), r.end(), lat_kind(l.la)) == r.end()) r.push_back(lat_kind(l.la));
+// latents of more than 256: 32 rows, the accumulators of 64 would not fit
+RowKind row_kind(const HyLatent& la) { return {la.H, 1, la.Rp > 256 ? 32 : 64}; }
+RowKind row_kind(const Hybrid& hy, const HyHeads& a) { return {a.H / a.G, a.G, heads_wide_rows(a.dkp, a.dvp, hy.elem()) ? 128 : 64}; }
+std::vector<RowKind> row_kinds(const Hybrid& hy) {
+  std::vector<RowKind> r;
+  for (auto& l : hy.layers) {
+    if (l.mixer == HY_MAMBA1) continue;
+    const RowKind k = l.mixer == HY_LATENT ? row_kind(l.la) : row_kind(hy, l.ha);
+    if (std::find(r.begin(), r.end(), k) == r.end()) r.push_back(k);
+  }
   return r;
 }
-// 64 rows per tile (32 for big latents, whose accumulators would not fit), or 16 where the rows of the segments would
+// big tiles, or 64 rows where 128 would not give every CU two workgroups, or 16 where the rows of the segments would
 // leave most of those empty
-void lat_tiles(const std::vector<int32_t>& seg_n, LatKind kind, int* cp, std::vector<int32_t>* tab) {
-  const int H = kind.first;
-  long rows = 0, t64 = 0;
+int row_tiles(const std::vector<int32_t>& seg_n, const RowKind& kind, std::vector<int32_t>* tab) {
+  long rows = 0, t64 = 0, big = 0;
   for (int n : seg_n) {
-    rows += (long)n * H;
-    t64 += ((long)n * H + 63) / 64;
+    rows += (long)n * kind.per;
+    t64 += ((long)n * kind.per + 63) / 64;
+    big += ((long)n * kind.per + kind.big - 1) / kind.big;
   }
-  *cp = t64 * 64 > 2 * rows ? 4 : (kind.second ? 2 : 1);
-  const int step = 64 / *cp;
+  const int step = t64 * 64 > 2 * rows ? 16 : (kind.big > 64 && big * kind.lanes < 512 ? 64 : kind.big);
   tab->clear();
   for (size_t s = 0; s < seg_n.size(); ++s)
-    for (int r = (seg_n[s] * H - 1) / step * step; r >= 0; r -= step) {  // the longest key ranges first
+    for (int r = (seg_n[s] * kind.per - 1) / step * step; r >= 0; r -= step) {  // the longest key ranges first
       tab->push_back((int)s);
       tab->push_back(r);
     }
+  return step;
 }
 
 // ---- the pass ----------------------------------------------------------------------------------------------------
@@ -103,27 +113,33 @@ struct Runner {
     a.ldo = ldo;
     return a;
   }
-  // x += everything pending (+ the loop entry); layer != nullptr: its two norms
-  int combine(const HyLayer* l, bool from_embed, int pass_no) {
+  // x += everything pending (+ the loop entry); layer != nullptr: its norms
+  int combine(const HyLayer* l, bool from_embed, int pass_no, T* cat = nullptr) {
     CombineArgs<T> a{};
     a.x = hy.x;
     a.x0 = hy.x0;
     a.add = pend;
     a.embed = (const T*)hy.embed.w;
+    a.pos_emb = (const T*)hy.pos_emb.w;
     a.tok = ps.p.tok;
+    a.pos = ps.p.pos;
+    a.cat = cat;
     a.W = hy.c.width;
     a.ld = hy.c.widthp;
     a.from_embed = from_embed;
-    a.add_x0 = pass_no > 0;
-    a.step = pass_no >= 0 ? hy.step.p + (size_t)pass_no * hy.c.widthp : nullptr;
+    a.add_x0 = pass_no > 0 && !hy.enter.N;
+    a.step = pass_no >= 0 && hy.step.on ? hy.step.p + (size_t)pass_no * hy.c.widthp : nullptr;
+    a.rms = hy.c.rms;
     a.eps = hy.c.eps;
+    a.mult = hy.c.mult;
+    a.emb_scale = hy.c.emb_scale;
     a.xn2_prev = (const T*)hy.xn2;
     a.xn1 = (T*)hy.xn1;
     a.xn2 = (T*)hy.xn2;
     if (l) {
       a.w1 = l->n1.p;
       a.b1 = l->n1b.p;
-      if (l->ff.on) {
+      if (l->ff.on && l->n2.on) {
         a.w2 = l->n2.p;
         a.b2 = l->n2b.p;
       }
@@ -131,6 +147,47 @@ struct Runner {
     pend = AddArgs<T>{};
     hipLaunchKernelGGL(k_combine<T>, dim3(ps.T), dim3(256), (size_t)hy.c.widthp * 4, s, a);
     return KH_OK;
+  }
+
+  // a pass of the loop starts: x <- W [x ; embedding output]
+  int enter(bool from_embed) {
+    const int Wp = hy.c.widthp;
+    TRY(combine(nullptr, from_embed, -1, (T*)hy.a2));
+    return lg_launch<T, LG_F32>(s, gemm(hy.enter, hy.a2, 2 * Wp, hy.x, Wp));
+  }
+
+  int heads(const HyRun& r, const HyHeads& ha, bool state_only) {
+    LgArgs pr = gemm(ha.qkvg, hy.xn1, hy.c.widthp, hy.a1, ha.qkvg.N);
+    pr.bias = ha.qkvg_b.p;
+    if (state_only) {  // key and value rows only
+      pr.W = (const T*)ha.qkvg.w + (size_t)ha.k_off() * ha.qkvg.ld;
+      pr.out = (T*)hy.a1 + ha.k_off();
+      pr.N = ha.g_off() - ha.k_off();
+      if (pr.bias) pr.bias += ha.k_off();
+    }
+    TRY((lg_launch<T, LG_T>(s, pr)));
+    HeadRowsArgs<T> hr{ha.head_row(hy.c.eps), (const T*)hy.a1, (T*)m->kcache + r.kv_off, hy.kv_slot, ha.qkvg.N, ps.T, ps.p};
+    hipLaunchKernelGGL(k_heads_rows<T>, dim3((ps.T * ha.G + 3) / 4), dim3(256), 0, s, hr);
+    if (state_only) return KH_OK;
+    const RowTiles* rt = row_tiles_of(row_kind(hy, ha));
+    if (!rt) return KH_ERR_INTERNAL;
+    HeadsArgs a = heads_args(hy, ha, (const T*)m->kcache + r.kv_off);
+    a.raw = hy.a1;
+    a.ldr = ha.qkvg.N;
+    a.out = hy.a0;
+    a.ldo = ha.o.ld;
+    a.nsplit = 1;
+    a.tiles = (const LatTile*)(ps.base + rt->off);
+    a.p = ps.p;
+    TRY(heads_attn_launch<T>(s, a, rt->n, rt->rows));
+    LgArgs o = gemm(ha.o, hy.a0, ha.o.ld, hy.mix, hy.c.widthp);
+    o.bias = ha.o_b.p;
+    return lg_launch<T, LG_F32>(s, o);
+  }
+  const RowTiles* row_tiles_of(const RowKind& k) const {
+    for (auto& t : ps.tiles)
+      if (t.kind == k) return &t;
+    return nullptr;
   }
 
   int mamba(const HyRun& r, const HyMamba& mb, bool state_only) {
@@ -254,9 +311,7 @@ struct Runner {
     }
     RopeQArgs<T> rq{(const T*)hy.a1, (T*)hy.a2, la.rope, H, la.dnp, la.dr, la.drp, la.Rp, la.dims, ps.p};
     if (la.drp) hipLaunchKernelGGL(k_rope_q<T>, dim3(ps.T), dim3(256), 0, s, rq);
-    const LatTiles* lt = nullptr;
-    for (auto& t : ps.lat)
-      if (LatKind(t.H, t.big) == lat_kind(la)) lt = &t;
+    const RowTiles* lt = row_tiles_of(row_kind(la));
     if (!lt) return KH_ERR_INTERNAL;
     LatArgs at{};
     at.Q = hy.a2;
@@ -271,7 +326,7 @@ struct Runner {
     at.nsplit = 1;
     at.scale2 = la.scale * 1.44269504088896f;
     at.p = ps.p;
-    TRY(lat_attn_launch<T>(s, at, lt->n, lt->cp));
+    TRY(lat_attn_launch<T>(s, at, lt->n, 64 / lt->rows));
     {  // values: per head, W_uv o
       LgArgs a = gemm(la.uv, hy.a0, H * la.Rp, hy.a1, H * la.dvp);
       a.N = la.dvp;
@@ -283,10 +338,23 @@ struct Runner {
     return lg_launch<T, LG_F32>(s, gemm(la.o, hy.a1, H * la.dvp, hy.mix, hy.c.widthp));
   }
 
-  int moe(const HyMoe& f) {
+  int feed_forward(const HyMoe& f, const void* in) {
+    if (f.top) TRY(experts(f, in));
+    if (f.sff) {
+      const int Wp = hy.c.widthp;
+      LgArgs a = gemm(f.sgu, in, Wp, hy.hs, f.sffp);
+      a.act = f.sact;
+      TRY((lg_launch<T, LG_GATED>(s, a)));
+      TRY((lg_launch<T, LG_T>(s, gemm(f.sdown, hy.hs, f.sffp, hy.sh, Wp))));
+      pend.sh = (const T*)hy.sh;
+      pend.sh_g = f.sgate ? hy.sh_g : nullptr;
+    }
+    return KH_OK;
+  }
+  int experts(const HyMoe& f, const void* in) {
     const int W = hy.c.width, Wp = hy.c.widthp;
-    TRY((lg_launch<T, LG_F32>(s, gemm(f.zr, hy.xn2, Wp, hy.z, f.zr.N))));
-    RouteArgs ra{hy.z, f.corr.p, hy.moe_id, hy.moe_w, hy.id_w, hy.sh_g, ps.T, f.zr.N, f.n_out(), f.E, f.top, f.sff > 0};
+    TRY((lg_launch<T, LG_F32>(s, gemm(f.zr, in, Wp, hy.z, f.zr.N))));
+    RouteArgs ra{hy.z, f.corr.p, hy.moe_id, hy.moe_w, hy.id_w, hy.sh_g, ps.T, f.zr.N, f.n_out(), f.E, f.top, f.sgate, f.over_chosen};
     moe_route_launch(s, ra);
     const int bm = lg_group_bm((long)ps.T * f.top, f.n_out());
     ListArgs li{hy.moe_id, hy.moe_rows, hy.moe_slot, hy.tiles, hy.n_tiles, ps.T, f.top, f.E, bm};
@@ -294,13 +362,14 @@ struct Runner {
     const long rows = (long)ps.T * f.top;
     const int mt = (int)(rows / bm + std::min<long>(f.E, rows));
     {
-      LgArgs a = gemm(f.gu, hy.xn2, Wp, hy.h, f.ffp);
+      LgArgs a = gemm(f.gu, in, Wp, hy.h, f.ffp);
       a.N = 2 * f.ffp;
+      a.act = f.act;
       a.tiles = hy.tiles;
       a.n_tiles = hy.n_tiles;
       a.gather = hy.moe_rows;
       a.w_group = (size_t)2 * f.ffp * f.gu.ld;
-      TRY((lg_launch<T, LG_SWIGLU>(s, a, 1, bm, mt)));
+      TRY((lg_launch<T, LG_GATED>(s, a, 1, bm, mt)));
     }
     {
       LgArgs a = gemm(f.down, hy.h, f.ffp, hy.y, Wp);
@@ -313,14 +382,8 @@ struct Runner {
     pend.y = (const T*)hy.y;
     pend.y_slot = hy.moe_slot;
     pend.y_w = hy.moe_w;
-    pend.id_w = hy.id_w;
+    pend.id_w = f.ident ? hy.id_w : nullptr;
     pend.top = f.top;
-    if (f.sff) {
-      TRY((lg_launch<T, LG_SWIGLU>(s, gemm(f.sgu, hy.xn2, Wp, hy.hs, f.sffp))));
-      TRY((lg_launch<T, LG_T>(s, gemm(f.sdown, hy.hs, f.sffp, hy.sh, Wp))));
-      pend.sh = (const T*)hy.sh;
-      pend.sh_g = hy.sh_g;
-    }
     return KH_OK;
   }
 
@@ -329,11 +392,14 @@ struct Runner {
       const HyRun& r = hy.runs[i];
       const HyLayer& l = hy.layers[(size_t)r.layer];
       const bool state_only = ps.no_logits && i + 1 == hy.runs.size() && !hy.probe;
-      TRY(combine(&l, i == 0, r.pass));
-      TRY(l.mixer == HY_MAMBA1 ? mamba(r, l.mb, state_only) : latent(r, l.la, state_only));
+      const bool through = r.pass >= 0 && hy.enter.N;
+      if (through) TRY(enter(i == 0));
+      TRY(combine(&l, i == 0 && !through, r.pass));
+      TRY(l.mixer == HY_MAMBA1 ? mamba(r, l.mb, state_only)
+          : l.mixer == HY_LATENT ? latent(r, l.la, state_only) : heads(r, l.ha, state_only));
       if (state_only) break;
       pend.mix = hy.mix;
-      if (l.ff.on) TRY(moe(l.ff));
+      if (l.ff.on) TRY(feed_forward(l.ff, l.n2.on ? hy.xn2 : hy.xn1));
       if (hy.probe) {
         TRY(combine(nullptr, false, -1));
         const int64_t n = (int64_t)ps.T * hy.c.width;
@@ -350,7 +416,7 @@ struct Runner {
   // logits of rows[0 .. n) (device list) -> out [n][vocab]; n <= wl_rows
   int logits(const int32_t* rows, int n, float* out) {
     hipLaunchKernelGGL(k_gather_norm<T>, dim3(n), dim3(256), 0, s, (const float*)hy.x, rows, hy.fnorm.p, hy.fnorm_b.p,
-                       (T*)hy.xw, hy.c.width, hy.c.widthp, hy.c.eps);
+                       (T*)hy.xw, hy.c.width, hy.c.widthp, hy.c.eps, (int)hy.c.rms);
     LgArgs a = gemm(hy.head, hy.xw, hy.c.widthp, out, hy.c.vocab);
     a.M = n;
     a.cap = hy.c.cap;
@@ -395,7 +461,7 @@ int hy_forward(kh_model* m, const HyEntry* e, int n, const int32_t* want, int n_
   Hybrid& hy = *m->hy;
   KH_CHECK_HIP(hipSetDevice(m->opts.device));
   KH_CHECK_HIP(hipStreamSynchronize(m->stream));  // the pinned tables of the call before are free again
-  const std::vector<LatKind> kinds = lat_kinds(hy);
+  const std::vector<RowKind> kinds = row_kinds(hy);
   // ---- cut the concatenated tokens into passes and build every pass's tables
   std::vector<Pass> passes;
   std::vector<int32_t> all;
@@ -468,12 +534,10 @@ int hy_forward(kh_model* m, const HyEntry* e, int n, const int32_t* want, int n_
     o.m0 = tb.put(m0);
     o.mn = tb.put(mn);
     o.want = tb.put(wr);
-    for (const LatKind& kd : kinds) {
-      LatTiles t{kd.first, kd.second, 0, 0, 0};
-      lat_tiles(sn, kd, &t.cp, &lt);
-      t.n = (int)lt.size() / 2;
+    for (const RowKind& kd : kinds) {
+      RowTiles t{kd, row_tiles(sn, kd, &lt), 0, (int)lt.size() / 2};
       t.off = tb.put(lt);
-      p.lat.push_back(t);
+      p.tiles.push_back(t);
     }
     bases.push_back((all.size() + 15) / 16 * 16);
     all.resize(bases.back() + tb.v.size());
@@ -525,13 +589,10 @@ int hy_unfused_step(kh_model* m) {
   Hybrid& hy = *m->hy;
   Pass p;
   std::vector<int32_t> tab{0, 0, 0, 0, 0, 1, 0, 0, 0, 0, 1, 3, 0, 0, 0, 0}, lt;
-  for (const LatKind& kd : lat_kinds(hy)) {
-    LatTiles t{kd.first, kd.second, 0, 0, 0};
-    lat_tiles({1}, kd, &t.cp, &lt);
-    t.n = (int)lt.size() / 2;
-    t.off = (int)tab.size();
+  for (const RowKind& kd : row_kinds(hy)) {
+    const int rows = row_tiles({1}, kd, &lt);
+    p.tiles.push_back({kd, rows, (int)tab.size(), (int)lt.size() / 2});
     tab.insert(tab.end(), lt.begin(), lt.end());
-    p.lat.push_back(t);
   }
   if (!hy.d_one) {
     TRY(dalloc(&hy.d_one, tab.size()));

@@ -40,8 +40,7 @@ template <class T>
 size_t vec_b(int n) { return Ld<T>::vec_bytes(n); }
 template <class T>
 size_t lds_out(const Hybrid& hy, const HyLayer& l, int B) {
-  const int nv = l.mixer == HY_MAMBA1 ? l.mb.innerp : l.la.H * l.la.dvp;
-  const int nbv = Ld<T>::blocks(nv);
+  const int nbv = Ld<T>::blocks(l.out_mat().ld);
   const int nf = l.ff.on ? l.ff.top * Ld<T>::blocks(l.ff.ffp) + (l.ff.sffp ? Ld<T>::blocks(l.ff.sffp) : 0) : 0;
   (void)hy;
   return ((size_t)B * nbv + nf) * Ld<T>::BE * 4;
@@ -50,6 +49,7 @@ template <class T>
 bool fits(const Hybrid& hy, int B) {
   const size_t room = kMaxLds - 2048;  // static shared memory of the kernels
   if (hy.c.widthp > 8192 || B * vec_b<T>(hy.c.widthp) > room) return false;
+  if (hy.enter.N && B * vec_b<T>(hy.enter.ld) > room) return false;
   for (auto& l : hy.layers) {
     if (lds_out<T>(hy, l, B) > room) return false;
     if (l.mixer == HY_MAMBA1 && B * vec_b<T>(l.mb.innerp) > room) return false;
@@ -109,6 +109,15 @@ int with_rp(int n_out, F&& f) {
   return f(std::integral_constant<int, 16>());
 }
 
+// waves of a row pair over nblk blocks (k_ld_out, k_ld_enter): as many as keep each wave's share within its two tiles and
+// give every CU a workgroup, while the launch has at most four per CU
+int split_waves(int rows, int nblk) {
+  int ks = 1;
+  while (ks < 8 && nblk >= 2 * ks && (nblk / ks > 8 || cdiv(cdiv(rows, 2) * ks, 8) < 256) && cdiv(cdiv(rows, 2) * ks * 2, 8) <= 1024)
+    ks *= 2;
+  return ks;
+}
+
 // One token of B sequences: tables at (tok, pos, slot); logits to `logits` [B][V]; argmax partials of sequence 0 to
 // the model's sampler buffers.
 template <class T, int B>
@@ -122,11 +131,19 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
     const HyRun& r = hy.runs[ri];
     const HyLayer& l = hy.layers[(size_t)r.layer];
     const HyMoe& f = l.ff;
-    const bool mamba = l.mixer == HY_MAMBA1;
-    const bool changed = ri == 0 || r.pass >= 0;
-    float* x_cur = changed ? st.x[2] : x_in;
+    const HyHeads& ha = l.ha;
+    const bool mamba = l.mixer == HY_MAMBA1, heads = l.mixer == HY_HEADS, through = r.pass >= 0 && hy.enter.N;
+    const bool changed = !through && (ri == 0 || r.pass >= 0);
+    float* x_cur = through || changed ? st.x[2] : x_in;
     float* x_out = x_in == st.x[0] ? st.x[1] : st.x[0];
-    const int in_ld = mamba ? 2 * l.mb.inner : l.la.dqkv.N;
+    const HyMat& w_in = mamba ? l.mb.in : (heads ? ha.qkvg : l.la.dqkv);
+    const int in_ld = w_in.N;
+    const LdEmbed emb{hy.embed.w, hy.pos_emb.w, hy.c.emb_scale};
+    if (through) {
+      LdEnterArgs a{hy.enter.w, ri == 0 ? nullptr : x_in, st.x[2], emb, W, Wp, 1, tb};
+      a.ks = split_waves(W, Ld<T>::blocks(hy.enter.ld));
+      TRY(go(k_ld_enter<T, B>, dim3(cdiv(cdiv(W, 2) * a.ks, 8)), 512, B * vec_b<T>(hy.enter.ld), s, a));
+    }
     {
       LdInArgs a{};
       auto seg = [&](const HyMat& w, float* out, int rows, int ldo, int kind, int norm2) {
@@ -138,13 +155,13 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
         g.kind = kind;
         g.norm2 = norm2;
       };
-      seg(mamba ? l.mb.in : l.la.dqkv, st.in, in_ld, in_ld, mamba ? LDI_CONV : LDI_PLAIN, 0);
-      if (f.on) {
-        seg(f.zr, st.z, f.zr.N, f.zr.N, LDI_PLAIN, 1);
-        if (f.sff) seg(f.sgu, st.hs, f.sffp, f.sffp, LDI_SWIGLU, 1);
-      }
+      seg(w_in, st.in, in_ld, in_ld, mamba ? LDI_CONV : LDI_PLAIN, 0);
+      if (heads) a.seg[0].bias = ha.qkvg_b.p;
+      if (f.top) seg(f.zr, st.z, f.zr.N, f.zr.N, LDI_PLAIN, 1);
+      if (f.sff) seg(f.sgu, st.hs, f.sffp, f.sffp, LDI_GATED, 1);
+      a.act = f.sact;
       int total = 0, wg = 0;
-      auto items = [&](const LdInSeg& g) { return cdiv(g.rows, g.kind == LDI_SWIGLU ? 2 : 4); };
+      auto items = [&](const LdInSeg& g) { return cdiv(g.rows, g.kind == LDI_GATED ? 2 : 4); };
       for (int i = 0; i < a.nseg; ++i) total += items(a.seg[i]);
       const int ipw = cdiv(total, 2048);
       for (int i = 0; i < a.nseg; ++i) {
@@ -152,19 +169,20 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
         a.seg[i].nwg = cdiv(items(a.seg[i]), 4 * ipw);
         wg += a.seg[i].nwg;
       }
-      a.x_in = x_in;
+      a.x_in = through ? x_cur : x_in;
       a.x_cur = changed ? x_cur : nullptr;
-      a.embed = hy.embed.w;
-      a.step = r.pass >= 0 ? hy.step.p + (size_t)r.pass * Wp : nullptr;
+      a.emb = emb;
+      a.step = r.pass >= 0 && hy.step.on ? hy.step.p + (size_t)r.pass * Wp : nullptr;
       a.w1 = l.n1.p;
       a.b1 = l.n1b.p;
-      a.w2 = f.on ? l.n2.p : nullptr;
-      a.b2 = f.on ? l.n2b.p : nullptr;
-      a.xn2 = f.on ? st.xn2 : nullptr;
+      a.w2 = l.norm2().p;
+      a.b2 = l.norm2_b().p;
+      a.xn2 = f.top ? st.xn2 : nullptr;
       a.W = W;
       a.ld = Wp;
-      a.from_embed = ri == 0;
-      a.add_x0 = r.pass > 0;
+      a.from_embed = ri == 0 && !through;
+      a.add_x0 = r.pass > 0 && !through;
+      a.rms = hy.c.rms;
       a.eps = hy.c.eps;
       a.t = tb;
       if (mamba) {
@@ -184,7 +202,7 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
       a.t = tb;
       a.eps = hy.c.eps;
       size_t lds = 0;
-      if (f.on) {
+      if (f.top) {
         a.z = st.z;
         a.corr = f.corr.p;
         a.xn2 = st.xn2;
@@ -196,7 +214,9 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
         a.top = f.top;
         a.n_out = f.n_out();
         a.n_expert = f.E;
-        a.shared = f.sff > 0;
+        a.shared = f.sgate;
+        a.over_chosen = f.over_chosen;
+        a.act = f.act;
         a.ffp = f.ffp;
         a.ldz = f.zr.N;
         a.W = W;
@@ -204,21 +224,30 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
         a.nwg_e = cdiv(f.ffp / 2, 4 * cdiv(B * f.top * f.ffp / 2, 3072));
         lds = vec_b<T>(Wp);
       }
-      const HyMat& wm = mamba ? l.mb.x : l.la.uq;
-      a.wm = wm.w;
-      a.rows = wm.N;
-      a.ldm = wm.ld;
-      a.n = mamba ? l.mb.inner : l.la.qr;
-      a.n4 = l.mb.innerp / 4;  // convolved inputs are padded with zeros
-      a.v = mamba ? st.xc : st.in;
       a.ldv = mamba ? l.mb.innerp : in_ld;
-      a.vnorm = mamba ? nullptr : l.la.qn.p;
-      a.om = st.mid;
-      a.ldo = wm.N;
-      a.nwg_m = std::min(cdiv(cdiv(wm.N, 4), 4), 512);
-      lds = std::max(lds, B * vec_b<T>(wm.ld));
       int extra = 0;
-      if (!mamba) {
+      if (heads) {
+        extra = cdiv(B * ha.G, 4);
+        a.heads = 1;
+        a.hr = ha.head_row(hy.c.eps);
+        a.raw = st.in;
+        a.cache = (T*)m->kcache + r.kv_off;
+        a.slot_elems = hy.kv_slot;
+      } else {
+        const HyMat& wm = mamba ? l.mb.x : l.la.uq;
+        a.wm = wm.w;
+        a.rows = wm.N;
+        a.ldm = wm.ld;
+        a.n = mamba ? l.mb.inner : l.la.qr;
+        a.n4 = l.mb.innerp / 4;  // convolved inputs are padded with zeros
+        a.v = mamba ? st.xc : st.in;
+        a.vnorm = mamba ? nullptr : l.la.qn.p;
+        a.om = st.mid;
+        a.ldo = wm.N;
+        a.nwg_m = std::min(cdiv(cdiv(wm.N, 4), 4), 512);
+        lds = std::max(lds, B * vec_b<T>(wm.ld));
+      }
+      if (l.mixer == HY_LATENT) {
         const HyLatent& la = l.la;
         extra = B;
         a.latent = 1;
@@ -235,7 +264,7 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
         a.dims = la.dims;
       }
       TRY(with_nv<T>(Wp, [&](auto nv) {
-        return with_rp(f.on ? f.n_out() : 1, [&](auto rp) {
+        return with_rp(f.top ? f.n_out() : 1, [&](auto rp) {
           return go(k_ld_mid<T, B, decltype(nv)::value, decltype(rp)::value>, dim3(B * a.top * a.nwg_e + a.nwg_m + extra), 256, lds,
                     s, a);
         });
@@ -246,6 +275,19 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
       LdScanArgs a{st.xc, st.in, st.mid, mb.dt.w, mb.dt_b.p, mb.A2.p, mb.D.p, hy.state + r.st_off, st.v, hy.st_slot,
                    mb.inner, mb.state, mb.rankp, mb.innerp, mb.innerp, tb};
       TRY(launch_scan<T>(a, B, s));
+    } else if (heads) {
+      HeadsArgs a = heads_args(hy, ha, (const T*)m->kcache + r.kv_off);
+      a.raw = st.in;
+      a.raw_f32 = 1;
+      a.ldr = in_ld;
+      a.part = st.part;
+      a.nsplit = ha.nsplit;
+      a.p.seg_slot = tb.slot;
+      a.p.seg_pos0 = tb.pos;
+      TRY(heads_attn_launch<T>(s, a, B * cdiv(ha.H / ha.G, 16), 16));
+      LdMergeArgs mg{st.part, ha.gate ? st.in + ha.g_off() : nullptr, st.v, ha.H, ha.nsplit, ha.dvp, ha.dvr, in_ld, ha.o.ld,
+                     ha.span, tb.pos};
+      TRY(go(k_ld_merge, dim3(ha.H, B), 256, 256 * 16, s, mg));
     } else {
       const HyLatent& la = l.la;
       LdAbsorbArgs ab{st.mid, la.ukT.w, la.rope, st.Q, la.H, std::max(1, std::min(cdiv(la.Rp, 32), cdiv(512, la.H * B))),
@@ -271,14 +313,16 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
       TRY(go(k_ld_values<T>, dim3(la.H * va.nwg, B), 256, vec_b<T>(la.Rp) + 256 * 16 + (size_t)la.Rp * 4, s, va));
     }
     {
-      const HyMat& wo = mamba ? l.mb.o : l.la.o;
+      const HyMat& wo = l.out_mat();
       LdOutArgs a{};
       a.wo = wo.w;
       a.v = st.v;
       a.n4v = wo.ld / 4;
       a.ld = Wp;
-      a.ld_v = mamba ? l.mb.innerp : l.la.H * l.la.dvp;
+      a.ld_v = wo.ld;
       a.ldv = wo.ld;
+      a.bias = heads ? ha.o_b.p : nullptr;
+      a.mult = hy.c.mult;
       a.x_cur = x_cur;
       a.x_out = x_out;
       a.W = W;
@@ -289,25 +333,20 @@ int step(kh_model* m, const LdTabs tb, float* logits) {
         a.he = st.he;
         a.hs = st.hs;
         a.ids = st.ids;
-        a.id_w = st.id_w;
-        a.sh_g = st.sh_g;
+        a.id_w = f.ident ? st.id_w : nullptr;
+        a.sh_g = f.sgate ? st.sh_g : nullptr;
         a.xn2 = st.xn2;
         a.top = f.top;
         a.ffp = f.ffp;
         a.sffp = f.sffp;
       }
-      // waves of a row pair: as many as keep each wave's share within its two tiles and give every CU a workgroup, while
-      // the launch has at most four per CU
-      const int nblk = Ld<T>::blocks(wo.ld) + (f.on ? f.top * Ld<T>::blocks(f.ffp) + (f.sff ? Ld<T>::blocks(f.sffp) : 0) : 0);
-      a.ks = 1;
-      while (a.ks < 8 && nblk >= 2 * a.ks && (nblk / a.ks > 8 || cdiv(cdiv(W, 2) * a.ks, 8) < 256) &&
-             cdiv(cdiv(W, 2) * a.ks * 2, 8) <= 1024)
-        a.ks *= 2;
+      a.ks = split_waves(W, Ld<T>::blocks(wo.ld) + (f.on ? f.top * Ld<T>::blocks(f.ffp) + (f.sff ? Ld<T>::blocks(f.sffp) : 0) : 0));
       TRY(go(k_ld_out<T, B>, dim3(cdiv(cdiv(W, 2) * a.ks, 8)), 512, lds_out<T>(hy, l, B), s, a));
     }
     x_in = x_out;
   }
-  LdHeadArgs h{x_in, hy.fnorm.p, hy.fnorm_b.p, hy.head.w, logits, m->part_val, m->part_idx, W, Wp, hy.c.vocab, hy.c.eps, hy.c.cap};
+  LdHeadArgs h{x_in, hy.fnorm.p, hy.fnorm_b.p, hy.head.w, logits, m->part_val, m->part_idx, W, Wp, hy.c.vocab, hy.c.rms, hy.c.eps,
+               hy.c.cap};
   return with_nv<T>(Wp, [&](auto nv) { return go(k_ld_head<T, B, decltype(nv)::value>, dim3(st.head_wg), 256, B * vec_b<T>(Wp), s, h); });
 }
 template <class T>
@@ -328,22 +367,24 @@ int hy_step_init(kh_model* m) {
   for (int B : {1, 2, 4})
     if (hy.f32 ? fits<float>(hy, B) : fits<bf16>(hy, B)) st.bmax = B;
   const size_t B = KH_HY_DECODE_B, W = (size_t)hy.c.widthp;
-  size_t in = 1, xc = 1, mid = 1, v = 1, he = 1, hs = 1, z = 1, top = 1, Q = 1, part = 1;
+  size_t in = 1, xc = 1, mid = 1, v = 1, he = 1, hs = 1, z = 1, top = 1, Q = 1, part = 1, hpart = 1;
   auto up = [](size_t& a, size_t n) { a = a > n ? a : n; };
-  int hmin = 1 << 30;
   for (auto& l : hy.layers) {
     if (l.mixer == HY_MAMBA1) {
       up(in, 2 * (size_t)l.mb.inner);
       up(xc, (size_t)l.mb.innerp);
       up(mid, (size_t)l.mb.x.N);
       up(v, (size_t)l.mb.innerp);
+    } else if (l.mixer == HY_HEADS) {
+      up(in, (size_t)l.ha.qkvg.N);
+      up(v, (size_t)l.ha.o.ld);
+      up(hpart, (size_t)l.ha.H * (l.ha.dvp + 4) * l.ha.nsplit);
     } else {
       up(in, (size_t)l.la.dqkv.N);
       up(mid, (size_t)l.la.uq.N);
       up(v, (size_t)l.la.H * l.la.dvp);
       up(Q, (size_t)l.la.H * l.la.row());
       up(part, (size_t)l.la.H * (l.la.Rp + 4));
-      hmin = std::min(hmin, l.la.H);
     }
     if (l.ff.on) {
       up(he, (size_t)l.ff.top * l.ff.ffp);
@@ -369,7 +410,7 @@ int hy_step_init(kh_model* m) {
   TRY(f(&st.z, B * z));
   TRY(f(&st.id_w, B));
   TRY(f(&st.sh_g, B));
-  TRY(f(&st.part, B * part * (size_t)st.nsplit));
+  TRY(f(&st.part, B * std::max(part * (size_t)st.nsplit, hpart)));
   TRY(f(&st.logits, B * (size_t)hy.c.vocab));
   TRY(f((float**)&st.Q, B * Q));
   TRY(dalloc(&st.ids, B * top));
@@ -398,7 +439,11 @@ void hy_launch_step(kh_model* m, int advance, int n_forced) {
 }
 int hy_launches(const kh_model* m) {
   int n = 2;
-  for (const HyRun& r : m->hy->runs) n += m->hy->layers[(size_t)r.layer].mixer == HY_MAMBA1 ? 4 : 6;
+  for (const HyRun& r : m->hy->runs) {
+    const int mixer = m->hy->layers[(size_t)r.layer].mixer;
+    n += mixer == HY_MAMBA1 ? 4 : (mixer == HY_LATENT ? 6 : 5);
+    if (r.pass >= 0 && m->hy->enter.N) ++n;
+  }
   return n;
 }
 int hy_decode_max(const kh_model* m) { return m->hy->step_st->bmax; }

@@ -1,20 +1,24 @@
 // kh_ldecode.h — fused decode step of the layer-list models: B sequences (1, 2 or 4), one token each.
 //
-// Per layer   mixer mamba1: 4 launches      latent attention: 6 launches
-//   k_ld_in   layer norms -> LDS ; every projection that reads them: mixer input, router (+ shared gate row), shared
-//             expert gate / up with SwiGLU ; mamba x rows go through the convolution and silu in the epilogue
-//   k_ld_mid  router choice, chosen experts' gate / up ; mamba: W_x ; latent: W_uq behind its RMS norm, cache row
+// Per layer   mixer mamba1: 4 launches      latent attention: 6      attention over heads: 5
+//   k_ld_in   norms -> LDS ; every projection that reads them: mixer input (+ bias), router (+ shared gate row), dense
+//             or shared feed-forward's gate / up ; mamba x rows go through the convolution and silu in the epilogue
+//   k_ld_mid  router choice, chosen experts' gate / up ; mamba: W_x ; latent: W_uq behind its RMS norm, cache row ;
+//             heads: cache row
 //   mamba     k_ld_scan   dt projection, softplus, one step of the selective scan, gate
 //   latent    k_ld_absorb W_uk^T q per head, rotation ; k_latent_attn (time splits) ; k_ld_values merge + W_uv per head
-//   k_ld_out  W_o . v + experts' down + shared down + identity experts + residual, one dot product per row over a
-//             concatenation of weight rows
-// then k_ld_head (final norm, head, soft cap, argmax partials) and the sampler of kh_fused.h.
+//   heads     k_heads_attn (time splits) ; k_ld_merge merge and output gate
+//   k_ld_out  W_o . v (+ bias) + experts' down + shared down + identity experts, times the residual multiplier, +
+//             residual: one dot product per row over a concatenation of weight rows
+// A loop that enters through a matrix: k_ld_enter in front of each pass.  Then k_ld_head (final norm, head, soft cap,
+// argmax partials) and the sampler of kh_fused.h.
 //
 // GEMV core: a wave owns R rows.  A row is cut into BLOCKS of 64 x 16 bytes; U blocks of R rows are requested together
 // (non-temporal), and the first tile of a wave is requested before the input vectors are staged.  Vectors lie in LDS
 // as fp32, block by block, split into planes of four so that a lane's reads are consecutive 16-byte slots; their tails
 // are zeros, so the clamped weight loads of a tail lane contribute nothing.  Accumulation is fp32.
 #pragma once
+#include "kh_heads.h"
 #include "kh_hybrid.h"
 
 namespace khm {
@@ -56,13 +60,13 @@ __device__ __forceinline__ void ld_stage(f32x4* xs, const float* src, int n4, in
       if (i0 + j * NT < total4) xs[ld_slot<T>(i0 + j * NT)] = v[j] * g;
   }
 }
-// Layer norm of one row (256 threads, NV float4 each, rows padded with zeros to ld) into LDS slots.  v: the row in
-// registers; returns the normalised values in v (also written to `out` when given).  Mean and variance come from ONE
-// workgroup reduction of (x - shift) and (x - shift)^2, shift = an element of the row: no cancellation beyond the
-// distance of that element from the mean.  red: 2 KH_WAVES_MAX floats.
+// Layer norm (rms: RMS norm, shift 0) of one row (256 threads, NV float4 each, rows padded with zeros to ld) into LDS
+// slots.  v: the row in registers; returns the normalised values in v (also written to `out` when given).  Mean and
+// variance come from ONE workgroup reduction of (x - shift) and (x - shift)^2, shift = an element of the row: no
+// cancellation beyond the distance of that element from the mean.  red: 2 KH_WAVES_MAX floats.
 template <class T, int NV>
-__device__ __forceinline__ void ld_norm(f32x4 (&v)[NV], const f32x4 (&w)[NV], const f32x4 (&b)[NV], float shift, int W, int n4,
-                                        int total4, float eps, float* red, f32x4* xs, f32x4* out) {
+__device__ __forceinline__ void ld_norm(f32x4 (&v)[NV], const f32x4 (&w)[NV], const f32x4 (&b)[NV], float shift, bool rms, int W,
+                                        int n4, int total4, float eps, float* red, f32x4* xs, f32x4* out) {
   float s1 = 0.f, s2 = 0.f;
 #pragma unroll
   for (int j = 0; j < NV; ++j) {
@@ -84,7 +88,7 @@ __device__ __forceinline__ void ld_norm(f32x4 (&v)[NV], const f32x4 (&w)[NV], co
   __syncthreads();
   s1 = (red[0] + red[1]) + (red[2] + red[3]);
   s2 = (red[KH_WAVES_MAX] + red[KH_WAVES_MAX + 1]) + (red[KH_WAVES_MAX + 2] + red[KH_WAVES_MAX + 3]);
-  const float m = s1 / (float)W, mean = shift + m;
+  const float m = rms ? 0.f : s1 / (float)W, mean = rms ? 0.f : shift + m;
   const float var = fmaxf(s2 / (float)W - m * m, 0.f);
   const float rstd = 1.0f / sqrtf(var + eps);
 #pragma unroll
@@ -173,12 +177,25 @@ struct LdTabs {
   const int32_t *tok, *pos, *slot;  // [B]
 };
 
+// The embedding output of a token: scale * embed[token] + pos_emb[position] (pos_emb nullptr: none), rows of ld elements
+struct LdEmbed {
+  const void *embed, *pos_emb;
+  float scale;
+};
+template <class T>
+__device__ __forceinline__ f32x4 ld_embed(const LdEmbed& e, int tok, int pos, int ld, int i4) {
+  f32x4 v = quad_f((const T*)e.embed + (size_t)tok * ld + 4 * i4) * e.scale;
+  if (e.pos_emb) v += quad_f((const T*)e.pos_emb + (size_t)pos * ld + 4 * i4);
+  return v;
+}
+
 // ---- k_ld_in -----------------------------------------------------------------------------------------------------
-enum LdInKind { LDI_PLAIN = 0, LDI_CONV = 1, LDI_SWIGLU = 2 };
+enum LdInKind { LDI_PLAIN = 0, LDI_CONV = 1, LDI_GATED = 2 };
 struct LdInSeg {
   const void* w;
   float* out;      // [B][ldo]
-  int rows, ldo, kind, norm2;  // rows: weight rows (SWIGLU: output columns); norm2: input is the second norm
+  const float* bias;  // LDI_PLAIN: one per row, or nullptr
+  int rows, ldo, kind, norm2;  // rows: weight rows (GATED: output columns); norm2: input is the second norm
   int wg0, nwg;
 };
 struct LdInArgs {
@@ -186,12 +203,13 @@ struct LdInArgs {
   int nseg;
   const float* x_in;   // [B][ld]
   float* x_cur;        // written by workgroup 0 when the input is modified
-  const void* embed;
+  LdEmbed emb;
   const float* step;
-  const float *w1, *b1, *w2, *b2;
-  float* xn2;          // [B][ld], written by the router's first workgroup (nullptr: no feed-forward)
-  int W, ld, from_embed, add_x0;
+  const float *w1, *b1, *w2, *b2;  // b: nullptr with rms
+  float* xn2;          // [B][ld], written by the router's first workgroup (nullptr: nobody reads it)
+  int W, ld, from_embed, add_x0, rms;
   float eps;
+  GateAct act;
   LdTabs t;
   // LDI_CONV
   const float *conv_w, *conv_b;
@@ -219,8 +237,9 @@ __global__ __launch_bounds__(256) void k_ld_in(const LdInArgs a) {
   const int norm2 = si == 0 ? a.seg[0].norm2 : si == 1 ? a.seg[1].norm2 : a.seg[2].norm2;
   const int wg0 = si == 0 ? a.seg[0].wg0 : si == 1 ? a.seg[1].wg0 : a.seg[2].wg0;
   const int nwg = si == 0 ? a.seg[0].nwg : si == 1 ? a.seg[1].nwg : a.seg[2].nwg;
+  const float* bias = si == 0 ? a.seg[0].bias : si == 1 ? a.seg[1].bias : a.seg[2].bias;
   const int nblk = Ld<T>::blocks(a.ld), nch = a.ld / Ld<T>::E;
-  const int per = kind == LDI_SWIGLU ? R / 2 : R;  // outputs per item
+  const int per = kind == LDI_GATED ? R / 2 : R;  // outputs per item
   const int items = (rows + per - 1) / per;
   int item = (wg - wg0) * 4 + wave;
   const T* row[R];
@@ -228,7 +247,7 @@ __global__ __launch_bounds__(256) void k_ld_in(const LdInArgs a) {
 #pragma unroll
     for (int r = 0; r < R; ++r) {
       int i;
-      if (kind == LDI_SWIGLU) {
+      if (kind == LDI_GATED) {
         int j = it * 2 + (r & 1);
         j = j < rows ? j : rows - 1;
         i = (j >> 4) * 32 + (j & 15) + (r >> 1) * 16;
@@ -269,14 +288,13 @@ __global__ __launch_bounds__(256) void k_ld_in(const LdInArgs a) {
     f32x4 nw[NV], nb[NV], v[NV];
     const f32x4 *wp = (const f32x4*)(norm2 ? a.w2 : a.w1), *bp = (const f32x4*)(norm2 ? a.b2 : a.b1);
     auto get = [&](int q) __attribute__((always_inline)) {
-      const T* e = (const T*)a.embed + (size_t)a.t.tok[q] * a.ld;
 #pragma unroll
       for (int j = 0; j < NV; ++j) {
         const int i = threadIdx.x + 256 * j;
         v[j] = f4_zero();
         if (i < n4) {
-          v[j] = a.from_embed ? quad_f(e + 4 * i) : ((const f32x4*)(a.x_in + (size_t)q * a.ld))[i];
-          if (a.add_x0) v[j] += quad_f(e + 4 * i);
+          v[j] = a.from_embed ? ld_embed<T>(a.emb, a.t.tok[q], a.t.pos[q], a.ld, i) : ((const f32x4*)(a.x_in + (size_t)q * a.ld))[i];
+          if (a.add_x0) v[j] += ld_embed<T>(a.emb, a.t.tok[q], a.t.pos[q], a.ld, i);
           if (a.step) v[j] += ((const f32x4*)a.step)[i];
         }
       }
@@ -286,7 +304,7 @@ __global__ __launch_bounds__(256) void k_ld_in(const LdInArgs a) {
     for (int j = 0; j < NV; ++j) {
       const int i = threadIdx.x + 256 * j;
       nw[j] = i < n4 ? wp[i] : f4_zero();
-      nb[j] = i < n4 ? bp[i] : f4_zero();
+      nb[j] = bp && i < n4 ? bp[i] : f4_zero();
     }
     for (int q = 0; q < B; ++q) {
       if (q) get(q);
@@ -297,14 +315,20 @@ __global__ __launch_bounds__(256) void k_ld_in(const LdInArgs a) {
       }
       // the router's first workgroup leaves the second norm for the launches that follow
       f32x4* keep = a.xn2 && wg == a.seg[1].wg0 ? (f32x4*)(a.xn2 + (size_t)q * a.ld) : nullptr;
-      float shift = a.from_embed ? (float)((const T*)a.embed)[(size_t)a.t.tok[q] * a.ld] : a.x_in[(size_t)q * a.ld];
+      float shift = 0.f;
+      if (!a.rms) shift = a.from_embed ? (float)((const T*)a.emb.embed)[(size_t)a.t.tok[q] * a.ld] : a.x_in[(size_t)q * a.ld];
       if (q) __syncthreads();  // red is free again
-      ld_norm<T, NV>(v, nw, nb, shift, a.W, n4, total4, a.eps, red, (f32x4*)(xs + (size_t)q * xstride), keep);
+      ld_norm<T, NV>(v, nw, nb, shift, a.rms, a.W, n4, total4, a.eps, red, (f32x4*)(xs + (size_t)q * xstride), keep);
     }
   }
   __syncthreads();
   while (item < items) {
     float acc[R][B] = {};
+    float bi = 0.f;
+    if (bias && lane < R * B) {
+      const int i = item * R + (lane & (R - 1));
+      bi = bias[i < rows ? i : rows - 1];
+    }
     ld_rows<T, R, U, B>(t, row, nblk, nch, xs, xstride, lane, acc);
     const int cur = item;
     item += nwg * 4;
@@ -315,11 +339,11 @@ __global__ __launch_bounds__(256) void k_ld_in(const LdInArgs a) {
     ld_reduce<R, B>(acc);
     if (lane < R * B) {
       const int r = lane & (R - 1), q = lane / R;
-      if (kind == LDI_SWIGLU) {
+      if (kind == LDI_GATED) {
         const int j = cur * 2 + r;
         if (r < 2 && j < rows) {
           const float g = ld_pick<R, B>(acc, r, q), u = ld_pick<R, B>(acc, r + 2, q);
-          out[(size_t)q * ldo + j] = silu1(g) * u;
+          out[(size_t)q * ldo + j] = gated1(a.act, g, u);
         }
       } else {
         const int i = cur * R + r;
@@ -353,7 +377,7 @@ __global__ __launch_bounds__(256) void k_ld_in(const LdInArgs a) {
             if (a.taps > 1) st[(size_t)(a.taps - 2) * a.inner] = v;
             a.xc[(size_t)q * a.xc_ld + i] = silu1(c);
           } else {
-            out[(size_t)q * ldo + i] = v;
+            out[(size_t)q * ldo + i] = v + bi;
           }
         }
       }
@@ -370,15 +394,17 @@ struct LdMidArgs {
   float* he;             // [B][top][ffp], weighted
   int32_t* ids;          // [B][top] (-1: identity), written for k_ld_out
   float *id_w, *sh_g;    // [B]
-  int nwg_e, top, n_out, n_expert, shared, ffp, ldz, W, ldw;
+  int nwg_e, top, n_out, n_expert, shared, ffp, ldz, W, ldw, over_chosen;
+  GateAct act;
   // mixer: workgroups [.., + nwg_m)
   const void* wm;        // rows x ld
   const float* v;        // [B][ldv] input vectors (n valid entries)
   const float* vnorm;    // RMS norm weight (nullptr: none)
   float* om;             // [B][ldo]
   int nwg_m, rows, ldm, n, n4, ldv, ldo;  // n4: float4 of a row that may be read (no norm)
-  // cache rows of latent attention: the last B workgroups
-  int latent;
+  // cache rows: the last workgroups (latent attention: one per sequence; heads: one wave per key / value head)
+  int latent, heads;
+  HeadRow hr;
   const float* raw;      // [B][ldv]: q latent, kv latent, rotated part
   const float* kvn;
   const float2* rope;
@@ -412,7 +438,8 @@ __global__ __launch_bounds__(256) void k_ld_mid(const LdMidArgs a) {
     // every wave makes the choice for itself: its weight loads leave without a barrier
     float idw = 0.f, w = 0.f;
     int id = -1;
-    moe_route<RP>(a.z + (size_t)q * a.ldz, a.corr, a.n_out, a.top, lane, [&](int kk, int i, float wt) __attribute__((always_inline)) {
+    const float wf = moe_route<RP>(a.z + (size_t)q * a.ldz, a.corr, a.n_out, a.top, a.over_chosen, lane,
+                                   [&](int kk, int i, float wt) __attribute__((always_inline)) {
       const bool ident = i >= a.n_expert;
       if (ident) idw += wt;
       if (kk == k) {
@@ -420,6 +447,8 @@ __global__ __launch_bounds__(256) void k_ld_mid(const LdMidArgs a) {
         w = wt;
       }
     });
+    w *= wf;
+    idw *= wf;
     if (part == 0 && threadIdx.x == 0) {
       a.ids[q * a.top + k] = id;
       if (k == 0) {
@@ -458,7 +487,7 @@ __global__ __launch_bounds__(256) void k_ld_mid(const LdMidArgs a) {
       ld_reduce<R, 1>(acc);
       if (lane < 2) {
         const float g = ld_pick<R, 1>(acc, lane, 0), u = ld_pick<R, 1>(acc, lane + 2, 0);
-        a.he[(size_t)pair * a.ffp + cur * 2 + lane] = w * (silu1(g) * u);
+        a.he[(size_t)pair * a.ffp + cur * 2 + lane] = w * gated1(a.act, g, u);
       }
     }
     return;
@@ -513,6 +542,12 @@ __global__ __launch_bounds__(256) void k_ld_mid(const LdMidArgs a) {
     return;
   }
   wg -= a.nwg_m;
+  if (a.heads) {
+    const int i = wg * 4 + wave, q = i / a.hr.G, g = i - q * a.hr.G;
+    if (q < B)
+      heads_cache_row(a.hr, a.raw + (size_t)q * a.ldv, (T*)a.cache + (size_t)a.t.slot[q] * a.slot_elems, a.t.pos[q], g, lane);
+    return;
+  }
   if (!a.latent || wg >= B) return;  // ---- cache row of sequence wg
   const float* rr = a.raw + (size_t)wg * a.ldv + a.qr;
   const int pos = a.t.pos[wg];
@@ -633,6 +668,43 @@ __global__ __launch_bounds__(256) void k_ld_absorb(const LdAbsorbArgs a) {
   }
 }
 
+// Merge of the time splits of one head: p [splits][C + 4] (C columns, running maximum, sum); its ns filled splits meet in
+// sum [256 / (C / 4) groups][C / 4], summed over the groups by the caller.  Returns 1 / sum of the weights and, in grp, the
+// number of groups.  fac: one factor per split, ns <= 256
+__device__ __forceinline__ float ld_merge_splits(const float* p, int ns, int C, float* fac, float* red, f32x4* sum, int& grp) {
+  float m = -INFINITY;
+  for (int s = threadIdx.x; s < ns; s += 256) m = fmaxf(m, p[(size_t)s * (C + 4) + C]);
+  m = block_max(m, red);
+  float l = 0.f;
+  for (int s = threadIdx.x; s < ns; s += 256) {
+    const float* ps = p + (size_t)s * (C + 4) + C;
+    const float f = __builtin_amdgcn_exp2f(ps[0] - m);  // an empty split: exp2(-inf) = 0
+    fac[s] = f;
+    l = __builtin_fmaf(f, ps[1], l);
+  }
+  l = block_sum(l, red);
+  // column groups of four; 256 / (C / 4) thread groups share the splits and meet in LDS
+  const int c4 = C >> 2, g = (int)threadIdx.x / c4;
+  grp = c4 < 256 ? 256 / c4 : 1;
+  if (g < grp) {
+    for (int i = (int)threadIdx.x - g * c4; i < c4; i += 256) {
+      f32x4 v = f4_zero();
+      int s = g;
+      for (; s + 7 * grp < ns; s += 8 * grp) {
+        f32x4 x[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] = *(const f32x4*)(p + (size_t)(s + j * grp) * (C + 4) + 4 * i);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v = fma_s(fac[s + j * grp], x[j], v);
+      }
+      for (; s < ns; s += grp) v = fma_s(fac[s], *(const f32x4*)(p + (size_t)s * (C + 4) + 4 * i), v);
+      sum[g * c4 + i] = v;
+    }
+  }
+  __syncthreads();
+  return 1.0f / l;
+}
+
 // ---- k_ld_values: merge of the time splits, then W_uv of the head.  grid (H nwg, B) ----------------------------------
 struct LdValuesArgs {
   const float* part;  // [B H][nsplit][Rp + 4]
@@ -664,38 +736,10 @@ __global__ __launch_bounds__(256) void k_ld_values(const LdValuesArgs a) {
     set_rows(item);
     ld_load<T, R, U>(t, row, 0, nblk, nch, lane);
   }
-  const int ns = lat_active_splits(a.pos[b] + 1, a.nsplit);
-  float m = -INFINITY;
-  for (int s = threadIdx.x; s < ns; s += 256) m = fmaxf(m, p[(size_t)s * (a.Rp + 4) + a.Rp]);
-  m = block_max(m, red);
-  float l = 0.f;
-  for (int s = threadIdx.x; s < ns; s += 256) {
-    const float* ps = p + (size_t)s * (a.Rp + 4) + a.Rp;
-    const float f = __builtin_amdgcn_exp2f(ps[0] - m);  // an empty split: exp2(-inf) = 0
-    fac[s] = f;
-    l = __builtin_fmaf(f, ps[1], l);
-  }
-  l = block_sum(l, red);
-  const float inv = 1.0f / l;
-  // column groups of four; 256 / (Rp / 4) thread groups share the splits and meet in LDS
-  const int c4 = a.Rp >> 2, grp = c4 < 256 ? 256 / c4 : 1, g = (int)threadIdx.x / c4;
+  const int c4 = a.Rp >> 2;
   f32x4* sum = (f32x4*)(xs + (size_t)nblk * Ld<T>::BE);  // [grp][c4]
-  if (g < grp) {
-    for (int i = (int)threadIdx.x - g * c4; i < c4; i += 256) {
-      f32x4 v = f4_zero();
-      int s = g;
-      for (; s + 7 * grp < ns; s += 8 * grp) {
-        f32x4 x[8];
-#pragma unroll
-        for (int j = 0; j < 8; ++j) x[j] = *(const f32x4*)(p + (size_t)(s + j * grp) * (a.Rp + 4) + 4 * i);
-#pragma unroll
-        for (int j = 0; j < 8; ++j) v = fma_s(fac[s + j * grp], x[j], v);
-      }
-      for (; s < ns; s += grp) v = fma_s(fac[s], *(const f32x4*)(p + (size_t)s * (a.Rp + 4) + 4 * i), v);
-      sum[g * c4 + i] = v;
-    }
-  }
-  __syncthreads();
+  int grp;
+  const float inv = ld_merge_splits(p, lat_active_splits(a.pos[b] + 1, a.nsplit), a.Rp, fac, red, sum, grp);
   for (int i = threadIdx.x; i < nblk * Ld<T>::BE / 4; i += 256) {
     f32x4 v = f4_zero();
     if (i < c4)
@@ -717,6 +761,86 @@ __global__ __launch_bounds__(256) void k_ld_values(const LdValuesArgs a) {
   }
 }
 
+// ---- k_ld_merge: attention over heads: merge of the time splits, output gate.  grid (H, B) --------------------------
+struct LdMergeArgs {
+  const float* part;  // [B H][nsplit][C + 4]
+  const float* gate;  // [B][ldg]: logits head by head, gs apart (nullptr: none)
+  float* o;           // [B][ldo], heads gs apart
+  int H, nsplit, C, gs, ldg, ldo;
+  KeySpan span;
+  const int32_t* pos;
+};
+static __global__ __launch_bounds__(256) void k_ld_merge(const LdMergeArgs a) {
+  extern __shared__ __attribute__((aligned(16))) char smem_raw[];
+  f32x4* sum = (f32x4*)smem_raw;
+  __shared__ float fac[256];
+  __shared__ float red[KH_WAVES_MAX];
+  const int b = blockIdx.y, h = blockIdx.x, pos = a.pos[b], i = (int)threadIdx.x, c4 = a.C >> 2;
+  f32x4 g = f4_zero();
+  const bool live = 4 * i < a.gs;
+  if (a.gate && live) g = *(const f32x4*)(a.gate + (size_t)b * a.ldg + (size_t)h * a.gs + 4 * i);
+  int grp;
+  const float inv = ld_merge_splits(a.part + ((size_t)b * a.H + h) * a.nsplit * (size_t)(a.C + 4),
+                                    lat_active_splits(pos + 1 - a.span.first(pos), a.nsplit), a.C, fac, red, sum, grp);
+  if (!live) return;
+  f32x4 v = f4_zero();
+  for (int k = 0; k < grp; ++k) v += sum[k * c4 + i];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) v[j] *= a.gate ? inv * sigmoid1(g[j]) : inv;
+  *(f32x4*)(a.o + (size_t)b * a.ldo + (size_t)h * a.gs + 4 * i) = v;
+}
+
+// ---- k_ld_enter: x_out = W [x ; embedding output], a pass of a loop that enters through a matrix --------------------
+struct LdEnterArgs {
+  const void* w;      // [W][2 ld]
+  const float* x;     // [B][ld] (nullptr: the embedding output itself)
+  float* x_out;       // [B][ld]
+  LdEmbed emb;
+  int W, ld, ks;
+  LdTabs t;
+};
+// Workgroup = 8 waves = 8 / ks groups of ks waves; a group owns R rows, its waves share the blocks.
+template <class T, int B>
+__global__ __launch_bounds__(512) void k_ld_enter(const LdEnterArgs a) {
+  constexpr int R = 2, U = 4, BE = Ld<T>::BE;
+  extern __shared__ __attribute__((aligned(16))) char smem_raw[];
+  float* xs = (float*)smem_raw;
+  __shared__ float comb[8][R * B];
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int K = 2 * a.ld, nblk = Ld<T>::blocks(K), nch = K / Ld<T>::E, n4 = a.ld >> 2;
+  const int kp = wave % a.ks, item = ((int)blockIdx.x * (8 / a.ks) + wave / a.ks) * R;
+  const int per = (nblk + a.ks - 1) / a.ks, b0 = kp * per, b1 = b0 + per < nblk ? b0 + per : nblk;
+  const T* row[R];
+#pragma unroll
+  for (int r = 0; r < R; ++r) row[r] = (const T*)a.w + (size_t)(item + r < a.W ? item + r : a.W - 1) * K;
+  LdTile<T, R, U> t;
+  ld_load<T, R, U>(t, row, b0, b1, nch, lane);
+  for (int q = 0; q < B; ++q) {
+    f32x4* xq = (f32x4*)(xs + (size_t)q * nblk * BE);
+    for (int i = threadIdx.x; i < nblk * BE / 4; i += 512) {
+      f32x4 v = f4_zero();
+      if (i < n4 && a.x) v = ((const f32x4*)(a.x + (size_t)q * a.ld))[i];
+      else if (i < 2 * n4) v = ld_embed<T>(a.emb, a.t.tok[q], a.t.pos[q], a.ld, i < n4 ? i : i - n4);
+      xq[ld_slot<T>(i)] = v;
+    }
+  }
+  __syncthreads();
+  float acc[R][B] = {};
+  for (int b = b0; b < b1; b += U) {
+    if (b != b0) ld_load<T, R, U>(t, row, b, b1, nch, lane);
+    ld_fma<T, R, U, B>(t, xs, nblk * BE, b, b1, lane, acc);
+  }
+  ld_reduce<R, B>(acc);
+  if (lane < R * B) comb[wave][lane] = ld_pick<R, B>(acc, lane & (R - 1), lane / R);
+  __syncthreads();
+  if (kp == 0 && lane < R * B) {
+    float v = 0.f;
+    for (int k = 0; k < a.ks; ++k) v += comb[wave + k][lane];
+    const int q = lane / R, i = item + (lane & (R - 1));
+    if (i < a.W) a.x_out[(size_t)q * a.ld + i] = v;
+  }
+}
+
 // ---- k_ld_out ----------------------------------------------------------------------------------------------------
 struct LdOutArgs {
   const void* wo;         // [W][ldv]
@@ -724,9 +848,11 @@ struct LdOutArgs {
   const void *down, *sdown;  // experts [W][ffp] each; shared [W][sffp]
   const float *he, *hs;   // [B][top][ffp] (weighted), [B][sffp]
   const int32_t* ids;     // [B][top]
-  const float *id_w, *sh_g, *xn2, *x_cur;
+  const float *id_w, *sh_g, *xn2, *x_cur;  // id_w, sh_g: nullptr = none, 1
+  const float* bias;      // of W_o, or nullptr
   float* x_out;           // [B][ld]
   int W, ld, n4v, ld_v, ldv, top, ffp, sffp, moe, ks;
+  float mult;             // of everything that is added to the residual
 };
 // Workgroup = 8 waves = 8 / ks groups of ks waves; a group owns R rows, its waves share the blocks of the concatenation
 // [mixer | shared | expert 0 | expert 1 ...] (blocks of identity experts are skipped).  Experts differ between
@@ -741,7 +867,7 @@ __global__ __launch_bounds__(512) void k_ld_out(const LdOutArgs a) {
   __shared__ float comb[8][R * B];
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int nbv = Ld<T>::blocks(a.ldv);
-  const int nbe = a.moe ? Ld<T>::blocks(a.ffp) : 1, nbs = a.moe && a.sffp ? Ld<T>::blocks(a.sffp) : 0;
+  const int nbe = a.moe && a.top ? Ld<T>::blocks(a.ffp) : 1, nbs = a.moe && a.sffp ? Ld<T>::blocks(a.sffp) : 0;
   const int nb = nbv + nbs + (a.moe ? a.top * nbe : 0);
   float* xv = (float*)smem_raw;
   float* xf = xv + (size_t)B * nbv * BE;
@@ -751,12 +877,13 @@ __global__ __launch_bounds__(512) void k_ld_out(const LdOutArgs a) {
 #pragma unroll
   for (int r = 0; r < R; ++r) ri[r] = item + r < a.W ? item + r : a.W - 1;
   // residual operands of the rows this wave will finish
-  float rx = 0.f, rn = 0.f, rw = 0.f;
+  float rx = 0.f, rn = 0.f, rw = 0.f, rb = 0.f;
   if (kp == 0 && lane < R * B) {
     const int q = lane / R, i = item + (lane & (R - 1));
     if (i < a.W) {
       rx = a.x_cur[(size_t)q * a.ld + i];
-      if (a.moe) {
+      if (a.bias) rb = a.bias[i];
+      if (a.id_w) {
         rn = a.xn2[(size_t)q * a.ld + i];
         rw = a.id_w[q];
       }
@@ -808,7 +935,8 @@ __global__ __launch_bounds__(512) void k_ld_out(const LdOutArgs a) {
       __syncthreads();  // the feed-forward vectors of the sequence before have been consumed
     }
     if (a.moe) {
-      if (nbs) ld_stage<T, 512>((f32x4*)xf, a.hs + (size_t)q * a.sffp, a.sffp >> 2, nbs * BE / 4, a.sh_g[q], threadIdx.x);
+      if (nbs) ld_stage<T, 512>((f32x4*)xf, a.hs + (size_t)q * a.sffp, a.sffp >> 2, nbs * BE / 4, a.sh_g ? a.sh_g[q] : 1.f,
+                                 threadIdx.x);
       for (int k = 0; k < a.top; ++k)
         ld_stage<T, 512>((f32x4*)(xf + (size_t)(nbs + k * nbe) * BE), a.he + (size_t)(q * a.top + k) * a.ffp, a.ffp >> 2,
                          nbe * BE / 4, 1.f, threadIdx.x);
@@ -846,19 +974,19 @@ __global__ __launch_bounds__(512) void k_ld_out(const LdOutArgs a) {
     float v = 0.f;
     for (int k = 0; k < a.ks; ++k) v += comb[wave + k][lane];
     const int q = lane / R, i = item + (lane & (R - 1));
-    if (i < a.W) a.x_out[(size_t)q * a.ld + i] = rx + __builtin_fmaf(rw, rn, v);
+    if (i < a.W) a.x_out[(size_t)q * a.ld + i] = __builtin_fmaf(a.mult, __builtin_fmaf(rw, rn, v) + rb, rx);
   }
 }
 
 // ---- k_ld_head ---------------------------------------------------------------------------------------------------
 struct LdHeadArgs {
   const float* x;        // [B][ld]
-  const float *w, *b;    // final norm
+  const float *w, *b;    // final norm (rms: b may be nullptr)
   const void* head;      // [V][ld]
   float* logits;         // [B][V]
   float* part_val;       // argmax partials of sequence 0 (nullptr: none)
   int32_t* part_idx;
-  int W, ld, V;
+  int W, ld, V, rms;
   float eps, cap;
 };
 template <class T, int B, int NV>
@@ -894,7 +1022,7 @@ __global__ __launch_bounds__(256) void k_ld_head(const LdHeadArgs a) {
     for (int j = 0; j < NV; ++j) {
       const int i = threadIdx.x + 256 * j;
       nw[j] = i < n4 ? ((const f32x4*)a.w)[i] : f4_zero();
-      nb[j] = i < n4 ? ((const f32x4*)a.b)[i] : f4_zero();
+      nb[j] = a.b && i < n4 ? ((const f32x4*)a.b)[i] : f4_zero();
     }
     for (int q = 0; q < B; ++q) {
 #pragma unroll
@@ -903,7 +1031,7 @@ __global__ __launch_bounds__(256) void k_ld_head(const LdHeadArgs a) {
         v[j] = i < n4 ? ((const f32x4*)(a.x + (size_t)q * a.ld))[i] : f4_zero();
       }
       if (q) __syncthreads();
-      ld_norm<T, NV>(v, nw, nb, a.x[(size_t)q * a.ld], a.W, n4, xstride >> 2, a.eps, red, (f32x4*)(xs + (size_t)q * xstride), nullptr);
+      ld_norm<T, NV>(v, nw, nb, a.rms ? 0.f : a.x[(size_t)q * a.ld], a.rms, a.W, n4, xstride >> 2, a.eps, red, (f32x4*)(xs + (size_t)q * xstride), nullptr);
     }
   }
   __syncthreads();

@@ -26,10 +26,10 @@
 namespace khm {
 
 enum LgEpi {
-  LG_T = 0,        // out T
-  LG_F32 = 1,      // out fp32
+  LG_T = 0,        // out T (+ bias)
+  LG_F32 = 1,      // out fp32 (+ bias)
   LG_SOFTPLUS = 2, // out fp32 = softplus(acc + bias[feature])
-  LG_SWIGLU = 3,   // weight rows come as 16 gate rows, 16 up rows, ...: out T = silu(gate) * up, half the features
+  LG_GATED = 3,    // weight rows come as 16 gate rows, 16 up rows, ...: out T = the gated unit, half the features
   LG_SPLIT = 4,    // features [0, n_split) -> out T, the rest -> out2 fp32
   LG_SOFTCAP = 5,  // out fp32 = cap * tanh(acc / cap); cap 0: plain
 };
@@ -43,7 +43,7 @@ struct LgArgs {
   const void* X;        // [M][ldx]
   void* out;            // [M][ldo]
   float* out2;          // LG_SPLIT: [M][ldo2]
-  const float* bias;    // LG_SOFTPLUS
+  const float* bias;    // LG_SOFTPLUS; LG_T / LG_F32: optional
   const int32_t* gather;   // row of X for row m (grouped, optional)
   const LgTile* tiles;     // grouped launch
   const int32_t* n_tiles;  // number of valid entries of tiles
@@ -51,6 +51,7 @@ struct LgArgs {
   size_t w_z, x_z, o_z; // batched: elements per blockIdx.z
   int M, N, K, ldw, ldx, ldo, ldo2, n_split;
   float cap;
+  GateAct act;          // LG_GATED
 };
 
 template <class T, int BM, int BN>
@@ -173,21 +174,25 @@ __global__ __launch_bounds__(256) void k_lgemm(const LgArgs a) {
   for (int m = 0; m < TM; ++m) {
     const int tok = mt0 + wm * (BM / 2) + m * 16 + fr;
     if (tok > m_last) continue;
-    if (EPI == LG_SWIGLU) {
+    if (EPI == LG_GATED) {
 #pragma unroll
       for (int n = 0; n + 1 < TN; n += 2) {
         const int f = f0 + wn * (BN / 2) + n * 16;  // a multiple of 32: gate tile; the up tile follows
         const int c = (f >> 1) + 4 * fh;
         f32x4 v;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = silu1(acc[n][m][i]) * acc[n + 1][m][i];
+        for (int i = 0; i < 4; ++i) v[i] = gated1(a.act, acc[n][m][i], acc[n + 1][m][i]);
         if (f < a.N) *(typename TL::quad*)((T*)a.out + (size_t)tok * a.ldo + c) = to_quad<T>(v);
       }
     } else {
 #pragma unroll
       for (int n = 0; n < TN; ++n) {
         const int f = f0 + wn * (BN / 2) + n * 16 + 4 * fh;
-        const f32x4 v = acc[n][m];
+        f32x4 v = acc[n][m];
+        if ((EPI == LG_T || EPI == LG_F32) && a.bias) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) v[i] += a.bias[f + i < a.N ? f + i : 0];
+        }
         if (EPI == LG_T) {
           T* o = (T*)a.out + (size_t)blockIdx.z * a.o_z + (size_t)tok * a.ldo + f;
           if (f + 3 < a.N && (a.ldo & 3) == 0) {
@@ -198,7 +203,7 @@ __global__ __launch_bounds__(256) void k_lgemm(const LgArgs a) {
               if (f + i < a.N) o[i] = (T)v[i];
           }
         } else {
-f32x4 y = v;
+          f32x4 y = v;
           if (EPI == LG_SOFTPLUS) {
 #pragma unroll
             for (int i = 0; i < 4; ++i) y[i] = softplus1(v[i] + a.bias[f + i < a.N ? f + i : 0]);

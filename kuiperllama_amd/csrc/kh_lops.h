@@ -1,5 +1,5 @@
-// kh_lops.h — per-token kernels of the layer-list models: embedding, the residual update fused with the two layer
-// norms of a parallel block, the causal convolution.  Everything that touches the residual stream is fp32.
+// kh_lops.h — per-token kernels of the layer-list models: embedding, the residual update fused with the one or two norms
+// of a parallel block (layer norm or RMS norm), the causal convolution.  Everything that touches the residual stream is fp32.
 #pragma once
 #include "kh_tile.h"
 
@@ -21,24 +21,26 @@ struct AddArgs {
   const float* y_w;       // [T][top]
   const float* id_w;      // [T]
   const T* sh;            // [T][ld] shared expert's output
-  const float* sh_g;      // [T] its gate
+  const float* sh_g;      // [T] its gate (nullptr: 1)
   int top;
 };
 
-// One workgroup per token.  x += pending; (loop entry) x += x0, x += step; then xn1 / xn2 = layer norms of x.
+// One workgroup per token.  x += mult * pending; (loop entry) x += x0, x += step; then xn1 / xn2 = norms of x, or
+// cat = [x | x0] for a loop that enters through a matrix.  The embedding output is scale * embed[token] + pos[position].
 // Rows of every array are ld (a multiple of KH_LPAD) elements with zeros behind the W valid ones.
 template <class T>
 struct CombineArgs {
   float *x, *x0;
   AddArgs<T> add;
-  const T* embed;
-  const int32_t* tok;
+  const T *embed, *pos_emb;                // pos_emb nullptr: none
+  const int32_t *tok, *pos;
   const float* step;                       // one row or nullptr
   const float *w1, *b1, *w2, *b2;          // norm parameters (w1 nullptr: no norm output)
   T *xn1, *xn2;
+  T* cat;                                  // [T][2 ld] or nullptr
   const T* xn2_prev;                       // identity experts' input: the xn2 the pending layer read
-  int W, ld, from_embed, add_x0;
-  float eps;
+  int W, ld, from_embed, add_x0, rms;      // rms: no mean, biases may be nullptr
+  float eps, mult, emb_scale;
 };
 template <class T>
 __device__ __forceinline__ f32x4 quad_f(const T* p) {
@@ -60,43 +62,43 @@ __global__ __launch_bounds__(256) void k_combine(const CombineArgs<T> a) {
   const size_t o = (size_t)t * a.ld;
   float s = 0.f;
   const T* e = a.from_embed ? a.embed + (size_t)a.tok[t] * a.ld : nullptr;
-  float idw = 0.f, shg = 0.f;
+  const T* ep = a.from_embed && a.pos_emb ? a.pos_emb + (size_t)a.pos[t] * a.ld : nullptr;
+  const float idw = a.add.y && a.add.id_w ? a.add.id_w[t] : 0.f, shg = a.add.sh && a.add.sh_g ? a.add.sh_g[t] : 1.f;
   const int top = a.add.y ? a.add.top : 0;
-  if (a.add.y) {
-    idw = a.add.id_w[t];
-    shg = a.add.sh ? a.add.sh_g[t] : 0.f;
-  }
   for (int i = threadIdx.x; i < n4; i += 256) {
     const int c = 4 * i;
     f32x4 v;
     if (a.from_embed) {
-      v = quad_f(e + c);
+      v = quad_f(e + c) * a.emb_scale;
+      if (ep) v += quad_f(ep + c);
       *(f32x4*)(a.x0 + o + c) = v;
     } else {
       v = *(const f32x4*)(a.x + o + c);
     }
     if (a.add.mix) {
       f32x4 d = *(const f32x4*)(a.add.mix + o + c);
-      if (a.add.y) {
-        f32x4 f = {0.f, 0.f, 0.f, 0.f};
-        for (int k = 0; k < top; ++k) {
-          const int sl = a.add.y_slot[(size_t)t * top + k];
-          if (sl >= 0) f = fma_s(a.add.y_w[(size_t)t * top + k], quad_f(a.add.y + (size_t)sl * a.ld + c), f);
-        }
-        if (idw != 0.f) f = fma_s(idw, quad_f(a.xn2_prev + o + c), f);
-        if (a.add.sh) f = fma_s(shg, quad_f(a.add.sh + o + c), f);
-        d += f;
+      f32x4 f = {0.f, 0.f, 0.f, 0.f};
+      for (int k = 0; k < top; ++k) {
+        const int sl = a.add.y_slot[(size_t)t * top + k];
+        if (sl >= 0) f = fma_s(a.add.y_w[(size_t)t * top + k], quad_f(a.add.y + (size_t)sl * a.ld + c), f);
       }
-      v += d;
+      if (idw != 0.f) f = fma_s(idw, quad_f(a.xn2_prev + o + c), f);
+      if (a.add.sh) f = fma_s(shg, quad_f(a.add.sh + o + c), f);
+      d += f;
+      v = fma_s(a.mult, d, v);
     }
     if (a.add_x0) v += *(const f32x4*)(a.x0 + o + c);
     if (a.step) v += *(const f32x4*)(a.step + c);
     *(f32x4*)(a.x + o + c) = v;
+    if (a.cat) {
+      *(typename Tile<T>::quad*)(a.cat + 2 * o + c) = to_quad<T>(v);
+      *(typename Tile<T>::quad*)(a.cat + 2 * o + a.ld + c) = to_quad<T>(a.from_embed ? v : *(const f32x4*)(a.x0 + o + c));
+    }
     row[i] = v;
     s += (v.x + v.y) + (v.z + v.w);
   }
   if (!a.w1) return;
-  const float mean = block_sum(s, red) / (float)a.W;
+  const float mean = a.rms ? 0.f : block_sum(s, red) / (float)a.W;
   float q = 0.f;
   for (int i = threadIdx.x; i < n4; i += 256) {
     const f32x4 v = row[i];
@@ -111,12 +113,13 @@ __global__ __launch_bounds__(256) void k_combine(const CombineArgs<T> a) {
     const int c = 4 * i;
     const f32x4 v = row[i];
     f32x4 y;
-    const f32x4 w1 = *(const f32x4*)(a.w1 + c), b1 = *(const f32x4*)(a.b1 + c);
+    const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+    const f32x4 w1 = *(const f32x4*)(a.w1 + c), b1 = a.b1 ? *(const f32x4*)(a.b1 + c) : zero;
 #pragma unroll
     for (int k = 0; k < 4; ++k) y[k] = (v[k] - mean) * rstd * w1[k] + b1[k];  // pads: weights and biases are zero
     *(typename Tile<T>::quad*)(a.xn1 + o + c) = to_quad<T>(y);
     if (a.w2) {
-      const f32x4 w2 = *(const f32x4*)(a.w2 + c), b2 = *(const f32x4*)(a.b2 + c);
+      const f32x4 w2 = *(const f32x4*)(a.w2 + c), b2 = a.b2 ? *(const f32x4*)(a.b2 + c) : zero;
 #pragma unroll
       for (int k = 0; k < 4; ++k) y[k] = (v[k] - mean) * rstd * w2[k] + b2[k];
       *(typename Tile<T>::quad*)(a.xn2 + o + c) = to_quad<T>(y);
@@ -124,15 +127,15 @@ __global__ __launch_bounds__(256) void k_combine(const CombineArgs<T> a) {
   }
 }
 
-// layer norm of gathered rows: out[r] = norm(x[rows[r]]); rows of ld elements on both sides
+// norm of gathered rows: out[r] = norm(x[rows[r]]); rows of ld elements on both sides.  rms: no mean, b may be nullptr
 template <class T>
 __global__ __launch_bounds__(256) void k_gather_norm(const float* x, const int32_t* rows, const float* w, const float* b,
-                                                     T* out, int W, int ld, float eps) {
+                                                     T* out, int W, int ld, float eps, int rms) {
   __shared__ float red[KH_WAVES_MAX];
   const float* r = x + (size_t)rows[blockIdx.x] * ld;
   float s = 0.f;
   for (int i = threadIdx.x; i < W; i += 256) s += r[i];
-  const float mean = block_sum(s, red) / (float)W;
+  const float mean = rms ? 0.f : block_sum(s, red) / (float)W;
   float q = 0.f;
   for (int i = threadIdx.x; i < W; i += 256) {
     const float d = r[i] - mean;
@@ -140,7 +143,7 @@ __global__ __launch_bounds__(256) void k_gather_norm(const float* x, const int32
   }
   const float rstd = 1.0f / sqrtf(block_sum(q, red) / (float)W + eps);
   for (int i = threadIdx.x; i < W; i += 256)
-    out[(size_t)blockIdx.x * ld + i] = (T)((r[i] - mean) * rstd * w[i] + b[i]);
+    out[(size_t)blockIdx.x * ld + i] = (T)((r[i] - mean) * rstd * w[i] + (b ? b[i] : 0.f));
 }
 
 // ---- causal depthwise convolution + silu -----------------------------------------------------------------------

@@ -1,6 +1,9 @@
 // kh_moe.h — expert router and dispatch lists.
-// Scores s = softmax(z) over all router outputs (fp32); the `top` largest s + correction are chosen, ties to the lower
-// index; the weights are the chosen s.  Outputs from n_expert on are identity experts (no tensors).
+// Two forms, both fp32, ties to the lower index:
+//   over all     scores s = softmax(z) over all router outputs; the `top` largest s + correction are chosen; the weights
+//                are the chosen s
+//   over chosen  the `top` largest z are chosen; the weights are the softmax over them alone
+// Outputs from n_expert on are identity experts (no tensors).
 #pragma once
 #include "kh_lgemm.h"
 
@@ -10,31 +13,37 @@
 namespace khm {
 
 // The choice for one token by one wave; z in LDS or global [n_out], n_out <= 64 PER.  Calls pick(k, id, weight) for
-// k = 0 .. top - 1 on every lane with wave-uniform values, in order of decreasing choice score.
+// k = 0 .. top - 1 on every lane with wave-uniform values, in order of decreasing choice score.  Weights are to be
+// multiplied by the returned factor.  corr nullptr: none.
 template <int PER, class F>
-__device__ __forceinline__ void moe_route(const float* z, const float* corr, int n_out, int top, int lane, F&& pick) {
+__device__ __forceinline__ float moe_route(const float* z, const float* corr, int n_out, int top, bool over_chosen, int lane,
+                                           F&& pick) {
   float s[PER], key[PER];
   float m = -INFINITY;
 #pragma unroll
   for (int j = 0; j < PER; ++j) {
     const int i = j * 64 + lane;
     s[j] = i < n_out ? z[i] : -INFINITY;
-    key[j] = i < n_out ? corr[i] : 0.f;
+    key[j] = corr && i < n_out ? corr[i] : 0.f;
     m = fmaxf(m, s[j]);
   }
   m = wave_max(m);
   float sum = 0.f;
 #pragma unroll
   for (int j = 0; j < PER; ++j) {
+    if (over_chosen) key[j] = s[j];
     s[j] = expf(s[j] - m);  // exp(-inf) = 0 beyond n_out
     sum += s[j];
   }
-  sum = wave_sum(sum);
+  if (!over_chosen) {
+    sum = wave_sum(sum);
 #pragma unroll
-  for (int j = 0; j < PER; ++j) {
-    s[j] /= sum;
-    key[j] = j * 64 + lane < n_out ? s[j] + key[j] : -INFINITY;
+    for (int j = 0; j < PER; ++j) {
+      s[j] /= sum;
+      key[j] = j * 64 + lane < n_out ? s[j] + key[j] : -INFINITY;
+    }
   }
+  float chosen = 0.f;
   for (int k = 0; k < top; ++k) {
     float v = key[0];
 #pragma unroll
@@ -53,34 +62,39 @@ __device__ __forceinline__ void moe_route(const float* z, const float* corr, int
       key[j] = mine ? -INFINITY : key[j];
     }
     w = wave_sum(w);  // one lane holds it, the others zero
+    chosen += w;
     pick(k, __builtin_amdgcn_readfirstlane(id), w);
   }
+  return over_chosen ? 1.0f / chosen : 1.0f;  // the largest z contributes exp(0)
 }
 
 struct RouteArgs {
   const float* z;        // [T][ldz]: router outputs, then (shared expert) its gate logit
-  const float* corr;     // [n_out]
+  const float* corr;     // [n_out] or nullptr
   int32_t* id;           // [T][top]
   float* w;              // [T][top]
   float* id_w;           // [T] summed weight of the chosen identity experts
   float* sh_g;           // [T] sigmoid of the shared expert's gate
-  int T, ldz, n_out, n_expert, top, shared;
+  int T, ldz, n_out, n_expert, top, shared, over_chosen;
 };
 template <int PER>
 __global__ __launch_bounds__(256) void k_moe_route(const RouteArgs a) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= a.T) return;
   const float* z = a.z + (size_t)t * a.ldz;
-  float idw = 0.f;
-  moe_route<PER>(z, a.corr, a.n_out, a.top, lane, [&](int k, int id, float w) __attribute__((always_inline)) {
+  float idw = 0.f, my_w = 0.f;
+  int my_id = 0;
+  const float f = moe_route<PER>(z, a.corr, a.n_out, a.top, a.over_chosen, lane, [&](int k, int id, float w) __attribute__((always_inline)) {
     if (id >= a.n_expert) idw += w;
-    if (lane == 0) {
-      a.id[(size_t)t * a.top + k] = id;
-      a.w[(size_t)t * a.top + k] = w;
-    }
+    my_id = lane == k ? id : my_id;  // top <= KH_MOE_MAX_TOP < 64: lane k keeps choice k
+    my_w = lane == k ? w : my_w;
   });
+  if (lane < a.top) {
+    a.id[(size_t)t * a.top + lane] = my_id;
+    a.w[(size_t)t * a.top + lane] = my_w * f;
+  }
   if (lane == 0) {
-    a.id_w[t] = idw;
+    a.id_w[t] = idw * f;
     if (a.shared) a.sh_g[t] = sigmoid1(z[a.n_out]);
   }
 }

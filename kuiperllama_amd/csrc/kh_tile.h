@@ -49,6 +49,16 @@ __device__ __forceinline__ typename Tile<T>::quad to_quad(f32x4 v) {
 
 __device__ __forceinline__ float sigmoid1(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu1(float z) { return z * sigmoid1(z); }
+// Gated unit of a feed-forward: gate times sigmoid(alpha gate) times (up + shift), both sides limited first.  SwiGLU is
+// {INFINITY, 1, 0}.
+struct GateAct {
+  float limit, alpha, shift;
+};
+__device__ __forceinline__ float gated1(const GateAct& c, float g, float u) {
+  g = fminf(g, c.limit);
+  u = fminf(fmaxf(u, -c.limit), c.limit);
+  return g * sigmoid1(c.alpha * g) * (u + c.shift);
+}
 // log(1 + e^z) without overflow
 __device__ __forceinline__ float softplus1(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 }  // namespace khm
