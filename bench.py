@@ -766,8 +766,18 @@ def assemble_line(spec, args, world, res, secondary, others, skipped, timing_bac
 
 
 # ---- layer-list models (--layers) ------------------------------------------------------------------------------------
-def layers_config(width: int, n_layers: int, vocab: int = 32000) -> dict:
-    """A Gufanex configuration with layers of a real model's proportions: mixers alternate, experts of half a width."""
+def layers_config(width: int, n_layers: int, vocab: int = 32000, arch: str = "Gufanex") -> dict:
+    """A configuration with layers of a real model's proportions: mixers alternate, experts of half a width."""
+    if arch == "Gusorax":
+        heads = width // 128
+        common = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5}
+        window = dict(common, mask={"size": 1024}, bias_max=512)
+        chunk = dict(common, mask={"size": 2048})
+        moe = {"kind": "moe", "expert": {"ff": width // 2, "limit": 7.0}, "router": {"experts": 32, "top": 7}}
+        return {"architecture": arch, "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "residual_mult": 0.5,
+                "embedding": {"scale": float(width) ** 0.5}, "max_positions": 4352,
+                "layers": [{"type": "attention_2" if i % 2 else "attention", "mixer": chunk if i % 2 else window,
+                            "mlp": {"kind": "dense", "ff": 7 * width // 2} if i == 0 else moe} for i in range(n_layers)]}
     ff, sff = width // 2, width
     mlp = {"kind": "moe", "expert": {"ff": ff}, "shared": {"ff": sff},
            "router": {"experts": 32, "identity": 4, "top": 6}}
@@ -789,7 +799,7 @@ def layers_tensors(cfg: dict, seed: int = 0) -> dict:
     rng_cfg = checkpoint.tensor_shapes(cfg)
     for k, sh in rng_cfg.items():
         if len(sh) == 2 and sh[0] * sh[1] > 1 << 16 and not k.endswith("A_log"):
-            sc = 1.0 if k == "embed" else sh[1] ** -0.5
+            sc = 1.0 / cfg.get("embedding", {}).get("scale", 1.0) if k == "embed" else sh[1] ** -0.5
             w = torch.randn(sh, device="cuda", generator=gen) * sc
             small[k] = w.to(torch.bfloat16).view(torch.int16).cpu().numpy().view(np.uint16)
         else:
@@ -804,45 +814,51 @@ def layers_work(cfg: dict) -> tuple:
     from kuiperllama_amd import checkpoint
     active, prompt, last = 0.0, 0.0, len(cfg["layers"]) - 1
     for k, sh in checkpoint.tensor_shapes(cfg).items():
-        if len(sh) != 2 or not k.startswith("l") or k == "loop.step" or k.endswith(("A_log", "conv")):
+        if len(sh) != 2 or not k.startswith("l") or k.startswith("loop") or k.endswith(("A_log", "conv", ".rel")):
             continue
         layer = int(k[1:k.index(".")])
         n = float(sh[0] * sh[1])
         if ".mlp.e" in k:
             r = cfg["layers"][layer]["mlp"]["router"]
-            n *= r["top"] / (r["experts"] + r["identity"])
+            n *= r["top"] / (r["experts"] + r.get("identity", 0))
         active += n
-        if layer < last or k.endswith((".mix.in", ".mix.x", ".mix.dt", ".mix.dq", ".mix.dkv")):
+        if layer < last or k.endswith((".mix.in", ".mix.x", ".mix.dt", ".mix.dq", ".mix.dkv", ".mix.k", ".mix.v")):
             prompt += n
     head = cfg["vocab"] * cfg["width"]
     return active + head, head, prompt
 
 
 def layers_bench(args) -> None:
-    """Decode and prefill throughput of layer-list models beside the llama family at equal weights per token."""
+    """Decode and prefill throughput of the layer-list models, and of the llama family at equal weights per token."""
     from kuiperllama_amd import checkpoint
     from kuiperllama_amd.model import KuiperModel
     rows = []
     rng = np.random.default_rng(1)
-    for width, n_layers in [(int(a), int(b)) for a, b in (x.split("x") for x in args.layers.split(","))]:
-        cfg = layers_config(width, n_layers)
-        elems, head, prompt_macs = layers_work(cfg)
-        t0 = time.time()
+
+    def layer_list(cfg):
         img = checkpoint.safetensors_image(layers_tensors(cfg))
-        m = KuiperModel.from_tensors(cfg, img, max_seq_len=4352)
-        del img
-        log(f"[bench] {width} x {n_layers}: built in {time.time() - t0:.1f} s, {m.cfg.weight_bytes / 1e9:.2f} GB")
+        return KuiperModel.from_tensors(cfg, img, max_seq_len=4352)
+
+    for width, n_layers in [(int(a), int(b)) for a, b in (x.split("x") for x in args.layers.split(","))]:
+        models = []
+        for arch in ("Gusorax", "Gufanex"):
+            cfg = layers_config(width, n_layers, arch=arch)
+            elems, head, prompt_macs = layers_work(cfg)
+            models.append((arch.lower(), lambda cfg=cfg: layer_list(cfg), elems * 2.0, prompt_macs, 2.5e15))
         hidden = int(((elems - head) / n_layers - 4 * width * width) / (3 * width)) // 64 * 64
         sp = binfmt.ModelSpec(width, hidden, n_layers, width // 128, width // 128, cfg["vocab"], 4352, False,
                               name=f"llama-{width}x{n_layers}")
-        for name, mk, wbytes, peak in (("gufanex", lambda: m, 2.0, 2.5e15),
-                                       ("llama", lambda: build_model(sp, 0)[0], 4.0, 157.3e12)):
-            mm = mk()
+        # every family leaves the last layer's output projections and feed-forward out of a prompt pass
+        models.append(("llama", lambda: build_model(sp, 0)[0], sp.weight_elems() * 4.0,
+                       (n_layers - 1) * (4 * width * width + 3 * width * hidden) + 3 * width * width, 157.3e12))
+        for name, make, nbytes, macs, peak in models:
+            t0 = time.time()
+            mm = make()
+            log(f"[bench] {name} {width} x {n_layers}: built in {time.time() - t0:.1f} s, {mm.cfg.weight_bytes / 1e9:.2f} GB")
             prompt = [int(t) for t in rng.integers(0, cfg["vocab"], 4096)]
             mm.generate(prompt[:2], 32, exec="graph")
             n = args.steps
             best = min(mm.generate(prompt[:2], n, exec="graph")[1] for _ in range(3)) / n
-            nbytes = (elems if name == "gufanex" else sp.weight_elems()) * wbytes
             row = {"model": name, "width": width, "layers": n_layers, "decode_us": round(best * 1e3, 1),
                    "decode_tok_s": round(1e3 / best, 1), "weight_mb_per_token": round(nbytes / 1e6, 1),
                    "decode_frac_of_8TBs": round(nbytes / (best * 1e-3) / 8e12, 3)}
@@ -850,11 +866,8 @@ def layers_bench(args) -> None:
             for T in (512, 2048, 4096):
                 mm.time_prefill(prompt[:T], 0, mode="gemm")
                 ms = min(mm.time_prefill(prompt[:T], 0, mode="gemm") for _ in range(3))
-                # both families leave the last layer's output projections and feed-forward out of a prompt pass
-                fl = 2.0 * T * (prompt_macs if name == "gufanex" else
-                                (n_layers - 1) * (4 * width * width + 3 * width * hidden) + 3 * width * width)
                 row[f"prefill{T}_tok_s"] = round(T / ms * 1e3)
-                row[f"prefill{T}_linear_frac_of_peak"] = round(fl / (ms * 1e-3) / peak, 3)
+                row[f"prefill{T}_linear_frac_of_peak"] = round(2.0 * T * macs / (ms * 1e-3) / peak, 3)
             mm.close()
             log("[bench] " + json.dumps(row))
             rows.append(row)
@@ -865,8 +878,8 @@ def layers_bench(args) -> None:
 def main(argv=None):
     ap = argparse.ArgumentParser()
     ap.add_argument("--layers", nargs="?", const="1024x8,2048x4,4096x2", default=None, metavar="WIDTHxLAYERS,...",
-                    help="measure layer-list models (Gufanex, bf16, random weights) of these sizes beside the llama "
-                         "family at equal weights per token instead of the default workload")
+                    help="measure the layer-list models (Gusorax, Gufanex; bf16, random weights) of these sizes beside the "
+                         "llama family at equal weights per token instead of the default workload")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=128)  # generate(model, "a", 128), main.cpp:69
     ap.add_argument("--warmup", type=int, default=16)

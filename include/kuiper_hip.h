@@ -380,10 +380,11 @@ int kh_plan_prefill_shape(int32_t epi, int32_t T, int32_t rows, int32_t K, int32
  * KH_ATTN_TLONG, KH_ATTN_DEFER (0 = never merge time splits in the wo kernel), KH_ATTN_DEFER_MAX (active splits up to
  * which it does), KH_PREFILL, KH_PG_<CHUNK|SHAPE_*|SOLO|KZ|ATTN|ATTN_QT|ROPE_FUSE|DEBUG>,
  * KH_SHAPE_DEBUG, KH_HY_DECODE (0 = single-token batches of layer-list models run on the pass kernels), KH_HY_EXPAND (0 = latent
- * attention of prompts in its absorbed form)) lives in ONE process-wide key -> value table, seeded once from the KH_* variables of
+ * attention of prompts in its absorbed form), KH_HY_TMAX (tokens of one pass, 32 ... 2048), KH_HY_ROWS (16, 64 or 128: row tiles
+ * of the attention kernels of a pass)) lives in ONE process-wide key -> value table, seeded once from the KH_* variables of
  * the environment when the library is first used and changed afterwards only through kh_debug_set
  * (value NULL = unset).  No launch path reads the environment.  Hooks that shape a model (KH_SHAPE_*,
- * KH_ATTN_*) are read by kh_model_create_*; the others by the call they affect.  Keys must start with "KH_". */
+ * KH_ATTN_*, KH_HY_TMAX) are read by kh_model_create_*; the others by the call they affect.  Keys must start with "KH_". */
 int kh_debug_set(const char* key, const char* value);
 const char* kh_debug_get(const char* key); /* NULL when unset */
 int64_t kh_debug_list(char* buf, int64_t cap); /* '\n'-separated names; returns bytes needed */

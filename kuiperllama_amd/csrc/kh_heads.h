@@ -94,9 +94,11 @@ struct HeadsArgs {
   PassTabs p;
 };
 
-// KN, KV: key and value size in units of 64.  CP = 4: 16 rows per workgroup; CP = 1: 64 MR rows
+// KN, KV: key and value size in units of 64.  CP = 4: 16 rows per workgroup; CP = 1: 64 MR rows.
+// Two waves per SIMD where the accumulators allow it: within 256 registers the compiler keeps them where the rescaling can
+// reach them (beyond, it moves them between two register files in every tile).
 template <class T, int KN, int KV, int CP, int MR>
-__global__ __launch_bounds__(256) void k_heads_attn(const HeadsArgs a) {
+__global__ __launch_bounds__(256, KN + KV > 4 ? 1 : 2) void k_heads_attn(const HeadsArgs a) {
   typedef Tile<T> TL;
   typedef typename TL::frag frag;
   constexpr int E = TL::N, KT = 4 * E, NS = KT / 16, ES = (int)sizeof(T);
@@ -106,17 +108,19 @@ __global__ __launch_bounds__(256) void k_heads_attn(const HeadsArgs a) {
   extern __shared__ __attribute__((aligned(1024))) char smem_raw[];
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int fr = lane & 15, fh = lane >> 4, wr = wave % WR, wc = wave / WR;
-  const int g = blockIdx.y, per = a.H / a.G;
+  const int g = blockIdx.x, per = a.H / a.G;
   LatTile tl;
   int n_rows, row0;
   if (a.tiles) {
-    tl = a.tiles[blockIdx.x];
+    // longest key ranges first; a launch of at most two workgroups per CU pairs the longest with the shortest instead
+    const int nt = (int)gridDim.y, half = (nt + 1) >> 1, y = (int)blockIdx.y;
+    tl = a.tiles[nt * a.G <= 512 && y >= half ? nt - 1 - (y - half) : y];
     n_rows = a.p.seg_n[tl.seg] * per;
     row0 = a.p.seg_row0[tl.seg];
   } else {
     const int nt = (per + ROWS - 1) / ROWS;
-    tl.seg = (int)blockIdx.x / nt;
-    tl.r0 = ((int)blockIdx.x - tl.seg * nt) * ROWS;
+    tl.seg = (int)blockIdx.y / nt;
+    tl.r0 = ((int)blockIdx.y - tl.seg * nt) * ROWS;
     n_rows = per;
     row0 = tl.seg;
   }
@@ -253,6 +257,9 @@ __global__ __launch_bounds__(256) void k_heads_attn(const HeadsArgs a) {
         const int k = n * 16 + fr;
         fk[b][n] = *(const frag*)(Kt + ((size_t)k * CB + ((4 * b + fh) ^ (k & 7))) * 16);
       }
+    frag fv[NT];  // requested with the keys: they arrive under the scores and the softmax
+#pragma unroll
+    for (int n = 0; n < NT; ++n) fv[n] = lat_col<CB>(Kt, DK + (wc * NT + n) * 16, lane, T());
 #pragma unroll
     for (int b = 0; b < NQ; ++b)
 #pragma unroll
@@ -265,21 +272,16 @@ __global__ __launch_bounds__(256) void k_heads_attn(const HeadsArgs a) {
     const bool near = a.bias && p_lo - (k0 + KT - 1) < a.nbias - 1;
 #pragma unroll
     for (int q = 0; q < MR; ++q) {
-      if (near) {
-        const float *bt = tab + (head[q] - g * per) * a.nbias, *bg = a.bias + (size_t)head[q] * a.nbias;
+      if (near) {  // two loads of known address space, not one of a selected address
+        const int d0 = my_pos[q] - k0 - 4 * fh;
+        auto add = [&](const float* row) __attribute__((always_inline)) {
 #pragma unroll
-        for (int n = 0; n < NS; ++n)
+          for (int n = 0; n < NS; ++n)
 #pragma unroll
-          for (int i = 0; i < 4; ++i) {
-            int d = my_pos[q] - (k0 + 16 * n + 4 * fh + i);
-            d = d < 0 ? 0 : (d < a.nbias ? d : a.nbias - 1);
-            s[q][n][i] += a.bias_lds ? bt[d] : bg[d];
-          }
-      } else if (a.bias) {
-#pragma unroll
-        for (int n = 0; n < NS; ++n)
-#pragma unroll
-          for (int i = 0; i < 4; ++i) s[q][n][i] += far[q];
+            for (int i = 0; i < 4; ++i) s[q][n][i] += row[min(max(d0 - 16 * n - i, 0), a.nbias - 1)];
+        };
+        if (a.bias_lds) add(tab + (head[q] - g * per) * a.nbias);
+        else add(a.bias + (size_t)head[q] * a.nbias);
       }
       if (edge) {
 #pragma unroll
@@ -290,11 +292,13 @@ __global__ __launch_bounds__(256) void k_heads_attn(const HeadsArgs a) {
             s[q][n][i] = k <= my_pos[q] && k >= my_first[q] && k < k_hi ? s[q][n][i] : -INFINITY;
           }
       }
+      const float add = near ? 0.f : far[q];  // the same for every key of a far tile: joins the maximum
       float mx = s[q][0][0];
 #pragma unroll
       for (int n = 0; n < NS; ++n)
 #pragma unroll
         for (int i = 0; i < 4; ++i) mx = fmaxf(mx, s[q][n][i]);
+      mx += add;
       // the running maximum rarely moves after the first tiles: rescale only when some row's does
       if (__any(mx > m[q])) {
         mx = fmaxf(mx, m[q]);
@@ -308,23 +312,22 @@ __global__ __launch_bounds__(256) void k_heads_attn(const HeadsArgs a) {
 #pragma unroll
           for (int i = 0; i < 4; ++i) o[q][n][i] *= f;
       }
+      const float base = m[q] - add;
       float sum = 0.f;
 #pragma unroll
       for (int n = 0; n < NS; ++n)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const float e = __builtin_amdgcn_exp2f(s[q][n][i] - m[q]);
+          const float e = __builtin_amdgcn_exp2f(s[q][n][i] - base);
           sum += e;
           p[q][4 * n + i] = (T)e;
         }
       l[q] += sum;
     }
 #pragma unroll
-    for (int n = 0; n < NT; ++n) {
-      const frag fv = lat_col<CB>(Kt, DK + (wc * NT + n) * 16, lane, T());
+    for (int n = 0; n < NT; ++n)
 #pragma unroll
-      for (int q = 0; q < MR; ++q) o[q][n] = TL::mma(fv, p[q], o[q][n]);
-    }
+      for (int q = 0; q < MR; ++q) o[q][n] = TL::mma(fv[n], p[q], o[q][n]);
   }
 #pragma unroll
   for (int q = 0; q < MR; ++q) {

@@ -27,7 +27,7 @@ int heads_attn_launch(hipStream_t s, HeadsArgs a, int ntiles, int rows) {
         done.push_back({dev, (const void*)kern, lds});
       }
     }
-    hipLaunchKernelGGL(kern, dim3(ntiles, a.G, a.nsplit), dim3(256), lds, s, a);
+    hipLaunchKernelGGL(kern, dim3(a.G, ntiles, a.nsplit), dim3(256), lds, s, a);
     return KH_OK;
   };
   auto by_rows = [&](auto kn, auto kv) -> int {

@@ -78,7 +78,8 @@ int row_tiles(const std::vector<int32_t>& seg_n, const RowKind& kind, std::vecto
     t64 += ((long)n * kind.per + 63) / 64;
     big += ((long)n * kind.per + kind.big - 1) / kind.big;
   }
-  const int step = t64 * 64 > 2 * rows ? 16 : (kind.big > 64 && big * kind.lanes < 512 ? 64 : kind.big);
+  int step = t64 * 64 > 2 * rows ? 16 : (kind.big > 64 && big * kind.lanes < 512 ? 64 : kind.big);
+  if (const char* e = dbg("KH_HY_ROWS")) step = atoi(e) == 16 ? 16 : std::min(atoi(e) == 128 ? 128 : 64, kind.big);
   tab->clear();
   for (size_t s = 0; s < seg_n.size(); ++s)
     for (int r = (seg_n[s] * kind.per - 1) / step * step; r >= 0; r -= step) {  // the longest key ranges first

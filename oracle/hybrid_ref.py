@@ -136,11 +136,9 @@ def heads(W, p, h, n, d):
 
 def softmax_extra(s, extra):
     """Rows of s [T, H, T] over the last axis with the constant `extra` in the denominator, in units of exp(0)."""
-    m = s.max(axis=-1)
-    if extra:
-        m = np.maximum(m, 0.0)
+    m = np.maximum(s.max(axis=-1), 0.0 if extra else -np.inf)
     e = np.exp(s - m[..., None])
-    return e / (e.sum(axis=-1) + extra * np.exp(-m))[..., None]
+    return e / (e.sum(axis=-1) + (extra * np.exp(-m) if extra else 0.0))[..., None]
 
 
 def grouped_attention(W, p, m, h, eps, seen, bias=None, extra=0.0, gate=False):

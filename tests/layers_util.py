@@ -37,6 +37,40 @@ def config(layers, width=88, vocab=101, eps=3e-5, cap=20.0, loop=None):
     return copy.deepcopy(c)
 
 
+def windowed(heads=6, kv_heads=2, dim=20, vdim=28, scale=0.3, window=11, rows=12, far=30.0):
+    return {"type": "attention", "mlp": None,
+            "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale, "mask": {"size": window},
+                      "rel_rows": rows, "bias_max": far}}
+
+
+def chunked(heads=4, kv_heads=2, dim=24, vdim=18, scale=0.25, chunk=19):
+    return {"type": "attention_2", "mlp": None,
+            "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale, "mask": {"size": chunk}}}
+
+
+def dense(ff=40):
+    return {"kind": "dense", "ff": ff}
+
+
+def clamped(experts=7, top=2, ff=24, limit=0.8):
+    return {"kind": "moe", "expert": {"ff": ff, "limit": limit}, "router": {"experts": experts, "top": top}}
+
+
+def gusorax(layers, width=72, vocab=93, eps=2e-4, mult=0.45, scale=6.5, positions=700, loop=None):
+    c = {"architecture": "Gusorax", "layers": layers, "width": width, "vocab": vocab, "norm": {"eps": eps}, "residual_mult": mult,
+         "embedding": {"scale": scale}, "max_positions": positions}
+    if loop is not None:
+        c["loop"] = dict(zip(("start", "stop", "times"), loop))
+    return copy.deepcopy(c)
+
+
+def heads_mixed(**kw):
+    """Both attention mixers, every feed-forward and none, a loop in the middle."""
+    return gusorax([dict(windowed(), mlp=dense()), dict(chunked(), mlp=clamped()), windowed(3, 3, 9, 40, 0.5, 33, 8, 20.0),
+                    dict(chunked(5, 1, 33, 7, 0.2, 40), mlp=clamped(4, 4, 10, 0.3)), dict(windowed(window=70), mlp=clamped(9, 1, 33))],
+                   loop=kw.pop("loop", (1, 4, 2)), **kw)
+
+
 def mixed(**kw):
     """Every mechanism and branch once: both mixers, with and without feed-forward, a loop in the middle."""
     return config([with_ff(mamba()), with_ff(latent()), mamba(40, 17, 3, 3), with_ff(latent(2, 36, 8, 16, 70, 50, 0.4), identity=0,

@@ -2,11 +2,12 @@
 """One workload of a layer-list model for rocprofv3, and the per-kernel summary of its trace.
 
     rocprofv3 --kernel-trace --stats -d OUT -o t -- python3 tools/layers_profile.py 2048 4 prefill 2048
-    rocprofv3 ...                                -- python3 tools/layers_profile.py 2048 4 decode 4096 [--llama]
+    rocprofv3 ...                                -- python3 tools/layers_profile.py 2048 4 decode 4096 [--gusorax | --llama]
     python3 tools/layers_profile.py --report OUT/t_results.db
 
 decode T: eager fused steps at positions T ... T + 63 (T <= 2: from an empty sequence); prefill T: four passes of a
-T-token prompt.  --llama: the llama-family model of equal weights per token (bench.py --layers).
+T-token prompt.  Default: the Gufanex model of bench.py --layers; --gusorax: the Gusorax one; --llama: the llama-family
+model of equal weights per token.
 """
 import os
 import sqlite3
@@ -33,7 +34,7 @@ def main() -> None:
     from kuiperllama_amd import binfmt, checkpoint
     from kuiperllama_amd.model import KuiperModel
     width, layers, mode, T = int(sys.argv[1]), int(sys.argv[2]), sys.argv[3], int(sys.argv[4])
-    cfg = bench.layers_config(width, layers)
+    cfg = bench.layers_config(width, layers, arch="Gusorax" if "--gusorax" in sys.argv else "Gufanex")
     if "--llama" in sys.argv:
         elems, head, _ = bench.layers_work(cfg)
         hidden = int(((elems - head) / layers - 4 * width * width) / (3 * width)) // 64 * 64
