@@ -1,9 +1,10 @@
 // kh_hybrid_load.hip — layer-list models: registry, config.json, model.safetensors -> padded weight rows in one HBM
-// arena, and the state manager (recurrent state and latent cache of every sequence slot).
+// arena, and the state manager (recurrent state, latent and key / value cache of every sequence slot).
 //
 // Weight rows are re-laid once at load for the kernels that read them: row lengths padded to KH_LPAD elements with
-// zeros, matrices that share an input stacked (router + shared gate; query and key/value down-projections), gate and
-// up rows interleaved in groups of 16, W_uk transposed per head, heads padded to KH_LPAD.
+// zeros, matrices that share an input stacked (router + shared gate; query and key/value down-projections; query, key,
+// value and gate heads), gate and up rows interleaved in groups of 16, W_uk transposed per head, latent heads padded to
+// KH_LPAD, plain heads to 16 rows.  A learned distance bias becomes a table by distance.
 #include <fcntl.h>
 #include <math.h>
 #include <stdio.h>

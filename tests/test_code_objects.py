@@ -1,8 +1,8 @@
 """The gfx950 code objects inside the built library: no kernel may use scratch memory (a register spill in a
 latency-bound decode kernel is a memory round trip per use), and the kernels the decode step launches exist.
 Reads the .hip_fatbin section of kuiperllama_amd/lib/libkuiper_hip.so with the LLVM tools of the ROCm install (no GPU).
-Round 6 found 20-24 bytes of scratch in six k_wo_comb instantiations after a branch had been removed from their
-merge loop (the compiler hoisted every factor read and crossed the 128-register cap): this test is the tripwire."""
+Six k_wo_comb instantiations once took 20-24 bytes of scratch after a branch had been removed from their merge loop (the
+compiler hoisted every factor read and crossed the 128-register cap): this test is the tripwire."""
 import os
 import re
 import shutil
@@ -61,5 +61,5 @@ def test_no_kernel_uses_scratch_and_step_kernels_exist():
     spilled = {k: v for k, v in kernels.items() if v}
     assert not spilled, f"kernels with scratch (bytes): {spilled}"
     for stem in ("k_qkv", "k_attn_decode", "k_gemv_res", "k_wo_comb", "k_ffn13", "k_ffn13_ring", "k_cls", "k_cls_ring",
-                 "k_sample", "k_pg_gemm", "k_pg_attn"):
+                 "k_sample", "k_pg_gemm", "k_pg_attn", "k_heads_attn", "k_heads_rows", "k_ld_merge", "k_ld_enter"):
         assert any(stem in k for k in kernels), f"no {stem} instantiation in the library"
