@@ -235,7 +235,8 @@ __global__ __launch_bounds__(256) void k_lgemm(const LgArgs a) {
   }
 }
 
-// Tile choice.  Plain / batched launches: the largest tile that still gives the chip enough workgroups.  Grouped
+// Tile choice.  Plain / batched launches: the largest tile that still gives the chip enough workgroups (one per CU is
+// not: nobody covers its barriers).  Grouped
 // launches: BM = the row granule the tile list was built with (lg_group_bm).
 static inline int lg_group_bm(long rows, int groups) {
   const long per = rows / (groups > 0 ? groups : 1);
@@ -265,7 +266,7 @@ int lg_launch(hipStream_t s, const LgArgs& a, int zdim = 1, int group_bm = 0, in
   if (a.tiles ? group_bm == 128 : a.M > 64 && tiles(128, 128) >= 400)
     return go(k_lgemm<T, 128, 128, EPI>, 128, 128, LgCfg<T, 128, 128>::LDS);
   if (a.tiles ? group_bm == 32 : a.M <= 32) return go(k_lgemm<T, 32, 64, EPI>, 32, 64, LgCfg<T, 32, 64>::LDS);
-  if (a.tiles || tiles(64, 128) >= 256) return go(k_lgemm<T, 64, 128, EPI>, 64, 128, LgCfg<T, 64, 128>::LDS);
+  if (a.tiles || tiles(64, 128) >= 400) return go(k_lgemm<T, 64, 128, EPI>, 64, 128, LgCfg<T, 64, 128>::LDS);
   return go(k_lgemm<T, 64, 64, EPI>, 64, 64, LgCfg<T, 64, 64>::LDS);
 }
 }  // namespace khm
